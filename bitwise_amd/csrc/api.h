@@ -112,10 +112,13 @@ int bw_norm_shift(const float* x, int ldx, const float* w, const float* mix, flo
 // with normaliser and running maximum.  state: [slots, state_ld] of S [heads][dim][vdim] (mode 1: then n [heads][dim], m [heads]).
 // mode 2: a decay per key channel exp(-exp(logit + bias)), the read-out taken before the update with the token's own
 // k v^T weighted by bias2 [heads*dim]; mode 3: one constant decay a head, bias [heads] (gate is not read).
-// q is multiplied by qscale, k by kscale.
+// mode 4: a step size per head, delta = softplus(logit at gate_off + head + bias[head]); decay exp(-bias2[head] delta), the
+// token enters as k (delta v)^T, skip[head] v (optional) joins the read-out.
+// q is multiplied by qscale, k by kscale; heads_per_key neighbouring heads share one q and one k.
 int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_off, int k_off, int v_off, const float* gate, int ldg,
                          int gate_off, int gate2_off, const float* bias, const float* bias2, float param, float qscale,
-                         float kscale, float* state, long long state_ld, float* out, int ldo, const int32_t* seq_rows,
+                         float kscale, const float* skip, int heads_per_key, float* state, long long state_ld, float* out,
+                         int ldo, const int32_t* seq_rows,
                          const int32_t* slots, const int32_t* positions, int nseq, int heads, int dim, int vdim,
                          const int32_t* chunks, int nchunks, const int32_t* spans, int nspans, float* scan_local,
                          float* scan_start, long long scan_floats, void* stream);
@@ -125,6 +128,12 @@ int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_off, int k_
 int bw_rotate_halves_rows(float* x, int ldx, int rows, int heads, int dim, int rot, int sections, int off0, int off1,
                           const float* cos_table, const float* sin_table, const int32_t* positions, void* stream);
 int bw_tanh_rows(float* x, int ld, int rows, int cols, void* stream);      // x <- tanh(x)
+// v = o * silu(z), each of a row's ``parts`` stretches of ``size`` elements divided by its own root mean square, times weight
+int bw_gated_part_norm(const float* o, int ldi, const float* z, int ldz, const float* weight, void* out, int out_is_bf16,
+                       int ldo, const int32_t* positions, int rows, int parts, int size, float eps, void* stream);
+// out = act(x); act 0: max(x, 0)^2, 1: x > 0: p0 x^2 + x/2, else (1/2 + p1) (e^x - 1 - x) + x/2
+int bw_activate(const float* x, int ldx, void* out, int out_is_bf16, int ldo, int rows, int cols, int act, float p0, float p1,
+                void* stream);
 int bw_head_norm_gate(const float* o, int ldi, const float* weight, int wstride, const float* g, int ldg, int gate, void* out,
                       int out_is_bf16, int ldo, const int32_t* positions, int rows, int heads, int vdim, float eps,
                       void* stream);
@@ -134,13 +143,19 @@ int bw_head_norm_gate(const float* o, int ldi, const float* weight, int wstride,
 int bw_glu(const float* gate_up, int ldg, void* h, int out_is_bf16, int rows, int inter, int act, float limit, float alpha,
            const float* row_gate, int ld_row_gate, void* stream);
 // Attention over a compressed cache shared by all heads (latent_attention.hip).
+// pairs 1: a rotated part's pairs are (2i, 2i+1) instead of (i, i + rotary/2).  q_rank > 0: the queries' own latent lies at
+// q_off and is normed into cq [rows, ldcq] (in the dtype qa_is_bf16 names); qa is not written.
 int bw_latent_prep(const float* proj, int ldp, int q_off, int dkv_off, const float* norm_w, float eps,
                    const float* cos_table, const float* sin_table, const int32_t* positions, const int32_t* row_seq,
                    const int32_t* block_table, int table_stride, void* cache, void* latent_t, int cache_is_bf16, void* qa, int qa_is_bf16, int ldqa,
-                   int rows, int heads, int dim, int rot, int rotary, int rank, int page_size, int write_cache,
-                   void* stream);
+                   int rows, int heads, int dim, int rot, int rotary, int rank, int page_size, int write_cache, int pairs,
+                   int q_rank, const float* q_norm_w, void* cq, int ldcq, void* stream);
+// gate (optional): head h's outputs are multiplied by sigmoid(gate[r * ldg + h]).  rot_n > 0: beside the product, the rot_n
+// elements at x[r][h*xhs + rot_src ..] are rotated at the row's position and stored at out[r][h*ohs + rot_dst ..].
 int bw_headwise_linear(const float* x, int ldx, int xhs, const void* wt, int w_is_bf16, int in, int outn, void* out,
-                       int out_is_bf16, int ldo, int ohs, int rows, int heads, void* stream);
+                       int out_is_bf16, int ldo, int ohs, int rows, int heads, const float* gate, int ldg, int rot_n,
+                       int rotary, int pairs, int rot_src, int rot_dst, const float* cos_table, const float* sin_table,
+                       const int32_t* positions, void* stream);
 int bw_shared_key_attention(const float* q, int ldq, const int32_t* positions, const int32_t* block_table,
                             int table_stride, const int32_t* tiles, int num_tiles, const void* cache, int cache_is_bf16,
                             int num_pages, const float* sink, float* out, int ldo, int heads, int dk, int dv,
@@ -155,7 +170,7 @@ int bw_shared_key_attention_mfma(const void* q, int ldq, const int32_t* position
 // above): a score per head that joins the softmax's denominator and has no value, or null.
 int bw_causal_conv(const float* x, int ldx, const float* in_bias, const void* w, const void* bias, int w_is_bf16, int taps, int channels,
                    float* state, long long state_ld, const int32_t* seq_rows, const int32_t* slots,
-                   const int32_t* positions, int nseq, int max_seq_rows, float* out, int ldo, void* stream);
+                   const int32_t* positions, int nseq, int max_seq_rows, float* out, int ldo, int silu, void* stream);
 int bw_pair_rope_unit(const float* src, int lds, const int32_t* positions, const int32_t* row_seq,
                       const int32_t* block_table, int table_stride, const float* cos_table, const float* sin_table,
                       void* q_out, void* k_cache, void* v_cache, int is_bf16, int rows, int heads, int kv_heads,
@@ -202,13 +217,17 @@ int bw_moe_route(const float* logits, int ld, int rows, int experts, int top, in
 int bw_moe_route_plan(const float* logits, int ld, int rows, int experts, int top, int groups, int keep, float weight_scale,
                       int score_kind, const float* correction, int group_best, int32_t* ids, float* wts, int32_t* sorted,
                       int32_t* place, int32_t* tiles, int32_t* meta, void* stream);
+// no router: row r's experts are table[token of r] ([vocab, top]), each weighs ``weight``; ids, wts and the plan in one launch
+int bw_moe_table_plan(const int32_t* tokens, const int32_t* feedback, int rows, const int32_t* table, int vocab, int top,
+                      int experts, float weight, int32_t* ids, float* wts, int32_t* sorted, int32_t* place, int32_t* tiles,
+                      int32_t* meta, void* stream);
 int bw_moe_max_tiles(int slots, int experts);
 int bw_moe_plan(const int32_t* ids, int slots, int experts, int32_t* sorted, int32_t* place, int32_t* tiles,
                 int32_t* meta, void* stream);
 int bw_moe_experts(const void* x, int x_is_bf16, int ldx, int x_rows, const void* w, int w_is_bf16, void* out, int ldo,
                    const int32_t* sorted, const int32_t* tiles, const int32_t* meta, int slots, int max_tiles, int top,
-                   int K, int N, int gate_up, float limit, float alpha, int round_out, void* stream);
-// (gate_up's activation: limit > 0: g = min(G, limit), u = clamp(U, -limit, limit), h = g sigmoid(alpha g) (u + 1);
+                   int K, int N, int form, float limit, float alpha, int round_out, void* stream);
+// (form 0: the down product; 1: gate and up stacked; 2: up without a gate, max(U, 0)^2.  The gated form's activation: limit > 0: g = min(G, limit), u = clamp(U, -limit, limit), h = g sigmoid(alpha g) (u + 1);
 // limit = 0: h = G sigmoid(alpha G) U)
 int bw_moe_tile_rows(int slots);
 int bw_moe_combine(const float* y, int ldy, const int32_t* place, const float* wts, int top, float* out, int ldo,

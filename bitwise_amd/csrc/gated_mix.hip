@@ -1,7 +1,7 @@
 // Kernels around mixers that convolve their projections over a few tokens, gate their outputs, or carry a
 // gated linear recurrence per channel; and the small row operations of a layer whose norm sits behind the sublayer.
 //
-//   causal_conv:   y_t[c] = sum_j w[c][j] * u_(t - taps + 1 + j)[c] (+ bias[c]); the last taps-1 inputs of every request
+//   causal_conv:   y_t[c] = sum_j w[c][j] * u_(t - taps + 1 + j)[c] (+ bias[c]), optionally through SiLU; the last taps-1 inputs of every request
 //                  live in its state slot, so a portion of any length continues where the last one stopped
 //   pair_rope_unit: rotation of neighbouring pairs (2i, 2i+1) of the first rot elements of each head at the row's
 //                  position, optional division by the head's root mean square, the cache write (keys and values padded
@@ -44,6 +44,7 @@ struct ConvArgs {
   const int32_t* positions;
   long long state_ld;
   int ldx, ldo, channels;
+  int silu;              // 1: every output goes through SiLU
 };
 
 template <int TAPS, typename WT>
@@ -81,6 +82,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(ConvArgs a) {
     }
     acc = fmaf(w[TAPS - 1], cur, acc);
     if (a.bias != nullptr) acc += bias;
+    if (a.silu) acc *= gm_sigmoid(acc);
     o[(size_t)t * a.ldo] = acc;
     if constexpr (TAPS > 1) {
 #pragma unroll
@@ -116,10 +118,10 @@ static int conv_launch(const ConvArgs& a, int taps, dim3 grid, hipStream_t s) {
 
 extern "C" int bw_causal_conv(const float* x, int ldx, const float* in_bias, const void* w, const void* bias, int w_is_bf16, int taps, int channels,
                               float* state, long long state_ld, const int32_t* seq_rows, const int32_t* slots,
-                              const int32_t* positions, int nseq, int max_seq_rows, float* out, int ldo, void* stream) {
+                              const int32_t* positions, int nseq, int max_seq_rows, float* out, int ldo, int silu, void* stream) {
   if (nseq <= 0 || channels <= 0 || max_seq_rows <= 0) return 0;
   if (taps < 1 || taps > CONV_MAX_TAPS || (taps > 1 && state == nullptr)) return -2;
-  ConvArgs a{x, w, bias, in_bias, state, out, seq_rows, slots, positions, state_ld, ldx, ldo, channels};
+  ConvArgs a{x, w, bias, in_bias, state, out, seq_rows, slots, positions, state_ld, ldx, ldo, channels, silu};
   const dim3 grid((channels + 255) / 256, nseq, (max_seq_rows + CONV_CHUNK - 1) / CONV_CHUNK);
   if (grid.y > 65535 || grid.z > 65535) return -2;
   return w_is_bf16 ? conv_launch<bf16_t>(a, taps, grid, (hipStream_t)stream) : conv_launch<float>(a, taps, grid, (hipStream_t)stream);

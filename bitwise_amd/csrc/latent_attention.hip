@@ -5,8 +5,10 @@
 // values afterwards: the cache is read once for all heads of a row tile.
 //
 //   latent_prep:         RMSNorm of the latent, rotation of the shared key part and of the queries' rotated
-//                        parts, cache write.
-//   headwise_linear:     out[r][h] = W[h] x[r][h], a product per head with weights of its own.
+//                        parts, cache write; where the queries go through a latent of their own, its RMSNorm
+//                        instead of the queries' rotation.
+//   headwise_linear:     out[r][h] = W[h] x[r][h], a product per head with weights of its own, optionally times a
+//                        sigmoid gate per head, optionally with the rotation of a query part beside it.
 //   shared_key_attention: causal softmax attention of all heads over the shared keys, values a prefix of
 //                        the key vector, with an optional sink per head in the denominator and an optional window.
 //
@@ -32,6 +34,20 @@ __device__ __forceinline__ void store_f(T* p, float v) {
 
 // ------------------------------------------------------------------------- prep
 
+// A rotated part's element i: of its first ``rotary`` elements, i and i + rotary/2 are a pair (pairs 0), or 2k and 2k + 1
+// (pairs 1), turned by column (i mod rotary/2, or k) of the position's row of the tables; the rest pass unchanged.
+__device__ __forceinline__ float rotated_element(const float* __restrict__ x, int i, int rotary, int pairs, const float* __restrict__ ct,
+                                                 const float* __restrict__ st) {
+  const int half = rotary / 2;
+  if (i >= rotary) return x[i];
+  if (pairs) {
+    const int k = i >> 1;
+    return (i & 1) ? x[i] * ct[k] + x[i - 1] * st[k] : x[i] * ct[k] - x[i + 1] * st[k];
+  }
+  if (i < half) return x[i] * ct[i] - x[i + half] * st[i];
+  return x[i] * ct[i - half] + x[i - half] * st[i - half];
+}
+
 struct PrepArgs {
   const float* proj;     // [rows, ldp]: q at q_off (heads x (dim + rot)), the down projection at dkv_off (rank + rot)
   int ldp, q_off, dkv_off;
@@ -45,11 +61,15 @@ struct PrepArgs {
   int table_stride;
   void* qa;              // [rows, ldqa] (32-bit, or bfloat16 for the matrix-core attention): head h at h * (rank + rot); the
   int ldqa, qa_is_bf16;  // rotated part goes to its last rot elements
-  int heads, dim, rot, rotary, rank, page_size, write_cache;
+  int heads, dim, rot, rotary, rank, page_size, write_cache, pairs;
+  // queries that go through a latent of their own (q_rank > 0; qa is not written then): the latent at q_off, normed into cq
+  int q_rank;
+  const float* q_norm_w;    // [q_rank]
+  void* cq;                 // [rows, ldcq] in the queries' dtype (qa_is_bf16)
+  int ldcq;
 };
 
-// A workgroup a row.  The rotated part: elements i and i + rotary/2 (i < rotary/2) are a pair; elements from
-// ``rotary`` on pass unchanged.
+// A workgroup a row.
 template <typename CT>
 __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a, CT* __restrict__ cache, CT* __restrict__ latent_t) {
   const int row = blockIdx.x;
@@ -75,22 +95,25 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a, CT* __rest
       for (int i = threadIdx.x; i < a.rank; i += blockDim.x) store_f(tp + (size_t)i * a.page_size, (dkv[i] * inv) * a.norm_w[i]);
     }
     const float* kr = dkv + a.rank;
-    for (int i = threadIdx.x; i < a.rot; i += blockDim.x) {
-      float v;
-      if (i < half) v = kr[i] * ct[i] - kr[i + half] * st[i];
-      else if (i < a.rotary) v = kr[i] * ct[i - half] + kr[i - half] * st[i - half];
-      else v = kr[i];
-      store_f(dst + a.rank + i, v);
+    for (int i = threadIdx.x; i < a.rot; i += blockDim.x) store_f(dst + a.rank + i, rotated_element(kr, i, a.rotary, a.pairs, ct, st));
+  }
+  if (a.q_rank > 0) {
+    const float* ql = pr + a.q_off;
+    float acc = 0.0f;
+    for (int i = lane; i < a.q_rank; i += 64) acc = fmaf(ql[i], ql[i], acc);
+    const float inv = 1.0f / sqrtf(wave_sum(acc) / (float)a.q_rank + a.eps);
+    for (int i = threadIdx.x; i < a.q_rank; i += blockDim.x) {
+      const float v = (ql[i] * inv) * a.q_norm_w[i];
+      const size_t at = (size_t)row * a.ldcq + i;
+      if (a.qa_is_bf16) reinterpret_cast<bf16_t*>(a.cq)[at] = f32_to_bf16(v);
+      else reinterpret_cast<float*>(a.cq)[at] = v;
     }
+    return;
   }
   const int per = a.dim + a.rot;
   for (int e = threadIdx.x; e < a.heads * a.rot; e += blockDim.x) {
     const int h = e / a.rot, i = e % a.rot;
-    const float* qr = pr + a.q_off + h * per + a.dim;
-    float v;
-    if (i < half) v = qr[i] * ct[i] - qr[i + half] * st[i];
-    else if (i < a.rotary) v = qr[i] * ct[i - half] + qr[i - half] * st[i - half];
-    else v = qr[i];
+    const float v = rotated_element(pr + a.q_off + h * per + a.dim, i, a.rotary, a.pairs, ct, st);
     const size_t at = (size_t)row * a.ldqa + h * width + a.rank + i;
     if (a.qa_is_bf16) reinterpret_cast<bf16_t*>(a.qa)[at] = f32_to_bf16(v);
     else reinterpret_cast<float*>(a.qa)[at] = v;
@@ -104,14 +127,37 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a, CT* __rest
 // per output, i ascending.
 // A workgroup is 64 outputs by four quarters of the inner size (a wave a quarter, eight weights asked for at a time); the
 // quarters' sums meet in LDS and are added in quarter order.
+// gate (optional): the outputs of head h are multiplied by sigmoid(gate[r][h]).  rot (optional): the workgroups of an extra
+// block of outputs write, for their rows and head, the rotated ``n`` elements at x[.. + src] to out[.. + dst].
+struct HeadExtras {
+  const float* gate;
+  int ldg;
+  int rot_n, rotary, pairs, src, dst;
+  const float* cos_table;
+  const float* sin_table;
+  const int32_t* positions;
+};
+
 #define HL_ROWS 8
 template <typename WT, typename OT>
 __global__ __launch_bounds__(256) void headwise_linear_kernel(const float* __restrict__ x, int ldx, int xhs,
                                                               const WT* __restrict__ wt, int in, int outn,
-                                                              OT* __restrict__ out, int ldo, int ohs, int rows) {
+                                                              OT* __restrict__ out, int ldo, int ohs, int rows, HeadExtras ex) {
   extern __shared__ float hl_x[];      // [HL_ROWS][in], then [4][HL_ROWS][64] partial sums
   float* hl_part = hl_x + HL_ROWS * in;
   const int r0 = blockIdx.x * HL_ROWS, h = blockIdx.y;
+  if ((int)blockIdx.z * 64 >= outn) {      // the extra block
+    const int half = ex.rotary / 2;
+    for (int e = threadIdx.x; e < HL_ROWS * ex.rot_n; e += 256) {
+      const int r = r0 + e / ex.rot_n, i = e % ex.rot_n;
+      const int pos = r < rows ? ex.positions[r] : -1;
+      if (pos < 0) continue;
+      store_f(out + (size_t)r * ldo + h * ohs + ex.dst + i,
+              rotated_element(x + (size_t)r * ldx + h * xhs + ex.src, i, ex.rotary, ex.pairs, ex.cos_table + (size_t)pos * half,
+                              ex.sin_table + (size_t)pos * half));
+    }
+    return;
+  }
   const int lane = threadIdx.x & 63, quarter = wave_index();
   const int o = blockIdx.z * 64 + lane;
   for (int e = threadIdx.x; e < HL_ROWS * in; e += 256) {
@@ -145,7 +191,9 @@ __global__ __launch_bounds__(256) void headwise_linear_kernel(const float* __res
   for (int r = 0; r < HL_ROWS; ++r) {
     const float sum = ((hl_part[r * 64 + lane] + hl_part[(HL_ROWS + r) * 64 + lane]) + hl_part[(2 * HL_ROWS + r) * 64 + lane]) +
                       hl_part[(3 * HL_ROWS + r) * 64 + lane];
-    if (r0 + r < rows) store_f(out + (size_t)(r0 + r) * ldo + h * ohs + o, sum);
+    if (r0 + r >= rows) continue;
+    const float gate = ex.gate != nullptr ? 1.0f / (1.0f + bw_expf(-ex.gate[(size_t)(r0 + r) * ex.ldg + h])) : 1.0f;
+    store_f(out + (size_t)(r0 + r) * ldo + h * ohs + o, sum * gate);
   }
 }
 
@@ -622,12 +670,13 @@ extern "C" int bw_latent_prep(const float* proj, int ldp, int q_off, int dkv_off
                               const float* cos_table, const float* sin_table, const int32_t* positions,
                               const int32_t* row_seq, const int32_t* block_table, int table_stride, void* cache,
                               void* latent_t, int cache_is_bf16, void* qa, int qa_is_bf16, int ldqa, int rows, int heads, int dim, int rot, int rotary,
-                              int rank, int page_size, int write_cache, void* stream) {
+                              int rank, int page_size, int write_cache, int pairs, int q_rank,
+                              const float* q_norm_w, void* cq, int ldcq, void* stream) {
   if (rows <= 0) return 0;
   if (heads <= 0 || dim < 0 || rot < 0 || rotary < 0 || rotary > rot || (rotary & 1) || rank <= 0 || page_size <= 0) return -2;
-  if (ldqa < heads * (rank + rot)) return -2;
+  if (q_rank < 0 || (q_rank > 0 ? (cq == nullptr || q_norm_w == nullptr || ldcq < q_rank) : ldqa < heads * (rank + rot))) return -2;
   PrepArgs a{proj, ldp, q_off, dkv_off, norm_w, eps, cos_table, sin_table, positions, row_seq, block_table, table_stride,
-             qa, ldqa, qa_is_bf16, heads, dim, rot, rotary, rank, page_size, write_cache};
+             qa, ldqa, qa_is_bf16, heads, dim, rot, rotary, rank, page_size, write_cache, pairs, q_rank, q_norm_w, cq, ldcq};
   hipStream_t s = (hipStream_t)stream;
   if (cache_is_bf16) hipLaunchKernelGGL(latent_prep_kernel<bf16_t>, dim3(rows), dim3(256), 0, s, a, (bf16_t*)cache, (bf16_t*)latent_t);
   else hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(rows), dim3(256), 0, s, a, (float*)cache, (float*)latent_t);
@@ -635,27 +684,29 @@ extern "C" int bw_latent_prep(const float* proj, int ldp, int q_off, int dkv_off
 }
 
 extern "C" int bw_headwise_linear(const float* x, int ldx, int xhs, const void* wt, int w_is_bf16, int in, int outn,
-                                  void* out, int out_is_bf16, int ldo, int ohs, int rows, int heads, void* stream) {
+                                  void* out, int out_is_bf16, int ldo, int ohs, int rows, int heads, const float* gate, int ldg,
+                                  int rot_n, int rotary, int pairs, int rot_src, int rot_dst, const float* cos_table,
+                                  const float* sin_table, const int32_t* positions, void* stream) {
   if (rows <= 0 || heads <= 0 || outn <= 0) return 0;
   if (in <= 0 || (size_t)HL_ROWS * in * sizeof(float) > 48 * 1024) return -2;
+  if (gate != nullptr && ldg < heads) return -2;
+  if (rot_n < 0 || (rot_n > 0 && (rotary < 0 || rotary > rot_n || (rotary & 1) || positions == nullptr ||
+                                  (rotary > 0 && (cos_table == nullptr || sin_table == nullptr)))))
+    return -2;
+  const HeadExtras ex{gate, ldg, rot_n, rotary, pairs, rot_src, rot_dst, cos_table, sin_table, positions};
   hipStream_t s = (hipStream_t)stream;
-  const dim3 grid((rows + HL_ROWS - 1) / HL_ROWS, heads, (outn + 63) / 64), block(256);
+  const dim3 grid((rows + HL_ROWS - 1) / HL_ROWS, heads, (outn + 63) / 64 + (rot_n > 0 ? 1 : 0)), block(256);
   const size_t bytes = (size_t)HL_ROWS * (in + 4 * 64) * sizeof(float);
+#define BW_HL_LAUNCH(WT, OT) \
+  hipLaunchKernelGGL((headwise_linear_kernel<WT, OT>), grid, block, bytes, s, x, ldx, xhs, (const WT*)wt, in, outn, (OT*)out, ldo, ohs, rows, ex)
   if (w_is_bf16) {
-    if (out_is_bf16)
-      hipLaunchKernelGGL((headwise_linear_kernel<bf16_t, bf16_t>), grid, block, bytes, s, x, ldx, xhs, (const bf16_t*)wt, in, outn,
-                         (bf16_t*)out, ldo, ohs, rows);
-    else
-      hipLaunchKernelGGL((headwise_linear_kernel<bf16_t, float>), grid, block, bytes, s, x, ldx, xhs, (const bf16_t*)wt, in, outn,
-                         (float*)out, ldo, ohs, rows);
+    if (out_is_bf16) BW_HL_LAUNCH(bf16_t, bf16_t);
+    else BW_HL_LAUNCH(bf16_t, float);
   } else {
-    if (out_is_bf16)
-      hipLaunchKernelGGL((headwise_linear_kernel<float, bf16_t>), grid, block, bytes, s, x, ldx, xhs, (const float*)wt, in, outn,
-                         (bf16_t*)out, ldo, ohs, rows);
-    else
-      hipLaunchKernelGGL((headwise_linear_kernel<float, float>), grid, block, bytes, s, x, ldx, xhs, (const float*)wt, in, outn,
-                         (float*)out, ldo, ohs, rows);
+    if (out_is_bf16) BW_HL_LAUNCH(float, bf16_t);
+    else BW_HL_LAUNCH(float, float);
   }
+#undef BW_HL_LAUNCH
   return BW_LAUNCH_CHECK();
 }
 

@@ -8,8 +8,10 @@
 //   plan:     the step's (row, choice) pairs ("slots") sorted by expert into runs, and the runs cut into tiles of
 //             16 or 128 slots (steps of few or of many slots): every tile belongs to one expert.  Built on the device; the products' grids are sized for
 //             the worst case and tiles past the last return at once.
+//   (or, without a router: the row's token id names its experts in a table, each weighs 1/top, and the plan is made at once)
 //   gate_up:  per tile, G = X W_gate^T and U = X W_up^T of its expert, then h = min(G, limit) * sigmoid(alpha * min(G, limit))
 //             * (clamp(U, -limit, limit) + 1), stored by the slot's place in the sorted order
+//             or, for experts without a gate, h = max(X W_up^T, 0)^2
 //   down:     per tile, h W_down^T of its expert, 32-bit sums by sorted place
 //   combine:  out[row] = sum over the row's choices, in the order they were chosen, of weight * its expert's output
 //
@@ -234,6 +236,35 @@ __global__ __launch_bounds__(1024) void moe_route_plan_kernel(const float* __res
   plan_body(ids, rows * top, E, segs, tm, 1, reinterpret_cast<int*>(both_lds + (size_t)rows * (2 * E + 2 * count)), sorted, place, tiles, meta);
 }
 
+// Routing by a table instead of a router: row r's experts are table[token of r][..], its weights ``weight`` each.  A token of
+// -2 is the one the step before sampled for the row (``feedback``).  A row without a token (padding) takes the experts of
+// the step's first row, so that it asks for no expert's weights that the step would not read anyway.  Entries are kept
+// inside 0 .. experts - 1.  One workgroup; the choices go to ``ids`` and the plan is made from there.
+__global__ __launch_bounds__(1024) void moe_table_plan_kernel(const int32_t* __restrict__ tokens, const int32_t* __restrict__ feedback,
+                                                              int rows, const int32_t* __restrict__ table, int vocab, int top, int E,
+                                                              float weight, int segs, int tm, int staged, int32_t* ids,
+                                                              float* __restrict__ wts, int32_t* __restrict__ sorted,
+                                                              int32_t* __restrict__ place, int32_t* __restrict__ tiles,
+                                                              int32_t* __restrict__ meta) {
+  extern __shared__ int table_lds[];    // [rows * top] if staged
+  auto token_of = [&](int r) {
+    int t = tokens[r];
+    if (t == -2 && feedback != nullptr) t = feedback[r];
+    return t;
+  };
+  const int n = rows * top;
+  for (int sidx = threadIdx.x; sidx < n; sidx += 1024) {
+    const int r = sidx / top;
+    int t = token_of(r);
+    if (t < 0 || t >= vocab) t = token_of(0);
+    if (t < 0 || t >= vocab) t = 0;
+    ids[sidx] = min(max(table[(size_t)t * top + sidx % top], 0), E - 1);
+    wts[sidx] = weight;
+  }
+  __syncthreads();                      // (written to memory by the workgroup's own threads, visible to all of them)
+  plan_body(ids, n, E, segs, tm, staged, table_lds, sorted, place, tiles, meta);
+}
+
 // Slots a tile: few slots a step (decoded tokens) get tiles of 16, whose kernel keeps many steps of weights in flight;
 // prompt portions get tiles of 128, which a workgroup stages in LDS.
 extern "C" int bw_moe_tile_rows(int slots) { return slots <= MOE_SMALL_SLOTS ? 16 : MOE_TM; }
@@ -251,6 +282,18 @@ extern "C" int bw_moe_plan(const int32_t* ids, int slots, int experts, int32_t* 
   const int staged = slots <= 12 * 1024;
   hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), staged ? (size_t)slots * sizeof(int) : 0, (hipStream_t)stream, ids, slots,
                      experts, segs, bw_moe_tile_rows(slots), staged, sorted, place, tiles, meta);
+  return BW_LAUNCH_CHECK();
+}
+
+extern "C" int bw_moe_table_plan(const int32_t* tokens, const int32_t* feedback, int rows, const int32_t* table, int vocab, int top,
+                                 int experts, float weight, int32_t* ids, float* wts, int32_t* sorted, int32_t* place, int32_t* tiles,
+                                 int32_t* meta, void* stream) {
+  if (rows <= 0) return 0;
+  if (experts < 1 || experts > MOE_MAX_EXPERTS || top < 1 || vocab < 1 || (long long)rows * top > 0x7fffffffLL) return -2;
+  const int slots = rows * top, staged = slots <= 12 * 1024;
+  hipLaunchKernelGGL(moe_table_plan_kernel, dim3(1), dim3(1024), staged ? (size_t)slots * sizeof(int) : 0, (hipStream_t)stream, tokens,
+                     feedback, rows, table, vocab, top, experts, weight, 1024 / experts, bw_moe_tile_rows(slots), staged, ids, wts, sorted,
+                     place, tiles, meta);
   return BW_LAUNCH_CHECK();
 }
 
@@ -280,7 +323,16 @@ __device__ __forceinline__ float moe_act(float g, float u, float limit, float al
   return (g * (1.0f / (1.0f + bw_expf(-alpha * g)))) * (u + 1.0f);
 }
 
+__device__ __forceinline__ float squared_relu(float z) {
+  const float m = fmaxf(z, 0.0f);
+  return m * m;
+}
+
 // ------------------------------------------------------------------------------ products on the matrix cores
+
+// FORM_DOWN: activations by sorted place times W [N, K].  FORM_GATED: rows times the stacked [2N, K] (gate rows, then up
+// rows), gated.  FORM_PLAIN: rows times W_up [N, K], squared ReLU.
+enum { FORM_DOWN = 0, FORM_GATED = 1, FORM_PLAIN = 2 };
 
 struct MoeArgs {
   const int32_t* sorted;   // [slots]
@@ -290,14 +342,14 @@ struct MoeArgs {
   float limit, alpha;
 };
 
-// A workgroup of four waves per (tile of 16 MB slots, 128 output columns); a wave owns 32 columns, for GATE_UP of
+// A workgroup of four waves per (tile of 16 MB slots, 128 output columns); a wave owns 32 columns, for FORM_GATED of
 // the gate and of the up matrix both, and all of the tile's rows.  Operands go from memory straight into registers: lane
 // (r, g) holds row r's (or column r's) elements k + 8g .. k + 8g + 7; a ring of DEPTH sets of operand registers keeps as
 // many steps of the inner size in flight.  MB blocks of 16 rows a tile: 1 with a deep ring for the few rows of decoded
 // tokens, where the weights stream from memory once and nothing is reused (prompt portions: moe_lds_kernel below).  Blocks of 16 rows past the tile's slots are skipped (a scalar
 // branch: the matrix cores ignore the execution mask); rows past them inside a block read the tile's first row and are
 // never stored.
-template <bool GATE_UP, int MB, int DEPTH, int CW>
+template <int FORM, int MB, int DEPTH, int CW>
 __global__ __launch_bounds__(256) void moe_mfma_kernel(MoeArgs a, const bf16_t* __restrict__ x, int ldx, int x_rows,
                                                        const bf16_t* __restrict__ w, void* __restrict__ out, int ldo, int max_tiles) {
   // Workgroups are dealt to the chip's eight dies in turn, and every die has an L2 of its own.  Workgroup L is the
@@ -312,7 +364,8 @@ __global__ __launch_bounds__(256) void moe_mfma_kernel(MoeArgs a, const bf16_t* 
             cnt = __builtin_amdgcn_readfirstlane(a.tiles[tile * 4 + 2]);
   const int n0 = col_block * (4 * CW) + wave * CW;         // CW columns a wave (32, or 16 where a step has very few slots
   if (n0 >= a.N) return;                                   // and more workgroups are worth more than wider ones)
-  constexpr int CB = CW / 16, NB = GATE_UP ? 2 * CB : CB;
+  constexpr bool GATED = FORM == FORM_GATED, GATHERS = FORM != FORM_DOWN;
+  constexpr int CB = CW / 16, NB = GATED ? 2 * CB : CB;
   const int mb_live = (cnt + 15) >> 4;                     // blocks of 16 rows that hold a slot
   // Every load goes through a buffer descriptor with a per-lane offset fixed for the whole kernel and the step's offset
   // in a scalar register: the loop spends no vector instruction on addresses and no branch on a load.  Rows of x are
@@ -325,15 +378,15 @@ __global__ __launch_bounds__(256) void moe_mfma_kernel(MoeArgs a, const bf16_t* 
   for (int i = 0; i < MB; ++i) {
     const int q = 16 * i + r;
     const int pq = p0 + (q < cnt ? q : 0);
-    const size_t row = GATE_UP ? (size_t)(a.sorted[pq] / a.top) : (size_t)pq;
+    const size_t row = GATHERS ? (size_t)(a.sorted[pq] / a.top) : (size_t)pq;
     voff_x[i] = i < mb_live ? (int)((row * ldx + 16 * g) * 2) : 0x7ffffff0;
   }
-  // weights of expert e: GATE_UP [2N, K] (gate rows, then up rows), else [N, K]
+  // weights of expert e: FORM_GATED [2N, K] (gate rows, then up rows), else [N, K]
   __amdgpu_buffer_rsrc_t rs_w[NB];
-  const size_t wbase = (size_t)e * (GATE_UP ? 2 : 1) * a.N * a.K;
+  const size_t wbase = (size_t)e * (GATED ? 2 : 1) * a.N * a.K;
 #pragma unroll
   for (int b = 0; b < NB; ++b) {
-    const int half = GATE_UP ? b / CB : 0, cb = GATE_UP ? b % CB : b;
+    const int half = GATED ? b / CB : 0, cb = GATED ? b % CB : b;
     const int nb0 = n0 + 16 * cb;
     const int rows_in = min(16, a.N - nb0);                // (may be <= 0: then nothing of the block is read)
     rs_w[b] = __builtin_amdgcn_make_buffer_rsrc((void*)(w + wbase + ((size_t)half * a.N + (rows_in > 0 ? nb0 : 0)) * a.K), 0,
@@ -408,8 +461,10 @@ __global__ __launch_bounds__(256) void moe_mfma_kernel(MoeArgs a, const bf16_t* 
       for (int cb = 0; cb < CB; ++cb) {
         const int n = n0 + 16 * cb + r;
         if (n >= a.N) continue;
-        if constexpr (GATE_UP)
+        if constexpr (GATED)
           reinterpret_cast<bf16_t*>(out)[(size_t)(p0 + m) * ldo + n] = f32_to_bf16(moe_act(acc[i][cb][q], acc[i][CB + cb][q], a.limit, a.alpha));
+        else if constexpr (GATHERS)
+          reinterpret_cast<bf16_t*>(out)[(size_t)(p0 + m) * ldo + n] = f32_to_bf16(squared_relu(acc[i][cb][q]));
         else
           reinterpret_cast<float*>(out)[(size_t)(p0 + m) * ldo + n] = acc[i][cb][q];
       }
@@ -418,7 +473,7 @@ __global__ __launch_bounds__(256) void moe_mfma_kernel(MoeArgs a, const bf16_t* 
 
 // ------------------------------------------------------------------------------ prompt portions: tiles staged in LDS
 
-// A workgroup of four waves per (tile of 128 slots, 128 output columns; GATE_UP: of the gate and of the up matrix both,
+// A workgroup of four waves per (tile of 128 slots, 128 output columns; FORM_GATED: of the gate and of the up matrix both,
 // 256 weight rows).  A step covers 64 elements of the inner size: the threads together copy the tile's 128 rows of x and
 // its weight rows, 128 bytes each, from memory into LDS (through registers: the next step's loads fly while this one is
 // multiplied; two stages, one barrier a step; rows 144 bytes apart against bank conflicts), and wave (wr, wc) multiplies
@@ -427,13 +482,14 @@ __global__ __launch_bounds__(256) void moe_mfma_kernel(MoeArgs a, const bf16_t* 
 // have the same bits as there.  87 flops for every byte that comes from L2, against 32 when every wave loads for itself.
 #define MOE_LDS_STRIDE 144
 
-template <bool GATE_UP>
+template <int FORM>
 __global__ __launch_bounds__(256) void moe_lds_kernel(MoeArgs a, const bf16_t* __restrict__ x, int ldx, int x_rows,
                                                       const bf16_t* __restrict__ w, void* __restrict__ out, int ldo, int max_tiles) {
-  constexpr int TM = MOE_TM, BR = GATE_UP ? 256 : 128, ROWS = TM + BR;
+  constexpr bool GATED = FORM == FORM_GATED, GATHERS = FORM != FORM_DOWN;
+  constexpr int TM = MOE_TM, BR = GATED ? 256 : 128, ROWS = TM + BR;
   constexpr int NCH = ROWS * 8 / 256;                       // 16-byte chunks a thread copies a step
   constexpr int STAGE = ROWS * MOE_LDS_STRIDE;
-  constexpr int NB = GATE_UP ? 8 : 4;
+  constexpr int NB = GATED ? 8 : 4;
   extern __shared__ __attribute__((aligned(16))) unsigned char moe_lds[];
   const int die = blockIdx.x & 7, nth = blockIdx.x >> 3;
   const int tile = nth % max_tiles, col_block = die + 8 * (nth / max_tiles);
@@ -446,9 +502,9 @@ __global__ __launch_bounds__(256) void moe_lds_kernel(MoeArgs a, const bf16_t* _
   const int K = a.K;
   const bool tail = (K & 63) != 0;
   const __amdgpu_buffer_rsrc_t rs_x = __builtin_amdgcn_make_buffer_rsrc((void*)x, 0, (int)((size_t)x_rows * ldx * 2), 0x00020000);
-  const size_t wbase = (size_t)e * (GATE_UP ? 2 : 1) * a.N * a.K;
+  const size_t wbase = (size_t)e * (GATED ? 2 : 1) * a.N * a.K;
   const __amdgpu_buffer_rsrc_t rs_w =
-      __builtin_amdgcn_make_buffer_rsrc((void*)(w + wbase), 0, (int)((size_t)(GATE_UP ? 2 : 1) * a.N * a.K * 2), 0x00020000);
+      __builtin_amdgcn_make_buffer_rsrc((void*)(w + wbase), 0, (int)((size_t)(GATED ? 2 : 1) * a.N * a.K * 2), 0x00020000);
   // chunk c = tid + 256 j: row c / 8 of the stage (x rows first, then weight rows), bytes 16 (c % 8) .. of the row's step
   int voff[NCH], lds_off[NCH];
 #pragma unroll
@@ -457,10 +513,10 @@ __global__ __launch_bounds__(256) void moe_lds_kernel(MoeArgs a, const bf16_t* _
     lds_off[j] = row * MOE_LDS_STRIDE + part * 16;
     if (row < TM) {
       const int pq = p0 + (row < cnt ? row : 0);
-      const size_t src = GATE_UP ? (size_t)(a.sorted[pq] / a.top) : (size_t)pq;
+      const size_t src = GATHERS ? (size_t)(a.sorted[pq] / a.top) : (size_t)pq;
       voff[j] = (int)((src * ldx) * 2) + part * 16;
     } else {
-      const int br = row - TM, half = GATE_UP ? br >> 7 : 0;
+      const int br = row - TM, half = GATED ? br >> 7 : 0;
       const int n = min(n0 + (br & 127), a.N - 1);
       voff[j] = (int)(((size_t)half * a.N + n) * a.K * 2) + part * 16;
     }
@@ -497,7 +553,7 @@ __global__ __launch_bounds__(256) void moe_lds_kernel(MoeArgs a, const bf16_t* _
   int b_off[NB];
 #pragma unroll
   for (int b = 0; b < NB; ++b) {
-    const int half = GATE_UP ? b >> 2 : 0, cb = b & 3;
+    const int half = GATED ? b >> 2 : 0, cb = b & 3;
     b_off[b] = (TM + 128 * half + 64 * wc + 16 * cb + r) * MOE_LDS_STRIDE + 32 * g;
   }
   auto multiply = [&](int stage) {
@@ -547,25 +603,27 @@ __global__ __launch_bounds__(256) void moe_lds_kernel(MoeArgs a, const bf16_t* _
       for (int cb = 0; cb < 4; ++cb) {
         const int n = n0 + 64 * wc + 16 * cb + r;
         if (n >= a.N) continue;
-        if constexpr (GATE_UP)
+        if constexpr (GATED)
           reinterpret_cast<bf16_t*>(out)[(size_t)(p0 + m) * ldo + n] = f32_to_bf16(moe_act(acc[i][cb][q], acc[i][4 + cb][q], a.limit, a.alpha));
+        else if constexpr (GATHERS)
+          reinterpret_cast<bf16_t*>(out)[(size_t)(p0 + m) * ldo + n] = f32_to_bf16(squared_relu(acc[i][cb][q]));
         else
           reinterpret_cast<float*>(out)[(size_t)(p0 + m) * ldo + n] = acc[i][cb][q];
       }
     }
 }
 
-template <bool GATE_UP>
+template <int FORM>
 static int moe_lds_launch(const MoeArgs& a, const bf16_t* x, int ldx, int x_rows, const bf16_t* w, void* out, int ldo, int max_tiles,
                           hipStream_t s) {
-  constexpr int BYTES = 2 * (MOE_TM + (GATE_UP ? 256 : 128)) * MOE_LDS_STRIDE;
+  constexpr int BYTES = 2 * (MOE_TM + (FORM == FORM_GATED ? 256 : 128)) * MOE_LDS_STRIDE;
   static bool allowed = false;
   if (!allowed) {
-    if (hipFuncSetAttribute((const void*)moe_lds_kernel<GATE_UP>, hipFuncAttributeMaxDynamicSharedMemorySize, BYTES) != hipSuccess) return -8;
+    if (hipFuncSetAttribute((const void*)moe_lds_kernel<FORM>, hipFuncAttributeMaxDynamicSharedMemorySize, BYTES) != hipSuccess) return -8;
     allowed = true;
   }
   const int col_blocks = (a.N + 127) / 128;
-  hipLaunchKernelGGL(moe_lds_kernel<GATE_UP>, dim3((unsigned)(8 * ((col_blocks + 7) / 8) * max_tiles)), dim3(256), BYTES, s, a, x, ldx, x_rows,
+  hipLaunchKernelGGL(moe_lds_kernel<FORM>, dim3((unsigned)(8 * ((col_blocks + 7) / 8) * max_tiles)), dim3(256), BYTES, s, a, x, ldx, x_rows,
                      w, out, ldo, max_tiles);
   return BW_LAUNCH_CHECK();
 }
@@ -575,75 +633,76 @@ static int moe_lds_launch(const MoeArgs& a, const bf16_t* x, int ldx, int x_rows
 // A thread an output (sorted place, column): one chain of fused multiply-adds over the inner size ascending.
 // ROUND: the activation is rounded to bfloat16 (and kept as a 32-bit value), for the bfloat16 mode of weights that the
 // matrix-core kernels do not take.
-template <bool GATE_UP, typename WT>
+template <int FORM, typename WT>
 __global__ __launch_bounds__(64) void moe_f32_kernel(MoeArgs a, const float* __restrict__ x, int ldx, const WT* __restrict__ w,
                                                      float* __restrict__ out, int ldo, int round_out) {
+  constexpr bool GATED = FORM == FORM_GATED, GATHERS = FORM != FORM_DOWN;
   const int tile = blockIdx.x;
   if (tile >= a.meta[0]) return;
   const int e = a.tiles[tile * 4], p0 = a.tiles[tile * 4 + 1], cnt = a.tiles[tile * 4 + 2];
   const int n = blockIdx.y * 64 + threadIdx.x;
   if (n >= a.N) return;
-  const size_t wbase = (size_t)e * (GATE_UP ? 2 : 1) * a.N * a.K;
+  const size_t wbase = (size_t)e * (GATED ? 2 : 1) * a.N * a.K;
   const WT* wg = w + wbase + (size_t)n * a.K;
   const WT* wu = wg + (size_t)a.N * a.K;
   for (int m = 0; m < cnt; ++m) {
-    const float* xr = x + (GATE_UP ? (size_t)(a.sorted[p0 + m] / a.top) : (size_t)(p0 + m)) * ldx;
+    const float* xr = x + (GATHERS ? (size_t)(a.sorted[p0 + m] / a.top) : (size_t)(p0 + m)) * ldx;
     float sg = 0.0f, su = 0.0f;
     for (int k = 0; k < a.K; ++k) {
       const float xv = xr[k];
       if constexpr (sizeof(WT) == 2) {
         sg = fmaf(xv, bf16_to_f32(wg[k]), sg);
-        if (GATE_UP) su = fmaf(xv, bf16_to_f32(wu[k]), su);
+        if (GATED) su = fmaf(xv, bf16_to_f32(wu[k]), su);
       } else {
         sg = fmaf(xv, wg[k], sg);
-        if (GATE_UP) su = fmaf(xv, wu[k], su);
+        if (GATED) su = fmaf(xv, wu[k], su);
       }
     }
-    float y = GATE_UP ? moe_act(sg, su, a.limit, a.alpha) : sg;
-    if (GATE_UP && round_out) y = bf16_to_f32(f32_to_bf16(y));
+    float y = GATED ? moe_act(sg, su, a.limit, a.alpha) : (GATHERS ? squared_relu(sg) : sg);
+    if (GATHERS && round_out) y = bf16_to_f32(f32_to_bf16(y));
     out[(size_t)(p0 + m) * ldo + n] = y;
   }
 }
 
-extern "C" int bw_moe_experts(const void* x, int x_is_bf16, int ldx, int x_rows, const void* w, int w_is_bf16, void* out, int ldo,
-                              const int32_t* sorted, const int32_t* tiles, const int32_t* meta, int slots, int max_tiles, int top,
-                              int K, int N, int gate_up, float limit, float alpha, int round_out, void* stream) {
-  const int tile_rows = bw_moe_tile_rows(slots);          // (as the plan was made)
-  if (max_tiles <= 0 || slots <= 0) return 0;
-  if (K <= 0 || N <= 0 || (N + 63) / 64 > 65535) return -2;
-  MoeArgs a{sorted, tiles, meta, top, K, N, limit, alpha};
-  hipStream_t s = (hipStream_t)stream;
+// The product over a plan's tiles for one form of it.
+template <int FORM>
+static int moe_experts_form(const MoeArgs& a, const void* x, int x_is_bf16, int ldx, int x_rows, const void* w, int w_is_bf16, void* out,
+                            int ldo, int slots, int max_tiles, int round_out, hipStream_t s) {
+  constexpr bool GATED = FORM == FORM_GATED;
   if (x_is_bf16) {
-    if (!w_is_bf16 || K % 8 || ldx % 8) return -3;
-    if ((size_t)x_rows * ldx * 2 >= (1ull << 31) || (size_t)16 * K * 2 >= (1ull << 31)) return -2;      // offsets inside a descriptor are 32-bit
-    if (tile_rows == 16) {
+    if (!w_is_bf16 || a.K % 8 || ldx % 8) return -3;
+    if ((size_t)x_rows * ldx * 2 >= (1ull << 31) || (size_t)16 * a.K * 2 >= (1ull << 31)) return -2;      // offsets inside a descriptor are 32-bit
+    if (bw_moe_tile_rows(slots) == 16) {                   // (as the plan was made)
       // very few slots (a step of up to 16 rows of four experts): 16 columns a wave, twice the workgroups
       const int cw = slots <= 64 ? 16 : 32;
-      const int col_blocks = (N + 4 * cw - 1) / (4 * cw);
+      const int col_blocks = (a.N + 4 * cw - 1) / (4 * cw);
       const dim3 grid((unsigned)(8 * ((col_blocks + 7) / 8) * max_tiles));
-      if (cw == 16) {
-        if (gate_up) hipLaunchKernelGGL((moe_mfma_kernel<true, 1, 6, 16>), grid, dim3(256), 0, s, a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles);
-        else hipLaunchKernelGGL((moe_mfma_kernel<false, 1, 8, 16>), grid, dim3(256), 0, s, a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles);
-      } else {
-        if (gate_up) hipLaunchKernelGGL((moe_mfma_kernel<true, 1, 4, 32>), grid, dim3(256), 0, s, a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles);
-        else hipLaunchKernelGGL((moe_mfma_kernel<false, 1, 6, 32>), grid, dim3(256), 0, s, a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles);
-      }
-    } else {
-      if ((size_t)2 * N * K * 2 >= (1ull << 31)) return -2;
-      return gate_up ? moe_lds_launch<true>(a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles, s)
-                     : moe_lds_launch<false>(a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles, s);
+      if (cw == 16)
+        hipLaunchKernelGGL((moe_mfma_kernel<FORM, 1, GATED ? 6 : 8, 16>), grid, dim3(256), 0, s, a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles);
+      else
+        hipLaunchKernelGGL((moe_mfma_kernel<FORM, 1, GATED ? 4 : 6, 32>), grid, dim3(256), 0, s, a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles);
+      return BW_LAUNCH_CHECK();
     }
-    return BW_LAUNCH_CHECK();
+    if ((size_t)2 * a.N * a.K * 2 >= (1ull << 31)) return -2;
+    return moe_lds_launch<FORM>(a, (const bf16_t*)x, ldx, x_rows, (const bf16_t*)w, out, ldo, max_tiles, s);
   }
-  const dim3 grid(max_tiles, (N + 63) / 64);
-  if (gate_up) {
-    if (w_is_bf16) hipLaunchKernelGGL((moe_f32_kernel<true, bf16_t>), grid, dim3(64), 0, s, a, (const float*)x, ldx, (const bf16_t*)w, (float*)out, ldo, round_out);
-    else hipLaunchKernelGGL((moe_f32_kernel<true, float>), grid, dim3(64), 0, s, a, (const float*)x, ldx, (const float*)w, (float*)out, ldo, round_out);
-  } else {
-    if (w_is_bf16) hipLaunchKernelGGL((moe_f32_kernel<false, bf16_t>), grid, dim3(64), 0, s, a, (const float*)x, ldx, (const bf16_t*)w, (float*)out, ldo, 0);
-    else hipLaunchKernelGGL((moe_f32_kernel<false, float>), grid, dim3(64), 0, s, a, (const float*)x, ldx, (const float*)w, (float*)out, ldo, 0);
-  }
+  const dim3 grid(max_tiles, (a.N + 63) / 64);
+  if (w_is_bf16) hipLaunchKernelGGL((moe_f32_kernel<FORM, bf16_t>), grid, dim3(64), 0, s, a, (const float*)x, ldx, (const bf16_t*)w, (float*)out, ldo, round_out);
+  else hipLaunchKernelGGL((moe_f32_kernel<FORM, float>), grid, dim3(64), 0, s, a, (const float*)x, ldx, (const float*)w, (float*)out, ldo, round_out);
   return BW_LAUNCH_CHECK();
+}
+
+extern "C" int bw_moe_experts(const void* x, int x_is_bf16, int ldx, int x_rows, const void* w, int w_is_bf16, void* out, int ldo,
+                              const int32_t* sorted, const int32_t* tiles, const int32_t* meta, int slots, int max_tiles, int top,
+                              int K, int N, int form, float limit, float alpha, int round_out, void* stream) {
+  if (max_tiles <= 0 || slots <= 0) return 0;
+  if (K <= 0 || N <= 0 || (N + 63) / 64 > 65535 || top < 1) return -2;
+  const MoeArgs a{sorted, tiles, meta, top, K, N, limit, alpha};
+  hipStream_t s = (hipStream_t)stream;
+  if (form == FORM_GATED) return moe_experts_form<FORM_GATED>(a, x, x_is_bf16, ldx, x_rows, w, w_is_bf16, out, ldo, slots, max_tiles, round_out, s);
+  if (form == FORM_PLAIN) return moe_experts_form<FORM_PLAIN>(a, x, x_is_bf16, ldx, x_rows, w, w_is_bf16, out, ldo, slots, max_tiles, round_out, s);
+  if (form == FORM_DOWN) return moe_experts_form<FORM_DOWN>(a, x, x_is_bf16, ldx, x_rows, w, w_is_bf16, out, ldo, slots, max_tiles, 0, s);
+  return -2;
 }
 
 // ------------------------------------------------------------------------------ combine

@@ -84,10 +84,13 @@ _SIGS = {
     "bw_norm_mean": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_void_p],
     "bw_norm_mean_add": [c_void_p, c_void_p, c_void_p, c_int, c_float, c_void_p, c_float, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
     "bw_linear_recurrence": [c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p,
-                             c_float, c_float, c_float, c_void_p, c_longlong, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
-                             c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_longlong, c_void_p],
+                             c_float, c_float, c_float, c_void_p, c_int, c_void_p, c_longlong, c_void_p, c_int, c_void_p, c_void_p,
+                             c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_longlong, c_void_p],
     "bw_head_norm_gate": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_int,
                           c_int, c_int, c_float, c_void_p],
+    "bw_gated_part_norm": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_float,
+                           c_void_p],
+    "bw_activate": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p],
     "bw_glu": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int, c_void_p],
     "bw_embed_sum": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                      c_float, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_void_p],
@@ -99,11 +102,11 @@ _SIGS = {
                                      c_void_p, c_longlong, c_void_p],
     "bw_latent_prep": [c_void_p, c_int, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                        c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                       c_void_p],
+                       c_int, c_int, c_void_p, c_void_p, c_int, c_void_p],
     "bw_headwise_linear": [c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int,
-                           c_int, c_void_p],
+                           c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p],
     "bw_causal_conv": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_longlong, c_void_p, c_void_p,
-                       c_void_p, c_int, c_int, c_void_p, c_int, c_void_p],
+                       c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p],
     "bw_pair_rope_unit": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                           c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
                           c_int, c_int, c_int, c_void_p],
@@ -117,6 +120,8 @@ _SIGS = {
     "bw_moe_route": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p],
     "bw_moe_route_plan": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_int, c_void_p, c_void_p,
                           c_void_p, c_void_p, c_void_p, c_void_p, c_void_p],
+    "bw_moe_table_plan": [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_void_p,
+                          c_void_p, c_void_p, c_void_p],
     "bw_moe_max_tiles": [c_int, c_int],
     "bw_moe_plan": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p],
     "bw_moe_experts": [c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
@@ -773,7 +778,7 @@ def gemm_qkv_rope_bf16(x: torch.Tensor, w_qkv: torch.Tensor, q_out: torch.Tensor
 
 # ------------------------------------------------------------------------------ mixers with a state per request
 
-RECUR_DECAY_PER_CHANNEL, RECUR_SCALAR_GATES, RECUR_BONUS_DECAY, RECUR_FIXED_DECAY = 0, 1, 2, 3
+RECUR_DECAY_PER_CHANNEL, RECUR_SCALAR_GATES, RECUR_BONUS_DECAY, RECUR_FIXED_DECAY, RECUR_STEP_DECAY = 0, 1, 2, 3, 4
 RECUR_MAX_DIM = 256          # key channels of a head that the recurrence keeps in a lane's registers
 GATE_SIGMOID, GATE_SILU = 0, 1
 ACT_SILU, ACT_GELU_TANH, ACT_CLAMPED_SWISH = 0, 1, 2
@@ -813,7 +818,8 @@ def norm_shift(x: torch.Tensor, weight: torch.Tensor, mix: torch.Tensor, state: 
 def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate: Optional[torch.Tensor], gate_off: int,
                       gate2_off: int, bias: torch.Tensor, bias2: Optional[torch.Tensor], param: float, qscale: float,
                       state: torch.Tensor, out: torch.Tensor, seq_rows: torch.Tensor, slots: torch.Tensor,
-                      positions: torch.Tensor, nseq: int, heads: int, dim: int, vdim: int, scan=None, kscale: float = 1.0) -> None:
+                      positions: torch.Tensor, nseq: int, heads: int, dim: int, vdim: int, scan=None, kscale: float = 1.0,
+                      heads_per_key: int = 1, skip: Optional[torch.Tensor] = None) -> None:
     """The recurrence S <- decay * S + k v^T, o = S^T (q * qscale) per head over every request's rows in order, from and
     to ``state`` [slots, elements].  RECUR_DECAY_PER_CHANNEL: decay = exp(logsigmoid(gate + bias) * param) per key
     channel (``gate`` [rows, >= gate_off + heads*dim]).  RECUR_SCALAR_GATES: capped input and forget gates per head
@@ -821,7 +827,10 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
     RECUR_BONUS_DECAY: decay = exp(-exp(gate + bias)) per key channel, and the read-out comes before the update:
     o = (S + diag(bias2) k v^T)^T q with the S the token before left (``bias2`` [heads*dim]: the weight of the token's own
     k v^T), then S <- decay * S + k v^T.  RECUR_FIXED_DECAY: one constant decay a head (``bias`` [heads]; ``gate`` None).
-    k is multiplied by ``kscale``.  ``state`` may be a column slice of a wider tensor.
+    RECUR_STEP_DECAY: a step size per head, delta = softplus(gate + bias) (``gate`` column gate_off + h, ``bias`` [heads]);
+    decay = exp(-bias2[h] delta) (``bias2`` [heads]: the rates), the token enters as k (delta v)^T, and ``skip`` [heads]
+    (optional) times v joins the read-out.
+    k is multiplied by ``kscale``; ``heads_per_key`` neighbouring heads share one q and one k.  ``state`` may be a column slice of a wider tensor.
 
     ``scan`` = (chunks [n, 4] int32 = (first row, rows, request, 1 if the request's last chunk), n, spans [k, 3] int32 =
     (request, its first chunk, its chunks), k, local, start): long portions run in three passes over their chunks (each
@@ -830,7 +839,7 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
     for those requests (nseq may be 0).  The result differs from the one-pass order by the rounding of the walk's sums."""
     _need_strided(proj, torch.float32, "proj")            # (may be a column slice of a wider product)
     if mode != RECUR_FIXED_DECAY:
-        _need(gate, torch.float32, "gate")
+        _need_strided(gate, torch.float32, "gate")
     _need(bias, torch.float32, "bias")
     _need_strided(state, torch.float32, "state")
     _need(out, torch.float32, "out")
@@ -845,6 +854,13 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
         if bias.numel() != heads or bias2.numel() != heads or max(gate_off, gate2_off) + heads > gate.shape[1]:
             raise ValueError("linear_recurrence: gates or biases do not fit the heads")
         need = heads * (dim * vdim + dim + 1)
+    elif mode == RECUR_STEP_DECAY:
+        if bias2 is None:
+            raise ValueError("linear_recurrence: a step size needs the decay's rates")
+        _need(bias2, torch.float32, "bias2")
+        if bias.numel() != heads or bias2.numel() != heads or gate_off + heads > gate.shape[1]:
+            raise ValueError("linear_recurrence: step sizes, their bias or the rates do not fit the heads")
+        need = heads * dim * vdim
     elif mode == RECUR_FIXED_DECAY:
         if bias.numel() != heads:
             raise ValueError("linear_recurrence: a constant decay a head is needed")
@@ -861,7 +877,13 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
         need = heads * dim * vdim
     if state.dim() != 2 or state.shape[1] < need:
         raise ValueError(f"linear_recurrence: a state slot needs {need} elements")
-    if max(q_off, k_off) + heads * dim > proj.shape[1] or v_off + heads * vdim > proj.shape[1] or out.shape[1] != heads * vdim:
+    if heads_per_key < 1 or heads % heads_per_key:
+        raise ValueError("linear_recurrence: the heads do not split into equal groups that share q and k")
+    if skip is not None:
+        _need(skip, torch.float32, "skip")
+        if skip.numel() != heads or mode != RECUR_STEP_DECAY:
+            raise ValueError("linear_recurrence: a weight a head for the token's own v, with step sizes only")
+    if max(q_off, k_off) + heads // heads_per_key * dim > proj.shape[1] or v_off + heads * vdim > proj.shape[1] or out.shape[1] != heads * vdim:
         raise ValueError("linear_recurrence: projections or out do not fit")
     if seq_rows.numel() < 2 * nseq or slots.numel() < nseq:
         raise ValueError("linear_recurrence: fewer request records than requests")
@@ -878,7 +900,8 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
     _check(_fn("bw_linear_recurrence")(int(mode), proj.data_ptr(), proj.stride(0), q_off, k_off, v_off,
                                        0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0),
                                        gate_off, gate2_off, bias.data_ptr(),
-                                       0 if bias2 is None else bias2.data_ptr(), float(param), float(qscale), float(kscale), state.data_ptr(),
+                                       0 if bias2 is None else bias2.data_ptr(), float(param), float(qscale), float(kscale),
+                                       0 if skip is None else skip.data_ptr(), int(heads_per_key), state.data_ptr(),
                                        state.stride(0), out.data_ptr(), out.stride(0), seq_rows.data_ptr(), slots.data_ptr(),
                                        positions.data_ptr(), nseq, heads, dim, vdim,
                                        0 if chunks is None else chunks.data_ptr(), nchunks,
@@ -978,6 +1001,37 @@ def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, per_head_weight: bool,
                                     heads, vdim, float(eps), _stream()), "head_norm_gate")
 
 
+def gated_part_norm(o: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, positions: torch.Tensor, rows: int,
+                    parts: int, eps: float) -> None:
+    """v = o * silu(z); every row's ``parts`` equal stretches of v are divided each by its own root mean square and multiplied
+    by ``weight`` [width].  o, z float32 (column slices will do), out float32 or bfloat16 (one rounding)."""
+    _need_strided(o, torch.float32, "o")
+    _need_strided(z, torch.float32, "z")
+    _need(weight, torch.float32, "weight")
+    _need(positions, torch.int32, "positions")
+    width = out.shape[1]
+    if width % parts or weight.numel() != width or o.shape[1] < width or z.shape[1] < width:
+        raise ValueError("gated_part_norm: o, z, weight and out do not fit, or the parts are not equal")
+    if min(o.shape[0], z.shape[0], out.shape[0], positions.numel()) < rows:
+        raise ValueError("gated_part_norm: buffers shorter than the rows")
+    _check(_fn("bw_gated_part_norm")(o.data_ptr(), o.stride(0), z.data_ptr(), z.stride(0), weight.data_ptr(), out.data_ptr(),
+                                     _act_out(out, "out"), out.stride(0), positions.data_ptr(), rows, int(parts), width // parts,
+                                     float(eps), _stream()), "gated_part_norm")
+
+
+PLAIN_RELU2, PLAIN_XIELU = 0, 1
+
+
+def activate(x: torch.Tensor, out: torch.Tensor, rows: int, act: int, p0: float = 0.0, p1: float = 0.0) -> None:
+    """out = act(x) of a 32-bit product, out float32 or bfloat16 (one rounding).  PLAIN_RELU2: max(x, 0)^2.  PLAIN_XIELU:
+    x > 0: p0 x^2 + x/2, else (1/2 + p1) (e^x - 1 - x) + x/2."""
+    _need_strided(x, torch.float32, "x")
+    if act not in (PLAIN_RELU2, PLAIN_XIELU) or x.shape[1] < out.shape[1] or min(x.shape[0], out.shape[0]) < rows:
+        raise ValueError("activate: an unknown activation, or out does not fit x")
+    _check(_fn("bw_activate")(x.data_ptr(), x.stride(0), out.data_ptr(), _act_out(out, "out"), out.stride(0), rows, out.shape[1],
+                              int(act), float(p0), float(p1), _stream()), "activate")
+
+
 def glu(gate_up: torch.Tensor, out: torch.Tensor, rows: int, act: int, limit: float = 0.0, alpha: float = 1.0,
         row_gate: Optional[torch.Tensor] = None) -> None:
     """out = act(gate) * up of the stacked 32-bit product [rows, >= 2*inter] (gate at column 0, up at column inter); out
@@ -1003,11 +1057,14 @@ def glu(gate_up: torch.Tensor, out: torch.Tensor, rows: int, act: int, limit: fl
 def latent_prep(proj: torch.Tensor, q_off: int, dkv_off: int, norm_w: torch.Tensor, eps: float, cos: torch.Tensor,
                 sin: torch.Tensor, positions: torch.Tensor, row_seq: torch.Tensor, block_table: torch.Tensor,
                 cache: torch.Tensor, qa: torch.Tensor, rows: int, heads: int, dim: int, rot: int, rotary: int, rank: int,
-                page_size: int, write_cache: bool = True, latent_t: Optional[torch.Tensor] = None) -> None:
+                page_size: int, write_cache: bool = True, latent_t: Optional[torch.Tensor] = None, pairs: bool = False,
+                q_latent: Optional[Tuple[torch.Tensor, torch.Tensor]] = None) -> None:
     """From the stacked projections: the latent (RMS-normed) and the rotated shared key part into the row's page slot
     ([pages, page_size * (rank + rot)]), and every head's rotated query part into ``qa`` [rows, heads * (rank + rot)]
     behind the place of its latent-space part.  ``latent_t`` [pages, rank * page_size]: the latent once more, transposed
-    within its page ([element][slot]), for the matrix-core attention."""
+    within its page ([element][slot]), for the matrix-core attention.  ``pairs``: elements 2i and 2i+1 of the rotated part
+    are turned together, instead of i and i + rotary/2.  ``q_latent`` = (weight [n], out [rows, n] in the queries' dtype):
+    what lies at q_off is no query but the queries' own latent, which is RMS-normed into ``out``; ``qa`` is not written."""
     _need(proj, torch.float32, "proj")
     _need(norm_w, torch.float32, "norm weight")
     _need(cos, torch.float32, "cos table")
@@ -1015,7 +1072,13 @@ def latent_prep(proj: torch.Tensor, q_off: int, dkv_off: int, norm_w: torch.Tens
     for t, what in ((positions, "positions"), (row_seq, "row_seq"), (block_table, "block_table")):
         _need(t, torch.int32, what)
     width = rank + rot
-    if q_off + heads * (dim + rot) > proj.shape[1] or dkv_off + width > proj.shape[1] or norm_w.numel() != rank:
+    q_rank, q_w, cq = 0, 0, None
+    if q_latent is not None:
+        _need(q_latent[0], torch.float32, "query norm weight")
+        q_rank, q_w, cq = q_latent[0].numel(), q_latent[0].data_ptr(), q_latent[1]
+        if cq.shape[1] != q_rank or cq.shape[0] < rows or cq.dtype != qa.dtype or not cq.is_contiguous():
+            raise ValueError("latent_prep: the queries' normed latent must be [rows, its size] in the queries' dtype")
+    if q_off + (q_rank or heads * (dim + rot)) > proj.shape[1] or dkv_off + width > proj.shape[1] or norm_w.numel() != rank:
         raise ValueError("latent_prep: projections or norm weight do not fit")
     if rotary % 2 or rotary > rot or (rotary and (cos.shape[1] != rotary // 2 or sin.shape != cos.shape)):
         raise ValueError("latent_prep: rotary tables must be [positions, rotary/2]")
@@ -1030,13 +1093,18 @@ def latent_prep(proj: torch.Tensor, q_off: int, dkv_off: int, norm_w: torch.Tens
                                  sin.data_ptr(), positions.data_ptr(), row_seq.data_ptr(), block_table.data_ptr(),
                                  block_table.stride(0), cache.data_ptr(), 0 if latent_t is None else latent_t.data_ptr(),
                                  _act_out(cache, "cache"), qa.data_ptr(), _act_out(qa, "qa"), qa.stride(0),
-                                 rows, heads, dim, rot, rotary, rank, page_size, int(write_cache), _stream()), "latent_prep")
+                                 rows, heads, dim, rot, rotary, rank, page_size, int(write_cache), int(pairs), q_rank, q_w,
+                                 0 if cq is None else cq.data_ptr(), 0 if cq is None else cq.stride(0), _stream()), "latent_prep")
 
 
 def headwise_linear(x: torch.Tensor, x_off: int, x_head_stride: int, wt: torch.Tensor, out: torch.Tensor, out_off: int,
-                    out_head_stride: int, rows: int) -> None:
+                    out_head_stride: int, rows: int, gate: Optional[torch.Tensor] = None, rotate=None) -> None:
     """out[r, out_off + h*out_head_stride + o] = sum_i wt[h, i, o] * x[r, x_off + h*x_head_stride + i]: a product per head,
-    weights input-major [heads, in, out] (bfloat16 or float32), 32-bit sums."""
+    weights input-major [heads, in, out] (bfloat16 or float32), 32-bit sums.  ``gate`` [rows, heads] (float32, a column slice
+    will do): head h's outputs are multiplied by sigmoid(gate[r, h]).  ``rotate`` = (n, rotary, pairs, src, dst, cos, sin,
+    positions): beside the product, in the same launch, the n elements at column x_off + h*x_head_stride + src of x are
+    rotated (pairs: neighbours; else i and i + rotary/2; elements from ``rotary`` on pass) and stored at column
+    out_off + h*out_head_stride + dst of out."""
     _need(x, torch.float32, "x")
     if wt.dim() != 3 or not wt.is_cuda or not wt.is_contiguous():
         raise ValueError("headwise_linear: weights must be a contiguous [heads, in, out] GPU tensor")
@@ -1045,10 +1113,27 @@ def headwise_linear(x: torch.Tensor, x_off: int, x_head_stride: int, wt: torch.T
         raise ValueError("headwise_linear: x or out narrower than the heads need")
     if x.shape[0] < rows or out.shape[0] < rows:
         raise ValueError("headwise_linear: buffers shorter than the rows")
+    gp, ldg = 0, 0
+    if gate is not None:
+        _need_strided(gate, torch.float32, "gate")
+        if gate.shape[1] < heads or gate.shape[0] < rows:
+            raise ValueError("headwise_linear: a gate a head is needed")
+        gp, ldg = gate.data_ptr(), gate.stride(0)
+    rot = (0, 0, 0, 0, 0, 0, 0, 0)
+    if rotate is not None and int(rotate[0]) > 0:
+        n, rotary, pairs, src, dst, cos, sin, positions = rotate
+        _need(cos, torch.float32, "cos table")
+        _need(sin, torch.float32, "sin table")
+        _need(positions, torch.int32, "positions")
+        if rotary % 2 or rotary > n or (rotary and (cos.shape[1] != rotary // 2 or sin.shape != cos.shape)) or positions.numel() < rows:
+            raise ValueError("headwise_linear: rotary tables must be [positions, rotary/2]")
+        if x_off + (heads - 1) * x_head_stride + src + n > x.shape[1] or out_off + (heads - 1) * out_head_stride + dst + n > out.shape[1]:
+            raise ValueError("headwise_linear: the rotated part does not fit x or out")
+        rot = (int(n), int(rotary), int(bool(pairs)), int(src), int(dst), cos.data_ptr(), sin.data_ptr(), positions.data_ptr())
     ob = _act_out(out, "out")
     _check(_fn("bw_headwise_linear")(x.data_ptr() + 4 * x_off, x.stride(0), x_head_stride, wt.data_ptr(), _is_bf16(wt, "weights"),
                                      inn, outn, out.data_ptr() + (2 if ob else 4) * out_off, ob, out.stride(0), out_head_stride,
-                                     rows, heads, _stream()), "headwise_linear")
+                                     rows, heads, gp, ldg, *rot, _stream()), "headwise_linear")
 
 
 def shared_key_attention(q: torch.Tensor, positions: torch.Tensor, block_table: torch.Tensor, tiles: Optional[torch.Tensor],
@@ -1142,12 +1227,13 @@ CONV_MAX_TAPS = 8
 
 def causal_conv(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
                 seq_rows: torch.Tensor, slots: torch.Tensor, positions: torch.Tensor, nseq: int, max_seq_rows: int,
-                out: torch.Tensor, in_bias: Optional[torch.Tensor] = None) -> None:
+                out: torch.Tensor, in_bias: Optional[torch.Tensor] = None, silu: bool = False) -> None:
     """out[t, c] = sum_j weight[c, j] * x[t - taps + 1 + j, c] (+ bias[c]) along every request's rows, the inputs before a
     portion's first row taken from ``state`` [slots, >= (taps - 1) * channels] (a view may start inside a wider slot),
     which then receives the portion's last taps - 1 inputs.  ``x`` [rows, >= channels] float32 (rows apart by its
     stride), ``out`` likewise.  ``max_seq_rows``: the most rows a request brings in this step.  ``in_bias`` [channels]
-    float32: added to every input on its way in (a projection's bias; the state then keeps inputs with it)."""
+    float32: added to every input on its way in (a projection's bias; the state then keeps inputs with it).  ``silu``: the outputs go
+    through SiLU."""
     if x.dtype != torch.float32 or out.dtype != torch.float32 or x.stride(1) != 1 or out.stride(1) != 1 or not (x.is_cuda and out.is_cuda):
         raise ValueError("causal_conv: x and out must be float32 GPU matrices with contiguous rows")
     if weight.dim() != 2 or not weight.is_cuda or not weight.is_contiguous():
@@ -1175,7 +1261,7 @@ def causal_conv(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tens
             raise ValueError("causal_conv: in_bias must be [channels]")
     _check(_fn("bw_causal_conv")(x.data_ptr(), x.stride(0), 0 if in_bias is None else in_bias.data_ptr(), weight.data_ptr(), 0 if bias is None else bias.data_ptr(), wb, taps,
                                  channels, sp, sld, seq_rows.data_ptr(), slots.data_ptr(), positions.data_ptr(), int(nseq),
-                                 int(max_seq_rows), out.data_ptr(), out.stride(0), _stream()), "causal_conv")
+                                 int(max_seq_rows), out.data_ptr(), out.stride(0), int(silu), _stream()), "causal_conv")
 
 
 def pair_rope_unit(src: torch.Tensor, positions: torch.Tensor, row_seq: torch.Tensor, block_table: torch.Tensor,
@@ -1435,24 +1521,52 @@ def moe_route_plan(logits: torch.Tensor, rows: int, top: int, groups: int, keep:
            "moe_route_plan")
 
 
+def moe_table_plan(tokens: torch.Tensor, feedback: Optional[torch.Tensor], rows: int, table: torch.Tensor, experts: int, weight: float,
+                   ids: torch.Tensor, wts: torch.Tensor, sorted_slots: torch.Tensor, place: torch.Tensor, tiles: torch.Tensor,
+                   meta: torch.Tensor) -> None:
+    """Routing by token id: row r's experts are ``table`` [vocab, top][token of r], each weighs ``weight``; choices, weights and
+    the plan in one launch.  Tokens as in ``embed``; a row without one takes the experts of the step's first row."""
+    _need(wts, torch.float32, "wts")
+    for t, what in ((tokens, "tokens"), (table, "table"), (ids, "ids"), (sorted_slots, "sorted"), (place, "place"), (tiles, "tiles"), (meta, "meta")):
+        _need(t, torch.int32, what)
+    vocab, top = table.shape
+    slots = rows * top
+    if tokens.numel() < rows or min(ids.numel(), wts.numel(), sorted_slots.numel(), place.numel()) < slots:
+        raise ValueError("moe_table_plan: buffers shorter than the rows")
+    if feedback is not None:
+        _need(feedback, torch.int32, "feedback")
+        if feedback.numel() < rows:
+            raise ValueError("moe_table_plan: feedback is shorter than the rows")
+    if tiles.numel() < 4 * moe_max_tiles(slots, experts) or meta.numel() < 1:
+        raise ValueError("moe_table_plan: the plan's tables are too small")
+    _check(_fn("bw_moe_table_plan")(tokens.data_ptr(), 0 if feedback is None else feedback.data_ptr(), rows, table.data_ptr(), vocab,
+                                    top, experts, float(weight), ids.data_ptr(), wts.data_ptr(), sorted_slots.data_ptr(),
+                                    place.data_ptr(), tiles.data_ptr(), meta.data_ptr(), _stream()), "moe_table_plan")
+
+
+MOE_DOWN, MOE_GATED, MOE_PLAIN = 0, 1, 2
+
+
 def moe_experts(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, sorted_slots: torch.Tensor, tiles: torch.Tensor,
-                meta: torch.Tensor, slots: int, top: int, gate_up: bool, limit: float = 0.0, alpha: float = 0.0,
+                meta: torch.Tensor, slots: int, top: int, form: int, limit: float = 0.0, alpha: float = 0.0,
                 round_out: bool = False) -> None:
-    """The experts' products over a plan's tiles.  ``gate_up``: x [rows, K] (a slot reads row slot // top), w [experts, 2N, K]
-    (gate rows, then up rows), out [slots, N] = the gated activation by sorted place.  Else: x [slots, K] by sorted place,
+    """The experts' products over a plan's tiles.  MOE_GATED: x [rows, K] (a slot reads row slot // top), w [experts, 2N, K]
+    (gate rows, then up rows), out [slots, N] = the gated activation by sorted place.  MOE_PLAIN: the same without a gate, w [experts, N, K], out = max(x W^T, 0)^2.  MOE_DOWN: x [slots, K] by sorted place,
     w [experts, N, K], out [slots, N] float32.  bfloat16 x runs on the matrix cores (bfloat16 weights, K a multiple of 8);
     float32 x runs 32-bit chains (``round_out``: the activation is rounded to bfloat16 values)."""
     if w.dim() != 3 or not w.is_cuda or not w.is_contiguous():
         raise ValueError("moe_experts: weights must be a contiguous [experts, N, K] GPU tensor")
     experts, N, K = w.shape
-    if gate_up:
+    if form not in (MOE_DOWN, MOE_GATED, MOE_PLAIN):
+        raise ValueError("moe_experts: an unknown form of the product")
+    if form == MOE_GATED:
         N //= 2
     xb, wb = _act_out(x, "x"), _is_bf16(w, "weights")
-    if x.shape[1] != K or out.shape[1] != N or out.shape[0] < slots or (not gate_up and x.shape[0] < slots):
+    if x.shape[1] != K or out.shape[1] != N or out.shape[0] < slots or (form == MOE_DOWN and x.shape[0] < slots):
         raise ValueError("moe_experts: x, w and out do not fit")
     if xb and (not wb or K % 8):
         raise ValueError("moe_experts: the matrix-core route takes bfloat16 weights and an inner size that is a multiple of 8")
-    want = torch.bfloat16 if (xb and gate_up) else torch.float32
+    want = torch.bfloat16 if (xb and form != MOE_DOWN) else torch.float32
     _need(out, want, "out")
     for t, what in ((sorted_slots, "sorted"), (tiles, "tiles"), (meta, "meta")):
         _need(t, torch.int32, what)
@@ -1460,7 +1574,7 @@ def moe_experts(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, sorted_slot
     if tiles.numel() < 4 * max_tiles or sorted_slots.numel() < slots:
         raise ValueError("moe_experts: the plan's tables are too small")
     _check(_fn("bw_moe_experts")(x.data_ptr(), xb, x.stride(0), x.shape[0], w.data_ptr(), wb, out.data_ptr(), out.stride(0), sorted_slots.data_ptr(),
-                                 tiles.data_ptr(), meta.data_ptr(), slots, max_tiles, top, K, N, int(gate_up), float(limit), float(alpha),
+                                 tiles.data_ptr(), meta.data_ptr(), slots, max_tiles, top, K, N, int(form), float(limit), float(alpha),
                                  int(round_out), _stream()), "moe_experts")
 
 

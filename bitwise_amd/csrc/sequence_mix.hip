@@ -22,6 +22,11 @@ __device__ __forceinline__ float log_sigmoid(float z) {
   return fminf(z, 0.0f) - log1pf(bw_expf(-fabsf(z)));
 }
 
+__device__ __forceinline__ float softplus(float z) {
+  // log(1 + e^z) = max(z, 0) + log1p(e^-|z|)
+  return fmaxf(z, 0.0f) + log1pf(bw_expf(-fabsf(z)));
+}
+
 template <typename OT>
 __device__ __forceinline__ void store_act(OT* p, float v) {
   if constexpr (sizeof(OT) == 2) *p = f32_to_bf16(v);
@@ -243,7 +248,7 @@ __global__ __launch_bounds__(256) void norm_shift_row_kernel(const float* __rest
 
 // ------------------------------------------------------------------------- the linear recurrence
 
-enum { RECUR_DECAY_PER_CHANNEL = 0, RECUR_SCALAR_GATES = 1, RECUR_BONUS_DECAY = 2, RECUR_FIXED_DECAY = 3 };
+enum { RECUR_DECAY_PER_CHANNEL = 0, RECUR_SCALAR_GATES = 1, RECUR_BONUS_DECAY = 2, RECUR_FIXED_DECAY = 3, RECUR_STEP_DECAY = 4 };
 
 // The sum over the lanes l, l + 64/SPLIT, ... that hold the parts of one column (every one of them gets it).
 template <int SPLIT>
@@ -265,8 +270,10 @@ struct RecurArgs {
   int ldp, q_off, k_off, v_off;
   const float* gate;       // per channel: decay logits [rows, ldg] at gate_off + head*dim + d;
   int ldg, gate_off, gate2_off;   // scalar gates: input gate at gate_off + head, forget gate at gate2_off + head
-  const float* bias;       // per channel: [heads*dim]; scalar gates: input-gate bias [heads]
-  const float* bias2;      // scalar gates: forget-gate bias [heads]
+  const float* bias;       // per channel: [heads*dim]; scalar gates: input-gate bias [heads]; step: bias of the step size [heads]
+  const float* bias2;      // scalar gates: forget-gate bias [heads]; step: the decay's rate [heads]
+  const float* skip;       // step: [heads], the weight of the token's own v in the read-out (null: none)
+  int heads_per_key;       // neighbouring heads that share one q and one k (1: every head has its own)
   float param;             // per channel: 1 / tau; scalar gates: the cap
   float qscale, kscale;
   float* state;            // [slots, state_ld]: S [heads][dim][vdim]; scalar gates also n [heads][dim] and m [heads]
@@ -298,6 +305,9 @@ struct RecurArgs {
 // RECUR_BONUS_DECAY:  alpha[d] = exp(-exp(z[d] + bias[d]));  o[j] = sum_d (S[d][j] + u[d] k[d] v[j]) q[d] with the S of the token
 //   before (the token's own k v^T is read through the bonus u = bias2 [heads*dim]), then S[d][j] <- alpha[d] S[d][j] + k[d] v[j].
 // RECUR_FIXED_DECAY:  as per channel with one constant decay a head, alpha[d] = bias[head]; no logits are read.
+// RECUR_STEP_DECAY:  a step size per head and token, delta = softplus(z + bias[head]) with z at gate_off + head;
+//   S[d][j] <- e^(-bias2[head] delta) S[d][j] + k[d] (delta v[j]),  o[j] = (S^T q)[j] + skip[head] v[j].
+// (a head's q and k are those of key group head / heads_per_key.)
 // (q is multiplied by qscale and k by kscale on their way into LDS.)
 //
 // A request's long portion can also run in three passes over chunks of its rows, which gives every chunk waves of its
@@ -310,7 +320,7 @@ struct RecurArgs {
 template <int MODE, int DPAD, int PHASE>
 __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a) {
   constexpr bool GATES = MODE == RECUR_SCALAR_GATES;
-  constexpr bool BONUS = MODE == RECUR_BONUS_DECAY, FIXED = MODE == RECUR_FIXED_DECAY;
+  constexpr bool BONUS = MODE == RECUR_BONUS_DECAY, FIXED = MODE == RECUR_FIXED_DECAY, STEP = MODE == RECUR_STEP_DECAY;
   constexpr int NN = (DPAD + 63) / 64;
   constexpr bool READ_OUT = PHASE != 1;
   // A column's key channels are split over SPLIT lanes (lane l, l + COLS, ... hold consecutive parts of column l mod COLS): a
@@ -321,7 +331,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   constexpr int DH = DPAD / SPLIT, COLS = 64 / SPLIT;
   __shared__ float qs[RC][DPAD];
   __shared__ float ks[RC][DPAD];
-  __shared__ float as[GATES ? 1 : RC][GATES ? 1 : DPAD];
+  __shared__ float as[GATES || STEP ? 1 : RC][GATES || STEP ? 1 : DPAD];
   __shared__ float gi[RC], gf[RC];
   __shared__ float vs[RW][RC][64];
   __shared__ float us[BONUS ? DPAD : 1];
@@ -380,6 +390,8 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
     for (int d = threadIdx.x; d < DPAD; d += 64 * RW) us[d] = d < dim ? a.bias2[h * dim + d] : 0.0f;
   }
   const float fixed_decay = FIXED ? a.bias[h] : 0.0f;
+  const float skip = STEP && a.skip != nullptr ? a.skip[h] : 0.0f;
+  const int hk = h / a.heads_per_key;
   for (int t0 = 0; t0 < count; t0 += RC) {
     const int tc = min(RC, count - t0);
     __syncthreads();
@@ -393,9 +405,9 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         const bool in = e < tc * DPAD && d < dim;
         const size_t row = (size_t)(first + t0 + min(t, tc - 1));
         const float* pr = a.proj + row * a.ldp;
-        qv[u] = in ? pr[a.q_off + h * dim + d] : 0.0f;
-        kv[u] = in ? pr[a.k_off + h * dim + d] : 0.0f;
-        if constexpr (!GATES && !FIXED) zv[u] = in ? a.gate[row * a.ldg + a.gate_off + h * dim + d] + a.bias[h * dim + d] : 0.0f;
+        qv[u] = in ? pr[a.q_off + hk * dim + d] : 0.0f;
+        kv[u] = in ? pr[a.k_off + hk * dim + d] : 0.0f;
+        if constexpr (!GATES && !FIXED && !STEP) zv[u] = in ? a.gate[row * a.ldg + a.gate_off + h * dim + d] + a.bias[h * dim + d] : 0.0f;
       }
 #pragma unroll
       for (int u = 0; u < 8; ++u) {
@@ -406,7 +418,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         ks[t][d] = kv[u] * a.kscale;
         if constexpr (FIXED) as[t][d] = d < dim ? fixed_decay : 0.0f;
         else if constexpr (BONUS) as[t][d] = d < dim ? bw_expf(-bw_expf(zv[u])) : 0.0f;
-        else if constexpr (!GATES) as[t][d] = d < dim ? bw_expf(log_sigmoid(zv[u]) * a.param) : 0.0f;
+        else if constexpr (!GATES && !STEP) as[t][d] = d < dim ? bw_expf(log_sigmoid(zv[u]) * a.param) : 0.0f;
       }
     }
     if constexpr (GATES) {
@@ -415,6 +427,14 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         const float cap = a.param;
         gi[lane] = cap * tanhf((pr[a.gate_off + h] + a.bias[h]) / cap);
         gf[lane] = log_sigmoid(cap * tanhf((pr[a.gate2_off + h] + a.bias2[h]) / cap));
+      }
+    }
+    if constexpr (STEP) {
+      if (wv == 0 && lane < tc) {
+        const float z = a.gate[(size_t)(first + t0 + lane) * a.ldg + a.gate_off + h] + a.bias[h];
+        const float delta = softplus(z);
+        gi[lane] = delta;
+        gf[lane] = bw_expf(-(a.bias2[h] * delta));
       }
     }
     // (a column's lanes read what its first lane wrote)
@@ -426,7 +446,20 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
     __syncthreads();
     for (int t = 0; t < tc; ++t) {
       float o = 0.0f;
-      if constexpr (!GATES) {
+      if constexpr (STEP) {
+        const float v = vs[wv][t][col];
+        const float fa = gf[t], bv = gi[t] * v;
+#pragma unroll
+        for (int d = 0; d < DH; ++d) {
+          Sreg[d] = fmaf(fa, Sreg[d], ks[t][dbase + d] * bv);
+          if constexpr (READ_OUT) o = fmaf(Sreg[d], qs[t][dbase + d], o);
+        }
+        if constexpr (PHASE == 1) {
+#pragma unroll
+          for (int i = 0; i < NN; ++i) nreg[i] *= fa;
+        }
+        if constexpr (READ_OUT) o = fmaf(skip, v, join_parts<SPLIT>(o));
+      } else if constexpr (!GATES) {
         const float v = vs[wv][t][col];
 #pragma unroll
         for (int d = 0; d < DH; ++d) {
@@ -473,7 +506,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         }
       }
       if constexpr (READ_OUT) {
-        if constexpr (!GATES) o = join_parts<SPLIT>(o);
+        if constexpr (!GATES && !STEP) o = join_parts<SPLIT>(o);
         if (live && lane < COLS) a.out[(size_t)(first + t0 + t) * a.ldo + h * vdim + j] = o;
       }
     }
@@ -599,6 +632,62 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   }
 }
 
+// ------------------------------------------------------------------------- output gate, then an RMS norm in equal parts
+
+// v = o[r][e] * silu(z[r][e]); out = v / sqrt(mean of v^2 over the part + eps) * weight[e], a row's parts being equal stretches
+// of ``size`` elements.  A workgroup per (row, part): thread t owns elements t, t + 256, ... (one chain over its squares),
+// the waves' sums are joined by wave_sum and added in wave order.  Parts of up to 256 GP_MAXV elements keep their values in
+// registers; the same chain either way.
+#define GP_MAXV 8
+template <typename OT>
+__global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __restrict__ o, int ldi, const float* __restrict__ z, int ldz,
+                                                              const float* __restrict__ weight, OT* __restrict__ out, int ldo,
+                                                              const int32_t* __restrict__ positions, int size, float eps) {
+  __shared__ float part[4];
+  const int row = blockIdx.x, base = blockIdx.y * size, tid = threadIdx.x;
+  if (positions[row] < 0) return;
+  const float* orow = o + (size_t)row * ldi + base;
+  const float* zrow = z + (size_t)row * ldz + base;
+  const float* wr = weight + base;
+  OT* dst = out + (size_t)row * ldo + base;
+  auto gated = [](float ov, float zv) { return ov * (zv * (1.0f / (1.0f + bw_expf(-zv)))); };
+  const bool small = size <= 256 * GP_MAXV;
+  float v[GP_MAXV];
+  float acc = 0.0f;
+  if (small) {
+    float ov[GP_MAXV], zv[GP_MAXV];
+#pragma unroll
+    for (int j = 0; j < GP_MAXV; ++j) {
+      const int e = min(tid + 256 * j, size - 1);
+      ov[j] = 256 * j < size ? orow[e] : 0.0f;
+      zv[j] = 256 * j < size ? zrow[e] : 0.0f;
+    }
+#pragma unroll
+    for (int j = 0; j < GP_MAXV; ++j) {
+      v[j] = tid + 256 * j < size ? gated(ov[j], zv[j]) : 0.0f;
+      acc = fmaf(v[j], v[j], acc);
+    }
+  } else {
+    for (int e = tid; e < size; e += 256) {
+      const float ve = gated(orow[e], zrow[e]);
+      acc = fmaf(ve, ve, acc);
+    }
+  }
+  acc = wave_sum(acc);
+  if ((tid & 63) == 0) part[tid >> 6] = acc;
+  __syncthreads();
+  const float inv = 1.0f / sqrtf((((part[0] + part[1]) + part[2]) + part[3]) / (float)size + eps);
+  if (small) {
+#pragma unroll
+    for (int j = 0; j < GP_MAXV; ++j) {
+      const int e = tid + 256 * j;
+      if (e < size) store_act(dst + e, (v[j] * inv) * wr[e]);
+    }
+  } else {
+    for (int e = tid; e < size; e += 256) store_act(dst + e, (gated(orow[e], zrow[e]) * inv) * wr[e]);
+  }
+}
+
 // ------------------------------------------------------------------------- gated unit
 
 enum { ACT_SILU = 0, ACT_GELU_TANH = 1, ACT_CLAMPED_SWISH = 2 };
@@ -624,6 +713,30 @@ __global__ void glu_kernel(const float* __restrict__ gu, int ldg, OT* __restrict
   store_act(hout + idx, h);
 }
 
+
+// ------------------------------------------------------------------------- activation without a gate
+
+// h = act(z) of a 32-bit product.  PLAIN_RELU2: max(z, 0)^2.  PLAIN_XIELU (p0 and p1 positive): z > 0: p0 z^2 + z/2;
+// z <= 0: (1/2 + p1) (e^z - 1 - z) + z/2.
+enum { PLAIN_RELU2 = 0, PLAIN_XIELU = 1 };
+
+template <typename OT>
+__global__ __launch_bounds__(256) void activate_kernel(const float* __restrict__ x, int ldx, OT* __restrict__ out, int ldo, int rows,
+                                                       int cols, int act, float p0, float p1) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= cols) return;
+  for (int r = blockIdx.y; r < rows; r += gridDim.y) {
+    const float z = x[(size_t)r * ldx + c];
+    float h;
+    if (act == PLAIN_XIELU) {
+      h = z > 0.0f ? fmaf(p0 * z, z, 0.5f * z) : fmaf(0.5f + p1, expm1f(z) - z, 0.5f * z);
+    } else {
+      const float m = fmaxf(z, 0.0f);
+      h = m * m;
+    }
+    store_act(out + (size_t)r * ldo + c, h);
+  }
+}
 
 // ------------------------------------------------------------------------- rotation of 32-bit projections in place
 
@@ -698,7 +811,7 @@ extern "C" int bw_norm_shift(const float* x, int ldx, const float* w, const floa
 
 extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_off, int k_off, int v_off, const float* gate,
                                     int ldg, int gate_off, int gate2_off, const float* bias, const float* bias2, float param,
-                                    float qscale, float kscale, float* state, long long state_ld, float* out, int ldo,
+                                    float qscale, float kscale, const float* skip, int heads_per_key, float* state, long long state_ld, float* out, int ldo,
                                     const int32_t* seq_rows, const int32_t* slots, const int32_t* positions, int nseq,
                                     int heads, int dim, int vdim, const int32_t* chunks, int nchunks, const int32_t* spans,
                                     int nspans, float* scan_local, float* scan_start, long long scan_floats, void* stream) {
@@ -707,18 +820,19 @@ extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_
     if (chunks == nullptr || spans == nullptr || nspans <= 0 || scan_local == nullptr || scan_start == nullptr) return -2;
     if (scan_floats < (long long)nchunks * heads * ((long long)dim * vdim + dim + 2)) return -6;
   }
-  if (heads <= 0 || dim <= 0 || vdim <= 0 || ldo < heads * vdim) return -2;
+  if (heads <= 0 || dim <= 0 || vdim <= 0 || ldo < heads * vdim || heads_per_key < 1 || heads % heads_per_key) return -2;
   const long long need = (long long)heads * dim * vdim + (mode == RECUR_SCALAR_GATES ? (long long)heads * dim + heads : 0);
   if (state_ld < need) return -2;
-  if (bias == nullptr || (mode != RECUR_FIXED_DECAY && gate == nullptr) || ((mode == RECUR_SCALAR_GATES || mode == RECUR_BONUS_DECAY) && bias2 == nullptr))
+  if (bias == nullptr || (mode != RECUR_FIXED_DECAY && gate == nullptr) || ((mode == RECUR_SCALAR_GATES || mode == RECUR_BONUS_DECAY || mode == RECUR_STEP_DECAY) && bias2 == nullptr))
     return -2;
-  RecurArgs a{proj, ldp, q_off, k_off, v_off, gate, ldg, gate_off, gate2_off, bias, bias2, param, qscale, kscale, state, state_ld,
+  RecurArgs a{proj, ldp, q_off, k_off, v_off, gate, ldg, gate_off, gate2_off, bias, bias2, skip, heads_per_key, param, qscale, kscale, state, state_ld,
               out, ldo, seq_rows, slots, positions, heads, dim, vdim, chunks, scan_local, scan_start};
   hipStream_t s = (hipStream_t)stream;
   if (mode == RECUR_SCALAR_GATES) return launch_recurrence_passes<RECUR_SCALAR_GATES>(a, nseq, nchunks, spans, nspans, s);
   if (mode == RECUR_DECAY_PER_CHANNEL) return launch_recurrence_passes<RECUR_DECAY_PER_CHANNEL>(a, nseq, nchunks, spans, nspans, s);
   if (mode == RECUR_BONUS_DECAY) return launch_recurrence_passes<RECUR_BONUS_DECAY>(a, nseq, nchunks, spans, nspans, s);
   if (mode == RECUR_FIXED_DECAY) return launch_recurrence_passes<RECUR_FIXED_DECAY>(a, nseq, nchunks, spans, nspans, s);
+  if (mode == RECUR_STEP_DECAY) return launch_recurrence_passes<RECUR_STEP_DECAY>(a, nseq, nchunks, spans, nspans, s);
   return -2;
 }
 
@@ -738,6 +852,20 @@ extern "C" int bw_head_norm_gate(const float* o, int ldi, const float* weight, i
   return BW_LAUNCH_CHECK();
 }
 
+extern "C" int bw_gated_part_norm(const float* o, int ldi, const float* z, int ldz, const float* weight, void* out, int out_is_bf16,
+                                  int ldo, const int32_t* positions, int rows, int parts, int size, float eps, void* stream) {
+  if (rows <= 0) return 0;
+  if (parts <= 0 || parts > 65535 || size <= 0 || ldi < parts * size || ldz < parts * size || ldo < parts * size) return -2;
+  const dim3 grid(rows, parts), block(256);
+  if (out_is_bf16)
+    hipLaunchKernelGGL(gated_part_norm_kernel<bf16_t>, grid, block, 0, (hipStream_t)stream, o, ldi, z, ldz, weight, (bf16_t*)out, ldo,
+                       positions, size, eps);
+  else
+    hipLaunchKernelGGL(gated_part_norm_kernel<float>, grid, block, 0, (hipStream_t)stream, o, ldi, z, ldz, weight, (float*)out, ldo,
+                       positions, size, eps);
+  return BW_LAUNCH_CHECK();
+}
+
 extern "C" int bw_glu(const float* gate_up, int ldg, void* h, int out_is_bf16, int rows, int inter, int act, float limit, float alpha,
                       const float* row_gate, int ld_row_gate, void* stream) {
   if (rows <= 0 || inter <= 0) return 0;
@@ -748,6 +876,16 @@ extern "C" int bw_glu(const float* gate_up, int ldg, void* h, int out_is_bf16, i
   const dim3 grid((unsigned)((n + 255) / 256)), block(256);
   if (out_is_bf16) hipLaunchKernelGGL(glu_kernel<bf16_t>, grid, block, 0, s, gate_up, ldg, (bf16_t*)h, n, inter, act, limit, alpha, row_gate, ld_row_gate);
   else hipLaunchKernelGGL(glu_kernel<float>, grid, block, 0, s, gate_up, ldg, (float*)h, n, inter, act, limit, alpha, row_gate, ld_row_gate);
+  return BW_LAUNCH_CHECK();
+}
+
+extern "C" int bw_activate(const float* x, int ldx, void* out, int out_is_bf16, int ldo, int rows, int cols, int act, float p0,
+                           float p1, void* stream) {
+  if (rows <= 0 || cols <= 0) return 0;
+  if (ldx < cols || ldo < cols || (act != PLAIN_RELU2 && act != PLAIN_XIELU)) return -2;
+  const dim3 grid((cols + 255) / 256, rows < 65535 ? rows : 65535), block(256);
+  if (out_is_bf16) hipLaunchKernelGGL(activate_kernel<bf16_t>, grid, block, 0, (hipStream_t)stream, x, ldx, (bf16_t*)out, ldo, rows, cols, act, p0, p1);
+  else hipLaunchKernelGGL(activate_kernel<float>, grid, block, 0, (hipStream_t)stream, x, ldx, (float*)out, ldo, rows, cols, act, p0, p1);
   return BW_LAUNCH_CHECK();
 }
 

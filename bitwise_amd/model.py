@@ -86,7 +86,7 @@ class Model:
         tensors = {}
         for name, ts in assembled.tensor_specs().items():
             if ts.kind == "int":
-                tensors[name] = torch.randint(0, 2 ** 15, ts.shape, generator=gen, dtype=torch.int32, device=rt.device)
+                tensors[name] = loader.random_table(ts, gen, rt.device)
                 continue
             z = torch.randn(ts.shape, generator=gen, dtype=torch.float32, device=rt.device)
             tensors[name] = loader.shape_values(ts.kind, z, sigma).to(wd)

@@ -24,10 +24,11 @@ class TensorSpec:
     "around_zero" (N(0, 0.1): a norm weight stored as its distance from 1), "unit_interval" (a mixing
     weight in (0, 1)), "bias" (N(0, 1): gate biases, sinks), "small_bias" (N(0, 0.1)), "conv" (taps of a short convolution,
     N(0, 0.5)), "router" (N(0, 0.3)), "gate_matrix" (N(0, 1/in): square matrices in front of a sigmoid) or "int" (integer
-    table, kept as int32).
+    table, kept as int32).  ``below`` (integer tables): the entries lie in 0 .. below - 1 and those of a row differ.
     """
     shape: Tuple[int, ...]
     kind: str = "linear"
+    below: int = 0
 
 
 @dataclass
@@ -282,6 +283,10 @@ class Mixer(Part):
 class FeedForward(Part):
     def forward_with_norm(self, ctx, x, norm, residual) -> bool:
         """As Mixer.forward_with_norm."""
+        return False
+
+    def forward_between_norms(self, ctx, x, norm, norm_behind) -> bool:
+        """As Mixer.forward_between_norms."""
         return False
 
     def forward(self, ctx, h, residual) -> None:

@@ -150,7 +150,7 @@ class SandwichBlock(Block):
             y = ctx.ws.buffer("sublayer_out", x.shape[1], torch.float32)
             self.mixer.forward_out(ctx, call, h, y)
             self.mixer_post_norm.add_normed(ctx, y, x)
-        if self.feed_forward is None:
+        if self.feed_forward is None or self.feed_forward.forward_between_norms(ctx, x, self.ffn_norm, self.ffn_post_norm):
             return
         h = self.ffn_norm.forward(ctx, x)
         if not self.feed_forward.forward_add_normed(ctx, h, self.ffn_post_norm, x):

@@ -3,9 +3,10 @@ part shared by all heads are cached; a head's key is [W_uk c | rotated part], it
 
 The scores are taken in the cache's own space: q_unrotated . (W_uk c) = (W_uk^T q_unrotated) . c, so a head's
 query becomes [W_uk^T q_unrotated | q_rotated] and one dot product with the cached vector is the score; the
-softmax-weighted sum of cached latents is projected to the head's values by W_uv afterwards.  The softmax has
+softmax-weighted sum of cached latents is projected to the head's values by W_uv afterwards.  The softmax may have
 a sink: one learned number per head that enters the denominator as exp(sink) beside the keys' terms (nothing is
-looked up for it, nothing is added to the output for it, and the score scale does not apply to it).
+looked up for it, nothing is added to the output for it, and the score scale does not apply to it).  The queries may go
+through an RMS-normed latent of their own, and a head's output may be multiplied by a sigmoid gate of the input.
 
 Rotations, the latent's norm, scores and softmax weights are 32-bit in both modes; the cache holds the mode's
 activation dtype.
@@ -53,9 +54,12 @@ def _tiles(ctx, rows_per_tile: int):
 class LatentAttention(Mixer):
     """params: width, heads, dim (unrotated query/key elements a head), rot_dim (rotated ones), vdim, kv_rank, scale, eps
     (of the latent's norm), window (None: all keys), position (PartSpec of the rotary tables; it may rotate fewer than
-    rot_dim elements, the rest of the rotated part passes unchanged).
-    tensors: q [heads*(dim+rot_dim), width]; dkv [kv_rank+rot_dim, width]; dkv.norm [kv_rank]; uk [heads*dim, kv_rank];
-    uv [heads*vdim, kv_rank]; sink [heads]; o [width, heads*vdim]."""
+    rot_dim elements, the rest of the rotated part passes unchanged; its pairs are neighbours if its ``layout`` says
+    "pairs", else half the rotated elements apart), q_rank (None: the queries are projected from the input), sink (True),
+    gate (False; True: one logit a head).
+    tensors: q [heads*(dim+rot_dim), width], or with q_rank dq [q_rank, width], dq.norm [q_rank] and uq
+    [heads*(dim+rot_dim), q_rank]; dkv [kv_rank+rot_dim, width]; dkv.norm [kv_rank]; uk [heads*dim, kv_rank];
+    uv [heads*vdim, kv_rank]; with sink: sink [heads]; with gate: g [heads, width]; o [width, heads*vdim]."""
 
     launches_through_ops = True
 
@@ -66,6 +70,8 @@ class LatentAttention(Mixer):
         self.dim, self.rot, self.vdim, self.rank = int(p["dim"]), int(p["rot_dim"]), int(p["vdim"]), int(p["kv_rank"])
         self.scale, self.eps = float(p["scale"]), float(p["eps"])
         self.window: Optional[int] = p.get("window")
+        self.q_rank = int(p.get("q_rank") or 0)
+        self.has_sink, self.has_gate = bool(p.get("sink", True)), bool(p.get("gate", False))
         self.key_width = self.rank + self.rot
         if self.rank > 512:
             raise ValueError(f"latent_attention: a latent of {self.rank} elements; the kernel takes up to 512")
@@ -74,10 +80,14 @@ class LatentAttention(Mixer):
         self.rotary = int(getattr(self.position, "rotary_dim", 0))
         if self.rotary % 2 or self.rotary > self.rot:
             raise ValueError(f"latent_attention: the position encoding rotates {self.rotary} elements, the rotated part has {self.rot}")
+        self.pairs = getattr(self.position, "layout", "halves") == "pairs"
         self.graph_safe = bool(getattr(self.position, "graph_safe", False))
         self.cos = self.sin = None
         self.proj: Optional[Linear] = None
+        self.uq: Optional[Linear] = None
         self.o: Optional[Linear] = None
+        self.sink: Optional[torch.Tensor] = None
+        self.q_norm: Optional[torch.Tensor] = None
         # bfloat16 mode: the attention runs on the matrix cores and keeps the latents a second time, transposed within
         # their pages, as the values (the page sizes it takes: multiples of 4); the 32-bit mode reads values and keys
         # from the one copy
@@ -88,27 +98,42 @@ class LatentAttention(Mixer):
             self.heads_per_group *= 2
 
     def tensors(self) -> Dict[str, TensorSpec]:
-        return {
-            "q": TensorSpec((self.heads * (self.dim + self.rot), self.width)),
-            "dkv": TensorSpec((self.key_width, self.width)),
-            "dkv.norm": TensorSpec((self.rank,), "norm"),
-            "uk": TensorSpec((self.heads * self.dim, self.rank)),
-            "uv": TensorSpec((self.heads * self.vdim, self.rank)),
-            "sink": TensorSpec((self.heads,), "bias"),
-            "o": TensorSpec((self.width, self.heads * self.vdim)),
-        }
+        nq = self.heads * (self.dim + self.rot)
+        out = {}
+        if self.q_rank:
+            out["dq"] = TensorSpec((self.q_rank, self.width))
+            out["dq.norm"] = TensorSpec((self.q_rank,), "norm")
+            out["uq"] = TensorSpec((nq, self.q_rank))
+        else:
+            out["q"] = TensorSpec((nq, self.width))
+        out["dkv"] = TensorSpec((self.key_width, self.width))
+        out["dkv.norm"] = TensorSpec((self.rank,), "norm")
+        out["uk"] = TensorSpec((self.heads * self.dim, self.rank))
+        out["uv"] = TensorSpec((self.heads * self.vdim, self.rank))
+        if self.has_sink:
+            out["sink"] = TensorSpec((self.heads,), "bias")
+        if self.has_gate:
+            out["g"] = TensorSpec((self.heads, self.width))
+        out["o"] = TensorSpec((self.width, self.heads * self.vdim))
+        return out
 
     def bind(self, tensors) -> None:
         self.cos, self.sin = self.position.tables()
-        q, dkv = tensors["q"], tensors["dkv"]
-        if q.dtype != dkv.dtype:
-            raise ValueError("q and dkv projections must be stored in one dtype to be stacked")
-        self.q_off, self.dkv_off = 0, q.shape[0]
-        self.proj = Linear(torch.cat([q, dkv], dim=0), self.rt)
+        # everything that reads the mixer's input is one product: [queries or their latent | down projection | gate]
+        stack = [tensors["dq" if self.q_rank else "q"], tensors["dkv"]] + ([tensors["g"]] if self.has_gate else [])
+        if len({t.dtype for t in stack}) != 1:
+            raise ValueError("the projections of the mixer's input must be stored in one dtype to be stacked")
+        self.q_off, self.dkv_off = 0, stack[0].shape[0]
+        self.gate_off = self.dkv_off + self.key_width
+        self.proj = Linear(torch.cat(stack, dim=0), self.rt)
+        if self.q_rank:
+            self.uq = Linear(tensors["uq"], self.rt)
+            self.q_norm = tensors["dq.norm"].to(self.rt.device).float().contiguous()
         self.o = Linear(tensors["o"], self.rt)
         dev = self.rt.device
         self.latent_norm = tensors["dkv.norm"].to(dev).float().contiguous()
-        self.sink = tensors["sink"].to(dev).float().contiguous()
+        if self.has_sink:
+            self.sink = tensors["sink"].to(dev).float().contiguous()
         # input-major per head: uk as stored is [head][dim][rank] (the transposed product wants exactly that);
         # uv [head][vdim][rank] is turned to [head][rank][vdim]
         self.uk_t = tensors["uk"].to(dev).view(self.heads, self.dim, self.rank).contiguous()
@@ -116,7 +141,8 @@ class LatentAttention(Mixer):
 
     def weight_bytes(self) -> int:
         small = self.uk_t.numel() * self.uk_t.element_size() + self.uv_t.numel() * self.uv_t.element_size()
-        return self.proj.nbytes() + self.o.nbytes() + small + 4 * (self.rank + self.heads)
+        return self.proj.nbytes() + (0 if self.uq is None else self.uq.nbytes()) + self.o.nbytes() + small + 4 * (
+            self.rank + self.q_rank + (self.heads if self.has_sink else 0))
 
     def cache_spec(self) -> CacheSpec:
         return CacheSpec(1, self.key_width, self.window, key_width=self.key_width,
@@ -125,19 +151,33 @@ class LatentAttention(Mixer):
     def page_sizes(self):
         return (4, 8, 16, 32, 64, 128) if self.on_matrix_cores else None
 
-    def forward(self, ctx, call, h, residual) -> None:
+    def _project(self, ctx, h) -> torch.Tensor:
+        y = ctx.ws.buffer("latent_proj", self.proj.out_features, torch.float32)
+        self.proj.store(ctx.ws, h, y, ctx.rows)
+        return y
+
+    def _run(self, ctx, call, y, target, add: bool) -> None:
+        """From the stacked product of the input (32-bit sums) to the mixer's output."""
         ws, rows = ctx.ws, ctx.rows
         table = ctx.block_tables[call.group]
-        y = ws.buffer("latent_proj", self.proj.out_features, torch.float32)
-        self.proj.store(ws, h, y, rows)
         mfma = self.on_matrix_cores
         # (the matrix-core kernel takes its queries rounded to bfloat16, so they are stored that way at once)
         qa = ws.buffer("latent_q", self.heads * self.key_width, torch.bfloat16 if mfma else torch.float32)
+        per = self.dim + self.rot
+        cq = ws.buffer("latent_cq", self.q_rank, qa.dtype) if self.q_rank else None
         ops.latent_prep(y, self.q_off, self.dkv_off, self.latent_norm, self.eps, self.cos, self.sin, ctx.positions, ctx.row_seq,
                         table, call.k_cache, qa, rows, self.heads, self.dim, self.rot, self.rotary, self.rank, ws.page_size,
-                        call.writes_cache, latent_t=call.v_cache if mfma else None)
-        # the unrotated query parts into the latent's space
-        ops.headwise_linear(y, self.q_off, self.dim + self.rot, self.uk_t, qa, 0, self.key_width, rows)
+                        call.writes_cache, latent_t=call.v_cache if mfma else None, pairs=self.pairs,
+                        q_latent=(self.q_norm, cq) if self.q_rank else None)
+        # the unrotated query parts into the latent's space (queries out of a latent of their own: their rotated parts are
+        # turned in the same launch)
+        if self.q_rank:
+            q = ws.buffer("latent_up_q", self.heads * per, torch.float32)
+            self.uq.store(ws, cq, q, rows)
+            ops.headwise_linear(q, 0, per, self.uk_t, qa, 0, self.key_width, rows,
+                                rotate=(self.rot, self.rotary, self.pairs, self.dim, self.rank, self.cos, self.sin, ctx.positions))
+        else:
+            ops.headwise_linear(y, self.q_off, per, self.uk_t, qa, 0, self.key_width, rows)
         lat = ws.buffer("latent_out", self.heads * self.rank, torch.float32)
         if mfma:
             self._attend_on_matrix_cores(ctx, call, qa, lat, table)
@@ -150,8 +190,28 @@ class LatentAttention(Mixer):
             if n_single:
                 ops.shared_key_attention(qa, ctx.positions, table, single, n_single, *common, 16)
         vals = ws.buffer("latent_values", self.heads * self.vdim, self.rt.act_dtype)
-        ops.headwise_linear(lat, 0, self.rank, self.uv_t, vals, 0, self.vdim, rows)
-        self.o.add_into(ws, vals, residual, rows)
+        ops.headwise_linear(lat, 0, self.rank, self.uv_t, vals, 0, self.vdim, rows,
+                            gate=y[:, self.gate_off:self.gate_off + self.heads] if self.has_gate else None)
+        if add:
+            self.o.add_into(ws, vals, target, rows)
+        else:
+            self.o.store(ws, vals, target, rows)
+
+    def forward(self, ctx, call, h, residual) -> None:
+        self._run(ctx, call, self._project(ctx, h), residual, True)
+
+    def forward_out(self, ctx, call, h, out) -> None:
+        self._run(ctx, call, self._project(ctx, h), out, False)
+
+    def forward_between_norms(self, ctx, call, x, norm, norm_behind) -> bool:
+        """Decode steps of few rows: the norm in front rides in the first product."""
+        y = ctx.ws.buffer("latent_proj", self.proj.out_features, torch.float32)
+        if not self.proj.store_normed(x, norm, y, ctx.rows):
+            return False
+        out = ctx.ws.buffer("sublayer_out", self.width, torch.float32)
+        self._run(ctx, call, y, out, False)
+        norm_behind.add_normed(ctx, out, x)
+        return True
 
     def _attend_on_matrix_cores(self, ctx, call, qa, lat, table) -> None:
         ws = ctx.ws

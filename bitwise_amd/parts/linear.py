@@ -67,6 +67,16 @@ class Linear:
             ops.gemm_f32(self._x32(ws, x, rows), self.weight, tmp, rows)
             ops.convert(tmp, out, rows)
 
+    def store_normed(self, x: torch.Tensor, norm, out: torch.Tensor, rows: int) -> bool:
+        """out[:rows] = norm(x[:rows]) @ W.T as one kernel (32-bit store), with the bits of the norm followed by ``store``.
+        False (and nothing is done) where the fused kernel does not take this step: many rows, the 32-bit mode, a norm of
+        another kind."""
+        from .norm import RMSNorm
+        if not (self.mfma and self.bias is None and type(norm) is RMSNorm and ops.can_fuse_norm(rows, self.weight, x)):
+            return False
+        ops.norm_gemm_bf16(x, norm.weight, norm.eps, self.weight, out, rows, ops.EPI_F32)
+        return True
+
     def add_into(self, ws, x: torch.Tensor, residual: torch.Tensor, rows: int) -> None:
         """residual[:rows] += x[:rows] @ W.T, the sum in 32-bit (src/model.cpp:300, :305)."""
         if self.bias is not None:

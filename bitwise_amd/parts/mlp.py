@@ -1,7 +1,7 @@
-"""Dense gated feed-forward (src/model.cpp:301-305, src/kernels.cpp:291-298):
+"""Dense feed-forwards.  The gated ones (src/model.cpp:301-305, src/kernels.cpp:291-298):
 one stacked product [gate; up], h = act(g) * u, down projection added into the residual stream.
 SwiGLU: act(g) = g * (1/(1+exp(-g))); the gated GELU uses the tanh form
-0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3)))."""
+0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))).  And one without a gate, h = act(W_up x)."""
 
 from __future__ import annotations
 
@@ -142,3 +142,79 @@ class ClampedGLU(GeGLU):
             self.down.add_into(ctx.ws, act, residual, ctx.rows)
         else:
             super().forward(ctx, h, residual)
+
+
+@register_feed_forward("mlp")
+class MLP(FeedForward):
+    """W_down act(W_up h), no gate.  ``act``: "relu2", max(z, 0)^2, or "xielu", the expanded integral of the exponential
+    linear unit with two learned numbers: z > 0: softplus(p) z^2 + z/2; z <= 0: (1/2 + softplus(q)) (e^z - 1 - z) + z/2.
+    params: width, inter, act, names (up, down and, for xielu, the tensor [p, q]).  The product leaves 32-bit sums, the
+    activation is one 32-bit kernel behind it, which rounds once for the down projection."""
+
+    graph_safe = True
+    launches_through_ops = True
+    ACTS = {"relu2": ops.PLAIN_RELU2, "xielu": ops.PLAIN_XIELU}
+
+    def __init__(self, params, runtime):
+        super().__init__(params, runtime)
+        self.width, self.inter = int(params["width"]), int(params["inter"])
+        if params.get("act") not in self.ACTS:
+            raise ValueError(f"mlp: the activation is one of {sorted(self.ACTS)}, not {params.get('act')!r}")
+        self.act = self.ACTS[params["act"]]
+        self.learned = self.act == ops.PLAIN_XIELU
+        self.names = tuple(params.get("names", ("up", "down", "act")))
+        if len(self.names) < (3 if self.learned else 2):
+            raise ValueError("mlp: tensors up, down and, where the activation has learned numbers, theirs")
+        self.coefficients = (0.0, 0.0)
+        self.up: Optional[Linear] = None
+        self.down: Optional[Linear] = None
+
+    def tensors(self) -> Dict[str, TensorSpec]:
+        out = {self.names[0]: TensorSpec((self.inter, self.width)), self.names[1]: TensorSpec((self.width, self.inter))}
+        if self.learned:
+            out[self.names[2]] = TensorSpec((2,), "bias")
+        return out
+
+    def bind(self, tensors) -> None:
+        self.up = Linear(tensors[self.names[0]], self.rt)
+        self.down = Linear(tensors[self.names[1]], self.rt)
+        if self.learned:
+            # (softplus in double precision on the host, rounded once where the kernel takes it)
+            p, q = torch.nn.functional.softplus(tensors[self.names[2]].detach().cpu().double()).tolist()
+            self.coefficients = (p, q)
+
+    def weight_bytes(self) -> int:
+        return self.up.nbytes() + self.down.nbytes()
+
+    def _activated(self, ctx, z) -> torch.Tensor:
+        act = ctx.ws.buffer("mlp_h", self.inter, self.rt.act_dtype)
+        ops.activate(z, act, ctx.rows, self.act, *self.coefficients)
+        return act
+
+    def _up(self, ctx, h) -> torch.Tensor:
+        z = ctx.ws.buffer("mlp_up", self.inter, torch.float32)
+        self.up.store(ctx.ws, h, z, ctx.rows)
+        return z
+
+    def forward(self, ctx, h, residual) -> None:
+        self.down.add_into(ctx.ws, self._activated(ctx, self._up(ctx, h)), residual, ctx.rows)
+
+    def forward_out(self, ctx, h, out) -> None:
+        self.down.store(ctx.ws, self._activated(ctx, self._up(ctx, h)), out, ctx.rows)
+
+    def forward_with_norm(self, ctx, x, norm, residual) -> bool:
+        z = ctx.ws.buffer("mlp_up", self.inter, torch.float32)
+        if not self.up.store_normed(x, norm, z, ctx.rows):
+            return False
+        self.down.add_into(ctx.ws, self._activated(ctx, z), residual, ctx.rows)
+        return True
+
+    def forward_between_norms(self, ctx, x, norm, norm_behind) -> bool:
+        """Decode steps of few rows: the norm in front rides in the up product."""
+        z = ctx.ws.buffer("mlp_up", self.inter, torch.float32)
+        if not self.up.store_normed(x, norm, z, ctx.rows):
+            return False
+        y = ctx.ws.buffer("sublayer_out", self.width, torch.float32)
+        self.down.store(ctx.ws, self._activated(ctx, z), y, ctx.rows)
+        norm_behind.add_normed(ctx, y, x)
+        return True

@@ -134,8 +134,10 @@ class _MatrixMemoryMixer(Mixer):
         self.proj.store(ctx.ws, h, y, ctx.rows)
         return y
 
-    def _recur(self, ctx, call, y, gate, gate_off, gate2_off, bias, bias2, param, raw, kscale: float = 1.0, at=None) -> None:
-        """``at``: where q (or r), k and v lie in a row of ``y``, if not at the stacked projection's own offsets."""
+    def _recur(self, ctx, call, y, gate, gate_off, gate2_off, bias, bias2, param, raw, kscale: float = 1.0, at=None, state=None,
+               heads_per_key: int = 1, skip=None) -> None:
+        """``at``: where q (or r), k and v lie in a row of ``y``, if not at the stacked projection's own
+        offsets.  ``state``: the memories' part of the slots, if they do not fill them."""
         at = self.offsets if at is None else at
         plan = _scan_plan(ctx)
         seq_rows, nseq, scan = ctx.seq_rows, ctx.nseq, None
@@ -147,8 +149,8 @@ class _MatrixMemoryMixer(Mixer):
             start = ctx.ws.buffer("recur_scan_start", most * rec, torch.float32, rows=1)
             scan = (chunks, nchunks, spans, nspans, local, start)
         ops.linear_recurrence(self.mode, y, at["r"] if "q" not in at else at["q"], at["k"], at["v"], gate, gate_off, gate2_off,
-                              bias, bias2, param, self.qscale, call.state, raw, seq_rows, ctx.slots, ctx.positions, nseq,
-                              self.heads, self.dim, self.vdim, scan=scan, kscale=kscale)
+                              bias, bias2, param, self.qscale, call.state if state is None else state, raw, seq_rows, ctx.slots, ctx.positions, nseq,
+                              self.heads, self.dim, self.vdim, scan=scan, kscale=kscale, heads_per_key=heads_per_key, skip=skip)
 
     def _finish(self, ctx, y, raw, target, add: bool = True, g_off: Optional[int] = None) -> None:
         act = ctx.ws.buffer("recur_gated", self.heads * self.vdim, self.rt.act_dtype)

@@ -52,6 +52,15 @@ def check_and_convert(specs: Mapping[str, TensorSpec], found: Mapping[str, torch
             if t.dtype not in (torch.int32, torch.int64):
                 wrong.append(f"{name}: stored as {t.dtype}, an integer table is needed")
                 continue
+            if spec.below:
+                bad = int(((t < 0) | (t >= spec.below)).sum())
+                if bad:
+                    wrong.append(f"{name}: {bad} entries outside 0 .. {spec.below - 1}")
+                    continue
+                ordered = t.reshape(-1, t.shape[-1]).sort(dim=-1).values
+                if bool((ordered[:, 1:] == ordered[:, :-1]).any()):
+                    wrong.append(f"{name}: a row names one entry twice")
+                    continue
             out[name] = t.to(torch.int32)
         elif t.dtype == torch.bfloat16 or t.dtype == torch.float32:
             out[name] = t
@@ -104,20 +113,31 @@ def shape_values(kind: str, z: torch.Tensor, sigma: float) -> torch.Tensor:
     return sigma * z
 
 
+def random_table(spec: TensorSpec, generator: torch.Generator, device="cpu") -> torch.Tensor:
+    """An integer table's random entries: uniform in [0, 2**15), or, bounded, the first of a random order of 0 .. below - 1."""
+    if not spec.below:
+        return torch.randint(0, 2 ** 15, spec.shape, generator=generator, dtype=torch.int32, device=device)
+    *rows, n = spec.shape
+    if n > spec.below:
+        raise ValueError(f"{n} different entries out of {spec.below}")
+    order = torch.rand((*rows, spec.below), generator=generator, device=device).argsort(dim=-1)
+    return order[..., :n].to(torch.int32).contiguous()
+
+
 def random_tensors(specs: Mapping[str, TensorSpec], seed: int, sigma: float = 0.02,
                    dtype: torch.dtype = torch.bfloat16) -> Iterator[Tuple[str, torch.Tensor]]:
     """Seeded random weights, one tensor after the other in the order of ``specs``.
 
     All draws come from one ``torch.Generator`` (CPU, ``manual_seed(seed)``) as float32
     standard normals in tensor order: linear and embedding weights are ``sigma * z``,
-    norm weights ``1 + 0.1 * z``, integer tables uniform in [0, 2**15).  Values are then
+    norm weights ``1 + 0.1 * z``, integer tables as ``random_table`` draws them.  Values are then
     rounded to ``dtype`` (round to nearest even for bfloat16).
     """
     g = torch.Generator(device="cpu")
     g.manual_seed(int(seed))
     for name, spec in specs.items():
         if spec.kind == "int":
-            yield name, torch.randint(0, 2 ** 15, spec.shape, generator=g, dtype=torch.int32)
+            yield name, random_table(spec, g)
             continue
         z = torch.randn(spec.shape, generator=g, dtype=torch.float32)
         yield name, shape_values(spec.kind, z, sigma).to(dtype)
