@@ -3,7 +3,7 @@
 random weights and uniform random token ids.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--dtype bf16|fp32] [--batch B] [--layers L]
-                    [--prefill-tokens T] [--no-points] [--shape smollm2|llama3_8b] [--trace-only] [--decode-phases] [--portion-align A] [--mixed] [--sweep] [--kuponex] [--sepedra] [--kikarax] [--vupolix]
+                    [--prefill-tokens T] [--no-points] [--shape smollm2|llama3_8b] [--trace-only] [--decode-phases] [--portion-align A] [--mixed] [--sweep] [--kuponex] [--sepedra] [--kikarax] [--vupolix] [--rasesun]
 
 A step is one decode step of the whole engine (scheduler, graph replay of the model, sampling,
 token hand-back) for a batch of B requests that each hold a 2,048-token context.  ``value`` is
@@ -226,6 +226,53 @@ def vupolix_comparison(bw, torch, steps: int, dtype: str, only: str = "") -> int
     return 0
 
 
+def rasesun_shape(width: int, expert_ff: int, experts: int = 32, top: int = 4, vocab: int = 32000) -> dict:
+    """A Rasesun of six layers (attention over a compressed cache, two state-space memories, and again) of which the third and
+    fourth run twice: eight layer runs.  Attention heads of 128 + 64 rotated elements behind a query latent, a latent of 512
+    elements, a window of 1,024 keys; memories of 128 x 64 a head, twice as wide as the model; a dense feed-forward as wide
+    as a token's experts together in the first layer, ``experts`` experts of which a token uses ``top`` in the others."""
+    big = width >= 4096
+    heads = width // 128
+    attention = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": 1536 if big else 768, "kv_rank": 512,
+                 "scale": 192 ** -0.5, "mask": {"size": 1024}, "rot": {"base": 500000.0, "dims": 64}}
+    memory = {"heads": width // 32, "vdim": 64, "state": 128, "groups": width // 512, "conv": 4, "norm_groups": width // 512}
+    dense = {"kind": "dense", "ff": top * expert_ff}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top}}
+    a = lambda mlp: {"type": "latent_attention", "mixer": dict(attention), "mlp": mlp}
+    m = {"type": "mamba2", "mixer": memory, "mlp": moe}
+    return {"architecture": "Rasesun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 8.0},
+            "logit_softcap": 30.0, "loop": {"start": 2, "stop": 4, "times": 2}, "layers": [a(dense), m, m, a(moe), m, m],
+            "max_positions": 16384, "eos_token_id": 2}
+
+
+def rasesun_comparison(bw, torch, steps: int, dtype: str, only: str = "") -> int:
+    """Prefill and decode of Rasesun at two layer sizes beside the Vupolix decoder (a norm on both sides of every sublayer,
+    matrix memories and windowed attention, routed experts, looped layers too) of equal width, depth and experts: one JSON
+    object a line."""
+    from bitwise_amd.measure import PEAK_FLOPS, measure_decode, measure_prefill
+    for name, width, expert_ff in (("2048x(4x2048 of 32)", 2048, 2048), ("4096x(4x3584 of 32)", 4096, 3584)):
+        for arch, cfg in (("Rasesun", rasesun_shape(width, expert_ff)), ("Vupolix", vupolix_shape(width, expert_ff))):
+            if only and only.lower() != arch.lower():
+                continue
+            model = bw.Model.random(cfg, seed=0, dtype=dtype, sigma=0.02, on_device=True)
+            for tokens in (512, 2048):
+                for exact in (True, False):
+                    # (exact_cuts False: the matrix memories run a long portion in three passes over chunks)
+                    m = measure_prefill(bw, torch, model, cfg, dtype, PEAK_FLOPS[dtype], tokens, exact_cuts=exact)
+                    print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "prefill_tokens": tokens, "exact_cuts": exact,
+                                      "ms": m["ms"], "tok_s": m["value"], "frac_of_matrix_peak": m["frac"]}), flush=True)
+            for batch in (1, 8, 64):
+                for exact in (True, False):
+                    # (exact_cuts False: a decoded token's keys of the compressed cache are cut into pieces)
+                    m = measure_decode(bw, torch, model, cfg, dtype, batch, steps, 4, context=2048, exact_cuts=exact)
+                    print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "decode_batch": batch, "context": 2048,
+                                      "exact_cuts": exact, "ms_per_step": m["ms_per_step"], "tok_s": m["tok_s"],
+                                      "frac_of_8_TBs": m["roofline"]["frac"]}), flush=True)
+            del model
+            torch.cuda.empty_cache()
+    return 0
+
+
 def sweep(bw, torch, steps: int, dtype: str) -> int:
     """Decode steps over batch and context, prefills over length: in bfloat16 at both shapes, in the 32-bit mode a
     coarser grid at the small one.  One JSON object a line."""
@@ -278,6 +325,9 @@ def main() -> int:
     ap.add_argument("--sepedra", nargs="?", const="both", default="", choices=["both", "sepedra", "llama"],
                     help="print a table instead of the line: prefill and decode of the Sepedra design at two layer sizes beside "
                          "the Llama decoder of equal width and depth with a feed-forward as wide as a token's experts together")
+    ap.add_argument("--rasesun", nargs="?", const="both", default="", choices=["both", "rasesun", "vupolix"],
+                    help="print a table instead of the line: prefill and decode of the Rasesun design at two layer sizes beside "
+                         "the Vupolix decoder of equal width, depth and experts (or one of the two)")
     ap.add_argument("--vupolix", nargs="?", const="both", default="", choices=["both", "vupolix", "sepedra"],
                     help="print a table instead of the line: prefill and decode of the Vupolix design at two layer sizes beside "
                          "the Sepedra decoder of equal width, depth and experts (or one of the two)")
@@ -302,6 +352,8 @@ def main() -> int:
     dtype = "bfloat16" if args.dtype == "bf16" else "float32"
     if args.sweep:
         return sweep(bw, torch, args.steps, dtype)
+    if args.rasesun:
+        return rasesun_comparison(bw, torch, min(args.steps, 32), dtype, "" if args.rasesun == "both" else args.rasesun)
     if args.vupolix:
         return vupolix_comparison(bw, torch, min(args.steps, 32), dtype, "" if args.vupolix == "both" else args.vupolix)
     if args.kikarax:

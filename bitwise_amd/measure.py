@@ -111,7 +111,35 @@ def vupolix_prefill_flops(cfg: dict, tokens: int) -> float:
     return total + 2 * w * cfg["vocab"]
 
 
+def rasesun_prefill_flops(cfg: dict, tokens: int) -> float:
+    """Multiply-adds times two of one prompt, every layer as often as it runs: every projection (the queries' two, the gates'),
+    the projections into and out of the latent's space, the attention's scores and weighted sums over the keys a query sees
+    (kv_rank + rot_dim and kv_rank elements a key and head, its window only), the memories' update and read-out of every
+    token (2 x state x vdim a head), the dense feed-forward, the chosen experts (the convolutions are left out)."""
+    w, total = cfg["width"], 0.0
+    loop = cfg.get("loop") or {"start": 0, "stop": 0, "times": 1}
+    for i, layer in enumerate(cfg["layers"]):
+        m, quadratic = layer["mixer"], 0.0
+        H, V = m["heads"], m["vdim"]
+        if layer["type"] == "mamba2":
+            N, inner = m["state"], H * V
+            per_token = w * (2 * inner + 2 * m["groups"] * N + H) + inner * w + 2 * H * N * V
+        else:
+            D, R, C, Q = m["dim"], m["rot_dim"], m["kv_rank"], m["q_rank"]
+            per_token = w * (Q + C + R + H) + Q * H * (D + R) + H * D * C + H * C * V + H * V * w
+            win = min((m.get("mask") or {"size": tokens})["size"], tokens)
+            quadratic = H * (2 * C + R) * (win * (win + 1) / 2 + (tokens - win) * win)
+        mlp = layer.get("mlp")
+        if mlp:
+            per_token += 2 * w * (mlp["ff"] if mlp["kind"] == "dense" else mlp["router"]["top"] * mlp["expert"]["ff"])
+        runs = loop["times"] if loop["start"] <= i < loop["stop"] else 1
+        total += runs * 2 * (per_token * tokens + quadratic)
+    return total + 2 * w * cfg["vocab"]
+
+
 def prefill_flops(cfg: dict, tokens: int) -> float:
+    if cfg.get("architecture") == "Rasesun":
+        return rasesun_prefill_flops(cfg, tokens)
     if cfg.get("architecture") == "Vupolix":
         return vupolix_prefill_flops(cfg, tokens)
     if cfg.get("architecture") == "Kikarax":
