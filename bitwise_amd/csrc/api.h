@@ -144,12 +144,12 @@ int bw_glu(const float* gate_up, int ldg, void* h, int out_is_bf16, int rows, in
            const float* row_gate, int ld_row_gate, void* stream);
 // Attention over a compressed cache shared by all heads (latent_attention.hip).
 // pairs 1: a rotated part's pairs are (2i, 2i+1) instead of (i, i + rotary/2).  q_rank > 0: the queries' own latent lies at
-// q_off and is normed into cq [rows, ldcq] (in the dtype qa_is_bf16 names); qa is not written.
+// q_off and is normed into cq [rows, ldcq]; qa is not written.
 int bw_latent_prep(const float* proj, int ldp, int q_off, int dkv_off, const float* norm_w, float eps,
                    const float* cos_table, const float* sin_table, const int32_t* positions, const int32_t* row_seq,
                    const int32_t* block_table, int table_stride, void* cache, void* latent_t, int cache_is_bf16, void* qa, int qa_is_bf16, int ldqa,
                    int rows, int heads, int dim, int rot, int rotary, int rank, int page_size, int write_cache, int pairs,
-                   int q_rank, const float* q_norm_w, void* cq, int ldcq, void* stream);
+                   int q_rank, const float* q_norm_w, void* cq, int cq_is_bf16, int ldcq, void* stream);
 // gate (optional): head h's outputs are multiplied by sigmoid(gate[r * ldg + h]).  rot_n > 0: beside the product, the rot_n
 // elements at x[r][h*xhs + rot_src ..] are rotated at the row's position and stored at out[r][h*ohs + rot_dst ..].
 int bw_headwise_linear(const float* x, int ldx, int xhs, const void* wt, int w_is_bf16, int in, int outn, void* out,

@@ -65,8 +65,8 @@ struct PrepArgs {
   // queries that go through a latent of their own (q_rank > 0; qa is not written then): the latent at q_off, normed into cq
   int q_rank;
   const float* q_norm_w;    // [q_rank]
-  void* cq;                 // [rows, ldcq] in the queries' dtype (qa_is_bf16)
-  int ldcq;
+  void* cq;                 // [rows, ldcq]
+  int ldcq, cq_is_bf16;
 };
 
 // A workgroup a row.
@@ -105,7 +105,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a, CT* __rest
     for (int i = threadIdx.x; i < a.q_rank; i += blockDim.x) {
       const float v = (ql[i] * inv) * a.q_norm_w[i];
       const size_t at = (size_t)row * a.ldcq + i;
-      if (a.qa_is_bf16) reinterpret_cast<bf16_t*>(a.cq)[at] = f32_to_bf16(v);
+      if (a.cq_is_bf16) reinterpret_cast<bf16_t*>(a.cq)[at] = f32_to_bf16(v);
       else reinterpret_cast<float*>(a.cq)[at] = v;
     }
     return;
@@ -671,12 +671,12 @@ extern "C" int bw_latent_prep(const float* proj, int ldp, int q_off, int dkv_off
                               const int32_t* row_seq, const int32_t* block_table, int table_stride, void* cache,
                               void* latent_t, int cache_is_bf16, void* qa, int qa_is_bf16, int ldqa, int rows, int heads, int dim, int rot, int rotary,
                               int rank, int page_size, int write_cache, int pairs, int q_rank,
-                              const float* q_norm_w, void* cq, int ldcq, void* stream) {
+                              const float* q_norm_w, void* cq, int cq_is_bf16, int ldcq, void* stream) {
   if (rows <= 0) return 0;
   if (heads <= 0 || dim < 0 || rot < 0 || rotary < 0 || rotary > rot || (rotary & 1) || rank <= 0 || page_size <= 0) return -2;
   if (q_rank < 0 || (q_rank > 0 ? (cq == nullptr || q_norm_w == nullptr || ldcq < q_rank) : ldqa < heads * (rank + rot))) return -2;
   PrepArgs a{proj, ldp, q_off, dkv_off, norm_w, eps, cos_table, sin_table, positions, row_seq, block_table, table_stride,
-             qa, ldqa, qa_is_bf16, heads, dim, rot, rotary, rank, page_size, write_cache, pairs, q_rank, q_norm_w, cq, ldcq};
+             qa, ldqa, qa_is_bf16, heads, dim, rot, rotary, rank, page_size, write_cache, pairs, q_rank, q_norm_w, cq, ldcq, cq_is_bf16};
   hipStream_t s = (hipStream_t)stream;
   if (cache_is_bf16) hipLaunchKernelGGL(latent_prep_kernel<bf16_t>, dim3(rows), dim3(256), 0, s, a, (bf16_t*)cache, (bf16_t*)latent_t);
   else hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(rows), dim3(256), 0, s, a, (float*)cache, (float*)latent_t);

@@ -102,7 +102,7 @@ _SIGS = {
                                      c_void_p, c_longlong, c_void_p],
     "bw_latent_prep": [c_void_p, c_int, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                        c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                       c_int, c_int, c_void_p, c_void_p, c_int, c_void_p],
+                       c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "bw_headwise_linear": [c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int,
                            c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p],
     "bw_causal_conv": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_longlong, c_void_p, c_void_p,
@@ -1063,7 +1063,7 @@ def latent_prep(proj: torch.Tensor, q_off: int, dkv_off: int, norm_w: torch.Tens
     ([pages, page_size * (rank + rot)]), and every head's rotated query part into ``qa`` [rows, heads * (rank + rot)]
     behind the place of its latent-space part.  ``latent_t`` [pages, rank * page_size]: the latent once more, transposed
     within its page ([element][slot]), for the matrix-core attention.  ``pairs``: elements 2i and 2i+1 of the rotated part
-    are turned together, instead of i and i + rotary/2.  ``q_latent`` = (weight [n], out [rows, n] in the queries' dtype):
+    are turned together, instead of i and i + rotary/2.  ``q_latent`` = (weight [n], out [rows, n]):
     what lies at q_off is no query but the queries' own latent, which is RMS-normed into ``out``; ``qa`` is not written."""
     _need(proj, torch.float32, "proj")
     _need(norm_w, torch.float32, "norm weight")
@@ -1076,8 +1076,8 @@ def latent_prep(proj: torch.Tensor, q_off: int, dkv_off: int, norm_w: torch.Tens
     if q_latent is not None:
         _need(q_latent[0], torch.float32, "query norm weight")
         q_rank, q_w, cq = q_latent[0].numel(), q_latent[0].data_ptr(), q_latent[1]
-        if cq.shape[1] != q_rank or cq.shape[0] < rows or cq.dtype != qa.dtype or not cq.is_contiguous():
-            raise ValueError("latent_prep: the queries' normed latent must be [rows, its size] in the queries' dtype")
+        if cq.shape[1] != q_rank or cq.shape[0] < rows or not cq.is_contiguous():
+            raise ValueError("latent_prep: the queries' normed latent must be [rows, its size]")
     if q_off + (q_rank or heads * (dim + rot)) > proj.shape[1] or dkv_off + width > proj.shape[1] or norm_w.numel() != rank:
         raise ValueError("latent_prep: projections or norm weight do not fit")
     if rotary % 2 or rotary > rot or (rotary and (cos.shape[1] != rotary // 2 or sin.shape != cos.shape)):
@@ -1094,7 +1094,8 @@ def latent_prep(proj: torch.Tensor, q_off: int, dkv_off: int, norm_w: torch.Tens
                                  block_table.stride(0), cache.data_ptr(), 0 if latent_t is None else latent_t.data_ptr(),
                                  _act_out(cache, "cache"), qa.data_ptr(), _act_out(qa, "qa"), qa.stride(0),
                                  rows, heads, dim, rot, rotary, rank, page_size, int(write_cache), int(pairs), q_rank, q_w,
-                                 0 if cq is None else cq.data_ptr(), 0 if cq is None else cq.stride(0), _stream()), "latent_prep")
+                                 0 if cq is None else cq.data_ptr(), 0 if cq is None else _act_out(cq, "cq"),
+                                 0 if cq is None else cq.stride(0), _stream()), "latent_prep")
 
 
 def headwise_linear(x: torch.Tensor, x_off: int, x_head_stride: int, wt: torch.Tensor, out: torch.Tensor, out_off: int,

@@ -164,7 +164,7 @@ class LatentAttention(Mixer):
         # (the matrix-core kernel takes its queries rounded to bfloat16, so they are stored that way at once)
         qa = ws.buffer("latent_q", self.heads * self.key_width, torch.bfloat16 if mfma else torch.float32)
         per = self.dim + self.rot
-        cq = ws.buffer("latent_cq", self.q_rank, qa.dtype) if self.q_rank else None
+        cq = ws.buffer("latent_cq", self.q_rank, self.rt.act_dtype) if self.q_rank else None
         ops.latent_prep(y, self.q_off, self.dkv_off, self.latent_norm, self.eps, self.cos, self.sin, ctx.positions, ctx.row_seq,
                         table, call.k_cache, qa, rows, self.heads, self.dim, self.rot, self.rotary, self.rank, ws.page_size,
                         call.writes_cache, latent_t=call.v_cache if mfma else None, pairs=self.pairs,
