@@ -160,11 +160,16 @@ int bw_shared_key_attention(const float* q, int ldq, const int32_t* positions, c
                             int table_stride, const int32_t* tiles, int num_tiles, const void* cache, int cache_is_bf16,
                             int num_pages, const float* sink, float* out, int ldo, int heads, int dk, int dv,
                             int page_size, int window, float scale, int heads_per_group, void* stream);
+int bw_headwise_linear_mfma(const void* x, int x_is_bf16, int ldx, int xhs, const void* w, int in, int outn, void* out,
+                            int out_is_bf16, int ldo, int ohs, int rows, int heads, const float* gate, int ldg, int rot_n,
+                            int rotary, int pairs, int rot_src, int rot_dst, const float* cos_table, const float* sin_table,
+                            const int32_t* positions, void* stream);
+int bw_shared_key_piece();      // keys of a piece: max_pieces below counts these
 int bw_shared_key_attention_mfma(const void* q, int ldq, const int32_t* positions, const int32_t* block_table,
                                  int table_stride, const int32_t* tiles, int num_tiles, const void* cache,
-                                 const void* latent_t, int num_pages, const float* sink, float* out, int ldo, int heads,
-                                 int dk, int dv, int page_size, int window, float scale, int heads_per_group, int nsplit,
-                                 int kchunk, float* partial, long long partial_floats, void* stream);
+                                 const void* latent_t, int num_pages, const float* sink, void* out, int out_is_bf16, int ldo,
+                                 int heads, int dk, int dv, int page_size, int window, float scale, int heads_per_group,
+                                 int max_pieces, float* partial, long long partial_floats, void* stream);
 // Mixers that convolve their projections over a few tokens, gate their outputs or carry a gated recurrence per channel,
 // and row operations of layers whose norm sits behind the sublayer (gated_mix.hip).  sink (the attention entry points
 // above): a score per head that joins the softmax's denominator and has no value, or null.

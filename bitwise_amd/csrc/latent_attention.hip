@@ -197,6 +197,107 @@ __global__ __launch_bounds__(256) void headwise_linear_kernel(const float* __res
   }
 }
 
+// The same product on the matrix cores, for bfloat16 weights that lie output-major, [head][outn][in] with in a multiple of 8:
+// x is rounded to bfloat16 where it enters (if it is not bfloat16 already), the sums are 32-bit, one chain of
+// v_mfma_f32_16x16x32_bf16 over the inner size ascending from zero for every block of 16 outputs x 16 rows, so a row's
+// bits depend neither on the rows beside it nor on the shape of the launch.  A wave owns 16 rows and 16 OB outputs; ROW_WAVES:
+// a workgroup's four waves are 64 rows (prompt portions), else 64 outputs of 16 rows.
+struct HeadGemmArgs {
+  const void* x;
+  int ldx, xhs;
+  const bf16_t* w;
+  int in, outn;
+  void* out;
+  int ldo, ohs, rows;
+  int aligned;             // rows and heads of out start at whole groups of four elements, outn is a multiple of 4
+};
+
+template <typename XT, typename OT, int OB, bool ROW_WAVES>
+__global__ __launch_bounds__(256) void headwise_mfma_kernel(HeadGemmArgs a, HeadExtras ex) {
+  const int lane = threadIdx.x & 63, n = lane & 15, g = lane >> 4, wv = wave_index();
+  const int h = blockIdx.y;
+  const XT* xh = reinterpret_cast<const XT*>(a.x) + (size_t)h * a.xhs;
+  OT* oh = reinterpret_cast<OT*>(a.out) + (size_t)h * a.ohs;
+  const int r_wg = blockIdx.x * (ROW_WAVES ? 64 : 16);
+  if ((int)blockIdx.z * 64 >= a.outn) {      // the extra block: the rotated part beside the product
+    if constexpr (sizeof(XT) == 4) {
+      const int half = ex.rotary / 2;
+      for (int e = threadIdx.x; e < (ROW_WAVES ? 64 : 16) * ex.rot_n; e += 256) {
+        const int r = r_wg + e / ex.rot_n, i = e % ex.rot_n;
+        const int pos = r < a.rows ? ex.positions[r] : -1;
+        if (pos < 0) continue;
+        store_f(oh + (size_t)r * a.ldo + ex.dst + i,
+                rotated_element(xh + (size_t)r * a.ldx + ex.src, i, ex.rotary, ex.pairs, ex.cos_table + (size_t)pos * half,
+                                ex.sin_table + (size_t)pos * half));
+      }
+    }
+    return;
+  }
+  const int r0 = r_wg + (ROW_WAVES ? 16 * wv : 0);
+  const int o0 = blockIdx.z * 64 + (ROW_WAVES ? 0 : 16 * wv);
+  if (r0 >= a.rows || o0 >= a.outn) return;
+  const XT* xr = xh + (size_t)min(r0 + n, a.rows - 1) * a.ldx;
+  const bf16_t* wr[OB];
+#pragma unroll
+  for (int b = 0; b < OB; ++b) wr[b] = a.w + ((size_t)h * a.outn + min(o0 + 16 * b + n, a.outn - 1)) * a.in;
+  f32x4 acc[OB];
+#pragma unroll
+  for (int b = 0; b < OB; ++b) acc[b] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  constexpr int U = 4;                       // steps of 32 elements whose loads are in flight together
+  for (int k0 = 0; k0 < a.in; k0 += 32 * U) {
+    u32x4 xf[U], wf[U][OB];
+#pragma unroll
+    for (int s = 0; s < U; ++s) {
+      const int k = k0 + 32 * s + 8 * g, kc = min(k, a.in - 8);
+#pragma unroll
+      for (int b = 0; b < OB; ++b) wf[s][b] = *reinterpret_cast<const u32x4*>(wr[b] + kc);
+      if constexpr (sizeof(XT) == 2) {
+        xf[s] = *reinterpret_cast<const u32x4*>(xr + kc);
+      } else {
+        const f32x4 lo = *reinterpret_cast<const f32x4*>(xr + kc), hi = *reinterpret_cast<const f32x4*>(xr + kc + 4);
+        xf[s] = (u32x4){pack_bf16x2(lo[0], lo[1]), pack_bf16x2(lo[2], lo[3]), pack_bf16x2(hi[0], hi[1]), pack_bf16x2(hi[2], hi[3])};
+      }
+      if (k >= a.in) xf[s] = (u32x4){0u, 0u, 0u, 0u};
+    }
+#pragma unroll
+    for (int s = 0; s < U; ++s)
+      if (k0 + 32 * s < a.in) {              // (scalar)
+#pragma unroll
+        for (int b = 0; b < OB; ++b)
+          acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(wf[s][b]), as_bf16x8(xf[s]), acc[b], 0, 0, 0);
+      }
+  }
+  const int r = r0 + n;
+  if (r >= a.rows) return;
+  const float gate = ex.gate != nullptr ? 1.0f / (1.0f + bw_expf(-ex.gate[(size_t)r * ex.ldg + h])) : 1.0f;
+#pragma unroll
+  for (int b = 0; b < OB; ++b) {
+    const int o = o0 + 16 * b + 4 * g;       // outputs o .. o + 3 of this lane's row
+    OT* dst = oh + (size_t)r * a.ldo + o;
+    if (a.aligned) {
+      if (o >= a.outn) continue;
+      if constexpr (sizeof(OT) == 2)
+        *reinterpret_cast<u32x2*>(dst) = (u32x2){pack_bf16x2(acc[b][0] * gate, acc[b][1] * gate), pack_bf16x2(acc[b][2] * gate, acc[b][3] * gate)};
+      else
+        *reinterpret_cast<f32x4*>(dst) = acc[b] * gate;
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (o + i < a.outn) store_f(dst + i, acc[b][i] * gate);
+    }
+  }
+}
+
+template <typename XT, typename OT>
+int launch_headwise_mfma(const HeadGemmArgs& a, const HeadExtras& ex, int heads, hipStream_t s) {
+  const int oz = (a.outn + 63) / 64 + (ex.rot_n > 0 ? 1 : 0);
+  if (a.rows > 64)
+    hipLaunchKernelGGL((headwise_mfma_kernel<XT, OT, 4, true>), dim3((a.rows + 63) / 64, heads, oz), dim3(256), 0, s, a, ex);
+  else
+    hipLaunchKernelGGL((headwise_mfma_kernel<XT, OT, 1, false>), dim3((a.rows + 15) / 16, heads, oz), dim3(256), 0, s, a, ex);
+  return BW_LAUNCH_CHECK();
+}
+
 // ------------------------------------------------------------------------- attention over shared keys
 
 struct SharedKeyArgs {
@@ -394,15 +495,22 @@ int launch_shared_key(const SharedKeyArgs& a, const CT* cache, int num_tiles, hi
 
 // ------------------------------------------------------------------------- the same attention on the matrix cores
 
-// bfloat16 caches whose key vectors are whole 16-byte groups.  A wave per (tile, group of heads, split of the keys): 16
-// query vectors (16 / hg rows x hg heads), keys in blocks of 64.  Scores: v_mfma_f32_16x16x32_bf16 with the keys as rows
-// (operand A, straight from the cache: a lane reads 8 consecutive elements of its key) and the queries as columns
-// (operand B, rounded to bfloat16 once, from LDS); 32-bit sums, scaled, masked, softmax in 32-bit with a running maximum.
-// The weighted sum takes the weights rounded to bfloat16 as columns and the values as rows d of a second copy of the
-// latent that the cache write leaves transposed, [page][d][slot]: a lane's 8 keys are two runs of 4 consecutive slots
-// (the keys of its four scores in two neighbouring sub-blocks of 16).  A lane's scores, sums and outputs all belong to
-// query (lane mod 16).  With nsplit > 1 a wave takes kchunk keys and leaves (maximum, denominator, sums) for
-// shared_key_combine_kernel; the sink joins where the result is finished.
+// bfloat16 caches whose key vectors are whole 16-byte groups.  A workgroup of four waves per (tile of rows, group of ``hg``
+// heads): 16 QT query vectors (16 QT / hg rows x hg heads).  The keys are cut into pieces of SK_PIECE keys at absolute
+// positions, and a piece is one unit of arithmetic: its scores, the largest of them that a query sees, the weights relative to
+// that maximum (32-bit, rounded to bfloat16 where they enter the product with the values), their sum, and the weighted sum of
+// the values as one chain over the piece's keys.  Pieces are then folded in order, (m, l, o) <- fold((m, l, o), piece) by
+// ``fold_piece``.  A prompt's tile walks the pieces of its window and folds as it goes; a single token's pieces get a workgroup
+// each, leave (maximum, sum, values) in memory, and shared_key_combine_kernel folds them by the same operations in the same
+// order: a position's bits do not depend on whether it came alone or inside a portion.
+//
+// Within a piece: scores by v_mfma_f32_16x16x32_bf16 with the keys as rows (operand A, straight from the cache: a wave takes 32
+// of the piece's keys, a lane reads 8 consecutive elements of its key) and the queries as columns (operand B, from LDS).  The
+// weights go through LDS; a wave then owns every fourth block of 16 value elements, read from the second copy of the latent that
+// the cache write leaves transposed, [page][element][slot]: a lane's 8 keys are 16 consecutive bytes of its element's row.
+#define SK_PIECE 128
+#define SK_PSTRIDE (SK_PIECE + 8)
+
 struct MfmaAttnArgs {
   const bf16_t* q;         // [rows, ldq] bfloat16: head h at h * dk
   int ldq;
@@ -411,10 +519,11 @@ struct MfmaAttnArgs {
   int table_stride;
   const int32_t* tiles;
   const float* sink;
-  float* out;
-  int ldo;
-  float* partial;          // [tiles][heads][nsplit][dv + 2]
-  int heads, dk, dv, page_size, window, hg, num_pages, nsplit, kchunk;
+  void* out;               // [rows, ldo], bfloat16 or 32-bit
+  int ldo, out_is_bf16;
+  float* partial;          // [tiles][heads][max_pieces][dv], then as many (maximum, sum)
+  float* partial_ml;
+  int heads, dk, dv, page_size, window, hg, num_pages, max_pieces;
   float scale;
 };
 
@@ -434,234 +543,355 @@ __device__ __forceinline__ float across_groups_sum(float v) {
   return a + b;
 }
 
-template <int NDT>
-__global__ __launch_bounds__(64) void shared_key_attention_mfma_kernel(MfmaAttnArgs a, const bf16_t* __restrict__ kc,
-                                                                       const bf16_t* __restrict__ vt) {
-  extern __shared__ bf16_t qs[];           // [16][qstride]
-  const int lane = threadIdx.x, n = lane & 15, g = lane >> 4;
-  const int t = blockIdx.x, h0 = blockIdx.y * a.hg, split = blockIdx.z;
+// A piece with maximum mp and sum lp joins what was folded so far: the factors for the old sums (c1) and the piece's (c2).
+__device__ __forceinline__ void fold_piece(float& m, float& l, float mp, float lp, float& c1, float& c2) {
+  const float mn = fmaxf(m, mp);
+  c1 = m == -INFINITY ? 0.0f : fast_exp(m - mn);
+  c2 = mp == -INFINITY ? 0.0f : fast_exp(mp - mn);
+  l = fmaf(lp, c2, l * c1);
+  m = mn;
+}
+
+// The factor on a query's folded sums: 1 / (denominator with the sink), scaled to the sink if that is larger.
+__device__ __forceinline__ float finish_softmax(float m, float l, float sk) {
+  const float mf = fmaxf(m, sk);
+  const float cm = m == -INFINITY ? 0.0f : fast_exp(m - mf);
+  const float lt = l * cm + (sk == -INFINITY ? 0.0f : fast_exp(sk - mf));
+  return lt > 0.0f ? cm / lt : 0.0f;
+}
+
+__device__ __forceinline__ void store_out(const MfmaAttnArgs& a, size_t at, float v) {
+  if (a.out_is_bf16) reinterpret_cast<bf16_t*>(a.out)[at] = f32_to_bf16(v);
+  else reinterpret_cast<float*>(a.out)[at] = v;
+}
+
+// NDT: blocks of 16 value elements a wave owns (wave w: blocks w, w + 4, ...).  QT 1: a workgroup a piece (single tokens).
+template <int QT, int NDT>
+__global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttnArgs a, const bf16_t* __restrict__ kc,
+                                                                        const bf16_t* __restrict__ vt) {
+  constexpr bool PIECES = QT == 1;
+  constexpr int NQ = 16 * QT;
+  extern __shared__ bf16_t sk_lds[];       // queries [NQ][qstride], weights [NQ][SK_PSTRIDE]
+  __shared__ float red_max[4][NQ], red_sum[4][NQ];
+  const int lane = threadIdx.x & 63, n = lane & 15, g = lane >> 4, wv = wave_index();
+  const int t = blockIdx.x, h0 = blockIdx.y * a.hg;
   int r0, nr, seq;
   if (a.tiles != nullptr) {
-    r0 = a.tiles[4 * t];
-    nr = a.tiles[4 * t + 1];
-    seq = a.tiles[4 * t + 2];
+    r0 = __builtin_amdgcn_readfirstlane(a.tiles[4 * t]);
+    nr = __builtin_amdgcn_readfirstlane(a.tiles[4 * t + 1]);
+    seq = __builtin_amdgcn_readfirstlane(a.tiles[4 * t + 2]);
   } else {
     r0 = t;
     nr = 1;
     seq = t;
   }
   if (nr <= 0) return;
-  const int pos0 = a.positions[r0];
+  const int pos0 = __builtin_amdgcn_readfirstlane(a.positions[r0]);
   if (pos0 < 0) return;
   const int pmax = pos0 + nr - 1;
-  const int rl = n / a.hg, h = h0 + n % a.hg;
-  const bool qok = rl < nr && h < a.heads;
-  const int qpos = qok ? pos0 + rl : -1;
-  const int qlo = a.window > 0 ? max(0, qpos - a.window + 1) : 0;
-  const int dkp = (a.dk + 31) & ~31, qstride = dkp + 8;
+  const int lo_first = a.window > 0 ? max(0, pos0 - a.window + 1) : 0;
+  int piece = lo_first / SK_PIECE;
+  const int last = pmax / SK_PIECE;
+  if constexpr (PIECES) {
+    piece += blockIdx.z;
+    if (piece > last) return;
+  }
+  const int dk = a.dk, dv = a.dv, ps = a.page_size;
+  const int dkp = (dk + 31) & ~31, qstride = dkp + 8;
+  bf16_t* qs = sk_lds;
+  bf16_t* pw = sk_lds + NQ * qstride;
   {
     const int groups = dkp >> 3;             // 16-byte groups of a query vector (dk is a multiple of 8)
-#pragma unroll 4
-    for (int e = lane; e < 16 * groups; e += 64) {
+    for (int e = threadIdx.x; e < NQ * groups; e += 256) {
       const int qn = e / groups, d = (e % groups) * 8;
       const int r2 = qn / a.hg, h2 = h0 + qn % a.hg;
       u32x4 v = {0u, 0u, 0u, 0u};
-      if (r2 < nr && h2 < a.heads && d < a.dk) v = *reinterpret_cast<const u32x4*>(a.q + (size_t)(r0 + r2) * a.ldq + h2 * a.dk + d);
+      if (r2 < nr && h2 < a.heads && d < dk) v = *reinterpret_cast<const u32x4*>(a.q + (size_t)(r0 + r2) * a.ldq + h2 * dk + d);
       *reinterpret_cast<u32x4*>(qs + qn * qstride + d) = v;
     }
   }
-  __syncthreads();
-
-  const int lo_first = a.window > 0 ? max(0, pos0 - a.window + 1) : 0;
-  int k_begin = lo_first & ~63, k_end = pmax + 1;
-  if (a.nsplit > 1) {
-    k_begin = max(k_begin, split * a.kchunk);
-    k_end = min(k_end, (split + 1) * a.kchunk);
+  const int qt_live = min(QT, (nr * a.hg + 15) >> 4);      // tiles of 16 queries that hold one (scalar)
+  int qpos[QT], qlo[QT];
+#pragma unroll
+  for (int c = 0; c < QT; ++c) {
+    const int qn = 16 * c + n, rl = qn / a.hg;
+    const bool ok = rl < nr && h0 + qn % a.hg < a.heads;
+    qpos[c] = ok ? pos0 + rl : -1;
+    qlo[c] = a.window > 0 ? max(0, qpos[c] - a.window + 1) : 0;
   }
   const int32_t* table = a.block_table + (size_t)seq * a.table_stride;
-  const int ps = a.page_size, dk = a.dk, dv = a.dv;
+  float m[QT], l[QT];
+  f32x4 acc[NDT][QT];
+#pragma unroll
+  for (int c = 0; c < QT; ++c) {
+    m[c] = -INFINITY;
+    l[c] = 0.0f;
+#pragma unroll
+    for (int j = 0; j < NDT; ++j) acc[j][c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  }
+  __syncthreads();
 
-  float m = -INFINITY, lsum = 0.0f;
-  f32x4 acc[NDT];
+  for (; piece <= last; ++piece) {
+    const int k0 = piece * SK_PIECE, kw = k0 + 32 * wv;
+    // where this lane's keys and runs of values lie
+    const bf16_t* krow[2];
 #pragma unroll
-  for (int dt = 0; dt < NDT; ++dt) acc[dt] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int u = 0; u < 2; ++u) {
+      const int kj = min(kw + 16 * u + n, pmax);
+      krow[u] = kc + ((size_t)min(max(table[kj / ps], 0), a.num_pages - 1) * ps + kj % ps) * dk;
+    }
+    const bf16_t* vrun[4];
+    int vpage2[4];                           // (pages of four slots: the run's second half lies in a page of its own)
+#pragma unroll
+    for (int sg = 0; sg < 4; ++sg) {
+      const int c = min(k0 + 32 * sg + 8 * g, pmax & ~7);
+      vrun[sg] = vt + (size_t)min(max(table[c / ps], 0), a.num_pages - 1) * dv * ps + c % ps;
+      vpage2[sg] = ps < 8 ? min(max(table[min(c + 4, pmax) / ps], 0), a.num_pages - 1) : 0;
+    }
+    auto load_values = [&](int sg, int j) -> u32x4 {
+      const int d = min(16 * (4 * j + wv) + n, dv - 1);     // (rows past the values are computed and never stored)
+      if (ps >= 8) return *reinterpret_cast<const u32x4*>(vrun[sg] + (size_t)d * ps);
+      const u32x2 lo = *reinterpret_cast<const u32x2*>(vrun[sg] + (size_t)d * ps);
+      const u32x2 hi = *reinterpret_cast<const u32x2*>(vt + (size_t)vpage2[sg] * dv * ps + (size_t)d * ps);
+      return (u32x4){lo[0], lo[1], hi[0], hi[1]};
+    };
 
-  for (int kb0 = k_begin; kb0 < k_end; kb0 += 64) {
-    const bf16_t* krow[4];
+    // ---- scores of this wave's 32 keys: lane (n, g) gets keys kw + 16u + 4g + i of query n of every tile
+    f32x4 st[2][QT];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int kj = min(kb0 + 16 * u + n, pmax);
-      const int page = min(max(table[kj / ps], 0), a.num_pages - 1);
-      krow[u] = kc + ((size_t)page * ps + kj % ps) * dk;
-    }
-    // (where the values' runs of 4 keys lie: asked of the table together with the keys' pages)
-    const bf16_t* vrun[2][2];
+    for (int u = 0; u < 2; ++u)
 #pragma unroll
-    for (int w = 0; w < 2; ++w)
+      for (int c = 0; c < QT; ++c) st[u][c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    if (kw <= pmax && kw + 31 >= lo_first) {                 // (scalar: some query of the tile may see one of them)
+      constexpr int KST = QT == 1 ? 18 : 9;                  // steps of 32 elements whose loads are in flight together
+      for (int d1 = 0; d1 < dkp; d1 += 32 * KST) {
+        u32x4 kf[KST][2];
 #pragma unroll
-      for (int x = 0; x < 2; ++x) {
-        const int c = min(kb0 + 32 * w + 16 * x + 4 * g, pmax & ~3);
-        vrun[w][x] = vt + (size_t)min(max(table[c / ps], 0), a.num_pages - 1) * dv * ps + c % ps;
-      }
-    f32x4 st[4];
+        for (int s4 = 0; s4 < KST; ++s4) {
+          // (elements past the key vector meet zeros in the query)
+          const int d0 = min(d1 + 32 * s4 + 8 * g, dk - 8);
+          if (d1 + 32 * s4 < dkp) {                          // (scalar)
+            kf[s4][0] = *reinterpret_cast<const u32x4*>(krow[0] + d0);
+            kf[s4][1] = *reinterpret_cast<const u32x4*>(krow[1] + d0);
+          }
+        }
 #pragma unroll
-    for (int u = 0; u < 4; ++u) st[u] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    // KST steps of 32 elements at a time: their 4 KST loads are in flight together (a single token's piece of 64 keys
-    // is one block, and what it waits for is memory)
-    constexpr int KST = NDT <= 16 ? 10 : 6;
-    for (int d1 = 8 * g; d1 < dkp; d1 += 32 * KST) {
-      u32x4 kf[KST][4], qf[KST];
+        for (int s4 = 0; s4 < KST; ++s4) {
+          if (d1 + 32 * s4 < dkp) {
 #pragma unroll
-      for (int s4 = 0; s4 < KST; ++s4) {
-        const int d0 = d1 + 32 * s4;
-        qf[s4] = d0 < dkp ? *reinterpret_cast<const u32x4*>(qs + n * qstride + d0) : (u32x4){0u, 0u, 0u, 0u};
-#pragma unroll
-        for (int u = 0; u < 4; ++u) kf[s4][u] = d0 < dk ? *reinterpret_cast<const u32x4*>(krow[u] + d0) : (u32x4){0u, 0u, 0u, 0u};
-      }
-#pragma unroll
-      for (int s4 = 0; s4 < KST; ++s4)
-#pragma unroll
-        for (int u = 0; u < 4; ++u)
-          st[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(kf[s4][u]), as_bf16x8(qf[s4]), st[u], 0, 0, 0);
-    }
-    // this lane: query n, keys kb0 + 16u + 4g + i
-    float mx = -INFINITY;
-#pragma unroll
-    for (int u = 0; u < 4; ++u)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int key = kb0 + 16 * u + 4 * g + i;
-        const bool valid = key <= qpos && key >= qlo && key < k_end;
-        const float sv = valid ? st[u][i] * a.scale : -INFINITY;
-        st[u][i] = sv;
-        mx = fmaxf(mx, sv);
-      }
-    mx = across_groups_max(mx);
-    const float mn = fmaxf(m, mx);
-    const float base = mn == -INFINITY ? 0.0f : mn;
-    const float corr = m == -INFINITY ? 0.0f : fast_exp(m - base);
-    float psum = 0.0f;
-#pragma unroll
-    for (int u = 0; u < 4; ++u)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const float pv = st[u][i] == -INFINITY ? 0.0f : fast_exp(st[u][i] - base);
-        st[u][i] = pv;
-        psum += pv;
-      }
-    lsum = lsum * corr + psum;
-    m = mn;
-#pragma unroll
-    for (int dt = 0; dt < NDT; ++dt) acc[dt] *= corr;
-    const bool ragged = kb0 + 63 > pmax || kb0 < lo_first;       // slots behind the last key, or before the window, may hold anything
-#pragma unroll
-    for (int w = 0; w < 2; ++w) {
-      const u32x4 pf = {pack_bf16x2(st[2 * w][0], st[2 * w][1]), pack_bf16x2(st[2 * w][2], st[2 * w][3]),
-                        pack_bf16x2(st[2 * w + 1][0], st[2 * w + 1][1]), pack_bf16x2(st[2 * w + 1][2], st[2 * w + 1][3])};
-      const int key0 = kb0 + 32 * w + 4 * g, key1 = key0 + 16;
-      const bf16_t* b0 = vrun[w][0];
-      const bf16_t* b1 = vrun[w][1];
-      uint32_t keep0[2] = {0xffffffffu, 0xffffffffu}, keep1[2] = {0xffffffffu, 0xffffffffu};
-      if (ragged) {
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const uint32_t bits = 0xffffu << (16 * (e & 1));
-          if (key0 + e > pmax || key0 + e < lo_first) keep0[e >> 1] &= ~bits;
-          if (key1 + e > pmax || key1 + e < lo_first) keep1[e >> 1] &= ~bits;
+            for (int c = 0; c < QT; ++c) {
+              if (c < qt_live) {                             // (scalar)
+                const u32x4 qf = *reinterpret_cast<const u32x4*>(qs + (16 * c + n) * qstride + d1 + 32 * s4 + 8 * g);
+                st[0][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(kf[s4][0]), as_bf16x8(qf), st[0][c], 0, 0, 0);
+                st[1][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(kf[s4][1]), as_bf16x8(qf), st[1][c], 0, 0, 0);
+              }
+            }
+          }
         }
       }
+    }
+    // the first blocks of values are asked for before the weights are formed
+    constexpr int AHEAD = NDT < 4 ? NDT : 4;
+    u32x4 vf[AHEAD][4];
 #pragma unroll
-      for (int dt = 0; dt < NDT; ++dt) {
-        const int d = 16 * dt + n;
-        u32x4 vf = {0u, 0u, 0u, 0u};
-        if (d < dv) {
-          const u32x2 x0 = *reinterpret_cast<const u32x2*>(b0 + (size_t)d * ps);
-          const u32x2 x1 = *reinterpret_cast<const u32x2*>(b1 + (size_t)d * ps);
-          vf = (u32x4){x0[0] & keep0[0], x0[1] & keep0[1], x1[0] & keep1[0], x1[1] & keep1[1]};
+    for (int j = 0; j < AHEAD; ++j)
+#pragma unroll
+      for (int sg = 0; sg < 4; ++sg) vf[j][sg] = load_values(sg, j);
+
+    // ---- the piece's softmax, relative to its own maximum
+#pragma unroll
+    for (int c = 0; c < QT; ++c) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int key = kw + 16 * u + 4 * g + i;
+          const float sv = key <= qpos[c] && key >= qlo[c] ? st[u][c][i] * a.scale : -INFINITY;
+          st[u][c][i] = sv;
+          mx = fmaxf(mx, sv);
         }
-        acc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(vf), as_bf16x8(pf), acc[dt], 0, 0, 0);
+      mx = across_groups_max(mx);
+      if (g == 0) red_max[wv][16 * c + n] = mx;
+    }
+    __syncthreads();
+    float mp[QT];
+#pragma unroll
+    for (int c = 0; c < QT; ++c) {
+      mp[c] = fmaxf(fmaxf(red_max[0][16 * c + n], red_max[1][16 * c + n]), fmaxf(red_max[2][16 * c + n], red_max[3][16 * c + n]));
+      const float base = mp[c] == -INFINITY ? 0.0f : mp[c];
+      float psum = 0.0f;
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        float p[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          p[i] = st[u][c][i] == -INFINITY ? 0.0f : fast_exp(st[u][c][i] - base);
+          psum += p[i];
+        }
+        *reinterpret_cast<u32x2*>(pw + (16 * c + n) * SK_PSTRIDE + 32 * wv + 16 * u + 4 * g) = (u32x2){pack_bf16x2(p[0], p[1]), pack_bf16x2(p[2], p[3])};
+      }
+      psum = across_groups_sum(psum);
+      if (g == 0) red_sum[wv][16 * c + n] = psum;
+    }
+    __syncthreads();
+    float c1[QT], c2[QT];
+    u32x4 pf[4][QT];
+#pragma unroll
+    for (int c = 0; c < QT; ++c) {
+      const float lp = ((red_sum[0][16 * c + n] + red_sum[1][16 * c + n]) + red_sum[2][16 * c + n]) + red_sum[3][16 * c + n];
+      fold_piece(m[c], l[c], mp[c], lp, c1[c], c2[c]);
+#pragma unroll
+      for (int sg = 0; sg < 4; ++sg) pf[sg][c] = *reinterpret_cast<const u32x4*>(pw + (16 * c + n) * SK_PSTRIDE + 32 * sg + 8 * g);
+    }
+
+    // ---- the weighted sum of the values: a chain over the piece's keys for every block of 16 elements, then the fold
+    const bool ragged = k0 + SK_PIECE - 1 > pmax || k0 < lo_first;       // slots outside may hold anything
+    uint32_t keep[4][4];
+#pragma unroll
+    for (int sg = 0; sg < 4; ++sg)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int key = k0 + 32 * sg + 8 * g + 2 * e;
+        keep[sg][e] = (key <= pmax && key >= lo_first ? 0xffffu : 0u) | (key + 1 <= pmax && key + 1 >= lo_first ? 0xffff0000u : 0u);
+      }
+#pragma unroll
+    for (int j = 0; j < NDT; ++j) {
+      u32x4 v[4];
+#pragma unroll
+      for (int sg = 0; sg < 4; ++sg) {
+        v[sg] = vf[j % AHEAD][sg];
+        if (j + AHEAD < NDT) vf[j % AHEAD][sg] = load_values(sg, j + AHEAD);
+      }
+      if (ragged) {                                          // (scalar)
+#pragma unroll
+        for (int sg = 0; sg < 4; ++sg)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[sg][e] &= keep[sg][e];
+      }
+#pragma unroll
+      for (int c = 0; c < QT; ++c) {
+        if (c < qt_live) {                                   // (scalar)
+          f32x4 pv = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int sg = 0; sg < 4; ++sg) pv = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(v[sg]), as_bf16x8(pf[sg][c]), pv, 0, 0, 0);
+          if constexpr (PIECES) {
+            acc[j][c] = pv;
+          } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) acc[j][c][i] = fmaf(pv[i], c2[c], acc[j][c][i] * c1[c]);
+          }
+        }
+      }
+    }
+    if constexpr (PIECES) {
+      if (qpos[0] < 0) return;
+      const size_t at = ((size_t)t * a.heads + h0 + n % a.hg) * a.max_pieces + blockIdx.z;
+      if (wv == 0 && g == 0) {
+        a.partial_ml[2 * at] = mp[0];
+        a.partial_ml[2 * at + 1] = ((red_sum[0][n] + red_sum[1][n]) + red_sum[2][n]) + red_sum[3][n];
+      }
+      float* part = a.partial + at * dv;
+#pragma unroll
+      for (int j = 0; j < NDT; ++j) {
+        const int d = 16 * (4 * j + wv) + 4 * g;
+        if ((dv & 3) == 0) {
+          if (d < dv) *reinterpret_cast<f32x4*>(part + d) = acc[j][0];
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (d + i < dv) part[d + i] = acc[j][0][i];
+        }
+      }
+      return;
+    }
+  }
+  if constexpr (!PIECES) {
+#pragma unroll
+    for (int c = 0; c < QT; ++c) {
+      if (qpos[c] < 0) continue;
+      const int qn = 16 * c + n, rl = qn / a.hg, h = h0 + qn % a.hg;
+      const float w = finish_softmax(m[c], l[c], a.sink != nullptr ? a.sink[h] : -INFINITY);
+      const size_t at = (size_t)(r0 + rl) * a.ldo + h * dv;
+#pragma unroll
+      for (int j = 0; j < NDT; ++j) {
+        const int d = 16 * (4 * j + wv) + 4 * g;
+        if (a.out_is_bf16 && (dv & 3) == 0 && (a.ldo & 3) == 0) {
+          if (d < dv)
+            *reinterpret_cast<u32x2*>(reinterpret_cast<bf16_t*>(a.out) + at + d) =
+                (u32x2){pack_bf16x2(acc[j][c][0] * w, acc[j][c][1] * w), pack_bf16x2(acc[j][c][2] * w, acc[j][c][3] * w)};
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (d + i < dv) store_out(a, at + d + i, acc[j][c][i] * w);
+        }
       }
     }
   }
-  lsum = across_groups_sum(lsum);
-  if (!qok) return;
-  if (a.nsplit > 1) {
-    float* part = a.partial + (((size_t)t * a.heads + h) * a.nsplit + split) * (dv + 2);
-    if (g == 0) {
-      part[0] = m;
-      part[1] = lsum;
-    }
-#pragma unroll
-    for (int dt = 0; dt < NDT; ++dt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = 16 * dt + 4 * g + i;
-        if (d < dv) part[2 + d] = acc[dt][i];
-      }
-    return;
-  }
-  const float sk = a.sink != nullptr ? a.sink[h] : -INFINITY;
-  const float mf = fmaxf(m, sk);
-  const float cm = m == -INFINITY ? 0.0f : fast_exp(m - mf);
-  const float lt = lsum * cm + (sk == -INFINITY ? 0.0f : fast_exp(sk - mf));
-  const float w = lt > 0.0f ? cm / lt : 0.0f;
-  float* orow = a.out + (size_t)(r0 + rl) * a.ldo + h * dv;
-#pragma unroll
-  for (int dt = 0; dt < NDT; ++dt)
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = 16 * dt + 4 * g + i;
-      if (d < dv) orow[d] = acc[dt][i] * w;
-    }
 }
 
-// The splits of one (single-row tile, head) joined: the largest maximum (the sink's score among them), every split's
-// denominator and sums scaled to it, in split order.
-__global__ __launch_bounds__(64) void shared_key_combine_kernel(MfmaAttnArgs a) {
+// The pieces of one (single-row tile, head) folded in order, a thread a value element.
+__global__ __launch_bounds__(256) void shared_key_combine_kernel(MfmaAttnArgs a) {
   const int t = blockIdx.x, h = blockIdx.y;
   const int r0 = a.tiles != nullptr ? a.tiles[4 * t] : t;
   if (a.tiles != nullptr && a.tiles[4 * t + 1] <= 0) return;
-  if (a.positions[r0] < 0) return;
-  const float* part = a.partial + ((size_t)t * a.heads + h) * a.nsplit * (a.dv + 2);
-  const int live = min(a.nsplit, a.positions[r0] / a.kchunk + 1);      // splits beyond the row's position hold nothing
-  const float sk = a.sink != nullptr ? a.sink[h] : -INFINITY;
-  // lane s holds split s's maximum and denominator (at most 64 splits); the weights of the splits go through LDS
-  __shared__ float wgt[64];
-  const int lane = threadIdx.x;
-  const float ms = lane < live ? part[(size_t)lane * (a.dv + 2)] : -INFINITY;
-  const float ls = lane < live ? part[(size_t)lane * (a.dv + 2) + 1] : 0.0f;
-  const float mt = fmaxf(sk, wave_max(ms));
-  const float ws = ms == -INFINITY ? 0.0f : fast_exp(ms - mt);
-  const float lt = wave_sum(ls * ws) + (sk == -INFINITY ? 0.0f : fast_exp(sk - mt));
-  wgt[lane] = ws;
-  __syncthreads();
-  const float inv = lt > 0.0f ? 1.0f / lt : 0.0f;
-  for (int d = lane; d < a.dv; d += 64) {
-    float o = 0.0f;
-    for (int s0 = 0; s0 < live; s0 += 8) {
-      float pv[8];
+  const int pos = a.positions[r0];
+  if (pos < 0) return;
+  const int d = blockIdx.z * 256 + threadIdx.x;
+  if (d >= a.dv) return;
+  const int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
+  const int np = pos / SK_PIECE - lo / SK_PIECE + 1;
+  const size_t at = ((size_t)t * a.heads + h) * a.max_pieces;
+  const float* ml = a.partial_ml + 2 * at;
+  const float* part = a.partial + at * a.dv + d;
+  float m = -INFINITY, l = 0.0f, o = 0.0f;
+  constexpr int UN = 8;
+  for (int p0 = 0; p0 < np; p0 += UN) {
+    float pv[UN], pm[UN], pl[UN];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) pv[u] = part[(size_t)min(s0 + u, live - 1) * (a.dv + 2) + 2 + d];
-#pragma unroll
-      for (int u = 0; u < 8; ++u)
-        if (s0 + u < live && wgt[s0 + u] != 0.0f) o = fmaf(pv[u], wgt[s0 + u], o);
+    for (int u = 0; u < UN; ++u) {
+      const int p = min(p0 + u, np - 1);
+      pv[u] = part[(size_t)p * a.dv];
+      pm[u] = ml[2 * p];
+      pl[u] = ml[2 * p + 1];
     }
-    a.out[(size_t)r0 * a.ldo + h * a.dv + d] = o * inv;
+#pragma unroll
+    for (int u = 0; u < UN; ++u) {
+      if (p0 + u < np) {
+        float c1, c2;
+        fold_piece(m, l, pm[u], pl[u], c1, c2);
+        o = fmaf(pv[u], c2, o * c1);
+      }
+    }
   }
+  store_out(a, (size_t)r0 * a.ldo + h * a.dv + d, o * finish_softmax(m, l, a.sink != nullptr ? a.sink[h] : -INFINITY));
 }
 
-int launch_shared_key_mfma(const MfmaAttnArgs& a, const bf16_t* kc, const bf16_t* vt, int num_tiles, hipStream_t s) {
+template <int QT, int NDT>
+int launch_shared_key_mfma_shape(const MfmaAttnArgs& a, const bf16_t* kc, const bf16_t* vt, int num_tiles, hipStream_t s) {
   const int dkp = (a.dk + 31) & ~31;
-  const size_t bytes = (size_t)16 * (dkp + 8) * sizeof(bf16_t);
-  const dim3 grid(num_tiles, (a.heads + a.hg - 1) / a.hg, a.nsplit), block(64);
-  const int ndt = (a.dv + 15) / 16;
-  if (ndt <= 4) hipLaunchKernelGGL(shared_key_attention_mfma_kernel<4>, grid, block, bytes, s, a, kc, vt);
-  else if (ndt <= 8) hipLaunchKernelGGL(shared_key_attention_mfma_kernel<8>, grid, block, bytes, s, a, kc, vt);
-  else if (ndt <= 16) hipLaunchKernelGGL(shared_key_attention_mfma_kernel<16>, grid, block, bytes, s, a, kc, vt);
-  else if (ndt <= 32) hipLaunchKernelGGL(shared_key_attention_mfma_kernel<32>, grid, block, bytes, s, a, kc, vt);
-  else return -4;
-  if (a.nsplit > 1) hipLaunchKernelGGL(shared_key_combine_kernel, dim3(num_tiles, a.heads), dim3(64), 0, s, a);
+  const size_t bytes = (size_t)16 * QT * (dkp + 8 + SK_PSTRIDE) * sizeof(bf16_t);
+  static bool allowed = false;
+  if (!allowed) {
+    if (hipFuncSetAttribute((const void*)shared_key_attention_mfma_kernel<QT, NDT>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                            150 * 1024) != hipSuccess)
+      return -8;
+    allowed = true;
+  }
+  if (bytes > 150 * 1024) return -8;
+  const dim3 grid(num_tiles, (a.heads + a.hg - 1) / a.hg, QT == 1 ? a.max_pieces : 1);
+  hipLaunchKernelGGL((shared_key_attention_mfma_kernel<QT, NDT>), grid, dim3(256), bytes, s, a, kc, vt);
   return BW_LAUNCH_CHECK();
+}
+
+template <int QT>
+int launch_shared_key_mfma(const MfmaAttnArgs& a, const bf16_t* kc, const bf16_t* vt, int num_tiles, hipStream_t s) {
+  const int per_wave = (a.dv + 63) / 64;     // blocks of 16 value elements a wave
+  if (per_wave <= 1) return launch_shared_key_mfma_shape<QT, 1>(a, kc, vt, num_tiles, s);
+  if (per_wave <= 2) return launch_shared_key_mfma_shape<QT, 2>(a, kc, vt, num_tiles, s);
+  if (per_wave <= 4) return launch_shared_key_mfma_shape<QT, 4>(a, kc, vt, num_tiles, s);
+  if (per_wave <= 8) return launch_shared_key_mfma_shape<QT, 8>(a, kc, vt, num_tiles, s);
+  return -4;
 }
 
 }  // namespace
@@ -726,26 +956,63 @@ extern "C" int bw_shared_key_attention(const float* q, int ldq, const int32_t* p
   return launch_shared_key<float>(a, (const float*)cache, num_tiles, s);
 }
 
+// The product per head on the matrix cores: weights [heads][outn][in] bfloat16, in a multiple of 8; x 32-bit (16-byte aligned
+// rows and heads) or bfloat16 (likewise).
+extern "C" int bw_headwise_linear_mfma(const void* x, int x_is_bf16, int ldx, int xhs, const void* w, int in, int outn, void* out,
+                                       int out_is_bf16, int ldo, int ohs, int rows, int heads, const float* gate, int ldg, int rot_n,
+                                       int rotary, int pairs, int rot_src, int rot_dst, const float* cos_table, const float* sin_table,
+                                       const int32_t* positions, void* stream) {
+  if (rows <= 0 || heads <= 0 || outn <= 0) return 0;
+  if (in < 8 || in % 8 || heads > 65535 || (outn + 63) / 64 > 65534) return -2;
+  const int unit = x_is_bf16 ? 8 : 4;
+  if (ldx % unit || xhs % unit || (reinterpret_cast<uintptr_t>(x) & 15) || (reinterpret_cast<uintptr_t>(w) & 15)) return -3;
+  if (gate != nullptr && ldg < heads) return -2;
+  if (rot_n < 0 || (rot_n > 0 && (x_is_bf16 || rotary < 0 || rotary > rot_n || (rotary & 1) || positions == nullptr ||
+                                  (rotary > 0 && (cos_table == nullptr || sin_table == nullptr)))))
+    return -2;
+  const uintptr_t mask = out_is_bf16 ? 7 : 15;
+  const int aligned = outn % 4 == 0 && ldo % 4 == 0 && ohs % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & mask) == 0;
+  const HeadGemmArgs a{x, ldx, xhs, (const bf16_t*)w, in, outn, out, ldo, ohs, rows, aligned};
+  const HeadExtras ex{gate, ldg, rot_n, rotary, pairs, rot_src, rot_dst, cos_table, sin_table, positions};
+  hipStream_t s = (hipStream_t)stream;
+  if (x_is_bf16) return out_is_bf16 ? launch_headwise_mfma<bf16_t, bf16_t>(a, ex, heads, s) : launch_headwise_mfma<bf16_t, float>(a, ex, heads, s);
+  return out_is_bf16 ? launch_headwise_mfma<float, bf16_t>(a, ex, heads, s) : launch_headwise_mfma<float, float>(a, ex, heads, s);
+}
+
+extern "C" int bw_shared_key_piece() { return SK_PIECE; }
+
 // The matrix-core route: bfloat16 cache with key vectors of a multiple of 8 elements, pages of a multiple of 4 slots, and the
-// transposed latents beside it.  nsplit > 1 (single-row tiles, 16 heads a group): every wave takes kchunk keys (a multiple
-// of 64) and ``partial`` holds tiles * heads * nsplit * (dv + 2) floats.
+// transposed latents beside it.  Prompt tiles (max_pieces 0): up to 64 / heads_per_group rows.  Single tokens (max_pieces > 0:
+// tiles of one row, 16 heads a group): ``partial`` holds tiles * heads * max_pieces * (dv + 2) floats, max_pieces covers the
+// pieces of SK_PIECE keys that a token's window, or its whole context, can touch.
 extern "C" int bw_shared_key_attention_mfma(const void* q, int ldq, const int32_t* positions, const int32_t* block_table,
                                             int table_stride, const int32_t* tiles, int num_tiles, const void* cache,
-                                            const void* latent_t, int num_pages, const float* sink, float* out, int ldo,
-                                            int heads, int dk, int dv, int page_size, int window, float scale,
-                                            int heads_per_group, int nsplit, int kchunk, float* partial,
-                                            long long partial_floats, void* stream) {
+                                            const void* latent_t, int num_pages, const float* sink, void* out, int out_is_bf16,
+                                            int ldo, int heads, int dk, int dv, int page_size, int window, float scale,
+                                            int heads_per_group, int max_pieces, float* partial, long long partial_floats,
+                                            void* stream) {
   if (num_tiles <= 0) return 0;
-  if (heads <= 0 || dk <= 0 || (dk % 8) || dv <= 0 || dv > dk || dv > 512 || page_size < 4 || (page_size % 4) || num_pages <= 0) return -2;
+  if (heads <= 0 || dk <= 0 || (dk % 8) || dv <= 0 || dv > dk || dv > 512 || page_size < 4 || (page_size & (page_size - 1)) || num_pages <= 0) return -2;
   if (heads_per_group < 1 || heads_per_group > 16 || (16 % heads_per_group)) return -2;
-  if (ldq < heads * dk || (ldq % 8) || ldo < heads * dv || nsplit < 1 || nsplit > 64) return -2;
+  if (ldq < heads * dk || (ldq % 8) || ldo < heads * dv || max_pieces < 0 || max_pieces > 65535) return -2;
   if (reinterpret_cast<uintptr_t>(q) & 15) return -3;
-  if (nsplit > 1) {
-    if (heads_per_group != 16 || kchunk < 64 || (kchunk % 64) || partial == nullptr) return -2;
-    if (partial_floats < (long long)num_tiles * heads * nsplit * (dv + 2)) return -6;
+  if ((reinterpret_cast<uintptr_t>(cache) & 15) || (reinterpret_cast<uintptr_t>(latent_t) & 15)) return -3;
+  const long long pieces = (long long)num_tiles * heads * max_pieces;
+  if (max_pieces > 0) {
+    if (heads_per_group != 16 || partial == nullptr || (reinterpret_cast<uintptr_t>(partial) & 15)) return -2;
+    // (what a block table can name; a window touches at most one piece more than it fills)
+    const long long span = ((long long)table_stride * page_size + SK_PIECE - 1) / SK_PIECE;
+    const long long in_window = window > 0 ? ((long long)window + SK_PIECE - 2) / SK_PIECE + 1 : span;
+    if (max_pieces < (span < in_window ? span : in_window)) return -2;
+    if (partial_floats < pieces * (dv + 2)) return -6;
   }
-  if ((reinterpret_cast<uintptr_t>(cache) & 15) || (reinterpret_cast<uintptr_t>(latent_t) & 7)) return -3;
-  MfmaAttnArgs a{(const bf16_t*)q, ldq, positions, block_table, table_stride, tiles, sink, out, ldo, partial, heads, dk, dv, page_size, window,
-                 heads_per_group, num_pages, nsplit, kchunk, scale};
-  return launch_shared_key_mfma(a, (const bf16_t*)cache, (const bf16_t*)latent_t, num_tiles, (hipStream_t)stream);
+  MfmaAttnArgs a{(const bf16_t*)q, ldq, positions, block_table, table_stride, tiles, sink, out, ldo, out_is_bf16, partial,
+                 partial == nullptr ? nullptr : partial + pieces * dv, heads, dk, dv, page_size, window, heads_per_group, num_pages,
+                 max_pieces, scale};
+  hipStream_t s = (hipStream_t)stream;
+  if (max_pieces == 0) return launch_shared_key_mfma<4>(a, (const bf16_t*)cache, (const bf16_t*)latent_t, num_tiles, s);
+  const int rc = launch_shared_key_mfma<1>(a, (const bf16_t*)cache, (const bf16_t*)latent_t, num_tiles, s);
+  if (rc != 0) return rc;
+  hipLaunchKernelGGL(shared_key_combine_kernel, dim3(num_tiles, heads, (dv + 255) / 256), dim3(256), 0, s, a);
+  return BW_LAUNCH_CHECK();
 }

@@ -98,8 +98,11 @@ _SIGS = {
                          c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                          c_int, c_int, c_void_p],
     "bw_shared_key_attention_mfma": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int,
-                                     c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int,
+                                     c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int,
                                      c_void_p, c_longlong, c_void_p],
+    "bw_shared_key_piece": [],
+    "bw_headwise_linear_mfma": [c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int,
+                                c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p],
     "bw_latent_prep": [c_void_p, c_int, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                        c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                        c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
@@ -140,7 +143,7 @@ _fns = {}
 _CHAIN_KEEPS = frozenset({
     "bw_gemm_bf16", "bw_gemm_add_bf16", "bw_norm_gemm_bf16", "bw_norm_qkv_rope_bf16",
     "bw_gemm_add_scratch", "bw_norm_gemm_supported", "bw_norm_gemm_wide_supported", "bw_attention_decode_scratch",
-    "bw_attention_fold_group_tiles", "bw_gemm_add_bf16_static_max", "bw_moe_max_tiles", "bw_chain_sync_words", "bw_chain_begin",
+    "bw_attention_fold_group_tiles", "bw_gemm_add_bf16_static_max", "bw_moe_max_tiles", "bw_shared_key_piece", "bw_chain_sync_words", "bw_chain_begin",
     "bw_chain_flush", "bw_chain_end",
 })
 _chain_open = False
@@ -1098,18 +1101,29 @@ def latent_prep(proj: torch.Tensor, q_off: int, dkv_off: int, norm_w: torch.Tens
                                  0 if cq is None else cq.stride(0), _stream()), "latent_prep")
 
 
+def headwise_mfma_ok(weights: torch.Tensor, inner: int, x_row_stride: int, x_head_stride: int) -> bool:
+    """Whether the product per head can run on the matrix cores: bfloat16 weights, an inner size in multiples of 8, and rows
+    and heads of a 32-bit x that start at whole 16 bytes."""
+    return weights.dtype == torch.bfloat16 and inner % 8 == 0 and x_row_stride % 4 == 0 and x_head_stride % 4 == 0
+
+
 def headwise_linear(x: torch.Tensor, x_off: int, x_head_stride: int, wt: torch.Tensor, out: torch.Tensor, out_off: int,
-                    out_head_stride: int, rows: int, gate: Optional[torch.Tensor] = None, rotate=None) -> None:
-    """out[r, out_off + h*out_head_stride + o] = sum_i wt[h, i, o] * x[r, x_off + h*x_head_stride + i]: a product per head,
-    weights input-major [heads, in, out] (bfloat16 or float32), 32-bit sums.  ``gate`` [rows, heads] (float32, a column slice
-    will do): head h's outputs are multiplied by sigmoid(gate[r, h]).  ``rotate`` = (n, rotary, pairs, src, dst, cos, sin,
-    positions): beside the product, in the same launch, the n elements at column x_off + h*x_head_stride + src of x are
-    rotated (pairs: neighbours; else i and i + rotary/2; elements from ``rotary`` on pass) and stored at column
-    out_off + h*out_head_stride + dst of out."""
-    _need(x, torch.float32, "x")
-    if wt.dim() != 3 or not wt.is_cuda or not wt.is_contiguous():
-        raise ValueError("headwise_linear: weights must be a contiguous [heads, in, out] GPU tensor")
-    heads, inn, outn = wt.shape
+                    out_head_stride: int, rows: int, gate: Optional[torch.Tensor] = None, rotate=None, matrix_cores: bool = False) -> None:
+    """out[r, out_off + h*out_head_stride + o] = sum_i W[h][i -> o] * x[r, x_off + h*x_head_stride + i]: a product per head,
+    32-bit sums.  ``wt``: input-major [heads, in, out] (bfloat16 or float32), x float32; with ``matrix_cores`` output-major
+    [heads, out, in] (bfloat16, in a multiple of 8), x float32 (rounded to bfloat16 where it enters) or bfloat16.
+    ``gate`` [rows, heads] (float32, a column slice will do): head h's outputs are multiplied by sigmoid(gate[r, h]).
+    ``rotate`` = (n, rotary, pairs, src, dst, cos, sin, positions): beside the product, in the same launch, the n elements at
+    column x_off + h*x_head_stride + src of x are rotated (pairs: neighbours; else i and i + rotary/2; elements from
+    ``rotary`` on pass) and stored at column out_off + h*out_head_stride + dst of out."""
+    if matrix_cores:
+        if not x.is_cuda or x.dtype not in (torch.float32, torch.bfloat16) or not x.is_contiguous():
+            raise ValueError("headwise_linear: x must be a contiguous float32 or bfloat16 GPU matrix")
+    else:
+        _need(x, torch.float32, "x")
+    if wt.dim() != 3 or not wt.is_cuda or not wt.is_contiguous() or (matrix_cores and wt.dtype != torch.bfloat16):
+        raise ValueError("headwise_linear: weights must be a contiguous [heads, in, out] GPU tensor (matrix cores: [heads, out, in] bfloat16)")
+    heads, inn, outn = (wt.shape[0], wt.shape[2], wt.shape[1]) if matrix_cores else wt.shape
     if x_off + (heads - 1) * x_head_stride + inn > x.shape[1] or out_off + (heads - 1) * out_head_stride + outn > out.shape[1]:
         raise ValueError("headwise_linear: x or out narrower than the heads need")
     if x.shape[0] < rows or out.shape[0] < rows:
@@ -1123,6 +1137,7 @@ def headwise_linear(x: torch.Tensor, x_off: int, x_head_stride: int, wt: torch.T
     rot = (0, 0, 0, 0, 0, 0, 0, 0)
     if rotate is not None and int(rotate[0]) > 0:
         n, rotary, pairs, src, dst, cos, sin, positions = rotate
+        _need(x, torch.float32, "x")
         _need(cos, torch.float32, "cos table")
         _need(sin, torch.float32, "sin table")
         _need(positions, torch.int32, "positions")
@@ -1132,9 +1147,16 @@ def headwise_linear(x: torch.Tensor, x_off: int, x_head_stride: int, wt: torch.T
             raise ValueError("headwise_linear: the rotated part does not fit x or out")
         rot = (int(n), int(rotary), int(bool(pairs)), int(src), int(dst), cos.data_ptr(), sin.data_ptr(), positions.data_ptr())
     ob = _act_out(out, "out")
+    op = out.data_ptr() + (2 if ob else 4) * out_off
+    if matrix_cores:
+        xb = _act_out(x, "x")
+        _check(_fn("bw_headwise_linear_mfma")(x.data_ptr() + (2 if xb else 4) * x_off, xb, x.stride(0), x_head_stride, wt.data_ptr(), inn,
+                                              outn, op, ob, out.stride(0), out_head_stride, rows, heads, gp, ldg, *rot, _stream()),
+               "headwise_linear")
+        return
     _check(_fn("bw_headwise_linear")(x.data_ptr() + 4 * x_off, x.stride(0), x_head_stride, wt.data_ptr(), _is_bf16(wt, "weights"),
-                                     inn, outn, out.data_ptr() + (2 if ob else 4) * out_off, ob, out.stride(0), out_head_stride,
-                                     rows, heads, gp, ldg, *rot, _stream()), "headwise_linear")
+                                     inn, outn, op, ob, out.stride(0), out_head_stride, rows, heads, gp, ldg, *rot, _stream()),
+           "headwise_linear")
 
 
 def shared_key_attention(q: torch.Tensor, positions: torch.Tensor, block_table: torch.Tensor, tiles: Optional[torch.Tensor],
@@ -1175,18 +1197,25 @@ def shared_key_mfma_ok(cache_dtype: torch.dtype, dk: int, dv: int, page_size: in
     return cache_dtype == torch.bfloat16 and dk % 8 == 0 and 0 < dv <= min(dk, 512) and page_size >= 4 and page_size % 4 == 0
 
 
+def shared_key_pieces(context: int, window: int) -> int:
+    """The most pieces of keys a single token can touch in a context of so many positions (window 0: it sees all of them)."""
+    piece = int(_fn("bw_shared_key_piece")())
+    span = -(-int(context) // piece)
+    return span if window <= 0 else min(span, (int(window) + piece - 2) // piece + 1)
+
+
 def shared_key_attention_mfma(q: torch.Tensor, positions: torch.Tensor, block_table: torch.Tensor, tiles: Optional[torch.Tensor],
                               num_tiles: int, cache: torch.Tensor, latent_t: torch.Tensor, sink: Optional[torch.Tensor],
                               out: torch.Tensor, heads: int, dk: int, dv: int, page_size: int, window: int, scale: float,
-                              heads_per_group: int, nsplit: int = 1, kchunk: int = 0,
-                              partial: Optional[torch.Tensor] = None) -> None:
+                              heads_per_group: int, max_pieces: int = 0, partial: Optional[torch.Tensor] = None) -> None:
     """``shared_key_attention`` on the matrix cores for a bfloat16 cache (``shared_key_mfma_ok``): queries and softmax
     weights are rounded to bfloat16 where they enter a product (``q`` arrives as bfloat16), sums are 32-bit.  ``latent_t`` [pages, dv * page_size]: the
-    values transposed within their pages.  Tiles hold up to 16 / heads_per_group rows.  nsplit > 1 (tiles of one row,
-    heads_per_group 16): wave s of a tile takes keys [s * kchunk, (s+1) * kchunk) and ``partial`` (float32, at least
-    tiles * heads * nsplit * (dv + 2)) holds the pieces that a second kernel joins."""
+    values transposed within their pages.  ``out`` float32 or bfloat16.  Tiles hold up to 64 / heads_per_group rows.
+    max_pieces > 0 (tiles of one row, heads_per_group 16): a workgroup for each of the ``shared_key_pieces`` runs of keys a
+    token can see, and ``partial`` (float32, at least tiles * heads * max_pieces * (dv + 2)) holds what they leave for a
+    second kernel that folds them; the bits of a row are those it gets in a tile."""
     _need(q, torch.bfloat16, "q")
-    _need(out, torch.float32, "out")
+    ob = _act_out(out, "out")
     _need(positions, torch.int32, "positions")
     _need(block_table, torch.int32, "block_table")
     _need(cache, torch.bfloat16, "cache")
@@ -1207,16 +1236,16 @@ def shared_key_attention_mfma(q: torch.Tensor, positions: torch.Tensor, block_ta
         raise ValueError("shared_key_attention_mfma: q or out do not fit")
     if cache.dim() != 2 or cache.shape[1] != page_size * dk or latent_t.shape != (cache.shape[0], page_size * dv):
         raise ValueError("shared_key_attention_mfma: cache or transposed values do not fit")
-    if nsplit > 1:
+    if max_pieces > 0:
         if partial is None:
-            raise ValueError("shared_key_attention_mfma: splits need room for their pieces")
+            raise ValueError("shared_key_attention_mfma: pieces need room for what they leave")
         _need(partial, torch.float32, "partial")
     _check(_fn("bw_shared_key_attention_mfma")(q.data_ptr(), q.stride(0), positions.data_ptr(), block_table.data_ptr(),
                                                block_table.stride(0), 0 if tiles is None else tiles.data_ptr(), num_tiles,
                                                cache.data_ptr(), latent_t.data_ptr(), cache.shape[0],
-                                               0 if sink is None else sink.data_ptr(), out.data_ptr(), out.stride(0), heads,
-                                               dk, dv, page_size, int(window), float(scale), int(heads_per_group), int(nsplit),
-                                               int(kchunk), 0 if partial is None else partial.data_ptr(),
+                                               0 if sink is None else sink.data_ptr(), out.data_ptr(), ob, out.stride(0), heads,
+                                               dk, dv, page_size, int(window), float(scale), int(heads_per_group), int(max_pieces),
+                                               0 if partial is None else partial.data_ptr(),
                                                0 if partial is None else partial.numel(), _stream()),
            "shared_key_attention_mfma")
 

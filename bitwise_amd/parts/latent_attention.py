@@ -24,7 +24,7 @@ from .base import CacheSpec, Mixer, TensorSpec, lookup, register_mixer, POSITION
 from .linear import Linear
 
 ROWS_PER_PROMPT_TILE = 4        # the 32-bit kernel: 16 query vectors a workgroup, 4 rows x 4 heads or a single token's 16 heads
-MAX_SPLITS = 64                 # pieces a single token's keys are cut into at most (each a multiple of 64 keys)
+QUERIES_PER_TILE = 64           # the matrix-core kernel: query vectors (rows x heads of a group) a workgroup in prompt portions
 
 
 def _tiles(ctx, rows_per_tile: int):
@@ -134,10 +134,16 @@ class LatentAttention(Mixer):
         self.latent_norm = tensors["dkv.norm"].to(dev).float().contiguous()
         if self.has_sink:
             self.sink = tensors["sink"].to(dev).float().contiguous()
-        # input-major per head: uk as stored is [head][dim][rank] (the transposed product wants exactly that);
-        # uv [head][vdim][rank] is turned to [head][rank][vdim]
-        self.uk_t = tensors["uk"].to(dev).view(self.heads, self.dim, self.rank).contiguous()
-        self.uv_t = tensors["uv"].to(dev).view(self.heads, self.vdim, self.rank).transpose(1, 2).contiguous()
+        # the products into and out of the latent's space.  On the matrix cores the weights lie output-major (uv as stored,
+        # [head][vdim][rank]; uk turned to [head][rank][dim]), else input-major (uk as stored, [head][dim][rank]; uv turned)
+        uk = tensors["uk"].to(dev).view(self.heads, self.dim, self.rank)
+        uv = tensors["uv"].to(dev).view(self.heads, self.vdim, self.rank)
+        per = self.dim + self.rot
+        query_stride = self.heads * per if self.q_rank else self.proj.out_features
+        self.uk_on_mfma = self.rt.bf16 and ops.headwise_mfma_ok(uk, self.dim, query_stride, per)
+        self.uv_on_mfma = self.rt.bf16 and ops.headwise_mfma_ok(uv, self.rank, self.heads * self.rank, self.rank)
+        self.uk_t = uk.transpose(1, 2).contiguous() if self.uk_on_mfma else uk.contiguous()
+        self.uv_t = uv.contiguous() if self.uv_on_mfma else uv.transpose(1, 2).contiguous()
 
     def weight_bytes(self) -> int:
         small = self.uk_t.numel() * self.uk_t.element_size() + self.uv_t.numel() * self.uv_t.element_size()
@@ -174,11 +180,12 @@ class LatentAttention(Mixer):
         if self.q_rank:
             q = ws.buffer("latent_up_q", self.heads * per, torch.float32)
             self.uq.store(ws, cq, q, rows)
-            ops.headwise_linear(q, 0, per, self.uk_t, qa, 0, self.key_width, rows,
+            ops.headwise_linear(q, 0, per, self.uk_t, qa, 0, self.key_width, rows, matrix_cores=self.uk_on_mfma,
                                 rotate=(self.rot, self.rotary, self.pairs, self.dim, self.rank, self.cos, self.sin, ctx.positions))
         else:
-            ops.headwise_linear(y, self.q_off, per, self.uk_t, qa, 0, self.key_width, rows)
-        lat = ws.buffer("latent_out", self.heads * self.rank, torch.float32)
+            ops.headwise_linear(y, self.q_off, per, self.uk_t, qa, 0, self.key_width, rows, matrix_cores=self.uk_on_mfma)
+        # (rounded where the next product would round it anyway)
+        lat = ws.buffer("latent_out", self.heads * self.rank, torch.bfloat16 if mfma and self.uv_on_mfma else torch.float32)
         if mfma:
             self._attend_on_matrix_cores(ctx, call, qa, lat, table)
         else:
@@ -190,7 +197,7 @@ class LatentAttention(Mixer):
             if n_single:
                 ops.shared_key_attention(qa, ctx.positions, table, single, n_single, *common, 16)
         vals = ws.buffer("latent_values", self.heads * self.vdim, self.rt.act_dtype)
-        ops.headwise_linear(lat, 0, self.rank, self.uv_t, vals, 0, self.vdim, rows,
+        ops.headwise_linear(lat, 0, self.rank, self.uv_t, vals, 0, self.vdim, rows, matrix_cores=self.uv_on_mfma,
                             gate=y[:, self.gate_off:self.gate_off + self.heads] if self.has_gate else None)
         if add:
             self.o.add_into(ws, vals, target, rows)
@@ -216,24 +223,18 @@ class LatentAttention(Mixer):
     def _attend_on_matrix_cores(self, ctx, call, qa, lat, table) -> None:
         ws = ctx.ws
         hg = self.heads_per_group
-        many, n_many, single, n_single = _tiles(ctx, 16 // hg)
-        common = (call.k_cache, call.v_cache, self.sink, lat, self.heads, self.key_width, self.rank, ws.page_size,
-                  int(self.window or 0), self.scale)
+        many, n_many, single, n_single = _tiles(ctx, QUERIES_PER_TILE // hg)
+        window = int(self.window or 0)
+        common = (call.k_cache, call.v_cache, self.sink, lat, self.heads, self.key_width, self.rank, ws.page_size, window, self.scale)
         if n_many:
             ops.shared_key_attention_mfma(qa, ctx.positions, table, many, n_many, *common, hg)
         if n_single:
-            # Single tokens: the keys a token can have (what its block table spans) are cut into pieces of a multiple of
-            # 64, at most MAX_SPLITS of them, a wave each; few tokens with long contexts still fill the chip.  The cut
-            # depends on the table's width alone, which a captured step fixes.
-            # The pieces are joined in another order than a wave walks its blocks of keys, so a position's last bits would depend
-            # on whether it came alone or inside a portion: an engine that promises bits under any cut (Workspace.exact_cuts)
-            # keeps single tokens on one wave per 16 heads.
-            span = table.shape[1] * ws.page_size
-            kchunk = 64 * max(1, -(-span // (64 * MAX_SPLITS)))
-            nsplit = 1 if getattr(ws, "exact_cuts", True) else max(1, -(-span // kchunk))
-            partial = None
-            if nsplit > 1:
-                # (room for the most pieces, for the power of two from this step's single tokens up: a few sizes at most)
-                tokens = 1 << max(0, n_single - 1).bit_length()
-                partial = ws.buffer("latent_split", tokens * MAX_SPLITS * self.heads * (self.rank + 2), torch.float32, rows=1)
-            ops.shared_key_attention_mfma(qa, ctx.positions, table, single, n_single, *common, 16, nsplit, kchunk, partial)
+            # Single tokens: a workgroup for every piece of keys the token can see, folded by a second launch; few tokens
+            # with long contexts still fill the chip.  Prompt tiles cut their keys at the same places and fold them by the
+            # same operations, so a position's bits do not depend on how it came.
+            pieces = ops.shared_key_pieces(table.shape[1] * ws.page_size, window)
+            # (room for the power of two from this step's single tokens up: a few sizes at most)
+            tokens = 1 << max(0, n_single - 1).bit_length()
+            widest = pieces if ws.max_table_width is None else ops.shared_key_pieces(ws.max_table_width * ws.page_size, window)
+            partial = ws.buffer("latent_pieces", tokens * max(pieces, widest) * self.heads * (self.rank + 2), torch.float32, rows=1)
+            ops.shared_key_attention_mfma(qa, ctx.positions, table, single, n_single, *common, 16, pieces, partial)

@@ -274,7 +274,7 @@ def test_randomized_scenarios_to_the_last_bit(gpu, dtype):
 
 def _attend(q, keys, sink, heads, dk, dv, scale, page, dtype, positions, window=0, matrix_cores=None):
     """shared_key_attention for single rows of one request at the given positions over ``keys`` [n, dk].  ``matrix_cores``:
-    (heads per group, splits) runs the matrix-core kernel instead."""
+    (heads per group, whether the keys' pieces get a workgroup each) runs the matrix-core kernel instead."""
     from bitwise_amd.csrc import ops
     dev = torch.device("cuda:0")
     n = keys.shape[0]
@@ -295,13 +295,12 @@ def _attend(q, keys, sink, heads, dk, dv, scale, page, dtype, positions, window=
         ops.shared_key_attention(q.float().to(dev).contiguous(), pos, table, tiles, rows, cache.to(dev), sk,
                                  out, heads, dk, dv, page, window, scale, 16)
     else:
-        hg, nsplit = matrix_cores
+        hg, in_pieces = matrix_cores
         vt = cache.view(pages, page, dk)[:, :, :dv].transpose(1, 2).contiguous().view(pages, dv * page)
-        kchunk = 64 * max(1, -(-(pages * page) // (64 * nsplit)))
-        nsplit = -(-(pages * page) // kchunk)
-        partial = torch.zeros(rows * heads * nsplit * (dv + 2), device=dev) if nsplit > 1 else None
+        pieces = ops.shared_key_pieces(pages * page, window) if in_pieces else 0
+        partial = torch.zeros(rows * heads * pieces * (dv + 2), device=dev) if pieces else None
         ops.shared_key_attention_mfma(q.bfloat16().to(dev).contiguous(), pos, table, tiles, rows, cache.to(dev), vt.to(dev), sk, out,
-                                      heads, dk, dv, page, window, scale, hg, nsplit, kchunk, partial)
+                                      heads, dk, dv, page, window, scale, hg, pieces, partial)
     return out.cpu().double().view(rows, heads, dv), cache
 
 
@@ -340,13 +339,15 @@ def test_a_far_key_among_hundreds_and_page_borders(gpu, dtype):
     for r, t in enumerate(targets):       # the probe's head returns (nearly) the value of its target
         assert (got[r, r % heads] - keys[t, :dv]).abs().max() < 0.05, t
     if dtype == torch.bfloat16:
-        # the matrix-core kernel: whole key range by one wave, and cut into pieces that a second kernel joins; queries and
-        # weights are rounded to bfloat16 on their way into the products
+        # the matrix-core kernel: a workgroup that walks the pieces of the keys, and one for each piece whose results a second
+        # kernel folds, which leaves the same bits; queries and weights are rounded to bfloat16 on their way into the products
         qr = q.bfloat16().double()
         want = _attend_plain(qr, keys, sink, heads, dk, dv, 0.2, positions)
-        for route in ((8, 1), (16, 1), (16, 4), (16, 11)):
+        first = None
+        for route in ((8, False), (16, False), (16, True)):
             got, _ = _attend(q, keys, sink, heads, dk, dv, 0.2, page, dtype, positions, matrix_cores=route)
-            assert (got - want).abs().max() < 1e-2 * want.abs().max(), route
+            first = got if first is None else first
+            assert torch.equal(got, first) and (got - want).abs().max() < 1e-2 * want.abs().max(), route
             for r, t in enumerate(targets):
                 assert (got[r, r % heads] - keys[t, :dv]).abs().max() < 0.05, (route, t)
 

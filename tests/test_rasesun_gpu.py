@@ -20,9 +20,9 @@ pytestmark = pytest.mark.gpu
 # float32: 32-bit sums against float64 ones, a few 1e-6 of a row.  bfloat16: activations rounded where the products and the
 # cache take them, carried through the layers and the loop's passes.  A row whose sublayer nearly cancels out is blown up
 # by the norm behind it, its roundings with it (the plain model with rounded activations has such rows too: one in a
-# hundred moves by a tenth or more of its size), so in that mode the 95th percentile carries the tight bound.
+# hundred moves by a tenth or more of its size), so in that mode the 90th percentile carries the tight bound.
 TOL = {"float32": 5e-5, "bfloat16": 0.08}
-MOST = {"float32": 1.0, "bfloat16": 0.95}
+MOST = {"float32": 1.0, "bfloat16": 0.9}
 TYPICAL = {"float32": 1e-5, "bfloat16": 2.5e-2}
 SIGMA = 0.15
 
@@ -511,29 +511,42 @@ def test_experts_by_table_against_plain(gpu, rows, top, experts):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("rows", [1, 9, 100])
+@pytest.mark.parametrize("rows", [1, 9, 40, 130])
 def test_products_per_head_with_rotation_and_gate(gpu, rows, dtype):
-    """A product per head into a wider row, with the rotation of neighbours beside it, and one with a gate per head."""
+    """A product per head into a wider row, with the rotation of neighbours beside it, and one with a gate per head: by
+    32-bit chains and on the matrix cores (whose rows do not depend on how many come together)."""
     from bitwise_amd.csrc import ops
     from bitwise_amd.parts.rope import PairRotaryTable
     from bitwise_amd.runtime import Runtime
     g = torch.Generator().manual_seed(rows)
-    for heads, dim, rot, rank in ((3, 16, 8, 40), (2, 128, 64, 512), (5, 10, 6, 7)):
+    for heads, dim, rot, rank in ((3, 16, 8, 40), (2, 128, 64, 512), (5, 10, 6, 7), (2, 264, 8, 30)):
         per, wide = dim + rot, rank + rot
         x, wk = torch.randn(rows, heads * per, generator=g), (torch.randn(heads, dim, rank, generator=g) * 0.1).to(torch.bfloat16)
-        table = PairRotaryTable({"base": 300.0, "dims": rot, "max_positions": 200}, Runtime("float32", gpu))
+        table = PairRotaryTable({"base": 300.0, "dims": rot, "max_positions": 300}, Runtime("float32", gpu))
         cos, sin = table.tables()
-        pos = torch.arange(60, 60 + rows)
-        out = torch.zeros(rows, heads * wide, dtype=dtype, device=gpu)
-        ops.headwise_linear(x.to(gpu), 0, per, wk.to(gpu), out, 0, wide, rows,
-                            rotate=(rot, rot, True, dim, rank, cos, sin, pos.to(torch.int32).to(gpu)))
-        xv = x.double().view(rows, heads, per)
-        want = torch.cat([torch.einsum("rhi,hio->rho", xv[..., :dim], wk.double()),
-                          pr.rotate_pairs(xv[..., dim:], 60, {"base": 300.0, "dims": rot})], -1).reshape(rows, -1)
-        tol = 1e-5 if dtype == torch.float32 else 0.02
-        assert (out.cpu().double() - want).abs().max() / want.abs().max() < tol
+        pos = torch.arange(60, 60 + rows).to(torch.int32).to(gpu)
         gate = torch.randn(rows, heads + 2, generator=g)
-        out = torch.zeros(rows, heads * rank, dtype=dtype, device=gpu)
-        ops.headwise_linear(x.to(gpu), 0, per, wk.to(gpu), out, 0, rank, rows, gate=gate.to(gpu)[:, 2:])
-        want = (torch.einsum("rhi,hio->rho", xv[..., :dim], wk.double()) * torch.sigmoid(gate[:, 2:].double())[..., None]).reshape(rows, -1)
-        assert (out.cpu().double() - want).abs().max() / want.abs().max() < tol
+        xv = x.double().view(rows, heads, per)
+        turned = pr.rotate_pairs(xv[..., dim:], 60, {"base": 300.0, "dims": rot})
+        for cores in ([False, True] if ops.headwise_mfma_ok(wk, dim, heads * per, per) else [False]):
+            wd = (wk.transpose(1, 2) if cores else wk).contiguous().to(gpu)
+            xin = pr.round_bf16(xv[..., :dim]) if cores else xv[..., :dim]
+            product = torch.einsum("rhi,hio->rho", xin, wk.double())
+            tol = 1e-5 if dtype == torch.float32 else 0.02
+            run = lambda n, ld, **kw: ops.headwise_linear(x[:n].to(gpu), 0, per, wd, out, 0, ld, n, matrix_cores=cores, **kw)
+            out = torch.zeros(rows, heads * wide, dtype=dtype, device=gpu)
+            run(rows, wide, rotate=(rot, rot, True, dim, rank, cos, sin, pos))
+            want = torch.cat([product, turned], -1).reshape(rows, -1)
+            assert (out.cpu().double() - want).abs().max() / want.abs().max() < tol, (heads, cores)
+            whole, out = out, torch.zeros(1, heads * wide, dtype=dtype, device=gpu)
+            run(1, wide, rotate=(rot, rot, True, dim, rank, cos, sin, pos))
+            assert torch.equal(out[0], whole[0])
+            out = torch.zeros(rows, heads * rank, dtype=dtype, device=gpu)
+            run(rows, rank, gate=gate.to(gpu)[:, 2:])
+            want = (product * torch.sigmoid(gate[:, 2:].double())[..., None]).reshape(rows, -1)
+            assert (out.cpu().double() - want).abs().max() / want.abs().max() < tol, (heads, cores)
+            if cores:
+                out = torch.zeros(rows, heads * rank, dtype=dtype, device=gpu)
+                ops.headwise_linear(x.to(torch.bfloat16).to(gpu), 0, per, wd, out, 0, rank, rows, matrix_cores=True)
+                want = product.reshape(rows, -1)
+                assert (out.cpu().double() - want).abs().max() / want.abs().max() < tol, heads
