@@ -109,7 +109,8 @@ int bw_norm_shift(const float* x, int ldx, const float* w, const float* mix, flo
                   void* out, int out_is_bf16, int ldo, int rows, int dim, float eps, int nmix, void* stream);
 // mode 0: a decay per key channel (gate: logits [rows, ldg] at gate_off, bias [heads*dim], param = 1/tau);
 // mode 1: scalar input and forget gates per head (columns gate_off and gate2_off of proj, biases bias and bias2, param = cap)
-// with normaliser and running maximum.  state: [slots, state_ld] of S [heads][dim][vdim] (mode 1: then n [heads][dim], m [heads]).
+// with normaliser and running maximum.  state: [slots, state_ld] of S [heads][vdim][dim] (mode 1: then n [heads][dim]
+// and m [heads] once for every workgroup of a head, which is what a slot smaller than needed is refused by).
 // mode 2: a decay per key channel exp(-exp(logit + bias)), the read-out taken before the update with the token's own
 // k v^T weighted by bias2 [heads*dim]; mode 3: one constant decay a head, bias [heads] (gate is not read).
 // mode 4: a step size per head, delta = softplus(logit at gate_off + head + bias[head]); decay exp(-bias2[head] delta), the
@@ -122,6 +123,7 @@ int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_off, int k_
                          const int32_t* slots, const int32_t* positions, int nseq, int heads, int dim, int vdim,
                          const int32_t* chunks, int nchunks, const int32_t* spans, int nspans, float* scan_local,
                          float* scan_start, long long scan_floats, void* stream);
+long long bw_recurrence_record(int dim, int vdim);      // floats that scan_local and scan_start hold per chunk and head
 // gate 0: sigmoid, 1: SiLU.  weight: [heads, wstride] (wstride 0: one weight vector for all heads).
 // Up to two sections of [heads][dim] 32-bit elements a row (at columns off0, off1) turned in place: of a head's first rot
 // elements, element i is paired with element i + rot/2; tables [positions, rot/2].

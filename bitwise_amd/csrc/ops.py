@@ -818,6 +818,26 @@ def norm_shift(x: torch.Tensor, weight: torch.Tensor, mix: torch.Tensor, state: 
            "norm_shift")
 
 
+@functools.lru_cache(maxsize=None)
+def recurrence_record(dim: int, vdim: int) -> int:
+    """Floats a chunk's record holds for one head in the three passes over chunks of ``linear_recurrence``."""
+    f = _build.load().bw_recurrence_record
+    f.argtypes, f.restype = [c_int, c_int], c_longlong
+    return int(f(int(dim), int(vdim)))
+
+
+def recurrence_state(mode: int, heads: int, dim: int, vdim: int) -> int:
+    """Floats of state a request holds: the memories, and with scalar gates a normaliser and a running maximum a head for
+    every workgroup that works on the head (copies, so that none reads what another has written)."""
+    n = heads * dim * vdim
+    if mode == RECUR_SCALAR_GATES:
+        # (a workgroup's value columns, as the kernel lays them out; the entry point refuses a slot that is too small)
+        padded = 16 if dim <= 16 else 32 if dim <= 32 else 64 if dim <= 64 else 128
+        columns = 256 // (16 if padded == 128 else padded // 8)
+        n += -(-vdim // columns) * heads * (dim + 1)
+    return n
+
+
 def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate: Optional[torch.Tensor], gate_off: int,
                       gate2_off: int, bias: torch.Tensor, bias2: Optional[torch.Tensor], param: float, qscale: float,
                       state: torch.Tensor, out: torch.Tensor, seq_rows: torch.Tensor, slots: torch.Tensor,
@@ -833,12 +853,13 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
     RECUR_STEP_DECAY: a step size per head, delta = softplus(gate + bias) (``gate`` column gate_off + h, ``bias`` [heads]);
     decay = exp(-bias2[h] delta) (``bias2`` [heads]: the rates), the token enters as k (delta v)^T, and ``skip`` [heads]
     (optional) times v joins the read-out.
-    k is multiplied by ``kscale``; ``heads_per_key`` neighbouring heads share one q and one k.  ``state`` may be a column slice of a wider tensor.
+    k is multiplied by ``kscale``; ``heads_per_key`` neighbouring heads share one q and one k.  A head's state lies as
+    [value column][key channel].  ``state`` may be a column slice of a wider tensor.
 
     ``scan`` = (chunks [n, 4] int32 = (first row, rows, request, 1 if the request's last chunk), n, spans [k, 3] int32 =
     (request, its first chunk, its chunks), k, local, start): long portions run in three passes over their chunks (each
     chunk from zero, a walk over a request's chunks that gives each its starting state, each chunk from there), with
-    ``local`` and ``start`` float32 of n * heads * (dim*vdim + dim + 2) elements each; ``seq_rows`` then carries no rows
+    ``local`` and ``start`` float32 of n * heads * ``recurrence_record(dim, vdim)`` elements each; ``seq_rows`` then carries no rows
     for those requests (nseq may be 0).  The result differs from the one-pass order by the rounding of the walk's sums."""
     _need_strided(proj, torch.float32, "proj")            # (may be a column slice of a wider product)
     if mode != RECUR_FIXED_DECAY:
@@ -856,7 +877,7 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
         _need(bias2, torch.float32, "bias2")
         if bias.numel() != heads or bias2.numel() != heads or max(gate_off, gate2_off) + heads > gate.shape[1]:
             raise ValueError("linear_recurrence: gates or biases do not fit the heads")
-        need = heads * (dim * vdim + dim + 1)
+        need = recurrence_state(mode, heads, dim, vdim)
     elif mode == RECUR_STEP_DECAY:
         if bias2 is None:
             raise ValueError("linear_recurrence: a step size needs the decay's rates")

@@ -15,6 +15,8 @@
 
 #include <math.h>
 
+#include <type_traits>
+
 namespace {
 
 __device__ __forceinline__ float log_sigmoid(float z) {
@@ -250,17 +252,19 @@ __global__ __launch_bounds__(256) void norm_shift_row_kernel(const float* __rest
 
 enum { RECUR_DECAY_PER_CHANNEL = 0, RECUR_SCALAR_GATES = 1, RECUR_BONUS_DECAY = 2, RECUR_FIXED_DECAY = 3, RECUR_STEP_DECAY = 4 };
 
-// The sum over the lanes l, l + 64/SPLIT, ... that hold the parts of one column (every one of them gets it).
+// The sum over the SPLIT lanes that hold the parts of one column, l, l + 64/SPLIT, ... (every one of them gets it).
 template <int SPLIT>
 __device__ __forceinline__ float join_parts(float v) {
   if constexpr (SPLIT >= 2) {
     float lower, upper;
     lane_halves<32>(v, lower, upper);
     v = lower + upper;
-    if constexpr (SPLIT == 4) {
+    if constexpr (SPLIT >= 4) {
       lane_halves<16>(v, lower, upper);
       v = lower + upper;
     }
+    if constexpr (SPLIT >= 8) v += lane_xor<8>(v);
+    if constexpr (SPLIT >= 16) v += lane_xor<4>(v);
   }
   return v;
 }
@@ -276,7 +280,8 @@ struct RecurArgs {
   int heads_per_key;       // neighbouring heads that share one q and one k (1: every head has its own)
   float param;             // per channel: 1 / tau; scalar gates: the cap
   float qscale, kscale;
-  float* state;            // [slots, state_ld]: S [heads][dim][vdim]; scalar gates also n [heads][dim] and m [heads]
+  float* state;            // [slots, state_ld]: S [heads][vdim][dim]; scalar gates then, per
+                           // workgroup of a head, n [heads][dim] and m [heads]
   long long state_ld;
   float* out;              // [rows, ldo]: head h at columns h*vdim ..
   int ldo;
@@ -285,16 +290,19 @@ struct RecurArgs {
   const int32_t* positions;
   int heads, dim, vdim;
   // long prompt portions in three passes (PHASE 1 to 3): chunks [n][4] = (first row, rows, request of the step, 1 if it is
-  // the request's last chunk); records of heads x (dim*vdim + dim + 2) floats per chunk: S, a vector, two scalars
+  // the request's last chunk); heads records of recur_record floats per chunk
   const int32_t* chunks;
-  float* local;            // per chunk, from zero state: S, and the decay over the chunk (per channel: the product of the
+  float* local;            // per chunk, from zero state: S [vdim][dim], and the decay over the chunk (per channel: the product of the
                            // decays; scalar gates: n, the maximum from -inf, the sum of the log forget gates)
   float* start;            // per chunk: the state it starts from (S; scalar gates: n, m)
 };
 
-// One wave per (request, head, block of 64, 32 or 16 value columns: see SPLIT).  Lane j keeps column j of the head's state matrix in
-// registers (one element per key channel), so the read-out S^T q needs no exchange between lanes; the tokens' q, k and
-// decays come through LDS in chunks of RC tokens and are read from there by all lanes at once.
+// A wave holds the state of 64 / SPLIT value columns of one head in registers: SPLIT lanes a column, each with DH consecutive
+// key channels, so that a head has many short waves; the parts' read-outs are added by lane exchanges in one order whatever
+// runs the head (a single token, a portion, a chunk): the split depends on the head's size alone.  The tokens' q, k, decays
+// and v come through LDS in chunks of RC tokens, shared by the workgroup's waves (neighbouring column blocks of one head);
+// the next chunk is on its way from memory while one is worked on.  In memory a column's channels lie side by side,
+// [column][channel], so a lane's part is a run of whole vectors.
 //
 // RECUR_DECAY_PER_CHANNEL:  S[d][j] <- alpha[d] S[d][j] + k[d] v[j],  alpha = exp(logsigmoid(z + bias) / tau);  o[j] = sum_d S[d][j] q[d].
 // RECUR_SCALAR_GATES:  i = cap tanh((gi + bi) / cap), f = logsigmoid(cap tanh((gf + bf) / cap)), m' = max(f + m, i),
@@ -316,29 +324,37 @@ struct RecurArgs {
 // chunk from there with the read-out, and the request's last chunk leaves the state in the slot.  PHASE 0 is the whole
 // portion by one wave.  The passes differ from PHASE 0 by the rounding of the scan's sums only.
 #define RC 16
-#define RW 4             // waves of a workgroup: neighbouring column blocks of one head, which share the staged tokens
+#define RW 4             // waves of a workgroup
+// floats of a chunk's record for one head: S, a vector, two scalars, in whole vectors of four
+__host__ __device__ __forceinline__ size_t recur_record(int dim, int vdim) { return ((size_t)dim * vdim + dim + 2 + 3) & ~(size_t)3; }
+
+__host__ __device__ constexpr int recur_split(int dpad) { return dpad >= 128 ? 16 : dpad / 8; }
+// value columns of a workgroup, and how many workgroups share a head
+__host__ __device__ constexpr int recur_columns(int dim) {
+  return RW * 64 / recur_split(dim <= 16 ? 16 : (dim <= 32 ? 32 : (dim <= 64 ? 64 : 128)));
+}
+__host__ __device__ constexpr int recur_blocks(int dim, int vdim) { return (vdim + recur_columns(dim) - 1) / recur_columns(dim); }
+
 template <int MODE, int DPAD, int PHASE>
 __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a) {
   constexpr bool GATES = MODE == RECUR_SCALAR_GATES;
   constexpr bool BONUS = MODE == RECUR_BONUS_DECAY, FIXED = MODE == RECUR_FIXED_DECAY, STEP = MODE == RECUR_STEP_DECAY;
+  constexpr bool CHANNELS = !GATES && !STEP;             // a decay per channel comes through LDS
   constexpr int NN = (DPAD + 63) / 64;
   constexpr bool READ_OUT = PHASE != 1;
-  // A column's key channels are split over SPLIT lanes (lane l, l + COLS, ... hold consecutive parts of column l mod COLS): a
-  // lane's part of the state is at most 64 registers and a token costs a lane DPAD / SPLIT steps, so a head has more and
-  // shorter waves.  The parts' read-outs are added by the swaps of the wave's halves and quarters, in one order whatever
-  // runs the head (a single token, a portion, a chunk): the split depends on the head's size alone.
-  constexpr int SPLIT = DPAD >= 64 ? 4 : (DPAD >= 32 ? 2 : 1);
-  constexpr int DH = DPAD / SPLIT, COLS = 64 / SPLIT;
-  __shared__ float qs[RC][DPAD];
-  __shared__ float ks[RC][DPAD];
-  __shared__ float as[GATES || STEP ? 1 : RC][GATES || STEP ? 1 : DPAD];
-  __shared__ float gi[RC], gf[RC];
-  __shared__ float vs[RW][RC][64];
-  __shared__ float us[BONUS ? DPAD : 1];
+  constexpr int SPLIT = recur_split(DPAD), DH = DPAD / SPLIT, COLS = 64 / SPLIT, WCOLS = RW * COLS;
+  constexpr int TU = SPLIT >= 4 ? 4 : 2;                 // tokens worked on together
+  constexpr int NQ = RC * DPAD / (64 * RW), NV = (RC * WCOLS + 64 * RW - 1) / (64 * RW);
+  static_assert(NQ * 64 * RW == RC * DPAD && RC % TU == 0, "a chunk is whole loads and whole groups of tokens");
+  __shared__ __attribute__((aligned(16))) float qs[2][RC][DPAD];
+  __shared__ __attribute__((aligned(16))) float ks[2][RC][DPAD];
+  __shared__ __attribute__((aligned(16))) float as[CHANNELS ? 2 : 1][CHANNELS ? RC : 1][CHANNELS ? DPAD : 4];
+  __shared__ float gi[2][RC], gf[2][RC];
+  __shared__ float vs[2][RC][WCOLS];
   const int lane = threadIdx.x & 63, wv = wave_index();
-  const int cb = blockIdx.x * RW + wv, h = blockIdx.y;
+  const int h = blockIdx.y;
   const int dim = a.dim, vdim = a.vdim;
-  const size_t rec = (size_t)dim * vdim + dim + 2;
+  const size_t rec = recur_record(dim, vdim);
   int first, count, slot;
   bool leaves_state = true;
   if constexpr (PHASE == 0) {
@@ -355,13 +371,16 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   }
   if (count <= 0 || slot < 0) return;
   if (a.positions[first] < 0) return;
-  const int col = lane % COLS, dbase = (lane / COLS) * DH;
-  const int j = cb * COLS + col;
+  const int col = lane % COLS, part = lane / COLS, dbase = part * DH;
+  const int j_wg = blockIdx.x * WCOLS, j_in = wv * COLS + col, j = j_wg + j_in;
   const bool live = j < vdim;
   float* st = a.state + (size_t)slot * a.state_ld;
   float* S = st + (size_t)h * dim * vdim;
-  float* nv = st + (size_t)a.heads * dim * vdim + (size_t)h * dim;
-  float* mv = st + (size_t)a.heads * dim * vdim + (size_t)a.heads * dim + h;
+  // (every workgroup of a head carries the normaliser and the maximum, so each keeps a copy of its own in the slot: one that
+  // starts late must not find what another has already written)
+  const size_t copy = (size_t)a.heads * dim + a.heads;
+  float* nv = st + (size_t)a.heads * dim * vdim + (GATES ? blockIdx.x * copy : 0) + (size_t)h * dim;
+  float* mv = st + (size_t)a.heads * dim * vdim + (GATES ? blockIdx.x * copy : 0) + (size_t)a.heads * dim + h;
   // where this wave's state comes from: the slot, nothing, or the chunk's start record
   const float* S_in = S;
   const float* nv_in = nv;
@@ -373,9 +392,20 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   }
 
   float Sreg[DH];
+  const bool in_vectors = (dim & 3) == 0 && (reinterpret_cast<uintptr_t>(S_in) & 15) == 0;     // (scalar)
+  if (PHASE != 1 && in_vectors) {
+    const f32x4* src = reinterpret_cast<const f32x4*>(S_in + (size_t)min(j, vdim - 1) * dim);
 #pragma unroll
-  for (int d = 0; d < DH; ++d) Sreg[d] = (PHASE != 1 && live && dbase + d < dim) ? S_in[(size_t)(dbase + d) * vdim + j] : 0.0f;
-  float nreg[NN];          // scalar gates: the normaliser; per channel in PHASE 1: the product of the chunk's decays
+    for (int d = 0; d < DH; d += 4) {
+      const f32x4 v = src[min(dbase + d, dim - 4) >> 2];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) Sreg[d + e] = live && dbase + d < dim ? v[e] : 0.0f;
+    }
+  } else {
+#pragma unroll
+    for (int d = 0; d < DH; ++d) Sreg[d] = (PHASE != 1 && live && dbase + d < dim) ? S_in[(size_t)j * dim + dbase + d] : 0.0f;
+  }
+  float nreg[NN];          // scalar gates: the normaliser; otherwise in PHASE 1: the product of the chunk's decays
   float m = 0.0f, fsum = 0.0f;
   if constexpr (GATES) {
 #pragma unroll
@@ -385,131 +415,196 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
 #pragma unroll
     for (int i = 0; i < NN; ++i) nreg[i] = 1.0f;
   }
-
+  float ureg[BONUS ? DH : 1];
   if constexpr (BONUS) {
-    for (int d = threadIdx.x; d < DPAD; d += 64 * RW) us[d] = d < dim ? a.bias2[h * dim + d] : 0.0f;
+#pragma unroll
+    for (int d = 0; d < DH; ++d) ureg[d] = dbase + d < dim ? a.bias2[h * dim + dbase + d] : 0.0f;
   }
   const float fixed_decay = FIXED ? a.bias[h] : 0.0f;
   const float skip = STEP && a.skip != nullptr ? a.skip[h] : 0.0f;
   const int hk = h / a.heads_per_key;
-  for (int t0 = 0; t0 < count; t0 += RC) {
+
+  // a chunk's operands on their way from memory (every load clamped into its row; what lies outside is zeroed on the way to LDS)
+  float rq[NQ], rk[NQ], rz[CHANNELS && !FIXED ? NQ : 1], rv[NV], rg[2];
+  auto fetch = [&](int t0) {
+    if (t0 >= count) return;                             // (scalar)
     const int tc = min(RC, count - t0);
-    __syncthreads();
-    // eight elements a lane at a time: their loads are all asked for before the first is used
-    for (int e0 = 0; e0 < tc * DPAD; e0 += 64 * RW * 8) {
-      float qv[8], kv[8], zv[8];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) {
-        const int e = e0 + 64 * RW * u + (int)threadIdx.x;
-        const int t = e / DPAD, d = e % DPAD;
-        const bool in = e < tc * DPAD && d < dim;
-        const size_t row = (size_t)(first + t0 + min(t, tc - 1));
+    for (int u = 0; u < NQ; ++u) {
+      if (64 * RW * u < tc * DPAD) {                     // (scalar)
+        const int e = 64 * RW * u + (int)threadIdx.x;
+        const size_t row = (size_t)(first + t0 + min(e / DPAD, tc - 1));
+        const int d = min(e % DPAD, dim - 1);
         const float* pr = a.proj + row * a.ldp;
-        qv[u] = in ? pr[a.q_off + hk * dim + d] : 0.0f;
-        kv[u] = in ? pr[a.k_off + hk * dim + d] : 0.0f;
-        if constexpr (!GATES && !FIXED && !STEP) zv[u] = in ? a.gate[row * a.ldg + a.gate_off + h * dim + d] + a.bias[h * dim + d] : 0.0f;
-      }
-#pragma unroll
-      for (int u = 0; u < 8; ++u) {
-        const int e = e0 + 64 * RW * u + (int)threadIdx.x;
-        if (e >= tc * DPAD) continue;
-        const int t = e / DPAD, d = e % DPAD;
-        qs[t][d] = qv[u] * a.qscale;
-        ks[t][d] = kv[u] * a.kscale;
-        if constexpr (FIXED) as[t][d] = d < dim ? fixed_decay : 0.0f;
-        else if constexpr (BONUS) as[t][d] = d < dim ? bw_expf(-bw_expf(zv[u])) : 0.0f;
-        else if constexpr (!GATES && !STEP) as[t][d] = d < dim ? bw_expf(log_sigmoid(zv[u]) * a.param) : 0.0f;
+        rq[u] = pr[a.q_off + hk * dim + d];
+        rk[u] = pr[a.k_off + hk * dim + d];
+        if constexpr (CHANNELS && !FIXED) rz[u] = a.gate[row * a.ldg + a.gate_off + h * dim + d] + a.bias[h * dim + d];
       }
     }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      if (64 * RW * u < tc * WCOLS) {
+        const int e = 64 * RW * u + (int)threadIdx.x;
+        const size_t row = (size_t)(first + t0 + min(e / WCOLS, tc - 1));
+        rv[u] = a.proj[row * a.ldp + a.v_off + h * vdim + min(j_wg + e % WCOLS, vdim - 1)];
+      }
+    }
+    if constexpr (GATES || STEP) {
+      const float* gr = a.gate + (size_t)(first + t0 + min((int)threadIdx.x, tc - 1)) * a.ldg;
+      rg[0] = gr[a.gate_off + h];
+      rg[1] = GATES ? gr[a.gate2_off + h] : 0.0f;
+    }
+  };
+  auto stash = [&](int t0, int buf) {
+    if (t0 >= count) return;
+    const int tc = min(RC, count - t0);
+#pragma unroll
+    for (int u = 0; u < NQ; ++u) {
+      if (64 * RW * u < tc * DPAD) {
+        const int e = 64 * RW * u + (int)threadIdx.x;
+        const int t = e / DPAD, d = e % DPAD;
+        const bool in = d < dim;
+        qs[buf][t][d] = in ? rq[u] * a.qscale : 0.0f;
+        ks[buf][t][d] = in ? rk[u] * a.kscale : 0.0f;
+        if constexpr (FIXED) as[buf][t][d] = in ? fixed_decay : 0.0f;
+        else if constexpr (BONUS) as[buf][t][d] = in ? bw_expf(-bw_expf(rz[u])) : 0.0f;
+        else if constexpr (CHANNELS) as[buf][t][d] = in ? bw_expf(log_sigmoid(rz[u]) * a.param) : 0.0f;
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int e = 64 * RW * u + (int)threadIdx.x;
+      if (64 * RW * u < tc * WCOLS && e < RC * WCOLS) vs[buf][e / WCOLS][e % WCOLS] = j_wg + e % WCOLS < vdim ? rv[u] : 0.0f;
+    }
     if constexpr (GATES) {
-      if (wv == 0 && lane < tc) {
-        const float* pr = a.proj + (size_t)(first + t0 + lane) * a.ldp;
+      if ((int)threadIdx.x < tc) {
         const float cap = a.param;
-        gi[lane] = cap * tanhf((pr[a.gate_off + h] + a.bias[h]) / cap);
-        gf[lane] = log_sigmoid(cap * tanhf((pr[a.gate2_off + h] + a.bias2[h]) / cap));
+        gi[buf][threadIdx.x] = cap * tanhf((rg[0] + a.bias[h]) / cap);
+        gf[buf][threadIdx.x] = log_sigmoid(cap * tanhf((rg[1] + a.bias2[h]) / cap));
       }
     }
     if constexpr (STEP) {
-      if (wv == 0 && lane < tc) {
-        const float z = a.gate[(size_t)(first + t0 + lane) * a.ldg + a.gate_off + h] + a.bias[h];
-        const float delta = softplus(z);
-        gi[lane] = delta;
-        gf[lane] = bw_expf(-(a.bias2[h] * delta));
+      if ((int)threadIdx.x < tc) {
+        const float delta = softplus(rg[0] + a.bias[h]);
+        gi[buf][threadIdx.x] = delta;
+        gf[buf][threadIdx.x] = bw_expf(-(a.bias2[h] * delta));
       }
     }
-    // (a column's lanes read what its first lane wrote)
-    if (lane < COLS) {
+  };
+
+  // N tokens from t on: their operands out of LDS together, then one after the other
+  auto tokens = [&](auto count_tag, int t0, int buf, int t) {
+    constexpr int N = decltype(count_tag)::value;
+    float kr[N][DH], qr[N][DH], ar[CHANNELS ? N : 1][CHANNELS ? DH : 1], vr[N], g1[N], g2[N], o[N];
 #pragma unroll
-      for (int t = 0; t < RC; ++t)
-        vs[wv][t][col] = (live && t < tc) ? a.proj[(size_t)(first + t0 + t) * a.ldp + a.v_off + h * vdim + j] : 0.0f;
+    for (int n = 0; n < N; ++n) {
+#pragma unroll
+      for (int d = 0; d < DH; d += 4) {
+        const f32x4 kv = *reinterpret_cast<const f32x4*>(&ks[buf][t + n][dbase + d]);
+        const f32x4 qv = *reinterpret_cast<const f32x4*>(&qs[buf][t + n][dbase + d]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          kr[n][d + e] = kv[e];
+          qr[n][d + e] = qv[e];
+        }
+        if constexpr (CHANNELS) {
+          const f32x4 av = *reinterpret_cast<const f32x4*>(&as[buf][t + n][dbase + d]);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) ar[n][d + e] = av[e];
+        }
+      }
+      vr[n] = vs[buf][t + n][j_in];
+      if constexpr (GATES || STEP) {
+        g1[n] = gi[buf][t + n];
+        g2[n] = gf[buf][t + n];
+      }
     }
-    __syncthreads();
-    for (int t = 0; t < tc; ++t) {
-      float o = 0.0f;
+#pragma unroll
+    for (int n = 0; n < N; ++n) {
+      o[n] = 0.0f;
       if constexpr (STEP) {
-        const float v = vs[wv][t][col];
-        const float fa = gf[t], bv = gi[t] * v;
+        const float fa = g2[n], bv = g1[n] * vr[n];
 #pragma unroll
         for (int d = 0; d < DH; ++d) {
-          Sreg[d] = fmaf(fa, Sreg[d], ks[t][dbase + d] * bv);
-          if constexpr (READ_OUT) o = fmaf(Sreg[d], qs[t][dbase + d], o);
+          Sreg[d] = fmaf(fa, Sreg[d], kr[n][d] * bv);
+          if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
         }
         if constexpr (PHASE == 1) {
 #pragma unroll
           for (int i = 0; i < NN; ++i) nreg[i] *= fa;
         }
-        if constexpr (READ_OUT) o = fmaf(skip, v, join_parts<SPLIT>(o));
       } else if constexpr (!GATES) {
-        const float v = vs[wv][t][col];
 #pragma unroll
         for (int d = 0; d < DH; ++d) {
+          const float kv = kr[n][d] * vr[n];
           if constexpr (BONUS) {
-            const float kv = ks[t][dbase + d] * v;
-            if constexpr (READ_OUT) o = fmaf(fmaf(us[dbase + d], kv, Sreg[d]), qs[t][dbase + d], o);
-            Sreg[d] = fmaf(as[t][dbase + d], Sreg[d], kv);
+            if constexpr (READ_OUT) o[n] = fmaf(fmaf(ureg[d], kv, Sreg[d]), qr[n][d], o[n]);
+            Sreg[d] = fmaf(ar[n][d], Sreg[d], kv);
           } else {
-            Sreg[d] = fmaf(as[t][dbase + d], Sreg[d], ks[t][dbase + d] * v);
-            if constexpr (READ_OUT) o = fmaf(Sreg[d], qs[t][dbase + d], o);
+            Sreg[d] = fmaf(ar[n][d], Sreg[d], kv);
+            if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
           }
         }
         if constexpr (PHASE == 1) {
 #pragma unroll
           for (int i = 0; i < NN; ++i)
-            if (lane + 64 * i < DPAD) nreg[i] *= as[t][lane + 64 * i];
+            if (lane + 64 * i < DPAD) nreg[i] *= as[buf][t + n][lane + 64 * i];
         }
       } else {
-        const float ig = gi[t], fg = gf[t];
+        const float ig = g1[n], fg = g2[n];
         const float mn = fmaxf(fg + m, ig);
         const float fa = bw_expf(fg + m - mn);
         const float ib = bw_expf(ig - mn);
         m = mn;
         fsum += fg;
-        const float bv = ib * vs[wv][t][col];
+        const float bv = ib * vr[n];
 #pragma unroll
         for (int d = 0; d < DH; ++d) {
-          Sreg[d] = fmaf(fa, Sreg[d], ks[t][dbase + d] * bv);
-          if constexpr (READ_OUT) o = fmaf(Sreg[d], qs[t][dbase + d], o);
+          Sreg[d] = fmaf(fa, Sreg[d], kr[n][d] * bv);
+          if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
         }
-        float part = 0.0f;
+        float sum = 0.0f;
 #pragma unroll
         for (int i = 0; i < NN; ++i) {
           const int d = lane + 64 * i;
           if (d < DPAD) {
-            nreg[i] = fmaf(fa, nreg[i], ib * ks[t][d]);
-            part = fmaf(nreg[i], qs[t][d], part);
+            nreg[i] = fmaf(fa, nreg[i], ib * ks[buf][t + n][d]);
+            sum = fmaf(nreg[i], qs[buf][t + n][d], sum);
           }
         }
         if constexpr (READ_OUT) {
-          o = join_parts<SPLIT>(o);
-          const float nq = wave_sum(part);
-          o = o / (fmaxf(fabsf(nq), bw_expf(-mn)) + 1e-6f);
+          o[n] = join_parts<SPLIT>(o[n]);
+          const float nq = wave_sum(sum);
+          o[n] = o[n] / (fmaxf(fabsf(nq), bw_expf(-mn)) + 1e-6f);
         }
       }
-      if constexpr (READ_OUT) {
-        if constexpr (!GATES && !STEP) o = join_parts<SPLIT>(o);
-        if (live && lane < COLS) a.out[(size_t)(first + t0 + t) * a.ldo + h * vdim + j] = o;
-      }
     }
+    if constexpr (READ_OUT) {
+      // (part n of a column stores token t + n)
+      float mine = 0.0f;
+#pragma unroll
+      for (int n = 0; n < N; ++n) {
+        float v = o[n];
+        if constexpr (!GATES) v = join_parts<SPLIT>(v);
+        if constexpr (STEP) v = fmaf(skip, vr[n], v);
+        mine = part == n ? v : mine;
+      }
+      if (live && part < N) a.out[(size_t)(first + t0 + t + part) * a.ldo + h * vdim + j] = mine;
+    }
+  };
+
+  fetch(0);
+  stash(0, 0);
+  __syncthreads();
+  int buf = 0;
+  for (int t0 = 0; t0 < count; t0 += RC, buf ^= 1) {
+    const int tc = min(RC, count - t0);
+    fetch(t0 + RC);
+    int t = 0;
+    for (; t + TU <= tc; t += TU) tokens(std::integral_constant<int, TU>{}, t0, buf, t);
+    for (; t < tc; ++t) tokens(std::integral_constant<int, 1>{}, t0, buf, t);
+    stash(t0 + RC, buf ^ 1);
+    __syncthreads();
   }
   // where the state goes: the slot (PHASE 3: from the request's last chunk only), or the chunk's own record
   float* S_out = S;
@@ -522,11 +617,18 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   }
   if (PHASE == 3 && !leaves_state) return;
   if (live) {
+    if ((dim & 3) == 0 && (reinterpret_cast<uintptr_t>(S_out) & 15) == 0) {
+      f32x4* dst = reinterpret_cast<f32x4*>(S_out + (size_t)j * dim);
 #pragma unroll
-    for (int d = 0; d < DH; ++d)
-      if (dbase + d < dim) S_out[(size_t)(dbase + d) * vdim + j] = Sreg[d];
+      for (int d = 0; d < DH; d += 4)
+        if (dbase + d < dim) dst[(dbase + d) >> 2] = (f32x4){Sreg[d], Sreg[d + 1], Sreg[d + 2], Sreg[d + 3]};
+    } else {
+#pragma unroll
+      for (int d = 0; d < DH; ++d)
+        if (dbase + d < dim) S_out[(size_t)j * dim + dbase + d] = Sreg[d];
+    }
   }
-  if (cb == 0 && (GATES || PHASE == 1)) {
+  if (wv == 0 && (PHASE == 1 ? blockIdx.x == 0 : GATES)) {
 #pragma unroll
     for (int i = 0; i < NN; ++i)
       if (lane + 64 * i < dim) nv_out[lane + 64 * i] = nreg[i];
@@ -549,7 +651,7 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurArgs a, const
   const int seq = spans[3 * blockIdx.z], c0 = spans[3 * blockIdx.z + 1], nc = spans[3 * blockIdx.z + 2];
   const int slot = a.slots[seq];
   if (slot < 0 || nc <= 0) return;
-  const size_t rec = (size_t)dim * vdim + dim + 2;
+  const size_t rec = recur_record(dim, vdim);
   const int e = blockIdx.x * 256 + threadIdx.x;
   const int sd = dim * vdim;
   const int mine = GATES ? sd + dim + 1 : sd;          // elements a head has to carry: S, and with scalar gates n and m
@@ -572,15 +674,14 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurArgs a, const
       m = mn;
     } else {
       out[e] = val;
-      val = fmaf(loc[sd + e / vdim], val, loc[e]);
+      val = fmaf(loc[sd + e % dim], val, loc[e]);
     }
   }
 }
 
 template <int MODE, int PHASE>
 int launch_recurrence(const RecurArgs& a, int units, hipStream_t s) {
-  const int cols = a.dim > 32 ? 16 : (a.dim > 16 ? 32 : 64);      // (columns a wave: linear_recurrence_kernel's COLS)
-  const dim3 grid((a.vdim + RW * cols - 1) / (RW * cols), a.heads, units), block(64 * RW);
+  const dim3 grid(recur_blocks(a.dim, a.vdim), a.heads, units), block(64 * RW);
   if (a.dim <= 16) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 16, PHASE>), grid, block, 0, s, a);
   else if (a.dim <= 32) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 32, PHASE>), grid, block, 0, s, a);
   else if (a.dim <= 64) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 64, PHASE>), grid, block, 0, s, a);
@@ -818,10 +919,10 @@ extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_
   if (nseq <= 0 && nchunks <= 0) return 0;
   if (nchunks > 0) {
     if (chunks == nullptr || spans == nullptr || nspans <= 0 || scan_local == nullptr || scan_start == nullptr) return -2;
-    if (scan_floats < (long long)nchunks * heads * ((long long)dim * vdim + dim + 2)) return -6;
+    if (scan_floats < (long long)nchunks * heads * (long long)recur_record(dim, vdim)) return -6;
   }
   if (heads <= 0 || dim <= 0 || vdim <= 0 || ldo < heads * vdim || heads_per_key < 1 || heads % heads_per_key) return -2;
-  const long long need = (long long)heads * dim * vdim + (mode == RECUR_SCALAR_GATES ? (long long)heads * dim + heads : 0);
+  const long long need = (long long)heads * dim * vdim + (mode == RECUR_SCALAR_GATES ? (long long)recur_blocks(dim, vdim) * ((long long)heads * dim + heads) : 0);
   if (state_ld < need) return -2;
   if (bias == nullptr || (mode != RECUR_FIXED_DECAY && gate == nullptr) || ((mode == RECUR_SCALAR_GATES || mode == RECUR_BONUS_DECAY || mode == RECUR_STEP_DECAY) && bias2 == nullptr))
     return -2;
@@ -835,6 +936,8 @@ extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_
   if (mode == RECUR_STEP_DECAY) return launch_recurrence_passes<RECUR_STEP_DECAY>(a, nseq, nchunks, spans, nspans, s);
   return -2;
 }
+
+extern "C" long long bw_recurrence_record(int dim, int vdim) { return (long long)recur_record(dim, vdim); }
 
 extern "C" int bw_head_norm_gate(const float* o, int ldi, const float* weight, int wstride, const float* g, int ldg, int gate,
                                  void* out, int out_is_bf16, int ldo, const int32_t* positions, int rows, int heads, int vdim,

@@ -117,10 +117,7 @@ class _MatrixMemoryMixer(Mixer):
         self.norm_weight = tensors["norm"].to(self.rt.device).float().contiguous()
 
     def state_spec(self) -> StateSpec:
-        n = self.heads * self.dim * self.vdim
-        if self.mode == ops.RECUR_SCALAR_GATES:
-            n += self.heads * self.dim + self.heads
-        return StateSpec((n,), "float32")
+        return StateSpec((ops.recurrence_state(self.mode, self.heads, self.dim, self.vdim),), "float32")
 
     def input_projection(self):
         return self.proj
@@ -143,7 +140,7 @@ class _MatrixMemoryMixer(Mixer):
         seq_rows, nseq, scan = ctx.seq_rows, ctx.nseq, None
         if plan is not None:
             seq_rows, nseq, chunks, nchunks, spans, nspans = plan
-            rec = self.heads * (self.dim * self.vdim + self.dim + 2)
+            rec = self.heads * ops.recurrence_record(self.dim, self.vdim)
             most = ctx.ws.max_rows // SCAN_CHUNK + ctx.ws.max_rows // SCAN_MIN_ROWS + 1     # chunks a step can bring
             local = ctx.ws.buffer("recur_scan_local", most * rec, torch.float32, rows=1)
             start = ctx.ws.buffer("recur_scan_start", most * rec, torch.float32, rows=1)

@@ -429,7 +429,7 @@ def test_recurrence_with_step_sizes_against_plain(gpu, heads, groups, dim, vdim)
             scan, seq_rows, nseq = None, dev([0, n]), 1
             if scan_from is not None and n >= scan_from:
                 chunks = [(c0, min(32, n - c0), 0, int(c0 + 32 >= n)) for c0 in range(0, n, 32)]
-                rec = heads * (dim * vdim + dim + 2)
+                rec = heads * ops.recurrence_record(dim, vdim)
                 scan = (dev(sum(chunks, ())), len(chunks), dev([0, 0, len(chunks)]), 1,
                         torch.zeros(len(chunks) * rec, device=gpu), torch.zeros(len(chunks) * rec, device=gpu))
                 seq_rows, nseq = dev([0, 0]), 0
