@@ -209,7 +209,7 @@ struct HeadGemmArgs {
   int in, outn;
   void* out;
   int ldo, ohs, rows;
-  int aligned;             // rows and heads of out start at whole groups of four elements, outn is a multiple of 4
+  int aligned;             // 1: rows and heads of out start at whole groups of four elements, outn is a multiple of 4; 2: of eight
 };
 
 template <typename XT, typename OT, int OB, bool ROW_WAVES>
@@ -237,9 +237,11 @@ __global__ __launch_bounds__(256) void headwise_mfma_kernel(HeadGemmArgs a, Head
   const int o0 = blockIdx.z * 64 + (ROW_WAVES ? 0 : 16 * wv);
   if (r0 >= a.rows || o0 >= a.outn) return;
   const XT* xr = xh + (size_t)min(r0 + n, a.rows - 1) * a.ldx;
+  // block b's row k of the product is output o0 + 4 OB (k / 4) + 4 b + k % 4: a lane's results are 4 OB neighbours
+  auto output_of = [](int b, int k) { return 4 * OB * (k >> 2) + 4 * b + (k & 3); };
   const bf16_t* wr[OB];
 #pragma unroll
-  for (int b = 0; b < OB; ++b) wr[b] = a.w + ((size_t)h * a.outn + min(o0 + 16 * b + n, a.outn - 1)) * a.in;
+  for (int b = 0; b < OB; ++b) wr[b] = a.w + ((size_t)h * a.outn + min(o0 + output_of(b, n), a.outn - 1)) * a.in;
   f32x4 acc[OB];
 #pragma unroll
   for (int b = 0; b < OB; ++b) acc[b] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -270,9 +272,20 @@ __global__ __launch_bounds__(256) void headwise_mfma_kernel(HeadGemmArgs a, Head
   const int r = r0 + n;
   if (r >= a.rows) return;
   const float gate = ex.gate != nullptr ? 1.0f / (1.0f + bw_expf(-ex.gate[(size_t)r * ex.ldg + h])) : 1.0f;
+  if constexpr (OB == 4 && sizeof(OT) == 2) {
+    if (a.aligned == 2 && o0 + 16 * g + 15 < a.outn) {
+      OT* dst = oh + (size_t)r * a.ldo + o0 + 16 * g;
+#pragma unroll
+      for (int b = 0; b < OB; b += 2)
+        *reinterpret_cast<u32x4*>(dst + 4 * b) = (u32x4){pack_bf16x2(acc[b][0] * gate, acc[b][1] * gate), pack_bf16x2(acc[b][2] * gate, acc[b][3] * gate),
+                                                         pack_bf16x2(acc[b + 1][0] * gate, acc[b + 1][1] * gate),
+                                                         pack_bf16x2(acc[b + 1][2] * gate, acc[b + 1][3] * gate)};
+      return;
+    }
+  }
 #pragma unroll
   for (int b = 0; b < OB; ++b) {
-    const int o = o0 + 16 * b + 4 * g;       // outputs o .. o + 3 of this lane's row
+    const int o = o0 + output_of(b, 4 * g);  // outputs o .. o + 3 of this lane's row
     OT* dst = oh + (size_t)r * a.ldo + o;
     if (a.aligned) {
       if (o >= a.outn) continue;
@@ -495,7 +508,7 @@ int launch_shared_key(const SharedKeyArgs& a, const CT* cache, int num_tiles, hi
 
 // ------------------------------------------------------------------------- the same attention on the matrix cores
 
-// bfloat16 caches whose key vectors are whole 16-byte groups.  A workgroup of four waves per (tile of rows, group of ``hg``
+// bfloat16 caches whose key vectors are whole 16-byte groups.  A workgroup of NW waves per (tile of rows, group of ``hg``
 // heads): 16 QT query vectors (16 QT / hg rows x hg heads).  The keys are cut into pieces of SK_PIECE keys at absolute
 // positions, and a piece is one unit of arithmetic: its scores, the largest of them that a query sees, the weights relative to
 // that maximum (32-bit, rounded to bfloat16 where they enter the product with the values), their sum, and the weighted sum of
@@ -504,11 +517,12 @@ int launch_shared_key(const SharedKeyArgs& a, const CT* cache, int num_tiles, hi
 // each, leave (maximum, sum, values) in memory, and shared_key_combine_kernel folds them by the same operations in the same
 // order: a position's bits do not depend on whether it came alone or inside a portion.
 //
-// Within a piece: scores by v_mfma_f32_16x16x32_bf16 with the keys as rows (operand A, straight from the cache: a wave takes 32
-// of the piece's keys, a lane reads 8 consecutive elements of its key) and the queries as columns (operand B, from LDS).  The
-// weights go through LDS; a wave then owns every fourth block of 16 value elements, read from the second copy of the latent that
+// Within a piece: scores by v_mfma_f32_16x16x32_bf16 with the keys as rows (operand A, straight from the cache: a wave takes
+// its share of the piece's keys in tiles of 16, a lane reads 8 consecutive elements of its key) and the queries as columns (operand B, from LDS).  The
+// weights go through LDS; a wave then owns every NW-th block of 16 value elements, read from the second copy of the latent that
 // the cache write leaves transposed, [page][element][slot]: a lane's 8 keys are 16 consecutive bytes of its element's row.
 #define SK_PIECE 128
+#define SK_TILE_QUERIES 32          // query vectors of a prompt tile's workgroup: two of them fit a compute unit's registers
 #define SK_PSTRIDE (SK_PIECE + 8)
 
 struct MfmaAttnArgs {
@@ -565,14 +579,16 @@ __device__ __forceinline__ void store_out(const MfmaAttnArgs& a, size_t at, floa
   else reinterpret_cast<float*>(a.out)[at] = v;
 }
 
-// NDT: blocks of 16 value elements a wave owns (wave w: blocks w, w + 4, ...).  QT 1: a workgroup a piece (single tokens).
-template <int QT, int NDT>
-__global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttnArgs a, const bf16_t* __restrict__ kc,
+// NDT: blocks of 16 value elements a wave owns (wave w: blocks w, w + NW, ...).  QT 1: a workgroup a piece (single tokens).
+// The sums of the weights are kept by tiles of 16 keys and added in tile order, whatever the number of waves.
+template <int QT, int NW, int NDT>
+__global__ __launch_bounds__(64 * NW, QT == 1 ? 1 : 2) void shared_key_attention_mfma_kernel(MfmaAttnArgs a, const bf16_t* __restrict__ kc,
                                                                         const bf16_t* __restrict__ vt) {
   constexpr bool PIECES = QT == 1;
   constexpr int NQ = 16 * QT;
+  constexpr int KT = SK_PIECE / 16, U = KT / NW;           // tiles of 16 keys: of a piece, of a wave
   extern __shared__ bf16_t sk_lds[];       // queries [NQ][qstride], weights [NQ][SK_PSTRIDE]
-  __shared__ float red_max[4][NQ], red_sum[4][NQ];
+  __shared__ float red_max[NW][NQ], red_sum[KT][NQ];
   const int lane = threadIdx.x & 63, n = lane & 15, g = lane >> 4, wv = wave_index();
   const int t = blockIdx.x, h0 = blockIdx.y * a.hg;
   int r0, nr, seq;
@@ -602,7 +618,7 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
   bf16_t* pw = sk_lds + NQ * qstride;
   {
     const int groups = dkp >> 3;             // 16-byte groups of a query vector (dk is a multiple of 8)
-    for (int e = threadIdx.x; e < NQ * groups; e += 256) {
+    for (int e = threadIdx.x; e < NQ * groups; e += 64 * NW) {
       const int qn = e / groups, d = (e % groups) * 8;
       const int r2 = qn / a.hg, h2 = h0 + qn % a.hg;
       u32x4 v = {0u, 0u, 0u, 0u};
@@ -610,7 +626,6 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
       *reinterpret_cast<u32x4*>(qs + qn * qstride + d) = v;
     }
   }
-  const int qt_live = min(QT, (nr * a.hg + 15) >> 4);      // tiles of 16 queries that hold one (scalar)
   int qpos[QT], qlo[QT];
 #pragma unroll
   for (int c = 0; c < QT; ++c) {
@@ -632,47 +647,43 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
   __syncthreads();
 
   for (; piece <= last; ++piece) {
-    const int k0 = piece * SK_PIECE, kw = k0 + 32 * wv;
+    const int k0 = piece * SK_PIECE, kw = k0 + 16 * U * wv;
     // where this lane's keys and runs of values lie
-    const bf16_t* krow[2];
+    const bf16_t* krow[U];
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
+    for (int u = 0; u < U; ++u) {
       const int kj = min(kw + 16 * u + n, pmax);
       krow[u] = kc + ((size_t)min(max(table[kj / ps], 0), a.num_pages - 1) * ps + kj % ps) * dk;
     }
     const bf16_t* vrun[4];
-    int vpage2[4];                           // (pages of four slots: the run's second half lies in a page of its own)
 #pragma unroll
     for (int sg = 0; sg < 4; ++sg) {
       const int c = min(k0 + 32 * sg + 8 * g, pmax & ~7);
       vrun[sg] = vt + (size_t)min(max(table[c / ps], 0), a.num_pages - 1) * dv * ps + c % ps;
-      vpage2[sg] = ps < 8 ? min(max(table[min(c + 4, pmax) / ps], 0), a.num_pages - 1) : 0;
     }
     auto load_values = [&](int sg, int j) -> u32x4 {
-      const int d = min(16 * (4 * j + wv) + n, dv - 1);     // (rows past the values are computed and never stored)
-      if (ps >= 8) return *reinterpret_cast<const u32x4*>(vrun[sg] + (size_t)d * ps);
-      const u32x2 lo = *reinterpret_cast<const u32x2*>(vrun[sg] + (size_t)d * ps);
-      const u32x2 hi = *reinterpret_cast<const u32x2*>(vt + (size_t)vpage2[sg] * dv * ps + (size_t)d * ps);
-      return (u32x4){lo[0], lo[1], hi[0], hi[1]};
+      // (rows past the values are computed and never stored)
+      const uint32_t d = (uint32_t)min(16 * (NW * j + wv) + n, dv - 1);
+      return *reinterpret_cast<const u32x4*>(vrun[sg] + d * (uint32_t)ps);
     };
 
-    // ---- scores of this wave's 32 keys: lane (n, g) gets keys kw + 16u + 4g + i of query n of every tile
-    f32x4 st[2][QT];
+    // ---- scores of this wave's keys: lane (n, g) gets keys kw + 16u + 4g + i of query n of every tile
+    f32x4 st[U][QT];
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
+    for (int u = 0; u < U; ++u)
 #pragma unroll
       for (int c = 0; c < QT; ++c) st[u][c] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    if (kw <= pmax && kw + 31 >= lo_first) {                 // (scalar: some query of the tile may see one of them)
-      constexpr int KST = QT == 1 ? 18 : 9;                  // steps of 32 elements whose loads are in flight together
+    if (kw <= pmax && kw + 16 * U - 1 >= lo_first) {                 // (scalar: some query of the tile may see one of them)
+      constexpr int KST = QT == 1 ? 18 : 6;                                // steps of 32 elements whose loads are in flight together
       for (int d1 = 0; d1 < dkp; d1 += 32 * KST) {
-        u32x4 kf[KST][2];
+        u32x4 kf[KST][U];
 #pragma unroll
         for (int s4 = 0; s4 < KST; ++s4) {
           // (elements past the key vector meet zeros in the query)
           const int d0 = min(d1 + 32 * s4 + 8 * g, dk - 8);
           if (d1 + 32 * s4 < dkp) {                          // (scalar)
-            kf[s4][0] = *reinterpret_cast<const u32x4*>(krow[0] + d0);
-            kf[s4][1] = *reinterpret_cast<const u32x4*>(krow[1] + d0);
+#pragma unroll
+            for (int u = 0; u < U; ++u) kf[s4][u] = *reinterpret_cast<const u32x4*>(krow[u] + d0);
           }
         }
 #pragma unroll
@@ -680,18 +691,23 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
           if (d1 + 32 * s4 < dkp) {
 #pragma unroll
             for (int c = 0; c < QT; ++c) {
-              if (c < qt_live) {                             // (scalar)
+              {
                 const u32x4 qf = *reinterpret_cast<const u32x4*>(qs + (16 * c + n) * qstride + d1 + 32 * s4 + 8 * g);
-                st[0][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(kf[s4][0]), as_bf16x8(qf), st[0][c], 0, 0, 0);
-                st[1][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(kf[s4][1]), as_bf16x8(qf), st[1][c], 0, 0, 0);
+#pragma unroll
+                for (int u = 0; u < U; ++u)
+                  st[u][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(kf[s4][u]), as_bf16x8(qf), st[u][c], 0, 0, 0);
               }
             }
           }
         }
+        __builtin_amdgcn_sched_barrier(0);
       }
     }
-    // the first blocks of values are asked for before the weights are formed
-    constexpr int AHEAD = NDT < 4 ? NDT : 4;
+    // the first blocks of values are asked for before the weights are formed (what is asked for when is as written: left to
+    // itself the scheduler asks for everything at once and runs out of registers)
+    __builtin_amdgcn_sched_barrier(0);
+    constexpr int MOST = QT == 1 ? 4 : 2;
+    constexpr int AHEAD = NDT < MOST ? NDT : MOST;
     u32x4 vf[AHEAD][4];
 #pragma unroll
     for (int j = 0; j < AHEAD; ++j)
@@ -703,7 +719,7 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
     for (int c = 0; c < QT; ++c) {
       float mx = -INFINITY;
 #pragma unroll
-      for (int u = 0; u < 2; ++u)
+      for (int u = 0; u < U; ++u)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int key = kw + 16 * u + 4 * g + i;
@@ -718,28 +734,31 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
     float mp[QT];
 #pragma unroll
     for (int c = 0; c < QT; ++c) {
-      mp[c] = fmaxf(fmaxf(red_max[0][16 * c + n], red_max[1][16 * c + n]), fmaxf(red_max[2][16 * c + n], red_max[3][16 * c + n]));
-      const float base = mp[c] == -INFINITY ? 0.0f : mp[c];
-      float psum = 0.0f;
+      mp[c] = red_max[0][16 * c + n];
 #pragma unroll
-      for (int u = 0; u < 2; ++u) {
-        float p[4];
+      for (int k = 1; k < NW; ++k) mp[c] = fmaxf(mp[c], red_max[k][16 * c + n]);
+      const float base = mp[c] == -INFINITY ? 0.0f : mp[c];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        float p[4], psum = 0.0f;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           p[i] = st[u][c][i] == -INFINITY ? 0.0f : fast_exp(st[u][c][i] - base);
           psum += p[i];
         }
-        *reinterpret_cast<u32x2*>(pw + (16 * c + n) * SK_PSTRIDE + 32 * wv + 16 * u + 4 * g) = (u32x2){pack_bf16x2(p[0], p[1]), pack_bf16x2(p[2], p[3])};
+        *reinterpret_cast<u32x2*>(pw + (16 * c + n) * SK_PSTRIDE + 16 * (U * wv + u) + 4 * g) = (u32x2){pack_bf16x2(p[0], p[1]), pack_bf16x2(p[2], p[3])};
+        psum = across_groups_sum(psum);
+        if (g == 0) red_sum[U * wv + u][16 * c + n] = psum;
       }
-      psum = across_groups_sum(psum);
-      if (g == 0) red_sum[wv][16 * c + n] = psum;
     }
     __syncthreads();
-    float c1[QT], c2[QT];
+    float c1[QT], c2[QT], lp = 0.0f;
     u32x4 pf[4][QT];
 #pragma unroll
     for (int c = 0; c < QT; ++c) {
-      const float lp = ((red_sum[0][16 * c + n] + red_sum[1][16 * c + n]) + red_sum[2][16 * c + n]) + red_sum[3][16 * c + n];
+      lp = red_sum[0][16 * c + n];
+#pragma unroll
+      for (int k = 1; k < KT; ++k) lp += red_sum[k][16 * c + n];
       fold_piece(m[c], l[c], mp[c], lp, c1[c], c2[c]);
 #pragma unroll
       for (int sg = 0; sg < 4; ++sg) pf[sg][c] = *reinterpret_cast<const u32x4*>(pw + (16 * c + n) * SK_PSTRIDE + 32 * sg + 8 * g);
@@ -747,14 +766,6 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
 
     // ---- the weighted sum of the values: a chain over the piece's keys for every block of 16 elements, then the fold
     const bool ragged = k0 + SK_PIECE - 1 > pmax || k0 < lo_first;       // slots outside may hold anything
-    uint32_t keep[4][4];
-#pragma unroll
-    for (int sg = 0; sg < 4; ++sg)
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int key = k0 + 32 * sg + 8 * g + 2 * e;
-        keep[sg][e] = (key <= pmax && key >= lo_first ? 0xffffu : 0u) | (key + 1 <= pmax && key + 1 >= lo_first ? 0xffff0000u : 0u);
-      }
 #pragma unroll
     for (int j = 0; j < NDT; ++j) {
       u32x4 v[4];
@@ -767,11 +778,14 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
 #pragma unroll
         for (int sg = 0; sg < 4; ++sg)
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[sg][e] &= keep[sg][e];
+          for (int e = 0; e < 4; ++e) {
+            const int key = k0 + 32 * sg + 8 * g + 2 * e;
+            v[sg][e] &= (key <= pmax && key >= lo_first ? 0xffffu : 0u) | (key + 1 <= pmax && key + 1 >= lo_first ? 0xffff0000u : 0u);
+          }
       }
 #pragma unroll
       for (int c = 0; c < QT; ++c) {
-        if (c < qt_live) {                                   // (scalar)
+        {
           f32x4 pv = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int sg = 0; sg < 4; ++sg) pv = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(v[sg]), as_bf16x8(pf[sg][c]), pv, 0, 0, 0);
@@ -780,21 +794,24 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
           } else {
 #pragma unroll
             for (int i = 0; i < 4; ++i) acc[j][c][i] = fmaf(pv[i], c2[c], acc[j][c][i] * c1[c]);
+            // (the fold happens here: put off to the end of the piece, every block's sums would be held twice)
+            asm volatile("" : "+v"(acc[j][c]));
           }
         }
       }
+      __builtin_amdgcn_sched_barrier(0);
     }
     if constexpr (PIECES) {
       if (qpos[0] < 0) return;
       const size_t at = ((size_t)t * a.heads + h0 + n % a.hg) * a.max_pieces + blockIdx.z;
       if (wv == 0 && g == 0) {
         a.partial_ml[2 * at] = mp[0];
-        a.partial_ml[2 * at + 1] = ((red_sum[0][n] + red_sum[1][n]) + red_sum[2][n]) + red_sum[3][n];
+        a.partial_ml[2 * at + 1] = lp;
       }
       float* part = a.partial + at * dv;
 #pragma unroll
       for (int j = 0; j < NDT; ++j) {
-        const int d = 16 * (4 * j + wv) + 4 * g;
+        const int d = 16 * (NW * j + wv) + 4 * g;
         if ((dv & 3) == 0) {
           if (d < dv) *reinterpret_cast<f32x4*>(part + d) = acc[j][0];
         } else {
@@ -815,7 +832,7 @@ __global__ __launch_bounds__(256) void shared_key_attention_mfma_kernel(MfmaAttn
       const size_t at = (size_t)(r0 + rl) * a.ldo + h * dv;
 #pragma unroll
       for (int j = 0; j < NDT; ++j) {
-        const int d = 16 * (4 * j + wv) + 4 * g;
+        const int d = 16 * (NW * j + wv) + 4 * g;
         if (a.out_is_bf16 && (dv & 3) == 0 && (a.ldo & 3) == 0) {
           if (d < dv)
             *reinterpret_cast<u32x2*>(reinterpret_cast<bf16_t*>(a.out) + at + d) =
@@ -867,30 +884,31 @@ __global__ __launch_bounds__(256) void shared_key_combine_kernel(MfmaAttnArgs a)
   store_out(a, (size_t)r0 * a.ldo + h * a.dv + d, o * finish_softmax(m, l, a.sink != nullptr ? a.sink[h] : -INFINITY));
 }
 
-template <int QT, int NDT>
+template <int QT, int NW, int NDT>
 int launch_shared_key_mfma_shape(const MfmaAttnArgs& a, const bf16_t* kc, const bf16_t* vt, int num_tiles, hipStream_t s) {
   const int dkp = (a.dk + 31) & ~31;
   const size_t bytes = (size_t)16 * QT * (dkp + 8 + SK_PSTRIDE) * sizeof(bf16_t);
   static bool allowed = false;
   if (!allowed) {
-    if (hipFuncSetAttribute((const void*)shared_key_attention_mfma_kernel<QT, NDT>, hipFuncAttributeMaxDynamicSharedMemorySize,
+    if (hipFuncSetAttribute((const void*)shared_key_attention_mfma_kernel<QT, NW, NDT>, hipFuncAttributeMaxDynamicSharedMemorySize,
                             150 * 1024) != hipSuccess)
       return -8;
     allowed = true;
   }
   if (bytes > 150 * 1024) return -8;
   const dim3 grid(num_tiles, (a.heads + a.hg - 1) / a.hg, QT == 1 ? a.max_pieces : 1);
-  hipLaunchKernelGGL((shared_key_attention_mfma_kernel<QT, NDT>), grid, dim3(256), bytes, s, a, kc, vt);
+  hipLaunchKernelGGL((shared_key_attention_mfma_kernel<QT, NW, NDT>), grid, dim3(64 * NW), bytes, s, a, kc, vt);
   return BW_LAUNCH_CHECK();
 }
 
 template <int QT>
 int launch_shared_key_mfma(const MfmaAttnArgs& a, const bf16_t* kc, const bf16_t* vt, int num_tiles, hipStream_t s) {
-  const int per_wave = (a.dv + 63) / 64;     // blocks of 16 value elements a wave
-  if (per_wave <= 1) return launch_shared_key_mfma_shape<QT, 1>(a, kc, vt, num_tiles, s);
-  if (per_wave <= 2) return launch_shared_key_mfma_shape<QT, 2>(a, kc, vt, num_tiles, s);
-  if (per_wave <= 4) return launch_shared_key_mfma_shape<QT, 4>(a, kc, vt, num_tiles, s);
-  if (per_wave <= 8) return launch_shared_key_mfma_shape<QT, 8>(a, kc, vt, num_tiles, s);
+  constexpr int NW = 4;
+  const int per_wave = (a.dv + 16 * NW - 1) / (16 * NW);     // blocks of 16 value elements a wave
+  if (per_wave <= 1) return launch_shared_key_mfma_shape<QT, NW, 1>(a, kc, vt, num_tiles, s);
+  if (per_wave <= 2) return launch_shared_key_mfma_shape<QT, NW, 2>(a, kc, vt, num_tiles, s);
+  if (per_wave <= 4) return launch_shared_key_mfma_shape<QT, NW, 4>(a, kc, vt, num_tiles, s);
+  if (per_wave <= 8) return launch_shared_key_mfma_shape<QT, NW, 8>(a, kc, vt, num_tiles, s);
   return -4;
 }
 
@@ -971,7 +989,8 @@ extern "C" int bw_headwise_linear_mfma(const void* x, int x_is_bf16, int ldx, in
                                   (rotary > 0 && (cos_table == nullptr || sin_table == nullptr)))))
     return -2;
   const uintptr_t mask = out_is_bf16 ? 7 : 15;
-  const int aligned = outn % 4 == 0 && ldo % 4 == 0 && ohs % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & mask) == 0;
+  int aligned = outn % 4 == 0 && ldo % 4 == 0 && ohs % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & mask) == 0;
+  if (aligned && outn % 8 == 0 && ldo % 8 == 0 && ohs % 8 == 0 && (reinterpret_cast<uintptr_t>(out) & 15) == 0) aligned = 2;
   const HeadGemmArgs a{x, ldx, xhs, (const bf16_t*)w, in, outn, out, ldo, ohs, rows, aligned};
   const HeadExtras ex{gate, ldg, rot_n, rotary, pairs, rot_src, rot_dst, cos_table, sin_table, positions};
   hipStream_t s = (hipStream_t)stream;
@@ -981,8 +1000,8 @@ extern "C" int bw_headwise_linear_mfma(const void* x, int x_is_bf16, int ldx, in
 
 extern "C" int bw_shared_key_piece() { return SK_PIECE; }
 
-// The matrix-core route: bfloat16 cache with key vectors of a multiple of 8 elements, pages of a multiple of 4 slots, and the
-// transposed latents beside it.  Prompt tiles (max_pieces 0): up to 64 / heads_per_group rows.  Single tokens (max_pieces > 0:
+// The matrix-core route: bfloat16 cache with key vectors of a multiple of 8 elements, pages of 8 slots or a larger power of two, and the
+// transposed latents beside it.  Prompt tiles (max_pieces 0): up to SK_TILE_QUERIES / heads_per_group rows.  Single tokens (max_pieces > 0:
 // tiles of one row, 16 heads a group): ``partial`` holds tiles * heads * max_pieces * (dv + 2) floats, max_pieces covers the
 // pieces of SK_PIECE keys that a token's window, or its whole context, can touch.
 extern "C" int bw_shared_key_attention_mfma(const void* q, int ldq, const int32_t* positions, const int32_t* block_table,
@@ -992,7 +1011,7 @@ extern "C" int bw_shared_key_attention_mfma(const void* q, int ldq, const int32_
                                             int heads_per_group, int max_pieces, float* partial, long long partial_floats,
                                             void* stream) {
   if (num_tiles <= 0) return 0;
-  if (heads <= 0 || dk <= 0 || (dk % 8) || dv <= 0 || dv > dk || dv > 512 || page_size < 4 || (page_size & (page_size - 1)) || num_pages <= 0) return -2;
+  if (heads <= 0 || dk <= 0 || (dk % 8) || dv <= 0 || dv > dk || dv > 512 || page_size < 8 || (page_size & (page_size - 1)) || num_pages <= 0) return -2;
   if (heads_per_group < 1 || heads_per_group > 16 || (16 % heads_per_group)) return -2;
   if (ldq < heads * dk || (ldq % 8) || ldo < heads * dv || max_pieces < 0 || max_pieces > 65535) return -2;
   if (reinterpret_cast<uintptr_t>(q) & 15) return -3;
@@ -1010,7 +1029,7 @@ extern "C" int bw_shared_key_attention_mfma(const void* q, int ldq, const int32_
                  partial == nullptr ? nullptr : partial + pieces * dv, heads, dk, dv, page_size, window, heads_per_group, num_pages,
                  max_pieces, scale};
   hipStream_t s = (hipStream_t)stream;
-  if (max_pieces == 0) return launch_shared_key_mfma<4>(a, (const bf16_t*)cache, (const bf16_t*)latent_t, num_tiles, s);
+  if (max_pieces == 0) return launch_shared_key_mfma<SK_TILE_QUERIES / 16>(a, (const bf16_t*)cache, (const bf16_t*)latent_t, num_tiles, s);
   const int rc = launch_shared_key_mfma<1>(a, (const bf16_t*)cache, (const bf16_t*)latent_t, num_tiles, s);
   if (rc != 0) return rc;
   hipLaunchKernelGGL(shared_key_combine_kernel, dim3(num_tiles, heads, (dv + 255) / 256), dim3(256), 0, s, a);

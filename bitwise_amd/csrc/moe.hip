@@ -171,6 +171,7 @@ __device__ __forceinline__ void plan_body(const int32_t* __restrict__ ids, int n
   const bool mine = g < segs;
   if (mine) {
     int c = 0;
+#pragma unroll 8
     for (int sidx = s0; sidx < s1; ++sidx) c += src[sidx] == e;
     seg_count[e * segs + g] = c;
   }
@@ -198,12 +199,19 @@ __device__ __forceinline__ void plan_body(const int32_t* __restrict__ ids, int n
   __syncthreads();
   if (mine) {
     int p = start[e] + seg_count[e * segs + g];
-    for (int sidx = s0; sidx < s1; ++sidx)
-      if (src[sidx] == e) {
-        sorted[p] = sidx;
-        place[sidx] = p;
-        ++p;
-      }
+    // (eight slots are read before the first is looked at)
+    for (int b = s0; b < s1; b += 8) {
+      int v[8];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[k] = src[min(b + k, s1 - 1)];
+#pragma unroll
+      for (int k = 0; k < 8; ++k)
+        if (b + k < s1 && v[k] == e) {
+          sorted[p] = b + k;
+          place[b + k] = p;
+          ++p;
+        }
+    }
   }
   for (int x = tid; x < E; x += 1024) {
     const int nt = (counts[x] + tm - 1) / tm;
@@ -253,13 +261,24 @@ __global__ __launch_bounds__(1024) void moe_table_plan_kernel(const int32_t* __r
     return t;
   };
   const int n = rows * top;
-  for (int sidx = threadIdx.x; sidx < n; sidx += 1024) {
-    const int r = sidx / top;
-    int t = token_of(r);
-    if (t < 0 || t >= vocab) t = token_of(0);
-    if (t < 0 || t >= vocab) t = 0;
-    ids[sidx] = min(max(table[(size_t)t * top + sidx % top], 0), E - 1);
-    wts[sidx] = weight;
+  int spare = token_of(0);
+  if (spare < 0 || spare >= vocab) spare = 0;
+  for (int b = threadIdx.x; b < n; b += 8 * 1024) {
+    // (eight slots' tokens, then their entries, are asked for together)
+    int t[8], e[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      t[k] = token_of(min(b + 1024 * k, n - 1) / top);
+      if (t[k] < 0 || t[k] >= vocab) t[k] = spare;
+    }
+#pragma unroll
+    for (int k = 0; k < 8; ++k) e[k] = table[(size_t)t[k] * top + min(b + 1024 * k, n - 1) % top];
+#pragma unroll
+    for (int k = 0; k < 8; ++k)
+      if (b + 1024 * k < n) {
+        ids[b + 1024 * k] = min(max(e[k], 0), E - 1);
+        wts[b + 1024 * k] = weight;
+      }
   }
   __syncthreads();                      // (written to memory by the workgroup's own threads, visible to all of them)
   plan_body(ids, n, E, segs, tm, staged, table_lds, sorted, place, tiles, meta);

@@ -1215,7 +1215,10 @@ def shared_key_attention(q: torch.Tensor, positions: torch.Tensor, block_table: 
 
 def shared_key_mfma_ok(cache_dtype: torch.dtype, dk: int, dv: int, page_size: int) -> bool:
     """Whether the matrix-core route of the attention over shared keys takes this cache."""
-    return cache_dtype == torch.bfloat16 and dk % 8 == 0 and 0 < dv <= min(dk, 512) and page_size >= 4 and page_size % 4 == 0
+    return cache_dtype == torch.bfloat16 and dk % 8 == 0 and 0 < dv <= min(dk, 512) and page_size >= 8 and page_size & (page_size - 1) == 0
+
+
+SHARED_KEY_TILE_QUERIES = 32      # query vectors (rows x heads of a group) of a prompt tile on the matrix cores
 
 
 def shared_key_pieces(context: int, window: int) -> int:
@@ -1231,7 +1234,7 @@ def shared_key_attention_mfma(q: torch.Tensor, positions: torch.Tensor, block_ta
                               heads_per_group: int, max_pieces: int = 0, partial: Optional[torch.Tensor] = None) -> None:
     """``shared_key_attention`` on the matrix cores for a bfloat16 cache (``shared_key_mfma_ok``): queries and softmax
     weights are rounded to bfloat16 where they enter a product (``q`` arrives as bfloat16), sums are 32-bit.  ``latent_t`` [pages, dv * page_size]: the
-    values transposed within their pages.  ``out`` float32 or bfloat16.  Tiles hold up to 64 / heads_per_group rows.
+    values transposed within their pages.  ``out`` float32 or bfloat16.  Tiles hold up to SHARED_KEY_TILE_QUERIES / heads_per_group rows.
     max_pieces > 0 (tiles of one row, heads_per_group 16): a workgroup for each of the ``shared_key_pieces`` runs of keys a
     token can see, and ``partial`` (float32, at least tiles * heads * max_pieces * (dv + 2)) holds what they leave for a
     second kernel that folds them; the bits of a row are those it gets in a tile."""

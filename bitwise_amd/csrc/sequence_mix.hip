@@ -328,12 +328,18 @@ struct RecurArgs {
 // floats of a chunk's record for one head: S, a vector, two scalars, in whole vectors of four
 __host__ __device__ __forceinline__ size_t recur_record(int dim, int vdim) { return ((size_t)dim * vdim + dim + 2 + 3) & ~(size_t)3; }
 
+// Lanes a column.  A portion walked whole (and a single token) gets many short waves; the passes over chunks have waves
+// enough and keep more of a column in a lane, which reads less through LDS for every multiply-add.
 __host__ __device__ constexpr int recur_split(int dpad) { return dpad >= 128 ? 16 : dpad / 8; }
+__host__ __device__ constexpr int recur_chunk_split(int dpad) { return dpad >= 64 ? 4 : (dpad >= 32 ? 2 : 1); }
 // value columns of a workgroup, and how many workgroups share a head
-__host__ __device__ constexpr int recur_columns(int dim) {
-  return RW * 64 / recur_split(dim <= 16 ? 16 : (dim <= 32 ? 32 : (dim <= 64 ? 64 : 128)));
+__host__ __device__ constexpr int recur_columns(int dim, bool chunks) {
+  const int dpad = dim <= 16 ? 16 : (dim <= 32 ? 32 : (dim <= 64 ? 64 : 128));
+  return RW * 64 / (chunks ? recur_chunk_split(dpad) : recur_split(dpad));
 }
-__host__ __device__ constexpr int recur_blocks(int dim, int vdim) { return (vdim + recur_columns(dim) - 1) / recur_columns(dim); }
+__host__ __device__ constexpr int recur_blocks(int dim, int vdim, bool chunks = false) {
+  return (vdim + recur_columns(dim, chunks) - 1) / recur_columns(dim, chunks);
+}
 
 template <int MODE, int DPAD, int PHASE>
 __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a) {
@@ -342,8 +348,9 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   constexpr bool CHANNELS = !GATES && !STEP;             // a decay per channel comes through LDS
   constexpr int NN = (DPAD + 63) / 64;
   constexpr bool READ_OUT = PHASE != 1;
-  constexpr int SPLIT = recur_split(DPAD), DH = DPAD / SPLIT, COLS = 64 / SPLIT, WCOLS = RW * COLS;
-  constexpr int TU = SPLIT >= 4 ? 4 : 2;                 // tokens worked on together
+  constexpr int SPLIT = PHASE == 0 ? recur_split(DPAD) : recur_chunk_split(DPAD);
+  constexpr int DH = DPAD / SPLIT, COLS = 64 / SPLIT, WCOLS = RW * COLS;
+  constexpr int TU = PHASE != 0 ? 1 : (SPLIT >= 4 ? 4 : 2);      // tokens worked on together
   constexpr int NQ = RC * DPAD / (64 * RW), NV = (RC * WCOLS + 64 * RW - 1) / (64 * RW);
   static_assert(NQ * 64 * RW == RC * DPAD && RC % TU == 0, "a chunk is whole loads and whole groups of tokens");
   __shared__ __attribute__((aligned(16))) float qs[2][RC][DPAD];
@@ -379,8 +386,9 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   // (every workgroup of a head carries the normaliser and the maximum, so each keeps a copy of its own in the slot: one that
   // starts late must not find what another has already written)
   const size_t copy = (size_t)a.heads * dim + a.heads;
-  float* nv = st + (size_t)a.heads * dim * vdim + (GATES ? blockIdx.x * copy : 0) + (size_t)h * dim;
-  float* mv = st + (size_t)a.heads * dim * vdim + (GATES ? blockIdx.x * copy : 0) + (size_t)a.heads * dim + h;
+  const size_t own = GATES && PHASE == 0 ? blockIdx.x * copy : 0;
+  float* nv = st + (size_t)a.heads * dim * vdim + own + (size_t)h * dim;
+  float* mv = st + (size_t)a.heads * dim * vdim + own + (size_t)a.heads * dim + h;
   // where this wave's state comes from: the slot, nothing, or the chunk's start record
   const float* S_in = S;
   const float* nv_in = nv;
@@ -628,13 +636,17 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         if (dbase + d < dim) S_out[(size_t)j * dim + dbase + d] = Sreg[d];
     }
   }
-  if (wv == 0 && (PHASE == 1 ? blockIdx.x == 0 : GATES)) {
+  if (wv == 0 && (PHASE == 0 ? GATES : blockIdx.x == 0 && (GATES || PHASE == 1))) {
+    // (the last of the passes leaves every workgroup's copy)
+    const int copies = PHASE == 3 ? recur_blocks(dim, vdim) : 1;
+    for (int k = 0; k < copies; ++k) {
 #pragma unroll
-    for (int i = 0; i < NN; ++i)
-      if (lane + 64 * i < dim) nv_out[lane + 64 * i] = nreg[i];
-    if (GATES && lane == 0) {
-      mv_out[0] = m;
-      if (PHASE == 1) mv_out[1] = fsum;
+      for (int i = 0; i < NN; ++i)
+        if (lane + 64 * i < dim) nv_out[k * copy + lane + 64 * i] = nreg[i];
+      if (GATES && lane == 0) {
+        mv_out[k * copy] = m;
+        if (PHASE == 1) mv_out[1] = fsum;
+      }
     }
   }
 }
@@ -681,7 +693,7 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurArgs a, const
 
 template <int MODE, int PHASE>
 int launch_recurrence(const RecurArgs& a, int units, hipStream_t s) {
-  const dim3 grid(recur_blocks(a.dim, a.vdim), a.heads, units), block(64 * RW);
+  const dim3 grid(recur_blocks(a.dim, a.vdim, PHASE != 0), a.heads, units), block(64 * RW);
   if (a.dim <= 16) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 16, PHASE>), grid, block, 0, s, a);
   else if (a.dim <= 32) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 32, PHASE>), grid, block, 0, s, a);
   else if (a.dim <= 64) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 64, PHASE>), grid, block, 0, s, a);

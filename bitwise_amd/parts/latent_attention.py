@@ -24,7 +24,6 @@ from .base import CacheSpec, Mixer, TensorSpec, lookup, register_mixer, POSITION
 from .linear import Linear
 
 ROWS_PER_PROMPT_TILE = 4        # the 32-bit kernel: 16 query vectors a workgroup, 4 rows x 4 heads or a single token's 16 heads
-QUERIES_PER_TILE = 64           # the matrix-core kernel: query vectors (rows x heads of a group) a workgroup in prompt portions
 
 
 def _tiles(ctx, rows_per_tile: int):
@@ -89,7 +88,7 @@ class LatentAttention(Mixer):
         self.sink: Optional[torch.Tensor] = None
         self.q_norm: Optional[torch.Tensor] = None
         # bfloat16 mode: the attention runs on the matrix cores and keeps the latents a second time, transposed within
-        # their pages, as the values (the page sizes it takes: multiples of 4); the 32-bit mode reads values and keys
+        # their pages, as the values (the page sizes it takes: powers of two from 8 on); the 32-bit mode reads values and keys
         # from the one copy
         self.on_matrix_cores = bool(runtime.bf16) and self.key_width % 8 == 0
         # heads that share a wave's 16 query vectors in prompt portions: the power of two from the number of heads up
@@ -155,7 +154,7 @@ class LatentAttention(Mixer):
                          value_width=self.rank if self.on_matrix_cores else 0)
 
     def page_sizes(self):
-        return (4, 8, 16, 32, 64, 128) if self.on_matrix_cores else None
+        return (8, 16, 32, 64, 128) if self.on_matrix_cores else None
 
     def _project(self, ctx, h) -> torch.Tensor:
         y = ctx.ws.buffer("latent_proj", self.proj.out_features, torch.float32)
@@ -223,7 +222,7 @@ class LatentAttention(Mixer):
     def _attend_on_matrix_cores(self, ctx, call, qa, lat, table) -> None:
         ws = ctx.ws
         hg = self.heads_per_group
-        many, n_many, single, n_single = _tiles(ctx, QUERIES_PER_TILE // hg)
+        many, n_many, single, n_single = _tiles(ctx, ops.SHARED_KEY_TILE_QUERIES // hg)
         window = int(self.window or 0)
         common = (call.k_cache, call.v_cache, self.sink, lat, self.heads, self.key_width, self.rank, ws.page_size, window, self.scale)
         if n_many:
