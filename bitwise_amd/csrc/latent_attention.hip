@@ -209,17 +209,23 @@ struct HeadGemmArgs {
   int in, outn;
   void* out;
   int ldo, ohs, rows;
+  int heads, oz;           // oz: blocks of 64 outputs (and one more for the rotated part)
   int aligned;             // 1: rows and heads of out start at whole groups of four elements, outn is a multiple of 4; 2: of eight
 };
 
 template <typename XT, typename OT, int OB, bool ROW_WAVES>
 __global__ __launch_bounds__(256) void headwise_mfma_kernel(HeadGemmArgs a, HeadExtras ex) {
   const int lane = threadIdx.x & 63, n = lane & 15, g = lane >> 4, wv = wave_index();
-  const int h = blockIdx.y;
+  // Workgroups are dealt to the eight dies in turn.  Of those of one die, the blocks of outputs of one (rows, head) follow each
+  // other: they read the same rows of x, from the die's own L2 after the first.
+  const int die = blockIdx.x & 7, nth = blockIdx.x >> 3;
+  const int zb = nth % a.oz, unit = (nth / a.oz) * 8 + die;
+  const int h = unit % a.heads, row_block = unit / a.heads;
+  const int r_wg = row_block * (ROW_WAVES ? 64 : 16);
+  if (r_wg >= a.rows) return;
   const XT* xh = reinterpret_cast<const XT*>(a.x) + (size_t)h * a.xhs;
   OT* oh = reinterpret_cast<OT*>(a.out) + (size_t)h * a.ohs;
-  const int r_wg = blockIdx.x * (ROW_WAVES ? 64 : 16);
-  if ((int)blockIdx.z * 64 >= a.outn) {      // the extra block: the rotated part beside the product
+  if (zb * 64 >= a.outn) {      // the extra block: the rotated part beside the product
     if constexpr (sizeof(XT) == 4) {
       const int half = ex.rotary / 2;
       for (int e = threadIdx.x; e < (ROW_WAVES ? 64 : 16) * ex.rot_n; e += 256) {
@@ -234,7 +240,7 @@ __global__ __launch_bounds__(256) void headwise_mfma_kernel(HeadGemmArgs a, Head
     return;
   }
   const int r0 = r_wg + (ROW_WAVES ? 16 * wv : 0);
-  const int o0 = blockIdx.z * 64 + (ROW_WAVES ? 0 : 16 * wv);
+  const int o0 = zb * 64 + (ROW_WAVES ? 0 : 16 * wv);
   if (r0 >= a.rows || o0 >= a.outn) return;
   const XT* xr = xh + (size_t)min(r0 + n, a.rows - 1) * a.ldx;
   // block b's row k of the product is output o0 + 4 OB (k / 4) + 4 b + k % 4: a lane's results are 4 OB neighbours
@@ -302,12 +308,13 @@ __global__ __launch_bounds__(256) void headwise_mfma_kernel(HeadGemmArgs a, Head
 }
 
 template <typename XT, typename OT>
-int launch_headwise_mfma(const HeadGemmArgs& a, const HeadExtras& ex, int heads, hipStream_t s) {
-  const int oz = (a.outn + 63) / 64 + (ex.rot_n > 0 ? 1 : 0);
+int launch_headwise_mfma(const HeadGemmArgs& a, const HeadExtras& ex, hipStream_t s) {
+  const int row_blocks = a.rows > 64 ? (a.rows + 63) / 64 : (a.rows + 15) / 16;
+  const dim3 grid((unsigned)((row_blocks * a.heads + 7) / 8 * 8 * a.oz));
   if (a.rows > 64)
-    hipLaunchKernelGGL((headwise_mfma_kernel<XT, OT, 4, true>), dim3((a.rows + 63) / 64, heads, oz), dim3(256), 0, s, a, ex);
+    hipLaunchKernelGGL((headwise_mfma_kernel<XT, OT, 4, true>), grid, dim3(256), 0, s, a, ex);
   else
-    hipLaunchKernelGGL((headwise_mfma_kernel<XT, OT, 1, false>), dim3((a.rows + 15) / 16, heads, oz), dim3(256), 0, s, a, ex);
+    hipLaunchKernelGGL((headwise_mfma_kernel<XT, OT, 1, false>), grid, dim3(256), 0, s, a, ex);
   return BW_LAUNCH_CHECK();
 }
 
@@ -981,7 +988,7 @@ extern "C" int bw_headwise_linear_mfma(const void* x, int x_is_bf16, int ldx, in
                                        int rotary, int pairs, int rot_src, int rot_dst, const float* cos_table, const float* sin_table,
                                        const int32_t* positions, void* stream) {
   if (rows <= 0 || heads <= 0 || outn <= 0) return 0;
-  if (in < 8 || in % 8 || heads > 65535 || (outn + 63) / 64 > 65534) return -2;
+  if (in < 8 || in % 8 || ((long long)rows / 16 + 1) * heads * ((outn + 63) / 64 + 1) > 0x3fffffffLL) return -2;
   const int unit = x_is_bf16 ? 8 : 4;
   if (ldx % unit || xhs % unit || (reinterpret_cast<uintptr_t>(x) & 15) || (reinterpret_cast<uintptr_t>(w) & 15)) return -3;
   if (gate != nullptr && ldg < heads) return -2;
@@ -991,11 +998,11 @@ extern "C" int bw_headwise_linear_mfma(const void* x, int x_is_bf16, int ldx, in
   const uintptr_t mask = out_is_bf16 ? 7 : 15;
   int aligned = outn % 4 == 0 && ldo % 4 == 0 && ohs % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & mask) == 0;
   if (aligned && outn % 8 == 0 && ldo % 8 == 0 && ohs % 8 == 0 && (reinterpret_cast<uintptr_t>(out) & 15) == 0) aligned = 2;
-  const HeadGemmArgs a{x, ldx, xhs, (const bf16_t*)w, in, outn, out, ldo, ohs, rows, aligned};
+  const HeadGemmArgs a{x, ldx, xhs, (const bf16_t*)w, in, outn, out, ldo, ohs, rows, heads, (outn + 63) / 64 + (rot_n > 0 ? 1 : 0), aligned};
   const HeadExtras ex{gate, ldg, rot_n, rotary, pairs, rot_src, rot_dst, cos_table, sin_table, positions};
   hipStream_t s = (hipStream_t)stream;
-  if (x_is_bf16) return out_is_bf16 ? launch_headwise_mfma<bf16_t, bf16_t>(a, ex, heads, s) : launch_headwise_mfma<bf16_t, float>(a, ex, heads, s);
-  return out_is_bf16 ? launch_headwise_mfma<float, bf16_t>(a, ex, heads, s) : launch_headwise_mfma<float, float>(a, ex, heads, s);
+  if (x_is_bf16) return out_is_bf16 ? launch_headwise_mfma<bf16_t, bf16_t>(a, ex, s) : launch_headwise_mfma<bf16_t, float>(a, ex, s);
+  return out_is_bf16 ? launch_headwise_mfma<float, bf16_t>(a, ex, s) : launch_headwise_mfma<float, float>(a, ex, s);
 }
 
 extern "C" int bw_shared_key_piece() { return SK_PIECE; }

@@ -150,68 +150,98 @@ extern "C" int bw_moe_route(const float* logits, int ld, int rows, int experts, 
 // ------------------------------------------------------------------------------ plan
 
 // One workgroup of 1024 threads.  sorted[p] = slot at sorted place p; place[slot] = p; tiles[t] = (expert, first place,
-// slots, 0) with up to tm slots a tile; meta[0] = number of tiles.  Thread (segment g, expert e) walks segment g of the
-// slots (from LDS, where the workgroup has put them if they fit) and counts those of expert e; after a prefix over
-// segments and experts it walks the segment again and hands out places.  Within an expert's run the slots ascend, so
-// the plan is the same from run to run.
-__device__ __forceinline__ void plan_body(const int32_t* __restrict__ ids, int n, int E, int segs, int tm, int staged, int* plan_ids,
-                                          int32_t* __restrict__ sorted, int32_t* __restrict__ place, int32_t* __restrict__ tiles,
-                                          int32_t* __restrict__ meta) {
-  __shared__ int seg_count[1024];       // [expert][segment]; after the prefix: slots of the expert in earlier segments
-  __shared__ int counts[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS], tile0[MOE_MAX_EXPERTS];
-  const int tid = threadIdx.x;
-  if (staged) {
-    for (int sidx = tid; sidx < n; sidx += 1024) plan_ids[sidx] = ids[sidx];
-    __syncthreads();
+// slots, 0) with up to tm slots a tile; meta[0] = number of tiles.  The slots are cut into one run per wave, and a wave walks its
+// run 64 slots at a time, a lane a slot: the lanes of one expert find each other by ballots over the expert number's bits, so a
+// lane knows its rank among them.  The first walk counts (hist [waves][E], in LDS), then a prefix over waves and experts gives
+// every (wave, expert) its first place, and the second walk hands out places.  Within an expert's run the slots ascend, so the
+// plan is the same from run to run.
+#define PLAN_WAVES 16
+
+// Very many experts: the counts take more dynamic LDS than a launch may ask for without saying so beforehand.
+static int plan_allow_lds(const void* kernel, size_t bytes) {
+  if (bytes <= 48 * 1024) return 0;
+  return hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes) == hipSuccess ? 0 : -8;
+}
+
+// Sum over lower lanes of the wave (exclusive) and over all of it.
+__device__ __forceinline__ int wave_prefix(int v, int lane, int& total) {
+  int x = v;
+#pragma unroll
+  for (int off = 1; off < 64; off <<= 1) {
+    const int y = __shfl_up(x, off, 64);
+    if (lane >= off) x += y;
   }
-  const int* src = staged ? plan_ids : ids;
-  const int e = tid % E, g = tid / E;
-  const int seg_len = (n + segs - 1) / segs;
-  const int s0 = g * seg_len, s1 = min(n, s0 + seg_len);
-  const bool mine = g < segs;
-  if (mine) {
-    int c = 0;
-#pragma unroll 8
-    for (int sidx = s0; sidx < s1; ++sidx) c += src[sidx] == e;
-    seg_count[e * segs + g] = c;
+  total = __shfl(x, 63, 64);
+  return x - v;
+}
+
+__device__ __forceinline__ void plan_body(const int32_t* __restrict__ ids, int n, int E, int tm, int* hist, int32_t* __restrict__ sorted,
+                                          int32_t* __restrict__ place, int32_t* __restrict__ tiles, int32_t* __restrict__ meta) {
+  __shared__ int counts[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS], tile0[MOE_MAX_EXPERTS];
+  const int tid = threadIdx.x, lane = tid & 63, wave = wave_index();
+  for (int k = tid; k < PLAN_WAVES * E; k += 1024) hist[k] = 0;
+  __syncthreads();
+  const int run = ((n + PLAN_WAVES - 1) / PLAN_WAVES + 63) & ~63;
+  const int s0 = wave * run, s1 = min(n, s0 + run);
+  int* mine = hist + wave * E;
+  int bits = 0;
+  while ((1 << bits) < E) ++bits;
+  // the lanes that hold a slot of this lane's expert
+  auto peers = [&](int e, bool live) -> unsigned long long {
+    unsigned long long m = __ballot(live);
+    for (int b = 0; b < bits; ++b) {
+      const unsigned long long one = __ballot(live && ((e >> b) & 1));
+      m &= ((e >> b) & 1) ? one : ~one;
+    }
+    return m;
+  };
+  const unsigned long long below = (1ull << lane) - 1ull;
+  for (int b = s0; b < s1; b += 64) {
+    const bool live = b + lane < s1;
+    const int e = live ? ids[b + lane] : 0;
+    const unsigned long long m = peers(e, live);
+    if (live && (m & below) == 0) mine[e] += __popcll(m);
+    __builtin_amdgcn_wave_barrier();
   }
   __syncthreads();
-  if (tid < E) {
+  for (int e = tid; e < E; e += 1024) {
     int c = 0;
-    for (int k = 0; k < segs; ++k) {
-      const int v = seg_count[tid * segs + k];
-      seg_count[tid * segs + k] = c;
+    for (int k = 0; k < PLAN_WAVES; ++k) {
+      const int v = hist[k * E + e];
+      hist[k * E + e] = c;
       c += v;
     }
-    counts[tid] = c;
+    counts[e] = c;
   }
   __syncthreads();
-  if (tid == 0) {
+  if (wave == 0) {
     int p = 0, t = 0;
-    for (int x = 0; x < E; ++x) {
-      start[x] = p;
-      tile0[x] = t;
-      p += counts[x];
-      t += (counts[x] + tm - 1) / tm;
+    for (int b = 0; b < E; b += 64) {
+      const int c = b + lane < E ? counts[b + lane] : 0;
+      int pt, tt;
+      const int pp = wave_prefix(c, lane, pt), tp = wave_prefix((c + tm - 1) / tm, lane, tt);
+      if (b + lane < E) {
+        start[b + lane] = p + pp;
+        tile0[b + lane] = t + tp;
+      }
+      p += pt;
+      t += tt;
     }
-    meta[0] = t;
+    if (lane == 0) meta[0] = t;
   }
   __syncthreads();
-  if (mine) {
-    int p = start[e] + seg_count[e * segs + g];
-    // (eight slots are read before the first is looked at)
-    for (int b = s0; b < s1; b += 8) {
-      int v[8];
-#pragma unroll
-      for (int k = 0; k < 8; ++k) v[k] = src[min(b + k, s1 - 1)];
-#pragma unroll
-      for (int k = 0; k < 8; ++k)
-        if (b + k < s1 && v[k] == e) {
-          sorted[p] = b + k;
-          place[b + k] = p;
-          ++p;
-        }
+  for (int b = s0; b < s1; b += 64) {
+    const bool live = b + lane < s1;
+    const int e = live ? ids[b + lane] : 0;
+    const unsigned long long m = peers(e, live);
+    if (live) {
+      const int p = start[e] + mine[e] + __popcll(m & below);
+      sorted[p] = b + lane;
+      place[b + lane] = p;
     }
+    __builtin_amdgcn_wave_barrier();
+    if (live && (m & below) == 0) mine[e] += __popcll(m);
+    __builtin_amdgcn_wave_barrier();
   }
   for (int x = tid; x < E; x += 1024) {
     const int nt = (counts[x] + tm - 1) / tm;
@@ -225,23 +255,22 @@ __device__ __forceinline__ void plan_body(const int32_t* __restrict__ ids, int n
   }
 }
 
-__global__ __launch_bounds__(1024) void moe_plan_kernel(const int32_t* __restrict__ ids, int n, int E, int segs, int tm, int staged,
-                                                        int32_t* __restrict__ sorted, int32_t* __restrict__ place,
-                                                        int32_t* __restrict__ tiles, int32_t* __restrict__ meta) {
-  extern __shared__ int plan_lds[];     // [n] if staged
-  plan_body(ids, n, E, segs, tm, staged, plan_lds, sorted, place, tiles, meta);
+__global__ __launch_bounds__(1024) void moe_plan_kernel(const int32_t* __restrict__ ids, int n, int E, int tm, int32_t* __restrict__ sorted,
+                                                        int32_t* __restrict__ place, int32_t* __restrict__ tiles, int32_t* __restrict__ meta) {
+  extern __shared__ int plan_lds[];     // [PLAN_WAVES][E]
+  plan_body(ids, n, E, tm, plan_lds, sorted, place, tiles, meta);
 }
 
 // Steps of up to 16 rows: route (a wave a row) and plan in one launch of one workgroup.
 __global__ __launch_bounds__(1024) void moe_route_plan_kernel(const float* __restrict__ logits, int ld, int rows, int E, int top, int count,
-                                                              int keep, float weight_scale, RouteRule rule, int32_t* __restrict__ ids, float* __restrict__ wts, int segs,
+                                                              int keep, float weight_scale, RouteRule rule, int32_t* __restrict__ ids, float* __restrict__ wts,
                                                               int tm, int32_t* __restrict__ sorted, int32_t* __restrict__ place,
                                                               int32_t* __restrict__ tiles, int32_t* __restrict__ meta) {
-  extern __shared__ float both_lds[];   // the waves' routing tables, then the plan's slots
+  extern __shared__ float both_lds[];   // the waves' routing tables, then the plan's counts in their place
   const int wave = wave_index(), lane = threadIdx.x & 63;
   if (wave < rows) route_row(logits, ld, wave, E, top, count, keep, weight_scale, rule, ids, wts, both_lds + (size_t)wave * (2 * E + 2 * count), lane);
   __syncthreads();                      // (the rows' choices, written to memory by their waves, are visible to the workgroup)
-  plan_body(ids, rows * top, E, segs, tm, 1, reinterpret_cast<int*>(both_lds + (size_t)rows * (2 * E + 2 * count)), sorted, place, tiles, meta);
+  plan_body(ids, rows * top, E, tm, reinterpret_cast<int*>(both_lds), sorted, place, tiles, meta);
 }
 
 // Routing by a table instead of a router: row r's experts are table[token of r][..], its weights ``weight`` each.  A token of
@@ -250,11 +279,11 @@ __global__ __launch_bounds__(1024) void moe_route_plan_kernel(const float* __res
 // inside 0 .. experts - 1.  One workgroup; the choices go to ``ids`` and the plan is made from there.
 __global__ __launch_bounds__(1024) void moe_table_plan_kernel(const int32_t* __restrict__ tokens, const int32_t* __restrict__ feedback,
                                                               int rows, const int32_t* __restrict__ table, int vocab, int top, int E,
-                                                              float weight, int segs, int tm, int staged, int32_t* ids,
+                                                              float weight, int tm, int32_t* ids,
                                                               float* __restrict__ wts, int32_t* __restrict__ sorted,
                                                               int32_t* __restrict__ place, int32_t* __restrict__ tiles,
                                                               int32_t* __restrict__ meta) {
-  extern __shared__ int table_lds[];    // [rows * top] if staged
+  extern __shared__ int table_lds[];    // [PLAN_WAVES][E]
   auto token_of = [&](int r) {
     int t = tokens[r];
     if (t == -2 && feedback != nullptr) t = feedback[r];
@@ -281,7 +310,7 @@ __global__ __launch_bounds__(1024) void moe_table_plan_kernel(const int32_t* __r
       }
   }
   __syncthreads();                      // (written to memory by the workgroup's own threads, visible to all of them)
-  plan_body(ids, n, E, segs, tm, staged, table_lds, sorted, place, tiles, meta);
+  plan_body(ids, n, E, tm, table_lds, sorted, place, tiles, meta);
 }
 
 // Slots a tile: few slots a step (decoded tokens) get tiles of 16, whose kernel keeps many steps of weights in flight;
@@ -297,10 +326,10 @@ extern "C" int bw_moe_plan(const int32_t* ids, int slots, int experts, int32_t* 
                            int32_t* meta, void* stream) {
   if (slots <= 0) return 0;
   if (experts < 1 || experts > MOE_MAX_EXPERTS) return -2;
-  const int segs = 1024 / experts;
-  const int staged = slots <= 12 * 1024;
-  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), staged ? (size_t)slots * sizeof(int) : 0, (hipStream_t)stream, ids, slots,
-                     experts, segs, bw_moe_tile_rows(slots), staged, sorted, place, tiles, meta);
+  const int allowed = plan_allow_lds((const void*)moe_plan_kernel, (size_t)PLAN_WAVES * experts * sizeof(int));
+  if (allowed != 0) return allowed;
+  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), (size_t)PLAN_WAVES * experts * sizeof(int), (hipStream_t)stream, ids, slots,
+                     experts, bw_moe_tile_rows(slots), sorted, place, tiles, meta);
   return BW_LAUNCH_CHECK();
 }
 
@@ -309,10 +338,11 @@ extern "C" int bw_moe_table_plan(const int32_t* tokens, const int32_t* feedback,
                                  int32_t* meta, void* stream) {
   if (rows <= 0) return 0;
   if (experts < 1 || experts > MOE_MAX_EXPERTS || top < 1 || vocab < 1 || (long long)rows * top > 0x7fffffffLL) return -2;
-  const int slots = rows * top, staged = slots <= 12 * 1024;
-  hipLaunchKernelGGL(moe_table_plan_kernel, dim3(1), dim3(1024), staged ? (size_t)slots * sizeof(int) : 0, (hipStream_t)stream, tokens,
-                     feedback, rows, table, vocab, top, experts, weight, 1024 / experts, bw_moe_tile_rows(slots), staged, ids, wts, sorted,
-                     place, tiles, meta);
+  const int slots = rows * top;
+  const int allowed = plan_allow_lds((const void*)moe_table_plan_kernel, (size_t)PLAN_WAVES * experts * sizeof(int));
+  if (allowed != 0) return allowed;
+  hipLaunchKernelGGL(moe_table_plan_kernel, dim3(1), dim3(1024), (size_t)PLAN_WAVES * experts * sizeof(int), (hipStream_t)stream, tokens,
+                     feedback, rows, table, vocab, top, experts, weight, bw_moe_tile_rows(slots), ids, wts, sorted, place, tiles, meta);
   return BW_LAUNCH_CHECK();
 }
 
@@ -320,7 +350,7 @@ extern "C" int bw_moe_route_plan(const float* logits, int ld, int rows, int expe
                                  float weight_scale, int score_kind, const float* correction, int group_best, int32_t* ids, float* wts,
                                  int32_t* sorted, int32_t* place, int32_t* tiles, int32_t* meta, void* stream) {
   if (rows <= 0) return 0;
-  const size_t bytes = ((size_t)rows * (2 * experts + 2 * groups) + (size_t)rows * top) * sizeof(float);
+  size_t bytes = (size_t)rows * (2 * experts + 2 * groups) * sizeof(float);
   if (rows > 16 || bytes > 48 * 1024) {
     const int rc = bw_moe_route(logits, ld, rows, experts, top, groups, keep, weight_scale, score_kind, correction, group_best, ids, wts, stream);
     return rc != 0 ? rc : bw_moe_plan(ids, rows * top, experts, sorted, place, tiles, meta, stream);
@@ -328,8 +358,11 @@ extern "C" int bw_moe_route_plan(const float* logits, int ld, int rows, int expe
   if (experts < 1 || experts > MOE_MAX_EXPERTS || top < 1 || groups < 1 || experts % groups || keep < 1 || keep > groups ||
       top > keep * (experts / groups) || score_kind < 0 || score_kind > 1 || group_best < 1 || group_best > 4)
     return -2;
+  if (bytes < (size_t)PLAN_WAVES * experts * sizeof(int)) bytes = (size_t)PLAN_WAVES * experts * sizeof(int);
+  const int allowed = plan_allow_lds((const void*)moe_route_plan_kernel, bytes);
+  if (allowed != 0) return allowed;
   hipLaunchKernelGGL(moe_route_plan_kernel, dim3(1), dim3(1024), bytes, (hipStream_t)stream, logits, ld, rows, experts, top, groups, keep,
-                     weight_scale, RouteRule{score_kind, correction, group_best}, ids, wts, 1024 / experts, bw_moe_tile_rows(rows * top), sorted, place, tiles, meta);
+                     weight_scale, RouteRule{score_kind, correction, group_best}, ids, wts, bw_moe_tile_rows(rows * top), sorted, place, tiles, meta);
   return BW_LAUNCH_CHECK();
 }
 

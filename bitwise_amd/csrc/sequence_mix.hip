@@ -351,13 +351,14 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   constexpr int SPLIT = PHASE == 0 ? recur_split(DPAD) : recur_chunk_split(DPAD);
   constexpr int DH = DPAD / SPLIT, COLS = 64 / SPLIT, WCOLS = RW * COLS;
   constexpr int TU = PHASE != 0 ? 1 : (SPLIT >= 4 ? 4 : 2);      // tokens worked on together
+  constexpr int BUFS = PHASE != 0 ? 1 : 2;               // (the passes over chunks hide the loads behind other waves)
   constexpr int NQ = RC * DPAD / (64 * RW), NV = (RC * WCOLS + 64 * RW - 1) / (64 * RW);
   static_assert(NQ * 64 * RW == RC * DPAD && RC % TU == 0, "a chunk is whole loads and whole groups of tokens");
-  __shared__ __attribute__((aligned(16))) float qs[2][RC][DPAD];
-  __shared__ __attribute__((aligned(16))) float ks[2][RC][DPAD];
-  __shared__ __attribute__((aligned(16))) float as[CHANNELS ? 2 : 1][CHANNELS ? RC : 1][CHANNELS ? DPAD : 4];
-  __shared__ float gi[2][RC], gf[2][RC];
-  __shared__ float vs[2][RC][WCOLS];
+  __shared__ __attribute__((aligned(16))) float qs[BUFS][RC][DPAD];
+  __shared__ __attribute__((aligned(16))) float ks[BUFS][RC][DPAD];
+  __shared__ __attribute__((aligned(16))) float as[CHANNELS ? BUFS : 1][CHANNELS ? RC : 1][CHANNELS ? DPAD : 4];
+  __shared__ float gi[BUFS][RC], gf[BUFS][RC];
+  __shared__ float vs[BUFS][RC][WCOLS];
   const int lane = threadIdx.x & 63, wv = wave_index();
   const int h = blockIdx.y;
   const int dim = a.dim, vdim = a.vdim;
@@ -601,18 +602,30 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
     }
   };
 
-  fetch(0);
-  stash(0, 0);
-  __syncthreads();
+  if constexpr (BUFS == 2) {
+    fetch(0);
+    stash(0, 0);
+    __syncthreads();
+  }
   int buf = 0;
-  for (int t0 = 0; t0 < count; t0 += RC, buf ^= 1) {
+  for (int t0 = 0; t0 < count; t0 += RC) {
     const int tc = min(RC, count - t0);
-    fetch(t0 + RC);
+    if constexpr (BUFS == 2) {
+      fetch(t0 + RC);
+    } else {
+      fetch(t0);
+      __syncthreads();
+      stash(t0, 0);
+      __syncthreads();
+    }
     int t = 0;
     for (; t + TU <= tc; t += TU) tokens(std::integral_constant<int, TU>{}, t0, buf, t);
     for (; t < tc; ++t) tokens(std::integral_constant<int, 1>{}, t0, buf, t);
-    stash(t0 + RC, buf ^ 1);
-    __syncthreads();
+    if constexpr (BUFS == 2) {
+      stash(t0 + RC, buf ^ 1);
+      __syncthreads();
+      buf ^= 1;
+    }
   }
   // where the state goes: the slot (PHASE 3: from the request's last chunk only), or the chunk's own record
   float* S_out = S;
