@@ -262,12 +262,9 @@ def rasesun_comparison(bw, torch, steps: int, dtype: str, only: str = "") -> int
                     print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "prefill_tokens": tokens, "exact_cuts": exact,
                                       "ms": m["ms"], "tok_s": m["value"], "frac_of_matrix_peak": m["frac"]}), flush=True)
             for batch in (1, 8, 64):
-                for exact in (True, False):
-                    # (exact_cuts False: a decoded token's keys of the compressed cache are cut into pieces)
-                    m = measure_decode(bw, torch, model, cfg, dtype, batch, steps, 4, context=2048, exact_cuts=exact)
-                    print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "decode_batch": batch, "context": 2048,
-                                      "exact_cuts": exact, "ms_per_step": m["ms_per_step"], "tok_s": m["tok_s"],
-                                      "frac_of_8_TBs": m["roofline"]["frac"]}), flush=True)
+                m = measure_decode(bw, torch, model, cfg, dtype, batch, steps, 4, context=2048)
+                print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "decode_batch": batch, "context": 2048,
+                                  "ms_per_step": m["ms_per_step"], "tok_s": m["tok_s"], "frac_of_8_TBs": m["roofline"]["frac"]}), flush=True)
             del model
             torch.cuda.empty_cache()
     return 0

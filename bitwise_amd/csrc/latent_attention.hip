@@ -85,6 +85,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a, CT* __rest
   if (a.write_cache) {
     // every wave sums the latent's squares in the same order; the lanes are joined by the butterflies of wave_sum
     float acc = 0.0f;
+#pragma unroll 8
     for (int i = lane; i < a.rank; i += 64) acc = fmaf(dkv[i], dkv[i], acc);
     const float inv = 1.0f / sqrtf(wave_sum(acc) / (float)a.rank + a.eps);
     const int page = a.block_table[(size_t)a.row_seq[row] * a.table_stride + pos / a.page_size];
@@ -100,6 +101,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a, CT* __rest
   if (a.q_rank > 0) {
     const float* ql = pr + a.q_off;
     float acc = 0.0f;
+#pragma unroll 8
     for (int i = lane; i < a.q_rank; i += 64) acc = fmaf(ql[i], ql[i], acc);
     const float inv = 1.0f / sqrtf(wave_sum(acc) / (float)a.q_rank + a.eps);
     for (int i = threadIdx.x; i < a.q_rank; i += blockDim.x) {

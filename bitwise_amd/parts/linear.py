@@ -70,7 +70,10 @@ class Linear:
     def store_normed(self, x: torch.Tensor, norm, out: torch.Tensor, rows: int) -> bool:
         """out[:rows] = norm(x[:rows]) @ W.T as one kernel (32-bit store), with the bits of the norm followed by ``store``.
         False (and nothing is done) where the fused kernel does not take this step: many rows, the 32-bit mode, a norm of
-        another kind."""
+        another kind; or few columns of a long inner size, whose fused kernel has too few workgroups to be worth the launch
+        it saves."""
+        if self.in_features > 1024 and self.out_features < 2048:
+            return False
         from .norm import RMSNorm
         if not (self.mfma and self.bias is None and type(norm) is RMSNorm and ops.can_fuse_norm(rows, self.weight, x)):
             return False
