@@ -90,7 +90,7 @@ def kuponex_comparison(bw, torch, steps: int, dtype: str, only: str = "") -> int
                     print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "prefill_tokens": tokens, "exact_cuts": exact,
                                       "ms": m["ms"], "tok_s": m["value"], "frac_of_matrix_peak": m["frac"]}), flush=True)
             for batch in (1, 8, 64):
-                m = measure_decode(bw, torch, model, cfg, dtype, batch, steps, 4, context=2048, exact_cuts=False)
+                m = measure_decode(bw, torch, model, cfg, dtype, batch, steps, 4, context=2048)
                 print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "decode_batch": batch, "context": 2048,
                                   "ms_per_step": m["ms_per_step"], "tok_s": m["tok_s"], "frac_of_8_TBs": m["roofline"]["frac"]}),
                       flush=True)

@@ -321,8 +321,8 @@ struct RecurArgs {
 // A request's long portion can also run in three passes over chunks of its rows, which gives every chunk waves of its
 // own: PHASE 1 runs every chunk from a zero state (no read-out) and leaves the chunk's own contribution and its decay;
 // recurrence_scan_kernel walks a request's chunks in order and leaves the state each one starts from; PHASE 3 runs every
-// chunk from there with the read-out, and the request's last chunk leaves the state in the slot.  PHASE 0 is the whole
-// portion by one wave.  The passes differ from PHASE 0 by the rounding of the scan's sums only.
+// chunk from there with the read-out, and the request's last chunk leaves the state in the slot.  PHASE 0 walks
+// the whole portion.  The passes differ from PHASE 0 by the rounding of the scan's sums only.
 #define RC 16
 #define RW 4             // waves of a workgroup
 // floats of a chunk's record for one head: S, a vector, two scalars, in whole vectors of four

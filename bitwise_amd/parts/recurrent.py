@@ -33,8 +33,9 @@ from .linear import Linear
 
 
 SCAN_CHUNK = 32          # rows of a chunk of a long portion
-SCAN_MIN_ROWS = 96       # portions from this many rows on run in three passes over chunks (shorter ones: one wave each),
+SCAN_MIN_ROWS = 96       # portions from this many rows on run in three passes over chunks (shorter ones are walked whole),
                          # where the engine allows logits to depend on the cut in their last bits (Workspace.exact_cuts False)
+SCAN_MAX_STATE = 1 << 20  # memories of a layer with so many elements and more fill the chip when a portion is walked whole: no passes
 
 
 def _scan_plan(ctx):
@@ -136,7 +137,7 @@ class _MatrixMemoryMixer(Mixer):
         """``at``: where q (or r), k and v lie in a row of ``y``, if not at the stacked projection's own
         offsets.  ``state``: the memories' part of the slots, if they do not fill them."""
         at = self.offsets if at is None else at
-        plan = _scan_plan(ctx)
+        plan = _scan_plan(ctx) if self.heads * self.dim * self.vdim < SCAN_MAX_STATE else None
         seq_rows, nseq, scan = ctx.seq_rows, ctx.nseq, None
         if plan is not None:
             seq_rows, nseq, chunks, nchunks, spans, nspans = plan
