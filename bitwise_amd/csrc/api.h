@@ -116,9 +116,10 @@ int bw_norm_shift(const float* x, int ldx, const float* w, const float* mix, flo
 // mode 4: a step size per head, delta = softplus(logit at gate_off + head + bias[head]); decay exp(-bias2[head] delta), the
 // token enters as k (delta v)^T, skip[head] v (optional) joins the read-out.
 // q is multiplied by qscale, k by kscale; heads_per_key neighbouring heads share one q and one k.
+// (silu 1, fixed decay only: q, k and v pass SiLU on their way in)
 int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_off, int k_off, int v_off, const float* gate, int ldg,
                          int gate_off, int gate2_off, const float* bias, const float* bias2, float param, float qscale,
-                         float kscale, const float* skip, int heads_per_key, float* state, long long state_ld, float* out,
+                         float kscale, const float* skip, int heads_per_key, int silu, float* state, long long state_ld, float* out,
                          int ldo, const int32_t* seq_rows,
                          const int32_t* slots, const int32_t* positions, int nseq, int heads, int dim, int vdim,
                          const int32_t* chunks, int nchunks, const int32_t* spans, int nspans, float* scan_local,
@@ -130,10 +131,13 @@ long long bw_recurrence_record(int dim, int vdim);      // floats that scan_loca
 int bw_rotate_halves_rows(float* x, int ldx, int rows, int heads, int dim, int rot, int sections, int off0, int off1,
                           const float* cos_table, const float* sin_table, const int32_t* positions, void* stream);
 int bw_tanh_rows(float* x, int ld, int rows, int cols, void* stream);      // x <- tanh(x)
-// v = o * silu(z), each of a row's ``parts`` stretches of ``size`` elements divided by its own root mean square, times weight
+int bw_silu_rows(float* x, int ld, int rows, int cols, void* stream);      // x <- silu(x)
+// v = o * act(z), each of a row's ``parts`` stretches of ``size`` elements divided by its own root mean square, times weight;
+// behind 1: v = o and the result is multiplied by act(z).  act: gate 0 sigmoid, 1 SiLU.
 int bw_gated_part_norm(const float* o, int ldi, const float* z, int ldz, const float* weight, void* out, int out_is_bf16,
-                       int ldo, const int32_t* positions, int rows, int parts, int size, float eps, void* stream);
-// out = act(x); act 0: max(x, 0)^2, 1: x > 0: p0 x^2 + x/2, else (1/2 + p1) (e^x - 1 - x) + x/2
+                       int ldo, const int32_t* positions, int rows, int parts, int size, float eps, int gate, int behind,
+                       void* stream);
+// out = act(x); act 0: max(x, 0)^2, 1: x > 0: p0 x^2 + x/2, else (1/2 + p1) (e^x - 1 - x) + x/2, 2: x/2 (1 + erf(x / sqrt 2))
 int bw_activate(const float* x, int ldx, void* out, int out_is_bf16, int ldo, int rows, int cols, int act, float p0, float p1,
                 void* stream);
 int bw_head_norm_gate(const float* o, int ldi, const float* weight, int wstride, const float* g, int ldg, int gate, void* out,
@@ -178,6 +182,13 @@ int bw_shared_key_attention_mfma(const void* q, int ldq, const int32_t* position
 int bw_causal_conv(const float* x, int ldx, const float* in_bias, const void* w, const void* bias, int w_is_bf16, int taps, int channels,
                    float* state, long long state_ld, const int32_t* seq_rows, const int32_t* slots,
                    const int32_t* positions, int nseq, int max_seq_rows, float* out, int ldo, int silu, void* stream);
+// The convolution with SiLU of causal_conv over [q heads | k heads | v] (key_heads heads of dim channels each, then v_channels),
+// q and k heads made unit vectors, x / sqrt(sum x^2 + eps), q times qscale; and per head of the memory, gates_out[r] =
+// [beta (heads) | g (heads)], beta = sigmoid(gate[b_off + h]), g = exp(-rate[h] softplus(gate[a_off + h] + dt_bias[h]))
+int bw_conv_heads(const float* x, int ldx, const float* w, int taps, int key_heads, int dim, int v_channels, float qscale, float eps,
+                  float* state, long long state_ld, const float* gate, int ldg, int a_off, int b_off, const float* dt_bias,
+                  const float* rate, int heads, float* gates_out, int ldgo, const int32_t* seq_rows, const int32_t* slots,
+                  const int32_t* positions, int nseq, int max_seq_rows, float* out, int ldo, void* stream);
 int bw_pair_rope_unit(const float* src, int lds, const int32_t* positions, const int32_t* row_seq,
                       const int32_t* block_table, int table_stride, const float* cos_table, const float* sin_table,
                       void* q_out, void* k_cache, void* v_cache, int is_bf16, int rows, int heads, int kv_heads,
@@ -188,13 +199,16 @@ int bw_pair_rope_unit(const float* src, int lds, const int32_t* positions, const
 // Queries and keys normed over their whole projection (all heads at once): x / sqrt(mean(x^2) + eps) * w; values as they
 // are or mixed with another layer's values of the same row, v <- (1 - lambda) v + lambda v_first (lambda: one number on
 // the device); the cache write and the queries' copy as bw_pair_rope_unit.  src: [q | k | v] at columns 0, heads*dim,
-// (heads + kv_heads)*dim.  v_keep (optional): receives the row's values as projected (32-bit, [rows, ldk]).
+// (heads + kv_heads)*dim.  v_keep (optional): receives the row's values as projected (32-bit, [rows, ldk]).  bias (optional,
+// [q | k | v]): added to the projections first.  rot > 0: the normed heads' first rot elements are turned at the row's
+// position, by the tables and layouts of bw_pair_rope_unit.
 int bw_whole_norm_kv(const float* src, int lds, const int32_t* positions, const int32_t* row_seq,
                      const int32_t* block_table, int table_stride, const float* q_w, const float* k_w, float eps,
                      const float* v_first, int ldf, const float* lambda, float* v_keep, int ldk, void* q_out,
                      void* k_cache, void* v_cache, int is_bf16, int rows, int heads, int kv_heads, int dim, int vdim,
-                     int hd, int page_size, int write_cache, void* stream);
-// per_head 1: g holds one logit a head ([rows, heads]) instead of one an element
+                     int hd, int page_size, int write_cache, const float* bias, const float* cos_table, const float* sin_table,
+                     int rot, int halves, void* stream);
+// g null: no gate, the heads are only compacted.  per_head 1: g holds one logit a head ([rows, heads]) instead of one an element
 int bw_gate_mul(const void* av, int a_is_bf16, int lda, int hd, const float* g, int ldg, void* out, int out_is_bf16,
                 int ldo, int rows, int heads, int vdim, int per_head, void* stream);
 // (y and gates are overwritten: y by its activation, the gates' logits by the recurrence's factor and addend)
@@ -212,6 +226,14 @@ int bw_norm_mean(const float* const* y, const int* ldy, const float* const* w, i
 // x[r] += scale * norm(that mean; w2, eps2), one launch, for rows of up to 2,048 elements: the bits of bw_norm_mean then bw_norm_add
 int bw_norm_mean_add(const float* const* y, const int* ldy, const float* const* w, int n, float eps, const float* w2, float eps2,
                      float scale, float* x, int ldx, int rows, int dim, void* stream);
+// out[r] = sum_b s[b] y[b][r], n <= 4 (host arrays)
+int bw_scaled_sum(const float* const* y, const int* ldy, const float* s, int n, float* out, int ldo, int rows, int dim, void* stream);
+// x[r] += scale * norm(that sum; w, eps), rounded as in bw_norm_add: one launch, the bits of bw_scaled_sum then bw_norm_add
+int bw_scaled_sum_norm_add(const float* const* y, const int* ldy, const float* s, int n, const float* w, float eps, float scale,
+                           float* x, int ldx, void* rounded, int ldr, int rows, int dim, void* stream);
+// out[r][d] = gelu_tanh(z[r][d]) * table[token of r][d] (table: a pointer into rows of ldt elements); negative tokens: zeros
+int bw_side_gate(const float* z, int ldz, const int32_t* tokens, const int32_t* feedback, const void* table, int table_is_bf16,
+                 int ldt, int vocab, void* out, int out_is_bf16, int ldo, int rows, int dim, void* stream);
 int bw_softcap(float* x, int ld, int rows, int cols, float cap, void* stream);
 int bw_scale_rows(float* x, int ld, int rows, int cols, float factor, void* stream);      // x *= factor
 // A feed-forward of routed experts (moe.hip).

@@ -20,6 +20,8 @@ typedef __attribute__((ext_vector_type(2))) uint32_t u32x2;
 // the same for all lanes, and everything derived from it (segments, strips, loop bounds) would
 // be computed per lane and branched on per lane.  A branch around a matrix instruction must be
 // scalar in particular: the matrix cores ignore the execution mask.
+#define BW_TOKEN_FROM_FEEDBACK (-2)      // a token id that means: take this row's token from the feedback array
+
 __device__ __forceinline__ int wave_index() { return __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)); }
 
 __device__ __forceinline__ float bf16_to_f32(bf16_t v) { return __uint_as_float(((uint32_t)v) << 16); }

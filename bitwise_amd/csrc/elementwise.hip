@@ -11,7 +11,6 @@
 
 // A token of -2 stands for "the token the last step sampled for this row": it is read from ``feedback`` (the
 // sampling kernel's output), so that a decode step can be launched before the host has seen the token.
-#define BW_TOKEN_FROM_FEEDBACK (-2)
 
 template <typename TableT>
 __global__ void embed_kernel(const int32_t* __restrict__ tokens, const int32_t* __restrict__ feedback,

@@ -6,7 +6,11 @@
 //   pair_rope_unit: rotation of neighbouring pairs (2i, 2i+1) of the first rot elements of each head at the row's
 //                  position, optional division by the head's root mean square, the cache write (keys and values padded
 //                  with zeros to the cache's head size) and the queries' copy
-//   gate_mul:      out = a * sigmoid(g), heads compacted from the attention's head size to the value size
+//   gate_mul:      out = a * sigmoid(g), heads compacted from the attention's head size to the value size (or only that)
+//   conv_heads:    the convolution with SiLU over heads of queries, keys and values, queries and keys made unit vectors, and
+//                  the step sizes and decays of a delta memory, in one launch
+//   scaled_sum:    out = sum_b s_b y_b, and scaled_sum_norm_add: x += that sum normed, one launch
+//   side_gate:     out = gelu_tanh(z) * the token's row of a table
 //   rglru_scan:    S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t with a_t = exp(c r_t), r and i sigmoids of block-diagonal
 //                  projections of u; out = S_t * gelu_tanh(y_t)
 //   norm_add:      x += y / sqrt(mean(y^2) + eps) * w (and, if asked, the new x once more rounded to bfloat16)
@@ -127,6 +131,163 @@ extern "C" int bw_causal_conv(const float* x, int ldx, const float* in_bias, con
   return w_is_bf16 ? conv_launch<bf16_t>(a, taps, grid, (hipStream_t)stream) : conv_launch<float>(a, taps, grid, (hipStream_t)stream);
 }
 
+// ------------------------------------------------------------------------------ what a delta memory reads
+
+// One launch for everything between the projections and a delta memory's recurrence: a causal convolution with SiLU per
+// channel over [q heads | k heads | v], every q and k head made a unit vector (x / sqrt(sum x^2 + eps), q then times qscale),
+// and a head's step size beta = sigmoid(zb) and decay g = exp(-rate softplus(za + dt_bias)).  A wave a head of q or k (its
+// channels lane, lane + 64, ...), a wave per 64 NC channels of v, a wave for the gates; CONV_HEADS_CHUNK tokens each.  The
+// convolution's sums are those of causal_conv.
+#define CONV_HEADS_CHUNK 16
+
+struct ConvHeadsArgs {
+  const float* x;          // [rows, ldx]: channel c at column c
+  const float* w;          // [channels, taps]
+  float* state;            // [slots, state_ld]: [taps - 1][channels] at the pointer, oldest first
+  float* out;              // [rows, ldo]
+  const int32_t* seq_rows;
+  const int32_t* slots;
+  const int32_t* positions;
+  const float* gate;       // [rows, ldg]: za of head h at a_off + h, zb at b_off + h
+  const float* dt_bias;    // [heads]
+  const float* rate;       // [heads]
+  float* gates_out;        // [rows, ldgo]: beta of head h at column h, g at heads + h
+  long long state_ld;
+  int ldx, ldo, channels, ldg, a_off, b_off, ldgo, heads, unit_heads, scaled_heads, dim, items;
+  float qscale, eps;
+};
+
+template <int TAPS, int NC>
+__global__ __launch_bounds__(256) void conv_heads_kernel(ConvHeadsArgs a) {
+  constexpr int P = TAPS > 1 ? TAPS - 1 : 1;
+  const int item = blockIdx.x * 4 + wave_index(), lane = threadIdx.x & 63;
+  const int seq = blockIdx.y, t0 = blockIdx.z * CONV_HEADS_CHUNK;
+  const int first = a.seq_rows[2 * seq], n = a.seq_rows[2 * seq + 1], slot = a.slots[seq];
+  if (item >= a.items || n <= 0 || slot < 0 || t0 >= n || a.positions[first] < 0) return;
+  const int t1 = min(n, t0 + CONV_HEADS_CHUNK);
+  if (item == a.items - 1) {
+    for (int e = lane; e < (t1 - t0) * a.heads; e += 64) {
+      const size_t row = (size_t)(first + t0 + e / a.heads);
+      const int h = e % a.heads;
+      const float za = a.gate[row * a.ldg + a.a_off + h] + a.dt_bias[h];
+      const float sp = fmaxf(za, 0.0f) + log1pf(bw_expf(-fabsf(za)));
+      a.gates_out[row * a.ldgo + h] = gm_sigmoid(a.gate[row * a.ldg + a.b_off + h]);
+      a.gates_out[row * a.ldgo + a.heads + h] = bw_expf(-(a.rate[h] * sp));
+    }
+    return;
+  }
+  const bool unit = item < a.unit_heads;
+  const int c0 = unit ? item * a.dim : a.unit_heads * a.dim + (item - a.unit_heads) * 64 * NC;
+  const int count = unit ? a.dim : min(64 * NC, a.channels - c0);
+  const float post = item < a.scaled_heads ? a.qscale : 1.0f;
+  float w[NC][TAPS], win[NC][P], old[NC][P];
+  int ch[NC];
+#pragma unroll
+  for (int i = 0; i < NC; ++i) {
+    ch[i] = c0 + min(lane + 64 * i, count - 1);
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[i][j] = a.w[(size_t)ch[i] * TAPS + j];
+  }
+  float* st = a.state + (size_t)slot * a.state_ld;
+  const float* x = a.x + (size_t)first * a.ldx;
+  // only the request's first chunk reaches back before the portion, and only its waves touch the slot
+#pragma unroll
+  for (int i = 0; i < NC; ++i) {
+#pragma unroll
+    for (int j = 0; j < P; ++j) old[i][j] = (TAPS > 1 && t0 == 0) ? st[(size_t)j * a.channels + ch[i]] : 0.0f;
+#pragma unroll
+    for (int j = 0; j < P; ++j) {
+      const int idx = t0 - (TAPS - 1) + j;
+      win[i][j] = idx >= 0 ? x[(size_t)idx * a.ldx + ch[i]] : old[i][(TAPS - 1 + idx) < 0 ? 0 : (TAPS - 1 + idx)];
+    }
+  }
+  float* o = a.out + (size_t)first * a.ldo;
+  constexpr int UN = 4;
+  for (int tb = t0; tb < t1; tb += UN) {
+    float cur[UN][NC];
+#pragma unroll
+    for (int u = 0; u < UN; ++u)
+#pragma unroll
+      for (int i = 0; i < NC; ++i) cur[u][i] = x[(size_t)min(tb + u, t1 - 1) * a.ldx + ch[i]];
+#pragma unroll
+    for (int u = 0; u < UN; ++u) {
+      if (tb + u >= t1) continue;                        // (scalar)
+      float y[NC], ss = 0.0f;
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        float acc = 0.0f;
+        if constexpr (TAPS > 1) {
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j) acc = fmaf(w[i][j], win[i][j], acc);
+        }
+        acc = fmaf(w[i][TAPS - 1], cur[u][i], acc);
+        acc *= gm_sigmoid(acc);
+        y[i] = acc;
+        if (lane + 64 * i < count) ss = fmaf(acc, acc, ss);
+        if constexpr (TAPS > 1) {
+#pragma unroll
+          for (int j = 0; j + 1 < TAPS - 1; ++j) win[i][j] = win[i][j + 1];
+          win[i][TAPS - 2] = cur[u][i];
+        }
+      }
+      float inv = 1.0f;
+      if (unit) inv = 1.0f / sqrtf(wave_sum(ss) + a.eps);
+#pragma unroll
+      for (int i = 0; i < NC; ++i)
+        if (lane + 64 * i < count) o[(size_t)(tb + u) * a.ldo + ch[i]] = unit ? (y[i] * inv) * post : y[i];
+    }
+  }
+  if (TAPS > 1 && t0 == 0) {
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      if (lane + 64 * i >= count) continue;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int idx = n - (TAPS - 1) + j;
+        float v = 0.0f;
+        if (idx >= 0) v = x[(size_t)idx * a.ldx + ch[i]];
+        else {
+#pragma unroll
+          for (int q = 0; q < P; ++q) v = (q == TAPS - 1 + idx) ? old[i][q] : v;
+        }
+        st[(size_t)j * a.channels + ch[i]] = v;
+      }
+    }
+  }
+}
+
+template <int NC>
+static int conv_heads_launch(const ConvHeadsArgs& a, int taps, dim3 grid, hipStream_t s) {
+  switch (taps) {
+#define CONV_CASE(T) case T: hipLaunchKernelGGL((conv_heads_kernel<T, NC>), grid, dim3(256), 0, s, a); break;
+    CONV_CASE(1) CONV_CASE(2) CONV_CASE(3) CONV_CASE(4) CONV_CASE(5) CONV_CASE(6) CONV_CASE(7) CONV_CASE(8)
+#undef CONV_CASE
+    default: return -2;
+  }
+  return BW_LAUNCH_CHECK();
+}
+
+extern "C" int bw_conv_heads(const float* x, int ldx, const float* w, int taps, int key_heads, int dim, int v_channels, float qscale,
+                             float eps, float* state, long long state_ld, const float* gate, int ldg, int a_off, int b_off,
+                             const float* dt_bias, const float* rate, int heads, float* gates_out, int ldgo, const int32_t* seq_rows,
+                             const int32_t* slots, const int32_t* positions, int nseq, int max_seq_rows, float* out, int ldo,
+                             void* stream) {
+  if (nseq <= 0 || max_seq_rows <= 0) return 0;
+  if (taps < 1 || taps > CONV_MAX_TAPS || (taps > 1 && state == nullptr) || key_heads < 1 || dim < 1 || dim > 256 || v_channels < 1 ||
+      heads < 1 || ldgo < 2 * heads)
+    return -2;
+  const int channels = 2 * key_heads * dim + v_channels, nc = (dim + 63) / 64;
+  if (ldx < channels || ldo < channels || (taps > 1 && state_ld < (long long)(taps - 1) * channels)) return -2;
+  const int items = 2 * key_heads + (v_channels + 64 * nc - 1) / (64 * nc) + 1;
+  ConvHeadsArgs a{x, w, state, out, seq_rows, slots, positions, gate, dt_bias, rate, gates_out, state_ld, ldx, ldo, channels, ldg,
+                  a_off, b_off, ldgo, heads, 2 * key_heads, key_heads, dim, items, qscale, eps};
+  const dim3 grid((items + 3) / 4, nseq, (max_seq_rows + CONV_HEADS_CHUNK - 1) / CONV_HEADS_CHUNK);
+  if (grid.y > 65535 || grid.z > 65535) return -2;
+  hipStream_t s = (hipStream_t)stream;
+  return nc == 1 ? conv_heads_launch<1>(a, taps, grid, s) : nc == 2 ? conv_heads_launch<2>(a, taps, grid, s)
+       : nc == 3 ? conv_heads_launch<3>(a, taps, grid, s) : conv_heads_launch<4>(a, taps, grid, s);
+}
+
 // ------------------------------------------------------------------------------ pair rotation, unit norm, cache write
 
 struct PairRopeArgs {
@@ -232,7 +393,7 @@ extern "C" int bw_pair_rope_unit(const float* src, int lds, const int32_t* posit
   return BW_LAUNCH_CHECK();
 }
 
-// ------------------------------------------------------------------------------ norm over whole projections, value mixing
+// ------------------------------------------------------------------------------ norm over whole projections, rotation, value mixing
 
 struct WholeNormArgs {
   const float* src;
@@ -247,7 +408,10 @@ struct WholeNormArgs {
   void* q_out;
   void* k_cache;
   void* v_cache;
-  int lds, ldf, ldk, heads, kv_heads, dim, vdim, hd, page_size, table_stride, write_cache;
+  const float* bias;           // [q | k | v] or null: added to the projections first
+  const float* cos_table;      // [positions, rot / 2]
+  const float* sin_table;
+  int lds, ldf, ldk, heads, kv_heads, dim, vdim, hd, page_size, table_stride, write_cache, rot, halves;
   float eps;
 };
 
@@ -261,6 +425,46 @@ __device__ __forceinline__ float workgroup_sum_256(float v, float* lds4) {
   return t;
 }
 
+// The normed heads of one projection, turned and padded: item i of ``heads * hd / 2`` is a pair of elements of one head, a
+// rotated pair for the first rot / 2 of a head, neighbours behind those (in either layout).  put(h, d, value) stores.
+template <typename Put>
+__device__ __forceinline__ void whole_norm_heads(const WholeNormArgs& a, const float* p, const float* b, const float* w, int heads,
+                                                 float inv, int pos, Put put) {
+  const int half = a.rot / 2, pairs = a.hd / 2;
+  const float* ct = a.cos_table + (size_t)pos * half;
+  const float* st = a.sin_table + (size_t)pos * half;
+  for (int i = threadIdx.x; i < heads * pairs; i += 256) {
+    const int h = i / pairs, r = i % pairs;
+    const bool turned = r < half;
+    const int d0 = a.halves && turned ? r : 2 * r, d1 = a.halves && turned ? r + half : 2 * r + 1;
+    float u = 0.0f, v = 0.0f;
+    if (d0 < a.dim) {
+      const int e = h * a.dim + d0;
+      u = ((b != nullptr ? p[e] + b[e] : p[e]) * inv) * w[e];
+    }
+    if (d1 < a.dim) {
+      const int e = h * a.dim + d1;
+      v = ((b != nullptr ? p[e] + b[e] : p[e]) * inv) * w[e];
+    }
+    if (turned) {
+      const float c = ct[r], s = st[r], u0 = u;
+      u = u0 * c - v * s;
+      v = v * c + u0 * s;
+    }
+    put(h, d0, u);
+    put(h, d1, v);
+  }
+}
+
+__device__ __forceinline__ float whole_norm_inv(const float* p, const float* b, int n, float eps, float* red) {
+  float acc = 0.0f;
+  for (int i = threadIdx.x; i < n; i += 256) {
+    const float v = b != nullptr ? p[i] + b[i] : p[i];
+    acc = fmaf(v, v, acc);
+  }
+  return 1.0f / sqrtf(workgroup_sum_256(acc, red) / (float)n + eps);
+}
+
 // A workgroup for each of a row's three parts (queries, keys, values): each is one chain of loads, a sum and stores.
 template <typename T>
 __global__ __launch_bounds__(256) void whole_norm_kv_kernel(WholeNormArgs a) {
@@ -271,14 +475,9 @@ __global__ __launch_bounds__(256) void whole_norm_kv_kernel(WholeNormArgs a) {
   const int qn = a.heads * a.dim, kn = a.kv_heads * a.dim;
   const float* q = a.src + (size_t)row * a.lds;
   if (part == 0) {
-    float acc = 0.0f;
-    for (int i = tid; i < qn; i += 256) acc = fmaf(q[i], q[i], acc);
-    const float inv_q = 1.0f / sqrtf(workgroup_sum_256(acc, red) / (float)qn + a.eps);
+    const float inv_q = whole_norm_inv(q, a.bias, qn, a.eps, red);
     T* qo = reinterpret_cast<T*>(a.q_out) + (size_t)row * a.heads * a.hd;
-    for (int i = tid; i < a.heads * a.hd; i += 256) {
-      const int h = i / a.hd, d = i % a.hd;
-      gm_store(qo + i, d < a.dim ? (q[h * a.dim + d] * inv_q) * a.q_w[h * a.dim + d] : 0.0f);
-    }
+    whole_norm_heads(a, q, a.bias, a.q_w, a.heads, inv_q, pos, [&](int h, int d, float v) { gm_store(qo + h * a.hd + d, v); });
     return;
   }
   if (!a.write_cache) return;
@@ -286,18 +485,16 @@ __global__ __launch_bounds__(256) void whole_norm_kv_kernel(WholeNormArgs a) {
   const int slot = pos % a.page_size;
   if (part == 1) {
     const float* k = q + qn;
-    float acc = 0.0f;
-    for (int i = tid; i < kn; i += 256) acc = fmaf(k[i], k[i], acc);
-    const float inv_k = 1.0f / sqrtf(workgroup_sum_256(acc, red) / (float)kn + a.eps);
+    const float* kb = a.bias != nullptr ? a.bias + qn : nullptr;
+    const float inv_k = whole_norm_inv(k, kb, kn, a.eps, red);
     T* kc = reinterpret_cast<T*>(a.k_cache);
-    for (int i = tid; i < a.kv_heads * a.hd; i += 256) {
-      const int h = i / a.hd, d = i % a.hd;
-      gm_store(kc + (((size_t)page * a.kv_heads + h) * a.page_size + slot) * a.hd + d,
-               d < a.dim ? (k[h * a.dim + d] * inv_k) * a.k_w[h * a.dim + d] : 0.0f);
-    }
+    whole_norm_heads(a, k, kb, a.k_w, a.kv_heads, inv_k, pos, [&](int h, int d, float v) {
+      gm_store(kc + (((size_t)page * a.kv_heads + h) * a.page_size + slot) * a.hd + d, v);
+    });
     return;
   }
   const float* v = q + qn + kn;
+  const float* vb = a.bias != nullptr ? a.bias + qn + kn : nullptr;
   T* vc = reinterpret_cast<T*>(a.v_cache);
   const float lam = a.v_first != nullptr ? a.lambda[0] : 0.0f;
   for (int i = tid; i < a.kv_heads * a.hd; i += 256) {
@@ -305,6 +502,7 @@ __global__ __launch_bounds__(256) void whole_norm_kv_kernel(WholeNormArgs a) {
     float val = 0.0f;
     if (d < a.vdim) {
       val = v[h * a.vdim + d];
+      if (vb != nullptr) val += vb[h * a.vdim + d];
       if (a.v_keep != nullptr) a.v_keep[(size_t)row * a.ldk + h * a.vdim + d] = val;
       if (a.v_first != nullptr) val = (1.0f - lam) * val + lam * a.v_first[(size_t)row * a.ldf + h * a.vdim + d];
     }
@@ -317,15 +515,17 @@ extern "C" int bw_whole_norm_kv(const float* src, int lds, const int32_t* positi
                                 const int32_t* block_table, int table_stride, const float* q_w, const float* k_w, float eps,
                                 const float* v_first, int ldf, const float* lambda, float* v_keep, int ldk, void* q_out,
                                 void* k_cache, void* v_cache, int is_bf16, int rows, int heads, int kv_heads, int dim, int vdim,
-                                int hd, int page_size, int write_cache, void* stream) {
+                                int hd, int page_size, int write_cache, const float* bias, const float* cos_table,
+                                const float* sin_table, int rot, int halves, void* stream) {
   if (rows <= 0) return 0;
-  if (heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || dim > hd || vdim > hd || page_size <= 0) return -2;
+  if (heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || dim > hd || vdim > hd || hd % 2 || page_size <= 0) return -2;
+  if (rot < 0 || rot % 2 || rot > dim || (rot > 0 && (cos_table == nullptr || sin_table == nullptr))) return -2;
   if (lds < heads * dim + (write_cache ? kv_heads * (dim + vdim) : 0)) return -2;
   if (v_first != nullptr && (lambda == nullptr || ldf < kv_heads * vdim)) return -2;
   if (v_keep != nullptr && ldk < kv_heads * vdim) return -2;
   if (v_keep != nullptr && v_keep == v_first) return -2;
-  WholeNormArgs a{src, positions, row_seq, block_table, q_w, k_w, v_first, lambda, v_keep, q_out, k_cache, v_cache, lds, ldf, ldk,
-                  heads, kv_heads, dim, vdim, hd, page_size, table_stride, write_cache, eps};
+  WholeNormArgs a{src, positions, row_seq, block_table, q_w, k_w, v_first, lambda, v_keep, q_out, k_cache, v_cache, bias, cos_table,
+                  sin_table, lds, ldf, ldk, heads, kv_heads, dim, vdim, hd, page_size, table_stride, write_cache, rot, halves, eps};
   if (is_bf16) hipLaunchKernelGGL(whole_norm_kv_kernel<bf16_t>, dim3(rows, 3), dim3(256), 0, (hipStream_t)stream, a);
   else hipLaunchKernelGGL(whole_norm_kv_kernel<float>, dim3(rows, 3), dim3(256), 0, (hipStream_t)stream, a);
   return BW_LAUNCH_CHECK();
@@ -341,7 +541,7 @@ __global__ __launch_bounds__(256) void gate_mul_kernel(const TI* __restrict__ av
   if (e >= heads * vdim) return;
   const int h = e / vdim, d = e % vdim;
   const float x = gm_load(av + (size_t)row * lda + (size_t)h * hd + d);
-  gm_store(out + (size_t)row * ldo + e, x * gm_sigmoid(g[(size_t)row * ldg + (per_head ? h : e)]));
+  gm_store(out + (size_t)row * ldo + e, g == nullptr ? x : x * gm_sigmoid(g[(size_t)row * ldg + (per_head ? h : e)]));
 }
 
 extern "C" int bw_gate_mul(const void* av, int a_is_bf16, int lda, int hd, const float* g, int ldg, void* out, int out_is_bf16,
@@ -683,6 +883,163 @@ extern "C" int bw_norm_mean(const float* const* y, const int* ldy, const float* 
   else if (n == 2) hipLaunchKernelGGL(norm_mean_kernel<2>, dim3(rows), dim3(256), 0, s, a);
   else if (n == 3) hipLaunchKernelGGL(norm_mean_kernel<3>, dim3(rows), dim3(256), 0, s, a);
   else hipLaunchKernelGGL(norm_mean_kernel<4>, dim3(rows), dim3(256), 0, s, a);
+  return BW_LAUNCH_CHECK();
+}
+
+// ------------------------------------------------------------------------------ a weighted sum of branches
+
+struct ScaledSumArgs {
+  const float* y[4];
+  int ldy[4];
+  float s[4];
+  int dim;
+};
+
+// out[r] = sum_b s_b y_b[r], b ascending (a product, then fused multiply-adds)
+template <int N>
+__global__ __launch_bounds__(256) void scaled_sum_kernel(ScaledSumArgs a, float* __restrict__ out, int ldo, int rows) {
+  const int e = blockIdx.x * 256 + threadIdx.x;
+  if (e >= a.dim) return;
+  for (int r = blockIdx.y; r < rows; r += gridDim.y) {
+    float z = a.s[0] * a.y[0][(size_t)r * a.ldy[0] + e];
+#pragma unroll
+    for (int b = 1; b < N; ++b) z = fmaf(a.s[b], a.y[b][(size_t)r * a.ldy[b] + e], z);
+    out[(size_t)r * ldo + e] = z;
+  }
+}
+
+// x[r] += scale * (z / sqrt(mean(z^2) + eps) * w) with z that sum: the norm behind the mixer in the same launch, rounded as in
+// norm_add.  A workgroup a row; rows of up to 2,048 elements stay in registers, longer ones are formed twice (the same
+// operations): the bits of scaled_sum_kernel followed by norm_add_kernel.
+template <int N>
+__global__ __launch_bounds__(256) void scaled_sum_norm_add_kernel(ScaledSumArgs a, const float* __restrict__ w, float eps, float scale,
+                                                                  float* __restrict__ x, int ldx, bf16_t* __restrict__ rounded, int ldr) {
+  __shared__ float part[4];
+  constexpr int MAXV = 8;
+  const int row = blockIdx.x, tid = threadIdx.x;
+  auto value = [&](int e) -> float {
+    float z = a.s[0] * a.y[0][(size_t)row * a.ldy[0] + e];
+#pragma unroll
+    for (int b = 1; b < N; ++b) z = fmaf(a.s[b], a.y[b][(size_t)row * a.ldy[b] + e], z);
+    return z;
+  };
+  float* xr = x + (size_t)row * ldx;
+  const bool small = a.dim <= 256 * MAXV;
+  float z[MAXV], xo[MAXV], wp[MAXV];
+  float acc = 0.0f;
+  if (small) {
+#pragma unroll
+    for (int j = 0; j < MAXV; ++j) {
+      const int e = min(tid + 256 * j, a.dim - 1);
+      const bool in = 256 * j < a.dim;                   // (scalar)
+      z[j] = in ? value(e) : 0.0f;
+      xo[j] = in ? xr[e] : 0.0f;
+      wp[j] = in ? w[e] : 0.0f;
+    }
+#pragma unroll
+    for (int j = 0; j < MAXV; ++j) {
+      if (tid + 256 * j >= a.dim) z[j] = 0.0f;
+      acc = fmaf(z[j], z[j], acc);
+    }
+  } else {
+    for (int e = tid; e < a.dim; e += 256) {
+      const float ze = value(e);
+      acc = fmaf(ze, ze, acc);
+    }
+  }
+  acc = wave_sum(acc);
+  if ((tid & 63) == 0) part[tid >> 6] = acc;
+  __syncthreads();
+  const float inv = 1.0f / sqrtf((((part[0] + part[1]) + part[2]) + part[3]) / (float)a.dim + eps);
+  auto store = [&](int e, float ze, float xe, float we) {
+    const float normed = (ze * inv) * we;
+    const float nx = scale == 1.0f ? xe + normed : fmaf(scale, normed, xe);
+    xr[e] = nx;
+    if (rounded != nullptr) rounded[(size_t)row * ldr + e] = f32_to_bf16(nx);
+  };
+  if (small) {
+#pragma unroll
+    for (int j = 0; j < MAXV; ++j)
+      if (tid + 256 * j < a.dim) store(tid + 256 * j, z[j], xo[j], wp[j]);
+  } else {
+    for (int e = tid; e < a.dim; e += 256) store(e, value(e), xr[e], w[e]);
+  }
+}
+
+static int scaled_sum_args(ScaledSumArgs& a, const float* const* y, const int* ldy, const float* s, int n, int dim) {
+  if (n < 1 || n > 4 || dim <= 0) return -2;
+  for (int b = 0; b < n; ++b) {
+    if (y[b] == nullptr || ldy[b] < dim) return -2;
+    a.y[b] = y[b];
+    a.ldy[b] = ldy[b];
+    a.s[b] = s[b];
+  }
+  a.dim = dim;
+  return 0;
+}
+
+extern "C" int bw_scaled_sum(const float* const* y, const int* ldy, const float* s, int n, float* out, int ldo, int rows, int dim,
+                             void* stream) {
+  if (rows <= 0) return 0;
+  ScaledSumArgs a{};
+  if (scaled_sum_args(a, y, ldy, s, n, dim) != 0 || ldo < dim) return -2;
+  const dim3 grid((dim + 255) / 256, rows < 65535 ? rows : 65535), block(256);
+  hipStream_t st = (hipStream_t)stream;
+  if (n == 1) hipLaunchKernelGGL(scaled_sum_kernel<1>, grid, block, 0, st, a, out, ldo, rows);
+  else if (n == 2) hipLaunchKernelGGL(scaled_sum_kernel<2>, grid, block, 0, st, a, out, ldo, rows);
+  else if (n == 3) hipLaunchKernelGGL(scaled_sum_kernel<3>, grid, block, 0, st, a, out, ldo, rows);
+  else hipLaunchKernelGGL(scaled_sum_kernel<4>, grid, block, 0, st, a, out, ldo, rows);
+  return BW_LAUNCH_CHECK();
+}
+
+extern "C" int bw_scaled_sum_norm_add(const float* const* y, const int* ldy, const float* s, int n, const float* w, float eps,
+                                      float scale, float* x, int ldx, void* rounded, int ldr, int rows, int dim, void* stream) {
+  if (rows <= 0) return 0;
+  ScaledSumArgs a{};
+  if (scaled_sum_args(a, y, ldy, s, n, dim) != 0 || w == nullptr || ldx < dim || (rounded != nullptr && ldr < dim)) return -2;
+  hipStream_t st = (hipStream_t)stream;
+  bf16_t* r = (bf16_t*)rounded;
+  if (n == 1) hipLaunchKernelGGL(scaled_sum_norm_add_kernel<1>, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr);
+  else if (n == 2) hipLaunchKernelGGL(scaled_sum_norm_add_kernel<2>, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr);
+  else if (n == 3) hipLaunchKernelGGL(scaled_sum_norm_add_kernel<3>, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr);
+  else hipLaunchKernelGGL(scaled_sum_norm_add_kernel<4>, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr);
+  return BW_LAUNCH_CHECK();
+}
+
+// ------------------------------------------------------------------------------ a token's row of a table behind a gate
+
+// out[r][d] = gelu_tanh(z[r][d]) * table[token of r][off + d]; rows of padding (a negative token) become zeros.  The token of
+// a row as in embed_kernel: a given id, or the one the step before sampled.
+template <typename TT, typename TO>
+__global__ __launch_bounds__(256) void side_gate_kernel(const float* __restrict__ z, int ldz, const int32_t* __restrict__ tokens,
+                                                        const int32_t* __restrict__ feedback, const TT* __restrict__ table, int ldt,
+                                                        int vocab, TO* __restrict__ out, int ldo, int rows, int dim) {
+  const int e = blockIdx.x * 256 + threadIdx.x;
+  if (e >= dim) return;
+  for (int row = blockIdx.y; row < rows; row += gridDim.y) {
+    int tok = tokens[row];
+    if (tok == BW_TOKEN_FROM_FEEDBACK && feedback != nullptr) tok = feedback[row];
+    float v = 0.0f;
+    if (tok >= 0 && tok < vocab) v = gm_gelu_tanh(z[(size_t)row * ldz + e]) * gm_load(table + (size_t)tok * ldt + e);
+    gm_store(out + (size_t)row * ldo + e, v);
+  }
+}
+
+extern "C" int bw_side_gate(const float* z, int ldz, const int32_t* tokens, const int32_t* feedback, const void* table,
+                            int table_is_bf16, int ldt, int vocab, void* out, int out_is_bf16, int ldo, int rows, int dim,
+                            void* stream) {
+  if (rows <= 0 || dim <= 0) return 0;
+  if (ldz < dim || ldt < dim || ldo < dim || vocab <= 0) return -2;
+  const dim3 grid((dim + 255) / 256, rows < 65535 ? rows : 65535), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (table_is_bf16 && out_is_bf16)
+    hipLaunchKernelGGL((side_gate_kernel<bf16_t, bf16_t>), grid, block, 0, s, z, ldz, tokens, feedback, (const bf16_t*)table, ldt, vocab, (bf16_t*)out, ldo, rows, dim);
+  else if (table_is_bf16)
+    hipLaunchKernelGGL((side_gate_kernel<bf16_t, float>), grid, block, 0, s, z, ldz, tokens, feedback, (const bf16_t*)table, ldt, vocab, (float*)out, ldo, rows, dim);
+  else if (out_is_bf16)
+    hipLaunchKernelGGL((side_gate_kernel<float, bf16_t>), grid, block, 0, s, z, ldz, tokens, feedback, (const float*)table, ldt, vocab, (bf16_t*)out, ldo, rows, dim);
+  else
+    hipLaunchKernelGGL((side_gate_kernel<float, float>), grid, block, 0, s, z, ldz, tokens, feedback, (const float*)table, ldt, vocab, (float*)out, ldo, rows, dim);
   return BW_LAUNCH_CHECK();
 }
 

@@ -81,22 +81,30 @@ _SIGS = {
                       c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
     "bw_rotate_halves_rows": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p],
     "bw_tanh_rows": [c_void_p, c_int, c_int, c_int, c_void_p],
+    "bw_silu_rows": [c_void_p, c_int, c_int, c_int, c_void_p],
+    "bw_conv_heads": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_longlong, c_void_p, c_int,
+                      c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p,
+                      c_int, c_void_p],
+    "bw_scaled_sum": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p],
+    "bw_scaled_sum_norm_add": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float, c_float, c_void_p, c_int, c_void_p, c_int, c_int,
+                               c_int, c_void_p],
+    "bw_side_gate": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
     "bw_norm_mean": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_void_p],
     "bw_norm_mean_add": [c_void_p, c_void_p, c_void_p, c_int, c_float, c_void_p, c_float, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
     "bw_linear_recurrence": [c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p,
-                             c_float, c_float, c_float, c_void_p, c_int, c_void_p, c_longlong, c_void_p, c_int, c_void_p, c_void_p,
+                             c_float, c_float, c_float, c_void_p, c_int, c_int, c_void_p, c_longlong, c_void_p, c_int, c_void_p, c_void_p,
                              c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_longlong, c_void_p],
     "bw_head_norm_gate": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_int,
                           c_int, c_int, c_float, c_void_p],
     "bw_gated_part_norm": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_float,
-                           c_void_p],
+                           c_int, c_int, c_void_p],
     "bw_activate": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p],
     "bw_glu": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_int, c_void_p],
     "bw_embed_sum": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                      c_float, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_void_p],
     "bw_whole_norm_kv": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_void_p, c_int,
                          c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                         c_int, c_int, c_void_p],
+                         c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "bw_shared_key_attention_mfma": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int,
                                      c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int,
                                      c_void_p, c_longlong, c_void_p],
@@ -782,6 +790,7 @@ def gemm_qkv_rope_bf16(x: torch.Tensor, w_qkv: torch.Tensor, q_out: torch.Tensor
 # ------------------------------------------------------------------------------ mixers with a state per request
 
 RECUR_DECAY_PER_CHANNEL, RECUR_SCALAR_GATES, RECUR_BONUS_DECAY, RECUR_FIXED_DECAY, RECUR_STEP_DECAY = 0, 1, 2, 3, 4
+RECUR_DELTA = 5
 RECUR_MAX_DIM = 256          # key channels of a head that the recurrence keeps in a lane's registers
 GATE_SIGMOID, GATE_SILU = 0, 1
 ACT_SILU, ACT_GELU_TANH, ACT_CLAMPED_SWISH = 0, 1, 2
@@ -839,10 +848,10 @@ def recurrence_state(mode: int, heads: int, dim: int, vdim: int) -> int:
 
 
 def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate: Optional[torch.Tensor], gate_off: int,
-                      gate2_off: int, bias: torch.Tensor, bias2: Optional[torch.Tensor], param: float, qscale: float,
+                      gate2_off: int, bias: Optional[torch.Tensor], bias2: Optional[torch.Tensor], param: float, qscale: float,
                       state: torch.Tensor, out: torch.Tensor, seq_rows: torch.Tensor, slots: torch.Tensor,
                       positions: torch.Tensor, nseq: int, heads: int, dim: int, vdim: int, scan=None, kscale: float = 1.0,
-                      heads_per_key: int = 1, skip: Optional[torch.Tensor] = None) -> None:
+                      heads_per_key: int = 1, skip: Optional[torch.Tensor] = None, silu: bool = False) -> None:
     """The recurrence S <- decay * S + k v^T, o = S^T (q * qscale) per head over every request's rows in order, from and
     to ``state`` [slots, elements].  RECUR_DECAY_PER_CHANNEL: decay = exp(logsigmoid(gate + bias) * param) per key
     channel (``gate`` [rows, >= gate_off + heads*dim]).  RECUR_SCALAR_GATES: capped input and forget gates per head
@@ -853,6 +862,9 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
     RECUR_STEP_DECAY: a step size per head, delta = softplus(gate + bias) (``gate`` column gate_off + h, ``bias`` [heads]);
     decay = exp(-bias2[h] delta) (``bias2`` [heads]: the rates), the token enters as k (delta v)^T, and ``skip`` [heads]
     (optional) times v joins the read-out.
+    RECUR_DELTA: a step size b and a decay a per head and token, as they are (``gate`` columns gate_off + h and gate2_off + h;
+    ``bias`` None): S <- a S, S <- S + k (b (v - S^T k))^T, then the read-out; always in one pass.
+    ``silu`` (fixed decay): q, k and v are the SiLU of what ``proj`` holds.
     k is multiplied by ``kscale``; ``heads_per_key`` neighbouring heads share one q and one k.  A head's state lies as
     [value column][key channel].  ``state`` may be a column slice of a wider tensor.
 
@@ -864,7 +876,10 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
     _need_strided(proj, torch.float32, "proj")            # (may be a column slice of a wider product)
     if mode != RECUR_FIXED_DECAY:
         _need_strided(gate, torch.float32, "gate")
-    _need(bias, torch.float32, "bias")
+    if bias is not None or mode != RECUR_DELTA:
+        _need(bias, torch.float32, "bias")
+    if silu and mode != RECUR_FIXED_DECAY:
+        raise ValueError("linear_recurrence: SiLU on the way in comes with a constant decay only")
     _need_strided(state, torch.float32, "state")
     _need(out, torch.float32, "out")
     for t, what in ((positions, "positions"), (seq_rows, "seq_rows"), (slots, "slots")):
@@ -884,6 +899,10 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
         _need(bias2, torch.float32, "bias2")
         if bias.numel() != heads or bias2.numel() != heads or gate_off + heads > gate.shape[1]:
             raise ValueError("linear_recurrence: step sizes, their bias or the rates do not fit the heads")
+        need = heads * dim * vdim
+    elif mode == RECUR_DELTA:
+        if max(gate_off, gate2_off) + heads > gate.shape[1] or scan is not None:
+            raise ValueError("linear_recurrence: step sizes and decays do not fit the heads, or passes over chunks were asked of a delta memory")
         need = heads * dim * vdim
     elif mode == RECUR_FIXED_DECAY:
         if bias.numel() != heads:
@@ -923,9 +942,9 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
             raise ValueError("linear_recurrence: the scan's tables or records do not fit")
     _check(_fn("bw_linear_recurrence")(int(mode), proj.data_ptr(), proj.stride(0), q_off, k_off, v_off,
                                        0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0),
-                                       gate_off, gate2_off, bias.data_ptr(),
+                                       gate_off, gate2_off, 0 if bias is None else bias.data_ptr(),
                                        0 if bias2 is None else bias2.data_ptr(), float(param), float(qscale), float(kscale),
-                                       0 if skip is None else skip.data_ptr(), int(heads_per_key), state.data_ptr(),
+                                       0 if skip is None else skip.data_ptr(), int(heads_per_key), int(silu), state.data_ptr(),
                                        state.stride(0), out.data_ptr(), out.stride(0), seq_rows.data_ptr(), slots.data_ptr(),
                                        positions.data_ptr(), nseq, heads, dim, vdim,
                                        0 if chunks is None else chunks.data_ptr(), nchunks,
@@ -960,6 +979,14 @@ def tanh_rows(x: torch.Tensor, rows: int) -> None:
     if x.shape[0] < rows:
         raise ValueError("tanh_rows: fewer rows than asked for")
     _check(_fn("bw_tanh_rows")(x.data_ptr(), x.stride(0), rows, x.shape[1], _stream()), "tanh_rows")
+
+
+def silu_rows(x: torch.Tensor, rows: int) -> None:
+    """x[:rows] <- silu(x[:rows]) in place; ``x`` float32 (a column slice will do)."""
+    _need_strided(x, torch.float32, "x")
+    if x.shape[0] < rows:
+        raise ValueError("silu_rows: x is shorter than the rows")
+    _check(_fn("bw_silu_rows")(x.data_ptr(), x.stride(0), rows, x.shape[1], _stream()), "silu_rows")
 
 
 def norm_mean(ys: Sequence[torch.Tensor], weights: Sequence[torch.Tensor], out: torch.Tensor, rows: int, eps: float) -> None:
@@ -1026,9 +1053,9 @@ def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, per_head_weight: bool,
 
 
 def gated_part_norm(o: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, positions: torch.Tensor, rows: int,
-                    parts: int, eps: float) -> None:
-    """v = o * silu(z); every row's ``parts`` equal stretches of v are divided each by its own root mean square and multiplied
-    by ``weight`` [width].  o, z float32 (column slices will do), out float32 or bfloat16 (one rounding)."""
+                    parts: int, eps: float, gate: int = GATE_SILU, behind: bool = False) -> None:
+    """v = o * act(z); every row's ``parts`` equal stretches of v are divided each by its own root mean square and multiplied
+    by ``weight`` [width].  ``behind``: v = o, and the normed row is multiplied by act(z).  act: ``gate``.  o, z float32 (column slices will do), out float32 or bfloat16 (one rounding)."""
     _need_strided(o, torch.float32, "o")
     _need_strided(z, torch.float32, "z")
     _need(weight, torch.float32, "weight")
@@ -1040,17 +1067,17 @@ def gated_part_norm(o: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, out:
         raise ValueError("gated_part_norm: buffers shorter than the rows")
     _check(_fn("bw_gated_part_norm")(o.data_ptr(), o.stride(0), z.data_ptr(), z.stride(0), weight.data_ptr(), out.data_ptr(),
                                      _act_out(out, "out"), out.stride(0), positions.data_ptr(), rows, int(parts), width // parts,
-                                     float(eps), _stream()), "gated_part_norm")
+                                     float(eps), int(gate), int(behind), _stream()), "gated_part_norm")
 
 
-PLAIN_RELU2, PLAIN_XIELU = 0, 1
+PLAIN_RELU2, PLAIN_XIELU, PLAIN_GELU_ERF = 0, 1, 2
 
 
 def activate(x: torch.Tensor, out: torch.Tensor, rows: int, act: int, p0: float = 0.0, p1: float = 0.0) -> None:
     """out = act(x) of a 32-bit product, out float32 or bfloat16 (one rounding).  PLAIN_RELU2: max(x, 0)^2.  PLAIN_XIELU:
-    x > 0: p0 x^2 + x/2, else (1/2 + p1) (e^x - 1 - x) + x/2."""
+    x > 0: p0 x^2 + x/2, else (1/2 + p1) (e^x - 1 - x) + x/2.  PLAIN_GELU_ERF: x/2 (1 + erf(x / sqrt 2))."""
     _need_strided(x, torch.float32, "x")
-    if act not in (PLAIN_RELU2, PLAIN_XIELU) or x.shape[1] < out.shape[1] or min(x.shape[0], out.shape[0]) < rows:
+    if act not in (PLAIN_RELU2, PLAIN_XIELU, PLAIN_GELU_ERF) or x.shape[1] < out.shape[1] or min(x.shape[0], out.shape[0]) < rows:
         raise ValueError("activate: an unknown activation, or out does not fit x")
     _check(_fn("bw_activate")(x.data_ptr(), x.stride(0), out.data_ptr(), _act_out(out, "out"), out.stride(0), rows, out.shape[1],
                               int(act), float(p0), float(p1), _stream()), "activate")
@@ -1318,6 +1345,43 @@ def causal_conv(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tens
                                  int(max_seq_rows), out.data_ptr(), out.stride(0), int(silu), _stream()), "causal_conv")
 
 
+def conv_heads(x: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tensor], gate: torch.Tensor, a_off: int, b_off: int,
+               dt_bias: torch.Tensor, rate: torch.Tensor, key_heads: int, dim: int, seq_rows: torch.Tensor, slots: torch.Tensor,
+               positions: torch.Tensor, nseq: int, max_seq_rows: int, out: torch.Tensor, gates: torch.Tensor, qscale: float,
+               eps: float) -> None:
+    """What a delta memory reads, in one launch.  ``x`` [rows, q | k | v] float32 (a column slice will do): ``key_heads`` heads of
+    ``dim`` channels of queries, as many of keys, then the values' channels.  Every channel passes the causal convolution of
+    ``causal_conv`` (weight [channels, taps] float32, ``state`` likewise) and SiLU; a head of q or k is then divided by
+    sqrt(sum x^2 + eps), q also multiplied by ``qscale``; to ``out``, x's layout.  ``gates`` [rows, 2*heads] receives
+    sigmoid(gate[:, b_off + h]) and, behind the heads, exp(-rate[h] * softplus(gate[:, a_off + h] + dt_bias[h]))."""
+    for t, what in ((x, "x"), (gate, "gate"), (out, "out"), (gates, "gates")):
+        _need_strided(t, torch.float32, what)
+    for t, what in ((weight, "weight"), (dt_bias, "dt_bias"), (rate, "rate")):
+        _need(t, torch.float32, what)
+    for t, what in ((seq_rows, "seq_rows"), (slots, "slots"), (positions, "positions")):
+        _need(t, torch.int32, what)
+    channels, taps = weight.shape
+    heads = dt_bias.numel()
+    if not 1 <= taps <= CONV_MAX_TAPS or not 1 <= dim <= RECUR_MAX_DIM:
+        raise ValueError(f"conv_heads: {taps} taps of heads of {dim}; the kernel takes 1 to {CONV_MAX_TAPS} and heads of up to {RECUR_MAX_DIM}")
+    if key_heads < 1 or channels <= 2 * key_heads * dim or x.shape[1] < channels or out.shape[1] < channels:
+        raise ValueError("conv_heads: x, out or the weight do not fit the heads")
+    if rate.numel() != heads or gates.shape[1] < 2 * heads or max(a_off, b_off) + heads > gate.shape[1] or min(a_off, b_off) < 0:
+        raise ValueError("conv_heads: gates, rates or biases do not fit the heads")
+    if seq_rows.numel() < 2 * nseq or slots.numel() < nseq:
+        raise ValueError("conv_heads: fewer request records than requests")
+    sp, sld = 0, 0
+    if taps > 1:
+        if state is None or state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < (taps - 1) * channels:
+            raise ValueError(f"conv_heads: a state slot needs {(taps - 1) * channels} float32 elements")
+        sp, sld = state.data_ptr(), state.stride(0)
+    _check(_fn("bw_conv_heads")(x.data_ptr(), x.stride(0), weight.data_ptr(), taps, int(key_heads), int(dim), channels - 2 * key_heads * dim,
+                                float(qscale), float(eps), sp, sld, gate.data_ptr(), gate.stride(0), int(a_off), int(b_off),
+                                dt_bias.data_ptr(), rate.data_ptr(), heads, gates.data_ptr(), gates.stride(0), seq_rows.data_ptr(),
+                                slots.data_ptr(), positions.data_ptr(), int(nseq), int(max_seq_rows), out.data_ptr(), out.stride(0),
+                                _stream()), "conv_heads")
+
+
 def pair_rope_unit(src: torch.Tensor, positions: torch.Tensor, row_seq: torch.Tensor, block_table: torch.Tensor,
                    cos: torch.Tensor, sin: torch.Tensor, q_out: torch.Tensor, k_cache: Optional[torch.Tensor],
                    v_cache: Optional[torch.Tensor], rows: int, heads: int, kv_heads: int, dim: int, vdim: int, head_size: int,
@@ -1367,13 +1431,16 @@ def whole_norm_kv(src: torch.Tensor, positions: torch.Tensor, row_seq: torch.Ten
                   q_weight: torch.Tensor, k_weight: torch.Tensor, eps: float, q_out: torch.Tensor, k_cache: torch.Tensor,
                   v_cache: torch.Tensor, rows: int, heads: int, kv_heads: int, dim: int, vdim: int, head_size: int,
                   page_size: int, write_cache: bool, v_first: Optional[torch.Tensor] = None,
-                  mix: Optional[torch.Tensor] = None, v_keep: Optional[torch.Tensor] = None) -> None:
+                  mix: Optional[torch.Tensor] = None, v_keep: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None,
+                  cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None, rot: int = 0, halves: bool = False) -> None:
     """Queries and keys of ``src`` [rows, q | k | v] (32-bit) normed over their whole projection, all heads at once,
     x / sqrt(mean(x^2) + eps) * weight; the queries go to ``q_out`` [rows, heads * head_size] and keys and values into
     the row's place in the paged cache, heads padded with zeros to ``head_size``.  ``v_first`` [rows, kv_heads * vdim]
     (32-bit) with ``mix`` (one 32-bit number on the device): the values are stored as (1 - mix) v + mix v_first.
-    ``v_keep``: receives the values as projected."""
-    _need(src, torch.float32, "src")
+    ``v_keep``: receives the values as projected.  ``bias`` [q | k | v] (32-bit; without ``write_cache`` q's part will do): added to the
+    projections first.  ``rot`` > 0: behind the norm the heads' first ``rot`` elements are rotated as in ``pair_rope_unit``.
+    ``src`` may be a column slice of a wider product."""
+    _need_strided(src, torch.float32, "src")
     _need(q_weight, torch.float32, "q_weight")
     _need(k_weight, torch.float32, "k_weight")
     for t, what in ((positions, "positions"), (row_seq, "row_seq"), (block_table, "block_table")):
@@ -1383,13 +1450,22 @@ def whole_norm_kv(src: torch.Tensor, positions: torch.Tensor, row_seq: torch.Ten
         raise ValueError("whole_norm_kv: the queries and the cache have one dtype")
     if src.shape[0] < rows or q_out.shape[0] < rows or q_out.shape[1] != heads * head_size:
         raise ValueError("whole_norm_kv: src or q_out do not fit")
-    if q_weight.numel() != heads * dim or k_weight.numel() != kv_heads * dim:
+    if q_weight.numel() != heads * dim or (write_cache and k_weight.numel() != kv_heads * dim):
         raise ValueError("whole_norm_kv: the norms' weights cover the whole projections")
     if src.shape[1] < heads * dim + (kv_heads * (dim + vdim) if write_cache else 0):
         raise ValueError("whole_norm_kv: src is narrower than the projections")
     page_elems = kv_heads * page_size * head_size
     if k_cache.shape[-1] != page_elems or v_cache.shape[-1] != page_elems:
         raise ValueError("whole_norm_kv: the cache's pages do not fit")
+    if bias is not None:
+        _need(bias, torch.float32, "bias")
+        if bias.numel() < heads * dim + (kv_heads * (dim + vdim) if write_cache else 0):
+            raise ValueError("whole_norm_kv: a bias for every projected channel")
+    if rot:
+        _need(cos, torch.float32, "cos table")
+        _need(sin, torch.float32, "sin table")
+        if rot % 2 or rot > dim or cos.shape[1] != rot // 2 or sin.shape != cos.shape:
+            raise ValueError("whole_norm_kv: rotary tables must be [positions, rot/2]")
     for t, what in ((v_first, "v_first"), (v_keep, "v_keep")):
         if t is not None:
             _need(t, torch.float32, what)
@@ -1405,20 +1481,22 @@ def whole_norm_kv(src: torch.Tensor, positions: torch.Tensor, row_seq: torch.Ten
                                    block_table.stride(0), q_weight.data_ptr(), k_weight.data_ptr(), float(eps), ptr(v_first),
                                    ld(v_first), ptr(mix) if v_first is not None else 0, ptr(v_keep), ld(v_keep), q_out.data_ptr(),
                                    k_cache.data_ptr(), v_cache.data_ptr(), is_bf16, rows, heads, kv_heads, dim, vdim, head_size,
-                                   page_size, int(bool(write_cache)), _stream()), "whole_norm_kv")
+                                   page_size, int(bool(write_cache)), ptr(bias), ptr(cos) if rot else 0, ptr(sin) if rot else 0,
+                                   int(rot), int(halves), _stream()), "whole_norm_kv")
 
 
-def gate_mul(av: torch.Tensor, head_size: int, g: torch.Tensor, out: torch.Tensor, rows: int, heads: int, vdim: int,
+def gate_mul(av: torch.Tensor, head_size: int, g: Optional[torch.Tensor], out: torch.Tensor, rows: int, heads: int, vdim: int,
              per_head: bool = False) -> None:
     """out[r, h*vdim + d] = av[r, h*head_size + d] * sigmoid(g[r, h*vdim + d]), or with ``per_head`` * sigmoid(g[r, h]);
-    ``g`` float32 (a column slice will do)."""
-    if g.dtype != torch.float32 or g.stride(1) != 1 or g.shape[1] < (heads if per_head else heads * vdim):
+    ``g`` float32 (a column slice will do), or None: the heads are only compacted."""
+    if g is not None and (g.dtype != torch.float32 or g.stride(1) != 1 or g.shape[1] < (heads if per_head else heads * vdim)):
         raise ValueError("gate_mul: g must be float32 with contiguous rows of heads*vdim (a gate a head: of heads)")
     if av.shape[1] != heads * head_size or out.shape[1] != heads * vdim or vdim > head_size:
         raise ValueError("gate_mul: av or out do not fit")
-    if min(av.shape[0], out.shape[0], g.shape[0]) < rows:
+    if min(av.shape[0], out.shape[0]) < rows or (g is not None and g.shape[0] < rows):
         raise ValueError("gate_mul: buffers shorter than the rows")
-    _check(_fn("bw_gate_mul")(av.data_ptr(), _act_out(av, "av"), av.stride(0), head_size, g.data_ptr(), g.stride(0), out.data_ptr(),
+    _check(_fn("bw_gate_mul")(av.data_ptr(), _act_out(av, "av"), av.stride(0), head_size, 0 if g is None else g.data_ptr(),
+                              0 if g is None else g.stride(0), out.data_ptr(),
                               _act_out(out, "out"), out.stride(0), rows, heads, vdim, int(per_head), _stream()), "gate_mul")
 
 
@@ -1482,6 +1560,67 @@ def norm_add(y: torch.Tensor, weight: torch.Tensor, x: torch.Tensor, rows: int, 
                               0 if rounded is None else rounded.data_ptr(), 0 if rounded is None else rounded.stride(0),
                               rows, dim, float(eps), 0 if place is None else place.data_ptr(), 0 if wts is None else wts.data_ptr(),
                               int(top), float(scale), _stream()), "norm_add")
+
+
+def _branches(ys: Sequence[torch.Tensor], scales: Sequence[float], rows: int, dim: int, what: str):
+    n = len(ys)
+    if not 1 <= n <= 4 or len(scales) != n:
+        raise ValueError(f"{what}: one to four inputs, a number each")
+    for y in ys:
+        _need_strided(y, torch.float32, "input")
+        if y.shape[1] != dim or y.shape[0] < rows:
+            raise ValueError(f"{what}: the inputs must have the output's width")
+    cast = lambda a: ctypes.cast(a, c_void_p)
+    return (cast((c_void_p * n)(*[y.data_ptr() for y in ys])), cast((c_int * n)(*[y.stride(0) for y in ys])),
+            cast((c_float * n)(*[float(s) for s in scales])), n)
+
+
+def scaled_sum(ys: Sequence[torch.Tensor], scales: Sequence[float], out: torch.Tensor, rows: int) -> None:
+    """out[:rows] = sum over b of scales[b] * ys[b][:rows], b ascending, 32-bit: up to four matrices of one width."""
+    _need(out, torch.float32, "out")
+    if out.shape[0] < rows:
+        raise ValueError("scaled_sum: out is shorter than the rows")
+    yp, ld, sc, n = _branches(ys, scales, rows, out.shape[1], "scaled_sum")
+    _check(_fn("bw_scaled_sum")(yp, ld, sc, n, out.data_ptr(), out.stride(0), rows, out.shape[1], _stream()), "scaled_sum")
+
+
+def scaled_sum_norm_add(ys: Sequence[torch.Tensor], scales: Sequence[float], weight: torch.Tensor, eps: float, scale: float,
+                        x: torch.Tensor, rows: int, rounded: Optional[torch.Tensor] = None) -> None:
+    """x[:rows] += scale * (z / sqrt(mean(z^2) + eps) * weight) with z the sum of ``scaled_sum``; ``rounded`` as in ``norm_add``: one
+    launch, the bits of ``scaled_sum`` followed by ``norm_add``."""
+    _need(x, torch.float32, "x")
+    _need(weight, torch.float32, "weight")
+    dim = x.shape[1]
+    if x.shape[0] < rows or weight.numel() != dim:
+        raise ValueError("scaled_sum_norm_add: weight and x do not fit")
+    if rounded is not None:
+        _need(rounded, torch.bfloat16, "rounded")
+        if rounded.shape[1] != dim or rounded.shape[0] < rows:
+            raise ValueError("scaled_sum_norm_add: the rounded copy does not fit")
+    yp, ld, sc, n = _branches(ys, scales, rows, dim, "scaled_sum_norm_add")
+    _check(_fn("bw_scaled_sum_norm_add")(yp, ld, sc, n, weight.data_ptr(), float(eps), float(scale), x.data_ptr(), x.stride(0),
+                                         0 if rounded is None else rounded.data_ptr(), 0 if rounded is None else rounded.stride(0),
+                                         rows, dim, _stream()), "scaled_sum_norm_add")
+
+
+def side_gate(z: torch.Tensor, tokens: torch.Tensor, feedback: Optional[torch.Tensor], table: torch.Tensor, out: torch.Tensor,
+              rows: int) -> None:
+    """out[r, d] = gelu_tanh(z[r, d]) * table[token of r, d]; ``z`` float32 and ``table`` [vocab, dim] may be column slices; tokens
+    as in ``embed`` (a negative one gives zeros, or the row's token from ``feedback``); out float32 or bfloat16."""
+    _need_strided(z, torch.float32, "z")
+    _need(tokens, torch.int32, "tokens")
+    if not table.is_cuda or table.dim() != 2 or table.stride(1) != 1:
+        raise ValueError("side_gate: the table must be a GPU matrix with contiguous rows")
+    dim = out.shape[1]
+    if z.shape[1] < dim or table.shape[1] != dim or min(z.shape[0], out.shape[0], tokens.numel()) < rows:
+        raise ValueError("side_gate: z, table and out do not fit")
+    if feedback is not None:
+        _need(feedback, torch.int32, "feedback")
+        if feedback.numel() < rows:
+            raise ValueError("side_gate: feedback is shorter than the rows")
+    _check(_fn("bw_side_gate")(z.data_ptr(), z.stride(0), tokens.data_ptr(), 0 if feedback is None else feedback.data_ptr(), table.data_ptr(),
+                               _is_bf16(table, "table"), table.stride(0), table.shape[0], out.data_ptr(), _act_out(out, "out"), out.stride(0),
+                               rows, dim, _stream()), "side_gate")
 
 
 def softcap(x: torch.Tensor, rows: int, cap: float) -> None:

@@ -29,6 +29,8 @@ __device__ __forceinline__ float softplus(float z) {
   return fmaxf(z, 0.0f) + log1pf(bw_expf(-fabsf(z)));
 }
 
+__device__ __forceinline__ float silu(float z) { return z * (1.0f / (1.0f + bw_expf(-z))); }
+
 template <typename OT>
 __device__ __forceinline__ void store_act(OT* p, float v) {
   if constexpr (sizeof(OT) == 2) *p = f32_to_bf16(v);
@@ -250,7 +252,7 @@ __global__ __launch_bounds__(256) void norm_shift_row_kernel(const float* __rest
 
 // ------------------------------------------------------------------------- the linear recurrence
 
-enum { RECUR_DECAY_PER_CHANNEL = 0, RECUR_SCALAR_GATES = 1, RECUR_BONUS_DECAY = 2, RECUR_FIXED_DECAY = 3, RECUR_STEP_DECAY = 4 };
+enum { RECUR_DECAY_PER_CHANNEL = 0, RECUR_SCALAR_GATES = 1, RECUR_BONUS_DECAY = 2, RECUR_FIXED_DECAY = 3, RECUR_STEP_DECAY = 4, RECUR_DELTA = 5 };
 
 // The sum over the SPLIT lanes that hold the parts of one column, l, l + 64/SPLIT, ... (every one of them gets it).
 template <int SPLIT>
@@ -280,6 +282,7 @@ struct RecurArgs {
   int heads_per_key;       // neighbouring heads that share one q and one k (1: every head has its own)
   float param;             // per channel: 1 / tau; scalar gates: the cap
   float qscale, kscale;
+  int silu;                // fixed decay: q, k and v pass SiLU on their way into LDS
   float* state;            // [slots, state_ld]: S [heads][vdim][dim]; scalar gates then, per
                            // workgroup of a head, n [heads][dim] and m [heads]
   long long state_ld;
@@ -315,6 +318,9 @@ struct RecurArgs {
 // RECUR_FIXED_DECAY:  as per channel with one constant decay a head, alpha[d] = bias[head]; no logits are read.
 // RECUR_STEP_DECAY:  a step size per head and token, delta = softplus(z + bias[head]) with z at gate_off + head;
 //   S[d][j] <- e^(-bias2[head] delta) S[d][j] + k[d] (delta v[j]),  o[j] = (S^T q)[j] + skip[head] v[j].
+// RECUR_DELTA:  a step size beta (at gate_off + head) and a decay a (at gate2_off + head) per head and token, as they are;
+//   u[j] = beta (v[j] - a (S^T k)[j]),  S[d][j] <- a S[d][j] + k[d] u[j],  o[j] = (S^T q)[j]: what k reads is replaced towards v.
+//   (The step of a chunk as a whole is a full matrix and not a decay, so there are no passes over chunks.)
 // (a head's q and k are those of key group head / heads_per_key.)
 // (q is multiplied by qscale and k by kscale on their way into LDS.)
 //
@@ -345,7 +351,8 @@ template <int MODE, int DPAD, int PHASE>
 __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a) {
   constexpr bool GATES = MODE == RECUR_SCALAR_GATES;
   constexpr bool BONUS = MODE == RECUR_BONUS_DECAY, FIXED = MODE == RECUR_FIXED_DECAY, STEP = MODE == RECUR_STEP_DECAY;
-  constexpr bool CHANNELS = !GATES && !STEP;             // a decay per channel comes through LDS
+  constexpr bool DELTA = MODE == RECUR_DELTA;
+  constexpr bool CHANNELS = !GATES && !STEP && !DELTA;   // a decay per channel comes through LDS
   constexpr int NN = (DPAD + 63) / 64;
   constexpr bool READ_OUT = PHASE != 1;
   constexpr int SPLIT = PHASE == 0 ? recur_split(DPAD) : recur_chunk_split(DPAD);
@@ -458,10 +465,10 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         rv[u] = a.proj[row * a.ldp + a.v_off + h * vdim + min(j_wg + e % WCOLS, vdim - 1)];
       }
     }
-    if constexpr (GATES || STEP) {
+    if constexpr (GATES || STEP || DELTA) {
       const float* gr = a.gate + (size_t)(first + t0 + min((int)threadIdx.x, tc - 1)) * a.ldg;
       rg[0] = gr[a.gate_off + h];
-      rg[1] = GATES ? gr[a.gate2_off + h] : 0.0f;
+      rg[1] = GATES || DELTA ? gr[a.gate2_off + h] : 0.0f;
     }
   };
   auto stash = [&](int t0, int buf) {
@@ -473,6 +480,12 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         const int e = 64 * RW * u + (int)threadIdx.x;
         const int t = e / DPAD, d = e % DPAD;
         const bool in = d < dim;
+        if constexpr (FIXED) {
+          if (a.silu) {                                  // (scalar)
+            rq[u] = silu(rq[u]);
+            rk[u] = silu(rk[u]);
+          }
+        }
         qs[buf][t][d] = in ? rq[u] * a.qscale : 0.0f;
         ks[buf][t][d] = in ? rk[u] * a.kscale : 0.0f;
         if constexpr (FIXED) as[buf][t][d] = in ? fixed_decay : 0.0f;
@@ -483,6 +496,9 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       const int e = 64 * RW * u + (int)threadIdx.x;
+      if constexpr (FIXED) {
+        if (a.silu) rv[u] = silu(rv[u]);
+      }
       if (64 * RW * u < tc * WCOLS && e < RC * WCOLS) vs[buf][e / WCOLS][e % WCOLS] = j_wg + e % WCOLS < vdim ? rv[u] : 0.0f;
     }
     if constexpr (GATES) {
@@ -490,6 +506,12 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         const float cap = a.param;
         gi[buf][threadIdx.x] = cap * tanhf((rg[0] + a.bias[h]) / cap);
         gf[buf][threadIdx.x] = log_sigmoid(cap * tanhf((rg[1] + a.bias2[h]) / cap));
+      }
+    }
+    if constexpr (DELTA) {
+      if ((int)threadIdx.x < tc) {
+        gi[buf][threadIdx.x] = rg[0];
+        gf[buf][threadIdx.x] = rg[1];
       }
     }
     if constexpr (STEP) {
@@ -523,7 +545,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         }
       }
       vr[n] = vs[buf][t + n][j_in];
-      if constexpr (GATES || STEP) {
+      if constexpr (GATES || STEP || DELTA) {
         g1[n] = gi[buf][t + n];
         g2[n] = gf[buf][t + n];
       }
@@ -541,6 +563,20 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         if constexpr (PHASE == 1) {
 #pragma unroll
           for (int i = 0; i < NN; ++i) nreg[i] *= fa;
+        }
+      } else if constexpr (DELTA) {
+        // (two chains over a lane's channels, then the column's lanes: the one sum the next token waits for)
+        float r0 = 0.0f, r1 = 0.0f;
+#pragma unroll
+        for (int d = 0; d < DH; d += 2) {
+          r0 = fmaf(Sreg[d], kr[n][d], r0);
+          r1 = fmaf(Sreg[d + 1], kr[n][d + 1], r1);
+        }
+        const float fa = g2[n], u = g1[n] * fmaf(-fa, join_parts<SPLIT>(r0 + r1), vr[n]);
+#pragma unroll
+        for (int d = 0; d < DH; ++d) {
+          Sreg[d] = fmaf(fa, Sreg[d], kr[n][d] * u);
+          o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
         }
       } else if constexpr (!GATES) {
 #pragma unroll
@@ -721,13 +757,17 @@ int launch_recurrence_passes(const RecurArgs& a, int nseq, int nchunks, const in
   int rc = 0;
   if (nseq > 0) rc = launch_recurrence<MODE, 0>(a, nseq, s);
   if (rc != 0 || nchunks <= 0) return rc;
-  rc = launch_recurrence<MODE, 1>(a, nchunks, s);
-  if (rc != 0) return rc;
-  const int mine = a.dim * a.vdim + (MODE == RECUR_SCALAR_GATES ? a.dim + 1 : 0);
-  hipLaunchKernelGGL(recurrence_scan_kernel<MODE>, dim3((mine + 255) / 256, a.heads, nspans), dim3(256), 0, s, a, spans);
-  rc = BW_LAUNCH_CHECK();
-  if (rc != 0) return rc;
-  return launch_recurrence<MODE, 3>(a, nchunks, s);
+  if constexpr (MODE == RECUR_DELTA) {
+    return -2;
+  } else {
+    rc = launch_recurrence<MODE, 1>(a, nchunks, s);
+    if (rc != 0) return rc;
+    const int mine = a.dim * a.vdim + (MODE == RECUR_SCALAR_GATES ? a.dim + 1 : 0);
+    hipLaunchKernelGGL(recurrence_scan_kernel<MODE>, dim3((mine + 255) / 256, a.heads, nspans), dim3(256), 0, s, a, spans);
+    rc = BW_LAUNCH_CHECK();
+    if (rc != 0) return rc;
+    return launch_recurrence<MODE, 3>(a, nchunks, s);
+  }
 }
 
 // ------------------------------------------------------------------------- per-head RMS norm and output gate
@@ -758,17 +798,18 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   }
 }
 
-// ------------------------------------------------------------------------- output gate, then an RMS norm in equal parts
+// ------------------------------------------------------------------------- output gate and an RMS norm in equal parts
 
-// v = o[r][e] * silu(z[r][e]); out = v / sqrt(mean of v^2 over the part + eps) * weight[e], a row's parts being equal stretches
-// of ``size`` elements.  A workgroup per (row, part): thread t owns elements t, t + 256, ... (one chain over its squares),
-// the waves' sums are joined by wave_sum and added in wave order.  Parts of up to 256 GP_MAXV elements keep their values in
-// registers; the same chain either way.
+// A row's parts are equal stretches of ``size`` elements.  BEHIND false: v = o[r][e] * act(z[r][e]), out = v / sqrt(mean of v^2
+// over the part + eps) * weight[e].  BEHIND true: v = o[r][e], and the norm's result is multiplied by act(z[r][e]).  act: SiLU
+// or sigmoid.  A workgroup per (row, part): thread t owns elements t, t + 256, ... (one chain over its squares), the waves'
+// sums are joined by wave_sum and added in wave order.  Parts of up to 256 GP_MAXV elements keep their values in registers;
+// the same chain either way.
 #define GP_MAXV 8
-template <typename OT>
+template <typename OT, bool BEHIND>
 __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __restrict__ o, int ldi, const float* __restrict__ z, int ldz,
                                                               const float* __restrict__ weight, OT* __restrict__ out, int ldo,
-                                                              const int32_t* __restrict__ positions, int size, float eps) {
+                                                              const int32_t* __restrict__ positions, int size, float eps, int gate) {
   __shared__ float part[4];
   const int row = blockIdx.x, base = blockIdx.y * size, tid = threadIdx.x;
   if (positions[row] < 0) return;
@@ -776,12 +817,20 @@ __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __res
   const float* zrow = z + (size_t)row * ldz + base;
   const float* wr = weight + base;
   OT* dst = out + (size_t)row * ldo + base;
-  auto gated = [](float ov, float zv) { return ov * (zv * (1.0f / (1.0f + bw_expf(-zv)))); };
+  auto act = [&](float zv) {
+    const float sg = 1.0f / (1.0f + bw_expf(-zv));
+    return gate == GATE_SILU ? zv * sg : sg;
+  };
+  auto before = [&](float ov, float zv) { return BEHIND ? ov : ov * act(zv); };
+  auto after = [&](float v, float inv, float we, float zv) {
+    const float y = (v * inv) * we;
+    return BEHIND ? y * act(zv) : y;
+  };
   const bool small = size <= 256 * GP_MAXV;
-  float v[GP_MAXV];
+  float v[GP_MAXV], zv[GP_MAXV];
   float acc = 0.0f;
   if (small) {
-    float ov[GP_MAXV], zv[GP_MAXV];
+    float ov[GP_MAXV];
 #pragma unroll
     for (int j = 0; j < GP_MAXV; ++j) {
       const int e = min(tid + 256 * j, size - 1);
@@ -790,12 +839,12 @@ __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __res
     }
 #pragma unroll
     for (int j = 0; j < GP_MAXV; ++j) {
-      v[j] = tid + 256 * j < size ? gated(ov[j], zv[j]) : 0.0f;
+      v[j] = tid + 256 * j < size ? before(ov[j], zv[j]) : 0.0f;
       acc = fmaf(v[j], v[j], acc);
     }
   } else {
     for (int e = tid; e < size; e += 256) {
-      const float ve = gated(orow[e], zrow[e]);
+      const float ve = before(orow[e], zrow[e]);
       acc = fmaf(ve, ve, acc);
     }
   }
@@ -807,10 +856,10 @@ __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __res
 #pragma unroll
     for (int j = 0; j < GP_MAXV; ++j) {
       const int e = tid + 256 * j;
-      if (e < size) store_act(dst + e, (v[j] * inv) * wr[e]);
+      if (e < size) store_act(dst + e, after(v[j], inv, wr[e], zv[j]));
     }
   } else {
-    for (int e = tid; e < size; e += 256) store_act(dst + e, (gated(orow[e], zrow[e]) * inv) * wr[e]);
+    for (int e = tid; e < size; e += 256) store_act(dst + e, after(before(orow[e], zrow[e]), inv, wr[e], zrow[e]));
   }
 }
 
@@ -843,8 +892,8 @@ __global__ void glu_kernel(const float* __restrict__ gu, int ldg, OT* __restrict
 // ------------------------------------------------------------------------- activation without a gate
 
 // h = act(z) of a 32-bit product.  PLAIN_RELU2: max(z, 0)^2.  PLAIN_XIELU (p0 and p1 positive): z > 0: p0 z^2 + z/2;
-// z <= 0: (1/2 + p1) (e^z - 1 - z) + z/2.
-enum { PLAIN_RELU2 = 0, PLAIN_XIELU = 1 };
+// z <= 0: (1/2 + p1) (e^z - 1 - z) + z/2.  PLAIN_GELU_ERF: z/2 (1 + erf(z / sqrt 2)).
+enum { PLAIN_RELU2 = 0, PLAIN_XIELU = 1, PLAIN_GELU_ERF = 2 };
 
 template <typename OT>
 __global__ __launch_bounds__(256) void activate_kernel(const float* __restrict__ x, int ldx, OT* __restrict__ out, int ldo, int rows,
@@ -856,6 +905,8 @@ __global__ __launch_bounds__(256) void activate_kernel(const float* __restrict__
     float h;
     if (act == PLAIN_XIELU) {
       h = z > 0.0f ? fmaf(p0 * z, z, 0.5f * z) : fmaf(0.5f + p1, expm1f(z) - z, 0.5f * z);
+    } else if (act == PLAIN_GELU_ERF) {
+      h = (0.5f * z) * (1.0f + erff(z * 0.7071067811865476f));
     } else {
       const float m = fmaxf(z, 0.0f);
       h = m * m;
@@ -905,6 +956,16 @@ __global__ __launch_bounds__(256) void tanh_rows_kernel(float* __restrict__ x, i
   *p = tanhf(*p);
 }
 
+// x <- silu(x) likewise
+__global__ __launch_bounds__(256) void silu_rows_kernel(float* __restrict__ x, int ld, int rows, int cols) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= cols) return;
+  for (int r = blockIdx.y; r < rows; r += gridDim.y) {
+    float* p = x + (size_t)r * ld + c;
+    *p = silu(*p);
+  }
+}
+
 }  // namespace
 
 extern "C" int bw_norm_shift(const float* x, int ldx, const float* w, const float* mix, float* state, long long state_ld,
@@ -937,7 +998,7 @@ extern "C" int bw_norm_shift(const float* x, int ldx, const float* w, const floa
 
 extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_off, int k_off, int v_off, const float* gate,
                                     int ldg, int gate_off, int gate2_off, const float* bias, const float* bias2, float param,
-                                    float qscale, float kscale, const float* skip, int heads_per_key, float* state, long long state_ld, float* out, int ldo,
+                                    float qscale, float kscale, const float* skip, int heads_per_key, int silu, float* state, long long state_ld, float* out, int ldo,
                                     const int32_t* seq_rows, const int32_t* slots, const int32_t* positions, int nseq,
                                     int heads, int dim, int vdim, const int32_t* chunks, int nchunks, const int32_t* spans,
                                     int nspans, float* scan_local, float* scan_start, long long scan_floats, void* stream) {
@@ -949,9 +1010,10 @@ extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_
   if (heads <= 0 || dim <= 0 || vdim <= 0 || ldo < heads * vdim || heads_per_key < 1 || heads % heads_per_key) return -2;
   const long long need = (long long)heads * dim * vdim + (mode == RECUR_SCALAR_GATES ? (long long)recur_blocks(dim, vdim) * ((long long)heads * dim + heads) : 0);
   if (state_ld < need) return -2;
-  if (bias == nullptr || (mode != RECUR_FIXED_DECAY && gate == nullptr) || ((mode == RECUR_SCALAR_GATES || mode == RECUR_BONUS_DECAY || mode == RECUR_STEP_DECAY) && bias2 == nullptr))
+  if (silu && mode != RECUR_FIXED_DECAY) return -2;
+  if ((bias == nullptr && mode != RECUR_DELTA) || (mode != RECUR_FIXED_DECAY && gate == nullptr) || ((mode == RECUR_SCALAR_GATES || mode == RECUR_BONUS_DECAY || mode == RECUR_STEP_DECAY) && bias2 == nullptr))
     return -2;
-  RecurArgs a{proj, ldp, q_off, k_off, v_off, gate, ldg, gate_off, gate2_off, bias, bias2, skip, heads_per_key, param, qscale, kscale, state, state_ld,
+  RecurArgs a{proj, ldp, q_off, k_off, v_off, gate, ldg, gate_off, gate2_off, bias, bias2, skip, heads_per_key, param, qscale, kscale, silu, state, state_ld,
               out, ldo, seq_rows, slots, positions, heads, dim, vdim, chunks, scan_local, scan_start};
   hipStream_t s = (hipStream_t)stream;
   if (mode == RECUR_SCALAR_GATES) return launch_recurrence_passes<RECUR_SCALAR_GATES>(a, nseq, nchunks, spans, nspans, s);
@@ -959,6 +1021,7 @@ extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_
   if (mode == RECUR_BONUS_DECAY) return launch_recurrence_passes<RECUR_BONUS_DECAY>(a, nseq, nchunks, spans, nspans, s);
   if (mode == RECUR_FIXED_DECAY) return launch_recurrence_passes<RECUR_FIXED_DECAY>(a, nseq, nchunks, spans, nspans, s);
   if (mode == RECUR_STEP_DECAY) return launch_recurrence_passes<RECUR_STEP_DECAY>(a, nseq, nchunks, spans, nspans, s);
+  if (mode == RECUR_DELTA) return launch_recurrence_passes<RECUR_DELTA>(a, nseq, nchunks, spans, nspans, s);
   return -2;
 }
 
@@ -981,16 +1044,21 @@ extern "C" int bw_head_norm_gate(const float* o, int ldi, const float* weight, i
 }
 
 extern "C" int bw_gated_part_norm(const float* o, int ldi, const float* z, int ldz, const float* weight, void* out, int out_is_bf16,
-                                  int ldo, const int32_t* positions, int rows, int parts, int size, float eps, void* stream) {
+                                  int ldo, const int32_t* positions, int rows, int parts, int size, float eps, int gate, int behind,
+                                  void* stream) {
   if (rows <= 0) return 0;
   if (parts <= 0 || parts > 65535 || size <= 0 || ldi < parts * size || ldz < parts * size || ldo < parts * size) return -2;
+  if (gate != GATE_SIGMOID && gate != GATE_SILU) return -2;
   const dim3 grid(rows, parts), block(256);
-  if (out_is_bf16)
-    hipLaunchKernelGGL(gated_part_norm_kernel<bf16_t>, grid, block, 0, (hipStream_t)stream, o, ldi, z, ldz, weight, (bf16_t*)out, ldo,
-                       positions, size, eps);
+  hipStream_t s = (hipStream_t)stream;
+  if (out_is_bf16 && behind)
+    hipLaunchKernelGGL((gated_part_norm_kernel<bf16_t, true>), grid, block, 0, s, o, ldi, z, ldz, weight, (bf16_t*)out, ldo, positions, size, eps, gate);
+  else if (out_is_bf16)
+    hipLaunchKernelGGL((gated_part_norm_kernel<bf16_t, false>), grid, block, 0, s, o, ldi, z, ldz, weight, (bf16_t*)out, ldo, positions, size, eps, gate);
+  else if (behind)
+    hipLaunchKernelGGL((gated_part_norm_kernel<float, true>), grid, block, 0, s, o, ldi, z, ldz, weight, (float*)out, ldo, positions, size, eps, gate);
   else
-    hipLaunchKernelGGL(gated_part_norm_kernel<float>, grid, block, 0, (hipStream_t)stream, o, ldi, z, ldz, weight, (float*)out, ldo,
-                       positions, size, eps);
+    hipLaunchKernelGGL((gated_part_norm_kernel<float, false>), grid, block, 0, s, o, ldi, z, ldz, weight, (float*)out, ldo, positions, size, eps, gate);
   return BW_LAUNCH_CHECK();
 }
 
@@ -1010,7 +1078,7 @@ extern "C" int bw_glu(const float* gate_up, int ldg, void* h, int out_is_bf16, i
 extern "C" int bw_activate(const float* x, int ldx, void* out, int out_is_bf16, int ldo, int rows, int cols, int act, float p0,
                            float p1, void* stream) {
   if (rows <= 0 || cols <= 0) return 0;
-  if (ldx < cols || ldo < cols || (act != PLAIN_RELU2 && act != PLAIN_XIELU)) return -2;
+  if (ldx < cols || ldo < cols || (act != PLAIN_RELU2 && act != PLAIN_XIELU && act != PLAIN_GELU_ERF)) return -2;
   const dim3 grid((cols + 255) / 256, rows < 65535 ? rows : 65535), block(256);
   if (out_is_bf16) hipLaunchKernelGGL(activate_kernel<bf16_t>, grid, block, 0, (hipStream_t)stream, x, ldx, (bf16_t*)out, ldo, rows, cols, act, p0, p1);
   else hipLaunchKernelGGL(activate_kernel<float>, grid, block, 0, (hipStream_t)stream, x, ldx, (float*)out, ldo, rows, cols, act, p0, p1);
@@ -1033,5 +1101,12 @@ extern "C" int bw_tanh_rows(float* x, int ld, int rows, int cols, void* stream) 
   if (ld < cols) return -2;
   const long long n = (long long)rows * cols;
   hipLaunchKernelGGL(tanh_rows_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, (hipStream_t)stream, x, ld, rows, cols);
+  return BW_LAUNCH_CHECK();
+}
+
+extern "C" int bw_silu_rows(float* x, int ld, int rows, int cols, void* stream) {
+  if (rows <= 0 || cols <= 0) return 0;
+  if (ld < cols) return -2;
+  hipLaunchKernelGGL(silu_rows_kernel, dim3((cols + 255) / 256, rows < 65535 ? rows : 65535), dim3(256), 0, (hipStream_t)stream, x, ld, rows, cols);
   return BW_LAUNCH_CHECK();
 }

@@ -273,8 +273,9 @@ class Mixer(Part):
         columns, a slice of a wider matrix): mixers that stand side by side on one input then share one product."""
         return None
 
-    def forward_add_normed(self, ctx, call, h, norm, x) -> bool:
-        """Optional: x += norm(mixer(h)) with the norm behind the mixer riding in the mixer's last kernel.  Return False
+    def forward_add_normed(self, ctx, call, h, norm, x, rounded=None) -> bool:
+        """Optional: x += norm(mixer(h)) with the norm behind the mixer riding in the mixer's last kernel (``rounded`` as in
+        ``Norm.add_normed``).  Return False
         (and do nothing) if this part or this norm cannot; the block then calls ``forward_out`` and the norm one after
         the other.  The result must be the same bits."""
         return False
@@ -305,11 +306,21 @@ class FeedForward(Part):
         return False
 
 
+class SideInput(Part):
+    """Something a layer adds to the stream beside its sublayers' outputs, out of the stream and what the step's rows are
+    (their token ids)."""
+
+    def forward_add(self, ctx, h, x, rounded=None) -> None:
+        """x += the side input; ``h``: the stream x as products take it (in bfloat16 mode rounded); ``rounded`` as in
+        ``Norm.add_normed``."""
+        raise NotImplementedError
+
+
 class Block(Part):
     """The arrangement of a layer's parts around the residual stream.
 
     ``roles`` names the parts an arrangement has and the kind of each ("mixer", "feed_forward",
-    "norm"), in the order their tensors are listed; the built parts become attributes of those
+    "norm", "side_input"), in the order their tensors are listed; the built parts become attributes of those
     names.  Every arrangement has a role "mixer"."""
 
     roles: Dict[str, str] = {}
@@ -338,12 +349,13 @@ class Block(Part):
 MIXERS: Dict[str, Type[Mixer]] = {}
 FEED_FORWARDS: Dict[str, Type[FeedForward]] = {}
 NORMS: Dict[str, Type[Norm]] = {}
+SIDE_INPUTS: Dict[str, Type[SideInput]] = {}
 POSITION_ENCODINGS: Dict[str, Type[PositionEncoding]] = {}
 BLOCKS: Dict[str, Type[Block]] = {}
 EMBEDDINGS: Dict[str, Type[Embedding]] = {}
 HEADS: Dict[str, Type[Head]] = {}
 # the registry of every kind of part a block's role may name
-KINDS: Dict[str, Dict[str, type]] = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS}
+KINDS: Dict[str, Dict[str, type]] = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS, "side_input": SIDE_INPUTS}
 
 
 def _register(table: Dict[str, type], what: str) -> Callable[[str], Callable[[type], type]]:
@@ -360,6 +372,7 @@ def _register(table: Dict[str, type], what: str) -> Callable[[str], Callable[[ty
 register_mixer = _register(MIXERS, "mixer")
 register_feed_forward = _register(FEED_FORWARDS, "feed-forward")
 register_norm = _register(NORMS, "norm")
+register_side_input = _register(SIDE_INPUTS, "side input")
 register_position_encoding = _register(POSITION_ENCODINGS, "position encoding")
 register_block = _register(BLOCKS, "block")
 register_embedding = _register(EMBEDDINGS, "embedding")

@@ -70,10 +70,11 @@ class ParallelBlock(Block):
 class PostNormBlock(Block):
     """x += norm1(mixer(x)); x += norm2(feed_forward(x)): the sublayers read the residual stream itself (in bfloat16
     mode its rounding, the only rounding between the stream and a sublayer's products), and each sublayer's output is
-    normed on its way back into the stream.  A layer may leave the feed-forward (and its norm) out."""
+    normed on its way back into the stream.  A layer may leave the feed-forward (and its norm) out; it may end with a side
+    input, which also reads the stream itself."""
 
-    roles = {"mixer_norm": "norm", "ffn_norm": "norm", "mixer": "mixer", "feed_forward": "feed_forward"}
-    optional_roles = ("ffn_norm", "feed_forward")
+    roles = {"mixer_norm": "norm", "ffn_norm": "norm", "mixer": "mixer", "feed_forward": "feed_forward", "side_input": "side_input"}
+    optional_roles = ("ffn_norm", "feed_forward", "side_input")
     graph_safe = True
     launches_through_ops = True
 
@@ -95,27 +96,37 @@ class PostNormBlock(Block):
         return h
 
     def _add(self, ctx, norm, y, x) -> None:
-        notes = getattr(ctx, "forward_notes", None)
-        if self.rt.bf16 and notes is not None:
-            norm.add_normed(ctx, y, x, rounded=ctx.ws.buffer("stream_rounded", x.shape[1], torch.bfloat16))
-            notes["stream_rounded"] = x
-        else:
-            norm.add_normed(ctx, y, x)
+        norm.add_normed(ctx, y, x, rounded=self._rounded(ctx, x))
+        self._note_rounded(ctx, x)
+
+    def _rounded(self, ctx, x):
+        """Where a kernel that adds into the stream leaves the rounded copy, or None."""
+        if not self.rt.bf16 or getattr(ctx, "forward_notes", None) is None:
+            return None
+        return ctx.ws.buffer("stream_rounded", x.shape[1], torch.bfloat16)
+
+    def _note_rounded(self, ctx, x) -> None:
+        if self.rt.bf16 and getattr(ctx, "forward_notes", None) is not None:
+            ctx.forward_notes["stream_rounded"] = x
 
     def forward(self, ctx, call, x) -> None:
         y = ctx.ws.buffer("sublayer_out", x.shape[1], torch.float32)
-        self.mixer.forward_out(ctx, call, self._input(ctx, x), y)
-        self._add(ctx, self.mixer_norm, y, x)
+        h = self._input(ctx, x)
+        if self.mixer.forward_add_normed(ctx, call, h, self.mixer_norm, x, self._rounded(ctx, x)):
+            self._note_rounded(ctx, x)
+        else:
+            self.mixer.forward_out(ctx, call, h, y)
+            self._add(ctx, self.mixer_norm, y, x)
         if self.feed_forward is not None:
             h = self._input(ctx, x)
-            notes = getattr(ctx, "forward_notes", None)
-            rounded = ctx.ws.buffer("stream_rounded", x.shape[1], torch.bfloat16) if (self.rt.bf16 and notes is not None) else None
-            if self.feed_forward.forward_add_normed(ctx, h, self.ffn_norm, x, rounded):
-                if rounded is not None:
-                    notes["stream_rounded"] = x
+            if self.feed_forward.forward_add_normed(ctx, h, self.ffn_norm, x, self._rounded(ctx, x)):
+                self._note_rounded(ctx, x)
             else:
                 self.feed_forward.forward_out(ctx, h, y)
                 self._add(ctx, self.ffn_norm, y, x)
+        if self.side_input is not None:
+            self.side_input.forward_add(ctx, self._input(ctx, x), x, self._rounded(ctx, x))
+            self._note_rounded(ctx, x)
 
 
 @register_block("sandwich")

@@ -14,7 +14,9 @@ from .linear import Linear
 @register_embedding("embedding")
 class TokenEmbedding(Embedding):
     """params: vocab, width; optional ``norm`` = {tensor, eps}: the gathered row is divided by its root mean square and
-    multiplied by that weight vector before it becomes the stream.  tensor: weight [vocab, width], gathered as 32-bit rows."""
+    multiplied by that weight vector before it becomes the stream; optional ``side`` = {tensor, width}: a second table [vocab,
+    width] whose rows are not gathered here: layers that take a side input read their own columns of a token's row
+    (``ctx.forward_notes["token_side_table"]``).  tensor: weight [vocab, width], gathered as 32-bit rows."""
 
     graph_safe = True
     launches_through_ops = True
@@ -26,9 +28,13 @@ class TokenEmbedding(Embedding):
         self.weight: Optional[torch.Tensor] = None
         self.norm = dict(params["norm"]) if params.get("norm") else None
         self.norm_weight: Optional[torch.Tensor] = None
+        self.side = dict(params["side"]) if params.get("side") else None
+        self.side_table: Optional[torch.Tensor] = None
 
     def tensors(self) -> Dict[str, TensorSpec]:
         out = {self.tensor: TensorSpec((self.vocab, self.width), "embedding")}
+        if self.side is not None:
+            out[str(self.side["tensor"])] = TensorSpec((self.vocab, int(self.side["width"])), "embedding")
         if self.norm is not None:
             out[str(self.norm["tensor"])] = TensorSpec((self.width,), "norm")
         return out
@@ -37,12 +43,19 @@ class TokenEmbedding(Embedding):
         self.weight = tensors[self.tensor].to(self.rt.device).contiguous()
         if self.norm is not None:
             self.norm_weight = tensors[str(self.norm["tensor"])].to(self.rt.device).float().contiguous()
+        if self.side is not None:
+            self.side_table = tensors[str(self.side["tensor"])].to(self.rt.device).contiguous()
 
     def weight_bytes(self) -> int:
         return 0      # a step reads one row per token, not the table
 
+    def _note_side_table(self, ctx) -> None:
+        if self.side_table is not None:
+            ctx.forward_notes["token_side_table"] = self.side_table
+
     def forward(self, ctx) -> torch.Tensor:
         x = ctx.ws.buffer("residual", self.width, torch.float32)
+        self._note_side_table(ctx)
         # (a step launched ahead of its tokens names them by the step before: ``ctx.token_feedback``)
         if self.norm is None:
             ops.embed(ctx.tokens[:ctx.rows], self.weight, x, getattr(ctx, "token_feedback", None))
@@ -100,6 +113,7 @@ class SummedEmbedding(TokenEmbedding):
 
     def forward(self, ctx) -> torch.Tensor:
         x = ctx.ws.buffer("residual", self.width, torch.float32)
+        self._note_side_table(ctx)
         state = getattr(ctx, "embedding_state", None)
         if self.pairs is not None and state is None:
             raise ValueError("embedding_sum: the step's context carries no state for the embedding (the token before)")

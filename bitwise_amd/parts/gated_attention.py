@@ -26,6 +26,9 @@ padding is zeros).  Further switches:
     sink "learned"         the sink is a tensor ``sink`` [heads], a number per head
     gate "head"            the gate is one number per head, sigmoid(W_g h) with W_g [heads, width]
     window W               the query at position i sees the keys i - W + 1 .. i
+    cache_window W         how far back the cache's readers look, where a layer that reads this one's keys looks further back
+                           than this layer itself (None: as far as the request goes)
+    bias                   q, k and v have biases (tensors q.b, k.b, v.b), added to the projections before anything else
   The last taps - 1 projected rows of a request are its state.  Convolution, rotation, norms, scores
 and softmax are 32-bit in both modes; the cache, the queries and the gated output have the mode's activation dtype.
 """
@@ -52,10 +55,10 @@ def max_seq_rows(ctx) -> int:
 @register_mixer("gated_attention")
 class GatedAttention(Mixer):
     """params: width, heads, kv_heads, dim, vdim, scale, eps, conv (taps), qk_norm, sink (None, a number or "learned"), gate
-    (False, True or "head"), values ("own" or "keys"), shared_kv, window, softcap, chunk, v_mix, position (PartSpec of a
-    position encoding with the layout "pairs" or "halves").
-    tensors: q, k, v [heads*dim | kv_heads*dim | kv_heads*vdim, width] (no v where the values are the keys); q.conv, k.conv,
-    v.conv [channels, taps]; g [heads*vdim, width] (a gate a head: [heads, width]); sink [heads] if learned;
+    (False, True or "head"), values ("own" or "keys"), shared_kv, window, cache_window, softcap, chunk, v_mix, bias, position
+    (PartSpec of a position encoding with the layout "pairs" or "halves").
+    tensors: q, k, v [heads*dim | kv_heads*dim | kv_heads*vdim, width] (no v where the values are the keys), with biases q.b,
+    k.b, v.b of as many elements; q.conv, k.conv, v.conv [channels, taps]; g [heads*vdim, width] (a gate a head: [heads, width]); sink [heads] if learned;
     o [width, heads*vdim]."""
 
     graph_safe = True
@@ -89,6 +92,10 @@ class GatedAttention(Mixer):
         self.learned_sink = p.get("sink") == "learned"
         self.sink_value: Optional[float] = None if p.get("sink") is None or self.learned_sink else float(p["sink"])
         self.window: Optional[int] = p.get("window")
+        self.cache_window: Optional[int] = p.get("cache_window", self.window)
+        if self.cache_window is not None and (self.window is None or self.cache_window < self.window):
+            raise ValueError("gated_attention: the cache keeps at least the layer's own window")
+        self.has_bias = bool(p.get("bias", False))
         if self.heads % self.kv_heads:
             raise ValueError(f"gated_attention: {self.heads} heads are no multiple of {self.kv_heads} kv heads")
         if not self.scale > 0:
@@ -109,8 +116,6 @@ class GatedAttention(Mixer):
                 raise ValueError(f"gated_attention rotates neighbouring pairs or halves; position encoding '{pos.kind}' is laid out otherwise")
             self.rot = int(self.position.rotary_dim)
         self.halves = getattr(self.position, "layout", None) == "halves"
-        if self.whole_norm and self.rot:
-            raise ValueError("gated_attention: the norm over whole projections comes without rotation")
         if self.rot > self.dim:
             raise ValueError(f"gated_attention: {self.rot} rotated elements in heads of {self.dim}")
         self.q_ch = self.heads * self.dim
@@ -120,7 +125,7 @@ class GatedAttention(Mixer):
         self.proj: Optional[Linear] = None
         self.o: Optional[Linear] = None
         self.conv_w = self.sink = self.cos = self.sin = None
-        self.q_norm_w = self.k_norm_w = self.mix_w = None
+        self.q_norm_w = self.k_norm_w = self.mix_w = self.bias = None
 
     def tensors(self) -> Dict[str, TensorSpec]:
         out = {"q": TensorSpec((self.q_ch, self.width))}
@@ -128,6 +133,12 @@ class GatedAttention(Mixer):
             out["k"] = TensorSpec((self.kv_heads * self.dim, self.width))
             if not self.values_are_keys:
                 out["v"] = TensorSpec((self.kv_heads * self.vdim, self.width))
+        if self.has_bias:
+            out["q.b"] = TensorSpec((self.q_ch,), "small_bias")
+            if not self.shared_kv:
+                out["k.b"] = TensorSpec((self.kv_heads * self.dim,), "small_bias")
+                if not self.values_are_keys:
+                    out["v.b"] = TensorSpec((self.kv_heads * self.vdim,), "small_bias")
         if self.learned_sink:
             out["sink"] = TensorSpec((self.heads,), "bias")
         if self.taps >= 1:
@@ -161,7 +172,14 @@ class GatedAttention(Mixer):
         stack = [tensors[n] for n in names]
         if len({t.dtype for t in stack}) != 1:
             raise ValueError("the projections of one mixer must be stored in one dtype to be stacked")
-        self.proj = Linear(torch.cat(stack, dim=0), self.rt)
+        bias = None
+        if self.has_bias:
+            bias = torch.cat([tensors[n + ".b"].to(dev).float() for n in names if n != "g"]).contiguous()      # (widening is exact)
+        if self.whole_norm:
+            self.bias, bias = bias, None                      # (rides in the kernel that norms)
+        elif bias is not None and self.gate:
+            bias = torch.cat([bias, torch.zeros(self.g_ch, device=dev)])
+        self.proj = Linear(torch.cat(stack, dim=0), self.rt, bias=bias)
         self.o = Linear(tensors["o"], self.rt)
         if self.taps >= 1:
             cn = ["q.conv"] + ([] if self.shared_kv else ["k.conv", "v.conv"])
@@ -175,7 +193,7 @@ class GatedAttention(Mixer):
         return self.proj.nbytes() + self.o.nbytes() + (0 if self.conv_w is None else self.conv_w.numel() * 4)
 
     def cache_spec(self) -> CacheSpec:
-        return CacheSpec(self.kv_heads, self.head_size, self.window)
+        return CacheSpec(self.kv_heads, self.head_size, self.cache_window)
 
     def page_sizes(self):
         return ops.PAGE_SIZES
@@ -184,8 +202,8 @@ class GatedAttention(Mixer):
         return StateSpec(((self.taps - 1) * self.conv_ch,), "float32") if self.taps > 1 else None
 
     def input_projection(self):
-        # (the plain arrangement only: rotation, cache write and gate read the product's columns by their stride)
-        return self.proj if self.proj is not None and self.taps < 1 and not self.whole_norm else None
+        # (no convolution and no bias in the product itself: norm, rotation, cache write and gate read its columns by their stride)
+        return self.proj if self.proj is not None and self.taps < 1 and self.proj.bias is None and self.v_mix is None else None
 
     def adopt_input_projection(self, weight) -> None:
         self.proj = Linear(weight, self.rt)
@@ -228,7 +246,8 @@ class GatedAttention(Mixer):
                         raise ValueError("gated_attention: a layer mixes values before any layer has kept its own")
             ops.whole_norm_kv(src, ctx.positions, ctx.row_seq, ctx.block_tables[call.group], self.q_norm_w, self.k_norm_w, self.eps,
                               q, call.k_cache, call.v_cache, rows, self.heads, self.kv_heads, self.dim, self.vdim, hs,
-                              ws.page_size, call.writes_cache, v_first=v_first, mix=self.mix_w, v_keep=v_keep)
+                              ws.page_size, call.writes_cache, v_first=v_first, mix=self.mix_w, v_keep=v_keep, bias=self.bias,
+                              cos=self.cos, sin=self.sin, rot=self.rot, halves=self.halves)
         else:
             ops.pair_rope_unit(src, ctx.positions, ctx.row_seq, ctx.block_tables[call.group], self.cos, self.sin, q, call.k_cache,
                                call.v_cache, rows, self.heads, self.kv_heads, self.dim, self.vdim, hs, self.rot, ws.page_size,
@@ -240,10 +259,7 @@ class GatedAttention(Mixer):
                chunk=self.chunk, softcap=self.softcap)
         if self.gate or hs != self.vdim:
             act = ws.buffer("gattn_gated", self.heads * self.vdim, rt.act_dtype)
-            if self.gate:
-                ops.gate_mul(av, hs, proj[:, self.conv_ch:], act, rows, self.heads, self.vdim, per_head=self.head_gate)
-            else:
-                act.view(-1, self.heads, self.vdim)[:rows].copy_(av.view(-1, self.heads, hs)[:rows, :, :self.vdim])
+            ops.gate_mul(av, hs, proj[:, self.conv_ch:] if self.gate else None, act, rows, self.heads, self.vdim, per_head=self.head_gate)
         else:
             act = av
         if add:

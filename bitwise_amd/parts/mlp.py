@@ -147,13 +147,14 @@ class ClampedGLU(GeGLU):
 @register_feed_forward("mlp")
 class MLP(FeedForward):
     """W_down act(W_up h), no gate.  ``act``: "relu2", max(z, 0)^2, or "xielu", the expanded integral of the exponential
-    linear unit with two learned numbers: z > 0: softplus(p) z^2 + z/2; z <= 0: (1/2 + softplus(q)) (e^z - 1 - z) + z/2.
+    linear unit with two learned numbers: z > 0: softplus(p) z^2 + z/2; z <= 0: (1/2 + softplus(q)) (e^z - 1 - z) + z/2;
+    or "gelu", z/2 (1 + erf(z / sqrt 2)).
     params: width, inter, act, names (up, down and, for xielu, the tensor [p, q]).  The product leaves 32-bit sums, the
     activation is one 32-bit kernel behind it, which rounds once for the down projection."""
 
     graph_safe = True
     launches_through_ops = True
-    ACTS = {"relu2": ops.PLAIN_RELU2, "xielu": ops.PLAIN_XIELU}
+    ACTS = {"relu2": ops.PLAIN_RELU2, "xielu": ops.PLAIN_XIELU, "gelu": ops.PLAIN_GELU_ERF}
 
     def __init__(self, params, runtime):
         super().__init__(params, runtime)

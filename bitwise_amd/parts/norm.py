@@ -14,8 +14,10 @@ from .base import Norm, StateSpec, TensorSpec, register_norm
 @register_norm("rmsnorm")
 class RMSNorm(Norm):
     """params: width, eps; optional ``offset`` (the stored weight w is applied as offset + w; 0 by default, 1 for a
-    weight kept as its distance from 1), ``tensor`` (the weight's name behind the prefix, "weight" by default) and
-    ``scale`` (1 by default): where the norm sits behind a sublayer, the stream receives scale * norm(y).
+    weight kept as its distance from 1), ``tensor`` (the weight's name behind the prefix, "weight" by default),
+    ``scale`` (1 by default): where the norm sits behind a sublayer, the stream receives scale * norm(y); and ``gain`` (the name
+    of a second vector: the norm's output is multiplied by it element by element; the two vectors' product, formed once in
+    32-bit, is what the kernels multiply by).
     The sum of squares, the root and both products are 32-bit; the output has the mode's activation dtype."""
 
     graph_safe = True
@@ -28,10 +30,14 @@ class RMSNorm(Norm):
         self.offset = float(params.get("offset", 0.0))
         self.tensor = str(params.get("tensor", "weight"))
         self.scale = float(params.get("scale", 1.0))
+        self.gain = params.get("gain")
         self.weight = None
 
     def tensors(self) -> Dict[str, TensorSpec]:
-        return {self.tensor: TensorSpec((self.width,), "around_zero" if self.offset else "norm")}
+        out = {self.tensor: TensorSpec((self.width,), "around_zero" if self.offset else "norm")}
+        if self.gain is not None:
+            out[str(self.gain)] = TensorSpec((self.width,), "norm")
+        return out
 
     def _applied(self, w: torch.Tensor) -> torch.Tensor:
         w = w.to(self.rt.device)
@@ -41,6 +47,8 @@ class RMSNorm(Norm):
 
     def bind(self, tensors) -> None:
         self.weight = self._applied(tensors[self.tensor])
+        if self.gain is not None:
+            self.weight = (self.weight.float() * tensors[str(self.gain)].to(self.rt.device).float()).contiguous()
 
     def weight_bytes(self) -> int:
         return self.weight.numel() * self.weight.element_size()
@@ -67,6 +75,8 @@ class ShiftedRMSNorm(RMSNorm):
 
     def __init__(self, params, runtime):
         super().__init__(params, runtime)
+        if self.gain is not None:
+            raise ValueError("rmsnorm_shift: no gain behind a shifted norm")
         many = params.get("mix_tensors")
         self.mix_tensors = [str(n) for n in many] if many else [str(params.get("mix_tensor", "shift"))]
         self.mix: Optional[torch.Tensor] = None

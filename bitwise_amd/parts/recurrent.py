@@ -1,6 +1,6 @@
 """Mixers with a matrix memory per head instead of a cache: S <- decay * S + k v^T, o = S^T q.
 
-Four kinds share the arrangement (one stacked projection of the mixer's input, the recurrence over each request's
+Five kinds share the arrangement (one stacked projection of the mixer's input, the recurrence over each request's
 rows in order from and to its state slot, a per-head RMS norm of the read-out with an output gate, the output
 projection added into the residual stream) and differ in the decay:
 
@@ -15,6 +15,8 @@ projection added into the residual stream) and differ in the decay:
   learned bonus: o = (S + diag(u) k v^T)^T r, then S <- diag(decay) S + k v^T; SiLU gate, norm weight over all heads.
 * ``retention``: one constant decay per head, queries and keys rotated by position (halves layout) and the keys scaled by
   dim^(-1/2) behind the rotation; the read-out norm has no weight and the gate is SiLU.
+* ``lightning``: one constant decay per head; queries, keys and values pass SiLU and nothing else; the heads' read-outs are
+  normed together (one root mean square, a weight over all heads) and the gate is a sigmoid.
 
 The state, the gates and everything between the projections and the read-out are 32-bit in both modes; the
 projections' sums arrive as 32-bit values and are not rounded on the way.
@@ -29,6 +31,7 @@ import torch
 
 from ..csrc import ops
 from .base import Mixer, POSITION_ENCODINGS, StateSpec, TensorSpec, lookup, register_mixer
+from .gated_attention import max_seq_rows
 from .linear import Linear
 
 
@@ -76,6 +79,7 @@ class _MatrixMemoryMixer(Mixer):
     mode = -1
     gate_kind = ops.GATE_SIGMOID
     per_head_norm_weight = True
+    passes = True                             # long portions may run in passes over chunks
 
     def __init__(self, params, runtime):
         super().__init__(params, runtime)
@@ -133,11 +137,11 @@ class _MatrixMemoryMixer(Mixer):
         return y
 
     def _recur(self, ctx, call, y, gate, gate_off, gate2_off, bias, bias2, param, raw, kscale: float = 1.0, at=None, state=None,
-               heads_per_key: int = 1, skip=None) -> None:
+               heads_per_key: int = 1, skip=None, silu: bool = False) -> None:
         """``at``: where q (or r), k and v lie in a row of ``y``, if not at the stacked projection's own
         offsets.  ``state``: the memories' part of the slots, if they do not fill them."""
         at = self.offsets if at is None else at
-        plan = _scan_plan(ctx) if self.heads * self.dim * self.vdim < SCAN_MAX_STATE else None
+        plan = _scan_plan(ctx) if self.passes and self.heads * self.dim * self.vdim < SCAN_MAX_STATE else None
         seq_rows, nseq, scan = ctx.seq_rows, ctx.nseq, None
         if plan is not None:
             seq_rows, nseq, chunks, nchunks, spans, nspans = plan
@@ -148,7 +152,7 @@ class _MatrixMemoryMixer(Mixer):
             scan = (chunks, nchunks, spans, nspans, local, start)
         ops.linear_recurrence(self.mode, y, at["r"] if "q" not in at else at["q"], at["k"], at["v"], gate, gate_off, gate2_off,
                               bias, bias2, param, self.qscale, call.state if state is None else state, raw, seq_rows, ctx.slots, ctx.positions, nseq,
-                              self.heads, self.dim, self.vdim, scan=scan, kscale=kscale, heads_per_key=heads_per_key, skip=skip)
+                              self.heads, self.dim, self.vdim, scan=scan, kscale=kscale, heads_per_key=heads_per_key, skip=skip, silu=silu)
 
     def _finish(self, ctx, y, raw, target, add: bool = True, g_off: Optional[int] = None) -> None:
         act = ctx.ws.buffer("recur_gated", self.heads * self.vdim, self.rt.act_dtype)
@@ -412,6 +416,60 @@ class Retention(_MatrixMemoryMixer):
         raw = ctx.ws.buffer("recur_out", self.heads * self.vdim, torch.float32)
         self._recur(ctx, call, y, None, 0, 0, self.decay, None, 0.0, raw, kscale=self.kscale)
         self._finish(ctx, y, raw, target, add)
+
+    def forward(self, ctx, call, h, residual) -> None:
+        self._run(ctx, call, h, residual, True)
+
+    def forward_out(self, ctx, call, h, out) -> None:
+        self._run(ctx, call, h, out, False)
+
+
+@register_mixer("lightning")
+class Lightning(_MatrixMemoryMixer):
+    """params: width, heads, dim, vdim, eps, decay (a number per head).
+    tensors: q, k [heads*dim, width]; v, g [heads*vdim, width]; norm [heads*vdim]; o [width, heads*vdim]."""
+
+    mode = ops.RECUR_FIXED_DECAY
+    STAGED_SILU_ROWS = 4      # steps whose requests bring up to so many rows each apply SiLU where the recurrence loads its operands
+
+    def __init__(self, params, runtime):
+        super().__init__(params, runtime)
+        self.qscale = 1.0
+        self.decay_values = [float(d) for d in params["decay"]]
+        if len(self.decay_values) != self.heads or any(not 0.0 <= d <= 1.0 for d in self.decay_values):
+            raise ValueError(f"lightning: a decay in [0, 1] for each of the {self.heads} heads is needed")
+        self.decay: Optional[torch.Tensor] = None
+
+    def _stack_sizes(self):
+        hd, hv = self.heads * self.dim, self.heads * self.vdim
+        return [("q", hd), ("k", hd), ("v", hv), ("g", hv)]
+
+    def bind(self, tensors) -> None:
+        self._bind_common(tensors)
+        self.decay = torch.tensor(self.decay_values, dtype=torch.float32, device=self.rt.device)
+
+    def weight_bytes(self) -> int:
+        return self.proj.nbytes() + self.o.nbytes() + 4 * self.norm_weight.numel()
+
+    def forward_out_projected(self, ctx, call, proj, out) -> None:
+        self._run(ctx, call, None, out, False, projected=proj)
+
+    def _run(self, ctx, call, h, target, add: bool, projected=None) -> None:
+        ws, rows, inner = ctx.ws, ctx.rows, self.heads * self.vdim
+        y = projected if projected is not None else self._project(ctx, h)
+        # (every block of a head's columns stages its q and k again, so a portion's are made once, in place; the same function)
+        staged = max_seq_rows(ctx) <= self.STAGED_SILU_ROWS
+        if not staged:
+            ops.silu_rows(y[:, :self.offsets["g"]], rows)
+        raw = ws.buffer("recur_out", inner, torch.float32)
+        self._recur(ctx, call, y, None, 0, 0, self.decay, None, 0.0, raw, silu=staged)
+        act = ws.buffer("recur_gated", inner, self.rt.act_dtype)
+        ops.gated_part_norm(raw, y[:, self.offsets["g"]:], self.norm_weight, act, ctx.positions, rows, 1, self.eps,
+                            gate=ops.GATE_SIGMOID, behind=True)
+        if add:
+            self.o.add_into(ws, act, target, rows)
+        else:
+            self.o.store(ws, act, target, rows)
 
     def forward(self, ctx, call, h, residual) -> None:
         self._run(ctx, call, h, residual, True)

@@ -1,7 +1,9 @@
-"""Several mixers side by side: all read the same input, each output is normed over the model width with a weight
-vector of its own, and the mixer's output is the mean of the normed outputs.
+"""Several mixers side by side: all read the same input, and their outputs become one, in one of two ways: each is normed
+over the model width with a weight vector of its own and the normed outputs are averaged, or (``scales``) they are added as
+they are, each times a number.
 
     out = (1/n) sum_b  y_b / sqrt(mean(y_b^2) + eps) * w_b,      y_b = branch_b(h)
+    out = sum_b  s_b y_b
 
 The branches are registered mixers of any kind; each keeps what it needs (pages of a cache, a slot of state) as it
 would alone.  Towards the engine the combination is one mixer: its cache is the one branch's that has one (at most one
@@ -21,14 +23,16 @@ from .linear import Linear
 
 @register_mixer("side_by_side")
 class SideBySide(Mixer):
-    """params: width, eps, branches: a list of (name, PartSpec of a mixer); a branch's tensors are its own behind
-    ``<name>.``, and ``<name>.out`` [width] is the weight of the norm behind it."""
+    """params: width, branches: a list of (name, PartSpec of a mixer); a branch's tensors are its own behind ``<name>.``; eps,
+    and ``<name>.out`` [width] is the weight of the norm behind a branch; or scales, a number per branch (no eps, no norms)."""
 
     SHARED_MAX_ROWS = 64       # steps of up to this many rows run the branches' first products as one
 
     def __init__(self, params, runtime):
         super().__init__(params, runtime)
-        self.width, self.eps = int(params["width"]), float(params["eps"])
+        self.width = int(params["width"])
+        self.scales: Optional[List[float]] = None if params.get("scales") is None else [float(s) for s in params["scales"]]
+        self.eps = float(params["eps"]) if self.scales is None else 0.0
         self.names: List[str] = []
         self.branches: List[Mixer] = []
         for name, spec in params["branches"]:
@@ -38,6 +42,8 @@ class SideBySide(Mixer):
             self.branches.append(lookup(MIXERS, "mixer", spec.kind)(spec.params, runtime))
         if not 1 <= len(self.branches) <= 4 or len(set(self.names)) != len(self.names):
             raise ValueError("side_by_side: one to four branches with names of their own")
+        if self.scales is not None and len(self.scales) != len(self.branches):
+            raise ValueError("side_by_side: scales are a number per branch")
         if sum(b.cache_spec() is not None for b in self.branches) > 1:
             raise ValueError("side_by_side: at most one branch may keep a paged cache")
         self.graph_safe = all(getattr(b, "graph_safe", False) for b in self.branches)
@@ -64,14 +70,15 @@ class SideBySide(Mixer):
         for name, b in zip(self.names, self.branches):
             for t, ts in b.tensors().items():
                 out[f"{name}.{t}"] = ts
-        for name in self.names:
+        for name in self.names if self.scales is None else ():
             out[f"{name}.out"] = TensorSpec((self.width,), "norm")
         return out
 
     def bind(self, tensors) -> None:
         for name, b in zip(self.names, self.branches):
             b.bind({t: tensors[f"{name}.{t}"] for t in b.tensors()})
-        self.out_weights = [tensors[f"{name}.out"].to(self.rt.device).float().contiguous() for name in self.names]
+        if self.scales is None:
+            self.out_weights = [tensors[f"{name}.out"].to(self.rt.device).float().contiguous() for name in self.names]
         # Branches whose whole reading of the input is one product each share one product: the matrices stacked (the
         # branches keep blocks of the stacked matrix, no copies), the branches read their columns of it.  A product's
         # column does not depend on the columns beside it, so these are the bits of a product each.
@@ -90,7 +97,7 @@ class SideBySide(Mixer):
 
     def weight_bytes(self) -> int:
         # (a branch counts its block of the shared matrix as its own projection)
-        return sum(b.weight_bytes() for b in self.branches) + 4 * self.width * len(self.branches)
+        return sum(b.weight_bytes() for b in self.branches) + 4 * self.width * len(self.out_weights)
 
     def cache_spec(self) -> Optional[CacheSpec]:
         for b in self.branches:
@@ -150,23 +157,32 @@ class SideBySide(Mixer):
         return ys
 
     def forward_out(self, ctx, call, h, out) -> None:
-        ops.norm_mean(self._branch_outputs(ctx, call, h), self.out_weights, out, ctx.rows, self.eps)
+        ys = self._branch_outputs(ctx, call, h)
+        if self.scales is not None:
+            ops.scaled_sum(ys, self.scales, out, ctx.rows)
+        else:
+            ops.norm_mean(ys, self.out_weights, out, ctx.rows, self.eps)
 
-    def _can_ride(self, norm) -> bool:
+    def _can_ride(self, norm, rounded=None) -> bool:
         from .norm import RMSNorm
-        return type(norm) is RMSNorm and self.width <= ops.NORM_MEAN_ADD_MAX_WIDTH
+        if self.scales is not None:
+            return type(norm) is RMSNorm
+        return type(norm) is RMSNorm and self.width <= ops.NORM_MEAN_ADD_MAX_WIDTH and rounded is None
 
-    def _mean_add(self, ctx, ys, norm, x) -> None:
+    def _mean_add(self, ctx, ys, norm, x, rounded=None) -> None:
         w32 = self._post_weights.get(id(norm))
         if w32 is None:
             w32 = self._post_weights[id(norm)] = norm.weight.float().contiguous()       # (widening is exact)
+        if self.scales is not None:
+            ops.scaled_sum_norm_add(ys, self.scales, w32, norm.eps, norm.scale, x, ctx.rows, rounded)
+            return
         ops.norm_mean_add(ys, self.out_weights, self.eps, w32, norm.eps, norm.scale, x, ctx.rows)
 
-    def forward_add_normed(self, ctx, call, h, norm, x) -> bool:
-        """The norm behind the mixer rides in the launch that norms and averages the branches (the same bits)."""
-        if not self._can_ride(norm):
+    def forward_add_normed(self, ctx, call, h, norm, x, rounded=None) -> bool:
+        """The norm behind the mixer rides in the launch that joins the branches (the same bits)."""
+        if not self._can_ride(norm, rounded):
             return False
-        self._mean_add(ctx, self._branch_outputs(ctx, call, h), norm, x)
+        self._mean_add(ctx, self._branch_outputs(ctx, call, h), norm, x, rounded)
         return True
 
     def forward_between_norms(self, ctx, call, x, norm, norm_behind) -> bool:

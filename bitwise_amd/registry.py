@@ -11,6 +11,7 @@ from typing import Any, Callable, Dict, Mapping, Optional
 
 from .config import kikarax as kikarax_config
 from .config import kuponex as kuponex_config
+from .config import nuzinex as nuzinex_config
 from .config import rasesun as rasesun_config
 from .config import sepedra as sepedra_config
 from .config import vupolix as vupolix_config
@@ -18,6 +19,7 @@ from .config.llama import ConfigError, LlamaConfig
 from .models.kikarax import TINY_KIKARAX, kikarax_spec
 from .models.kuponex import TINY_KUPONEX, kuponex_spec
 from .models.llama import TINY_LLAMA, llama_spec
+from .models.nuzinex import TINY_NUZINEX, nuzinex_spec
 from .models.rasesun import TINY_RASESUN, rasesun_spec
 from .models.sepedra import TINY_SEPEDRA, sepedra_spec
 from .models.vupolix import TINY_VUPOLIX, vupolix_spec
@@ -88,3 +90,4 @@ register_architecture(kikarax_config.ARCHITECTURE, kikarax_config.KikaraxConfig.
 register_architecture(vupolix_config.ARCHITECTURE, vupolix_config.VupolixConfig.from_dict, vupolix_spec, TINY_VUPOLIX,
                       vupolix_config.sizes_from_tensors)
 register_architecture(rasesun_config.ARCHITECTURE, rasesun_config.RasesunConfig.from_dict, rasesun_spec, TINY_RASESUN)
+register_architecture(nuzinex_config.ARCHITECTURE, nuzinex_config.NuzinexConfig.from_dict, nuzinex_spec, TINY_NUZINEX)
