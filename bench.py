@@ -3,7 +3,7 @@
 random weights and uniform random token ids.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--dtype bf16|fp32] [--batch B] [--layers L]
-                    [--prefill-tokens T] [--no-points] [--shape smollm2|llama3_8b] [--trace-only] [--decode-phases] [--portion-align A] [--mixed] [--sweep] [--kuponex] [--sepedra] [--kikarax] [--vupolix] [--rasesun]
+                    [--prefill-tokens T] [--no-points] [--shape smollm2|llama3_8b] [--trace-only] [--decode-phases] [--portion-align A] [--mixed] [--sweep] [--kuponex] [--sepedra] [--kikarax] [--vupolix] [--rasesun] [--nuzinex]
 
 A step is one decode step of the whole engine (scheduler, graph replay of the model, sampling,
 token hand-back) for a batch of B requests that each hold a 2,048-token context.  ``value`` is
@@ -270,6 +270,50 @@ def rasesun_comparison(bw, torch, steps: int, dtype: str, only: str = "") -> int
     return 0
 
 
+def nuzinex_shape(width: int, ff: int, vocab: int = 32000) -> dict:
+    """A Nuzinex of eight layers: windowed attention, lightning attention, full attention beside a gated delta memory, an
+    attention layer that reads the first one's cache, and again lightning, side by side, side by side, lightning.  Attention
+    heads of 128 with a quarter as many key heads, a window of 1,024 keys; delta memories of 128 x 128 a head, twice as wide as
+    the model, two heads a key head; lightning heads of 128 x 128; a side input of 256 columns a layer."""
+    heads = width // 128
+    att = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+           "rot": {"base": 500000.0, "dims": 128}}
+    mlp = {"kind": "dense", "ff": ff}
+    local = lambda **more: {"type": "attention", "mixer": dict(att, mask={"size": 1024}, **more), "mlp": mlp}
+    both = {"type": "parallel", "mlp": mlp,
+            "mixer": {"left": dict(att), "left_scale": 0.6, "right_scale": 0.5,
+                      "right": {"heads": 2 * heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4}}}
+    fading = {"type": "lightning", "mlp": mlp,
+              "mixer": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 0.5 ** (1 + 8 * (h + 1) / heads) for h in range(heads)]}}
+    return {"architecture": "Nuzinex", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "token_side": {"dim": 256},
+            "layers": [local(), fading, both, local(kv_from=0), fading, both, both, fading], "max_positions": 16384, "eos_token_id": 2}
+
+
+def nuzinex_comparison(bw, torch, steps: int, dtype: str, only: str = "") -> int:
+    """Prefill and decode of Nuzinex at two layer sizes beside the Kuponex decoder (dense feed-forwards, matrix memories and
+    attention too) of equal width and depth, with feed-forwards of equal weights (two matrices there, three here): one JSON
+    object a line."""
+    from bitwise_amd.measure import PEAK_FLOPS, measure_decode, measure_prefill
+    for name, width, ff in (("2048x12288", 2048, 12288), ("4096x21504", 4096, 21504)):
+        for arch, cfg in (("Nuzinex", nuzinex_shape(width, ff)), ("Kuponex", kuponex_shape(width, 2 * ff // 3, 2))):
+            if only and only.lower() != arch.lower():
+                continue
+            model = bw.Model.random(cfg, seed=0, dtype=dtype, sigma=0.02, on_device=True)
+            for tokens in (512, 2048):
+                for exact in (True, False):
+                    # (exact_cuts False: matrix memories whose decay is a number run a long portion in three passes over chunks)
+                    m = measure_prefill(bw, torch, model, cfg, dtype, PEAK_FLOPS[dtype], tokens, exact_cuts=exact)
+                    print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "prefill_tokens": tokens, "exact_cuts": exact,
+                                      "ms": m["ms"], "tok_s": m["value"], "frac_of_matrix_peak": m["frac"]}), flush=True)
+            for batch in (1, 8, 64):
+                m = measure_decode(bw, torch, model, cfg, dtype, batch, steps, 4, context=2048)
+                print(json.dumps({"shape": name, "model": arch, "dtype": dtype, "decode_batch": batch, "context": 2048,
+                                  "ms_per_step": m["ms_per_step"], "tok_s": m["tok_s"], "frac_of_8_TBs": m["roofline"]["frac"]}), flush=True)
+            del model
+            torch.cuda.empty_cache()
+    return 0
+
+
 def sweep(bw, torch, steps: int, dtype: str) -> int:
     """Decode steps over batch and context, prefills over length: in bfloat16 at both shapes, in the 32-bit mode a
     coarser grid at the small one.  One JSON object a line."""
@@ -322,6 +366,9 @@ def main() -> int:
     ap.add_argument("--sepedra", nargs="?", const="both", default="", choices=["both", "sepedra", "llama"],
                     help="print a table instead of the line: prefill and decode of the Sepedra design at two layer sizes beside "
                          "the Llama decoder of equal width and depth with a feed-forward as wide as a token's experts together")
+    ap.add_argument("--nuzinex", nargs="?", const="both", default="", choices=["both", "nuzinex", "kuponex"],
+                    help="print a table instead of the line: prefill and decode of the Nuzinex design at two layer sizes beside "
+                         "the Kuponex decoder of equal width, depth and feed-forward weights (or one of the two)")
     ap.add_argument("--rasesun", nargs="?", const="both", default="", choices=["both", "rasesun", "vupolix"],
                     help="print a table instead of the line: prefill and decode of the Rasesun design at two layer sizes beside "
                          "the Vupolix decoder of equal width, depth and experts (or one of the two)")
@@ -349,6 +396,8 @@ def main() -> int:
     dtype = "bfloat16" if args.dtype == "bf16" else "float32"
     if args.sweep:
         return sweep(bw, torch, args.steps, dtype)
+    if args.nuzinex:
+        return nuzinex_comparison(bw, torch, min(args.steps, 32), dtype, "" if args.nuzinex == "both" else args.nuzinex)
     if args.rasesun:
         return rasesun_comparison(bw, torch, min(args.steps, 32), dtype, "" if args.rasesun == "both" else args.rasesun)
     if args.vupolix:

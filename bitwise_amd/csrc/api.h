@@ -38,6 +38,8 @@ int bw_gemm_bf16(const void* x, const void* w, void* out, int M, int N, int K, i
 int bw_gemm_clamped_glu_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo, float limit,
                              float alpha, void* stream);
 int bw_gemm_add_scratch(int M, int N, int K, long long* scratch_floats, int* counters);
+int bw_gemm_store_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo, float* scratch,
+                       long long scratch_floats, int32_t* counters, int num_counters, void* stream);   // (bw_gemm_bf16's 32-bit store)
 int bw_gemm_add_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo, float* scratch,
                      long long scratch_floats, int32_t* counters, int num_counters, void* stream);
 // No counterpart in the reference.  For callers that cannot allocate device memory and cannot bring a

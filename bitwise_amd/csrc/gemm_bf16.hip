@@ -163,7 +163,8 @@ static int chain_record_rows(int kind, const RowsCall& c, int wgs, int waves, in
 // as there are compute units, if the product has them), a workgroup per tile and segment of K if there are several
 // (they meet in device scratch the caller brings).  tiles 0: it does not run there.
 // out = (((out + p[0]) + p[1]) + ...) + p[S-1], element by element: the segments of a residual add that
-// gemm_bf16_big_kernel left in scratch ([S][M][N]), joined in segment order.
+// gemm_bf16_big_kernel left in scratch ([S][M][N]), joined in segment order (ADD false: a store, the chain starts at p[0]).
+template <bool ADD>
 __global__ __launch_bounds__(256) void add_segments_kernel(float* __restrict__ out, const float* __restrict__ parts, int S,
                                                            int M, int N, int ldo) {
   const size_t quads = (size_t)M * (N >> 2);
@@ -171,8 +172,8 @@ __global__ __launch_bounds__(256) void add_segments_kernel(float* __restrict__ o
   if (i >= quads) return;
   const int m = (int)(i / (N >> 2)), n = 4 * (int)(i % (N >> 2));
   float* o = out + (size_t)m * ldo + n;
-  f32x4 y = *reinterpret_cast<const f32x4*>(o);
-  for (int sg = 0; sg < S; ++sg) y = y + *reinterpret_cast<const f32x4*>(parts + ((size_t)sg * M + m) * N + n);
+  f32x4 y = *reinterpret_cast<const f32x4*>(ADD ? o : parts + (size_t)m * N + n);
+  for (int sg = ADD ? 0 : 1; sg < S; ++sg) y = y + *reinterpret_cast<const f32x4*>(parts + ((size_t)sg * M + m) * N + n);
   *reinterpret_cast<f32x4*>(o) = y;
 }
 
@@ -258,6 +259,8 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
                             size_t scratch_floats = 0, int num_counters = 0) {
   const int S = (K + GEMM_SEG - 1) / GEMM_SEG;
   constexpr int NB = epi_is_glu(EPI) ? 2 : 1;
+  // a 32-bit store may give the segments of K workgroups of their own, too, where the caller brings the scratch
+  const bool split_ok = sp.scratch != nullptr && sp.counters != nullptr;
   if (M <= 64) {
     // (the rotary epilogue belongs to the wide kernel; the clamped unit of few rows is a kernel behind the 32-bit product)
     if constexpr (EPI == EPI_QKV_ROPE || EPI == EPI_CLAMPED_GLU_BF16) return -2;
@@ -268,7 +271,11 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
       // (the descriptors of W cover a tile's rows each, so only the rows of x have to fit 31 bits of offset)
       const bool fits = (size_t)M * ldx * 2 < ((size_t)1 << 31);
       // (a residual add of several segments starts its chain at the residual: the kernels further down do that)
-      if ((S == 1 || EPI != EPI_ADD_F32) && K % 64 == 0 && wgs >= 64 && fits) {
+      // (and so does a 32-bit store of up to 16 rows, whose segments those kernels give waves of their own, or with scratch
+      // of up to 64 and four segments: 4,096 columns of K = 21,504 at 8 rows took 65 us as 64 workgroups with all of K
+      // each, 29 as strips; at 64 rows of K = 8,192 21 us and 17.5, of K = 21,504, where the join weighs more, 33 and 39)
+      const bool whole_k = S == 1 || (EPI != EPI_ADD_F32 && !(EPI == EPI_F32 && (M <= 16 ? S <= 40 : split_ok && S <= 4)));
+      if (whole_k && K % 64 == 0 && wgs >= 64 && fits) {
         if (M <= 16) return launch_mid<EPI, 1, false>(x, w, out, M, N, K, ldx, ldo, wgs, s);
         if (M <= 32) return launch_mid<EPI, 2, false>(x, w, out, M, N, K, ldx, ldo, wgs, s);
         // 33 to 64 rows and so few columns that twice the workgroups still fit the chip at once: two blocks of 32 rows,
@@ -283,11 +290,11 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
       }
       // a residual add of more than 16 rows and fewer columns (the other kernel for it fetches W once per block of
       // 16 rows): narrower tiles, and several segments if the caller brought scratch for them to meet in
-      if constexpr (EPI == EPI_ADD_F32) {
+      if constexpr (EPI == EPI_ADD_F32 || EPI == EPI_F32) {
         int tiles;
         bool narrow;
         add_rows_shape(M, N, K, tiles, narrow);
-        if (tiles && fits && (S == 1 || (sp.scratch != nullptr && sp.counters != nullptr))) {
+        if (tiles && fits && (S == 1 || split_ok)) {
           if (S > 1 && (scratch_floats < (size_t)tiles * S * 4096 || num_counters < tiles)) return -6;
           const MidNormArgs na{};
           const QkvRopeArgs no{};
@@ -344,7 +351,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
     }
 #undef BW_SKINNY
   } else {
-    if constexpr (EPI == EPI_ADD_F32) {
+    if constexpr (EPI == EPI_ADD_F32 || EPI == EPI_F32) {
       // Few enough workgroups to be on the chip at once (the output projection of a short prompt is 16 tiles of 128 x 128
       // for 128 rows and 2048 columns, whatever is idle): the kernel for up to 64 rows, a workgroup per block of 64 rows,
       // 64 or 32 columns and segment of K, all blocks in one launch.
@@ -356,7 +363,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
         int tiles, zb;
         bool narrow;
         add_blocks_shape(M, N, K, tiles, narrow, zb);
-        const bool scratch_ok = S == 1 || (sp.scratch != nullptr && sp.counters != nullptr &&
+        const bool scratch_ok = S == 1 || (split_ok &&
                                            scratch_floats >= (size_t)tiles * zb * S * 4096 && num_counters >= tiles * zb);
         if (tiles && scratch_ok) {
           const MidNormArgs na{};
@@ -366,8 +373,10 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
         }
       }
       int tiles;
-      const AddRoute route = add_route(M, N, K, ldo, tiles);
-      if (route == ADD_ROW_BLOCKS && (size_t)M * ldx * 2 < ((size_t)1 << 31) &&
+      AddRoute route = add_route(M, N, K, ldo, tiles);
+      // (a store has whole-K kernels with larger tiles further down: it splits only what leaves compute units idle there)
+      if (EPI == EPI_F32 && ((M + 127) / 128) * ((N + 127) / 128) >= 256) route = ADD_WHOLE;
+      if (EPI == EPI_ADD_F32 && route == ADD_ROW_BLOCKS && (size_t)M * ldx * 2 < ((size_t)1 << 31) &&
           (S == 1 || (sp.scratch != nullptr && sp.counters != nullptr && scratch_floats >= (size_t)tiles * S * 4096 &&
                       num_counters >= tiles))) {
         for (int m0 = 0; m0 < M; m0 += 64) {
@@ -377,7 +386,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
         }
         return 0;
       }
-      if (route == ADD_TILE256) return launch_tile256<EPI>(x, w, out, M, N, K, ldx, ldo, s);
+      if (EPI == EPI_ADD_F32 && route == ADD_TILE256) return launch_tile256<EPI>(x, w, out, M, N, K, ldx, ldo, s);
       if (route == ADD_BIG_SPLIT && sp.scratch != nullptr && ((uintptr_t)out & 15) == 0) {
         if (scratch_floats < (size_t)S * M * N) return -6;
         const int bm = (M + BIG_BM - 1) / BIG_BM, bn = (N + 255) / 256;
@@ -390,7 +399,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
         BW_LAUNCH((gemm_bf16_big_kernel<EPI_F32>), dim3(bm * bn, S), dim3(512), BIG_SLOTS * BIG_SLOT, s, x, w,
                            (void*)sp.scratch, M, N, K, ldx, N, bm, bn, rp, (size_t)M * N);
         const size_t quads = (size_t)M * (N >> 2);
-        BW_LAUNCH(add_segments_kernel, dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, s, (float*)out, sp.scratch, S,
+        BW_LAUNCH(add_segments_kernel<EPI == EPI_ADD_F32>, dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, s, (float*)out, sp.scratch, S,
                            M, N, ldo);
         return BW_LAUNCH_CHECK();
       }
@@ -399,7 +408,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
         const int rc = launch_tile256<EPI_F32>(x, w, (void*)sp.scratch, M, N, K, ldx, N, s, QkvRopeArgs{}, S, (size_t)M * N);
         if (rc) return rc;
         const size_t quads = (size_t)M * (N >> 2);
-        BW_LAUNCH(add_segments_kernel, dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, s, (float*)out, sp.scratch, S,
+        BW_LAUNCH(add_segments_kernel<EPI == EPI_ADD_F32>, dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, s, (float*)out, sp.scratch, S,
                            M, N, ldo);
         return BW_LAUNCH_CHECK();
       }
@@ -415,7 +424,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
         BW_LAUNCH((gemm_bf16_tile128_kernel<EPI_F32>), dim3(mt * nt, S), dim3(512), T128_STAGES * T128_STAGE, s, x, w,
                            (void*)sp.scratch, M, N, K, ldx, N, mt, nt, rp, (size_t)M * N);
         const size_t quads = (size_t)M * (N >> 2);
-        BW_LAUNCH(add_segments_kernel, dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, s, (float*)out, sp.scratch, S,
+        BW_LAUNCH(add_segments_kernel<EPI == EPI_ADD_F32>, dim3((unsigned)((quads + 255) / 256)), dim3(256), 0, s, (float*)out, sp.scratch, S,
                            M, N, ldo);
         return BW_LAUNCH_CHECK();
       }
@@ -524,6 +533,16 @@ extern "C" int bw_gemm_add_bf16(const void* x, const void* w, void* out, int M, 
   if ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) return -3;
   return launch_gemm_bf16<EPI_ADD_F32>((const bf16_t*)x, (const bf16_t*)w, out, M, N, K, ldx, ldo, (hipStream_t)stream,
                                        QkvRopeArgs{}, MidSplitArgs{scratch, counters}, (size_t)scratch_floats, num_counters);
+}
+
+// out = x W^T (32-bit store) with that scratch: the bits of bw_gemm_bf16's store.
+extern "C" int bw_gemm_store_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo,
+                                  float* scratch, long long scratch_floats, int32_t* counters, int num_counters, void* stream) {
+  if (M <= 0 || N <= 0) return 0;
+  if (K <= 0 || (K % 8) || (ldx % 8) || ldx < K || ldo < N) return -2;
+  if ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) return -3;
+  return launch_gemm_bf16<EPI_F32>((const bf16_t*)x, (const bf16_t*)w, out, M, N, K, ldx, ldo, (hipStream_t)stream,
+                                   QkvRopeArgs{}, MidSplitArgs{scratch, counters}, (size_t)scratch_floats, num_counters);
 }
 
 extern "C" int bw_gemm_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo,

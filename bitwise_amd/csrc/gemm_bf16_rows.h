@@ -453,7 +453,7 @@ __device__ __forceinline__ void mid_body(const bf16_t* __restrict__ x, const bf1
     }
   } else {
     const int n = n0 + 16 * strip + r;
-    if constexpr (EPI == EPI_ADD_F32 && !NORM) {
+    if constexpr ((EPI == EPI_ADD_F32 || EPI == EPI_F32) && !NORM) {
       const int nseg = cc.gy;
       if (nseg > 1) {
         // Every segment's workgroup leaves its sums in device scratch (stores of device scope: they write through,
@@ -483,9 +483,10 @@ __device__ __forceinline__ void mid_body(const bf16_t* __restrict__ x, const bf1
 #pragma unroll
           for (int q = 0; q < 4; ++q) {
             const int m = 16 * (a_block0 + i) + 4 * g + q;
-            y[q] = (m < M && n < N) ? ((const float*)out)[(size_t)m * ldo + n] : 0.0f;   // the chain starts at the residual
+            y[q] = (EPI == EPI_ADD_F32 && m < M && n < N) ? ((const float*)out)[(size_t)m * ldo + n] : 0.0f;   // the chain starts at the residual
           }
-          for (int sg = 0; sg < nseg; ++sg)
+          if constexpr (EPI == EPI_F32) y = __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(rs_s, mine + i * 1024, 0, 16));
+          for (int sg = EPI == EPI_F32 ? 1 : 0; sg < nseg; ++sg)
             y = y + __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(rs_s, mine + i * 1024, sg * cell, 16));
 #pragma unroll
           for (int q = 0; q < 4; ++q) {

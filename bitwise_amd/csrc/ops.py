@@ -51,6 +51,8 @@ _SIGS = {
     "bw_gemm_add_scratch": [c_int, c_int, c_int, c_void_p, c_void_p],
     "bw_gemm_add_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_longlong, c_void_p,
                          c_int, c_void_p],
+    "bw_gemm_store_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_longlong, c_void_p,
+                           c_int, c_void_p],
     "bw_gemm_add_bf16_static": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "bw_gemm_add_bf16_static_max": [c_void_p, c_void_p],
     "bw_gemm_qkv_rope_bf16": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
@@ -149,7 +151,7 @@ _fns = {}
 # path that sends the waiting phases first, or launch nothing).  Every other one is a launch that must come after
 # what waits.
 _CHAIN_KEEPS = frozenset({
-    "bw_gemm_bf16", "bw_gemm_add_bf16", "bw_norm_gemm_bf16", "bw_norm_qkv_rope_bf16",
+    "bw_gemm_bf16", "bw_gemm_add_bf16", "bw_gemm_store_bf16", "bw_norm_gemm_bf16", "bw_norm_qkv_rope_bf16",
     "bw_gemm_add_scratch", "bw_norm_gemm_supported", "bw_norm_gemm_wide_supported", "bw_attention_decode_scratch",
     "bw_attention_fold_group_tiles", "bw_gemm_add_bf16_static_max", "bw_moe_max_tiles", "bw_shared_key_piece", "bw_chain_sync_words", "bw_chain_begin",
     "bw_chain_flush", "bw_chain_end",
@@ -456,7 +458,7 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, rows: int, ep
               scratch: Optional[Tuple[torch.Tensor, torch.Tensor]] = None) -> None:
     """out[:rows] = epilogue(x[:rows] @ w.T) on the matrix cores; see gemm_bf16.hip for the
     arithmetic.  EPI_SWIGLU_BF16 takes the stacked weight [2N, K] (gate rows, then up rows).
-    ``scratch`` (EPI_ADD_F32 only): the tensors ``gemm_add_scratch`` asks for (float32, int32
+    ``scratch`` (EPI_ADD_F32 and EPI_F32): the tensors ``gemm_add_scratch`` asks for (float32, int32
     zeros); the bits do not depend on it.  ``x`` may be a column slice of a wider matrix that starts at a multiple of 8
     elements, and with a 32-bit store ``out`` may be a column slice too."""
     _need_strided(x, torch.bfloat16, "x")
@@ -477,12 +479,13 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, rows: int, ep
         raise ValueError(f"gemm_bf16: x {tuple(x.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)} do not match")
     if K % 8:
         raise ValueError(f"gemm_bf16: inner size {K} must be a multiple of 8 (16-byte operand loads)")
-    if scratch is not None and epilogue == EPI_ADD_F32:
+    if scratch is not None and epilogue in (EPI_ADD_F32, EPI_F32):
         sc_f, sc_c = scratch
         _need(sc_f, torch.float32, "scratch")
         _need(sc_c, torch.int32, "scratch counters")
-        _check(_fn("bw_gemm_add_bf16")(x.data_ptr(), w.data_ptr(), out.data_ptr(), rows, N, K, x.stride(0), out.stride(0),
-                                       sc_f.data_ptr(), sc_f.numel(), sc_c.data_ptr(), sc_c.numel(), _stream()), "gemm_bf16")
+        entry = "bw_gemm_add_bf16" if epilogue == EPI_ADD_F32 else "bw_gemm_store_bf16"
+        _check(_fn(entry)(x.data_ptr(), w.data_ptr(), out.data_ptr(), rows, N, K, x.stride(0), out.stride(0),
+                          sc_f.data_ptr(), sc_f.numel(), sc_c.data_ptr(), sc_c.numel(), _stream()), "gemm_bf16")
         return
     _check(_fn("bw_gemm_bf16")(x.data_ptr(), w.data_ptr(), out.data_ptr(), rows, N, K, x.stride(0), out.stride(0),
                                epilogue, _stream()), "gemm_bf16")

@@ -137,7 +137,39 @@ def rasesun_prefill_flops(cfg: dict, tokens: int) -> float:
     return total + 2 * w * cfg["vocab"]
 
 
+def nuzinex_prefill_flops(cfg: dict, tokens: int) -> float:
+    """Multiply-adds times two of one prompt: every projection (the gates', the step sizes' and the side input's), the
+    feed-forwards, the attention's scores and weighted sums over the keys a query sees, and for the memories the update and
+    the read-out of every token (2 x dim x vdim a head; the delta memory reads once more) (the convolutions are left out)."""
+    w, side, total = cfg["width"], cfg["token_side"]["dim"], 0.0
+
+    def attention(m, gate):
+        H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        own = 0 if m.get("kv_from") is not None else G * (D + V)
+        win = min((m.get("mask") or {"size": tokens})["size"], tokens)
+        return (w * (H * D + own + (H * V if gate else 0)) + H * V * w, H * (D + V) * (win * (win + 1) / 2 + (tokens - win) * win))
+
+    for layer in cfg["layers"]:
+        m, quadratic = layer["mixer"], 0.0
+        if layer["type"] == "attention":
+            per_token, quadratic = attention(m, False)
+        elif layer["type"] == "parallel":
+            per_token, quadratic = attention(m["left"], True)
+            r = m["right"]
+            H, G, D, V = r["heads"], r["kv_heads"], r["dim"], r["vdim"]
+            per_token += w * (2 * G * D + 2 * H * V + 2 * H) + H * V * w + 3 * H * D * V
+        else:
+            H, D, V = m["heads"], m["dim"], m["vdim"]
+            per_token = w * H * (2 * D + 2 * V) + H * V * w + 2 * H * D * V
+        if layer.get("mlp"):
+            per_token += 2 * w * layer["mlp"]["ff"]
+        total += 2 * ((per_token + 2 * w * side) * tokens + quadratic)
+    return total + 2 * w * cfg["vocab"]
+
+
 def prefill_flops(cfg: dict, tokens: int) -> float:
+    if cfg.get("architecture") == "Nuzinex":
+        return nuzinex_prefill_flops(cfg, tokens)
     if cfg.get("architecture") == "Rasesun":
         return rasesun_prefill_flops(cfg, tokens)
     if cfg.get("architecture") == "Vupolix":

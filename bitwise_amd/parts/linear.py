@@ -45,6 +45,23 @@ class Linear:
         ops.convert(x, buf, rows)
         return buf
 
+    def _scratch(self, ws, rows: int):
+        """17 rows or more and a long inner size: every 2048-segment of it gets workgroups of its own, which meet in device
+        scratch.  For up to 64 rows (or a few blocks of 64) that is a fixed size; for a prompt portion it holds the
+        segments' sums whole and is sized for the longest step, so that one buffer serves every portion."""
+        if rows <= 16:
+            return None
+        floats, counters = ops.gemm_add_scratch(rows, self.out_features, self.in_features)
+        if floats and rows > 64:
+            longest = ops.gemm_add_scratch(ws.max_rows, self.out_features, self.in_features)
+            floats, counters = max(floats, longest[0]), max(counters, longest[1])
+            if floats > longest[0]:        # (the longest step needs none: a size per power of two, not one per number of rows)
+                floats = 1 << (floats - 1).bit_length()
+        if not floats:
+            return None
+        return (ws.buffer("gemm_add_split", floats, torch.float32, rows=1),
+                ws.buffer("gemm_add_split_count", counters, torch.int32, rows=1))
+
     def store(self, ws, x: torch.Tensor, out: torch.Tensor, rows: int) -> None:
         """out[:rows] = x[:rows] @ W.T (out float32, or bfloat16 on the matrix-core path).  ``ws`` is the
         step's workspace (temporaries for a weight whose dtype is not the mode's)."""
@@ -59,7 +76,10 @@ class Linear:
             if y is not out:
                 ops.convert(y, out, rows)
         elif self.mfma:
-            ops.gemm_bf16(x, self.weight, out, rows, ops.EPI_BF16 if out.dtype == torch.bfloat16 else ops.EPI_F32)
+            if out.dtype == torch.bfloat16:
+                ops.gemm_bf16(x, self.weight, out, rows, ops.EPI_BF16)
+            else:
+                ops.gemm_bf16(x, self.weight, out, rows, ops.EPI_F32, scratch=self._scratch(ws, rows))
         elif out.dtype == torch.float32:
             ops.gemm_f32(self._x32(ws, x, rows), self.weight, out, rows)
         else:
@@ -88,18 +108,6 @@ class Linear:
             ops.add_(residual, y, rows)
             return
         if self.mfma:
-            # 17 rows or more and a long inner size: every 2048-segment of it gets workgroups of its own, which meet
-            # in device scratch.  For up to 64 rows (or a few blocks of 64) that is a fixed size; for a prompt portion
-            # it holds the segments' sums whole and is sized for the longest step, so that one buffer serves every
-            # portion.
-            scratch = None
-            floats, counters = ops.gemm_add_scratch(rows, self.out_features, self.in_features) if rows > 16 else (0, 0)
-            if floats and rows > 64:
-                longest = ops.gemm_add_scratch(ws.max_rows, self.out_features, self.in_features)
-                floats, counters = max(floats, longest[0]), max(counters, longest[1])
-            if floats:
-                scratch = (ws.buffer("gemm_add_split", floats, torch.float32, rows=1),
-                           ws.buffer("gemm_add_split_count", counters, torch.int32, rows=1))
-            ops.gemm_bf16(x, self.weight, residual, rows, ops.EPI_ADD_F32, scratch=scratch)
+            ops.gemm_bf16(x, self.weight, residual, rows, ops.EPI_ADD_F32, scratch=self._scratch(ws, rows))
         else:
             ops.gemm_f32(self._x32(ws, x, rows), self.weight, residual, rows, accumulate=True)
