@@ -425,48 +425,94 @@ __device__ __forceinline__ float workgroup_sum_256(float v, float* lds4) {
   return t;
 }
 
-// The normed heads of one projection, turned and padded: item i of ``heads * hd / 2`` is a pair of elements of one head, a
-// rotated pair for the first rot / 2 of a head, neighbours behind those (in either layout).  put(h, d, value) stores.
-template <typename Put>
+// One projection (the queries or the keys) normed over all its heads, turned and padded.  Item i of ``heads * ceil(dim / 2)`` is a
+// pair of elements of one head: a rotated pair for the first rot / 2 of a head, neighbours behind those (in either layout).
+// Thread t owns pairs t, t + 256, ...: its sum of squares is one chain over them, the waves' sums are added in wave order.
+// Projections of up to 256 PV pairs keep them in registers, everything they need asked for before anything is used; longer
+// ones are read twice (the same operations).  put(h, d, value) stores.
+template <int PV, typename Put>
 __device__ __forceinline__ void whole_norm_heads(const WholeNormArgs& a, const float* p, const float* b, const float* w, int heads,
-                                                 float inv, int pos, Put put) {
-  const int half = a.rot / 2, pairs = a.hd / 2;
+                                                 int pos, float* red, Put put) {
+  const int half = a.rot / 2, per = (a.dim + 1) / 2, pairs = heads * per, tid = threadIdx.x;
   const float* ct = a.cos_table + (size_t)pos * half;
   const float* st = a.sin_table + (size_t)pos * half;
-  for (int i = threadIdx.x; i < heads * pairs; i += 256) {
-    const int h = i / pairs, r = i % pairs;
-    const bool turned = r < half;
-    const int d0 = a.halves && turned ? r : 2 * r, d1 = a.halves && turned ? r + half : 2 * r + 1;
-    float u = 0.0f, v = 0.0f;
-    if (d0 < a.dim) {
-      const int e = h * a.dim + d0;
-      u = ((b != nullptr ? p[e] + b[e] : p[e]) * inv) * w[e];
-    }
-    if (d1 < a.dim) {
-      const int e = h * a.dim + d1;
-      v = ((b != nullptr ? p[e] + b[e] : p[e]) * inv) * w[e];
-    }
-    if (turned) {
-      const float c = ct[r], s = st[r], u0 = u;
+  struct Pair { int h, r, d0, d1; };
+  auto place = [&](int i) {
+    Pair q;
+    q.h = i / per;
+    q.r = i - q.h * per;
+    const bool apart = a.halves && q.r < half;
+    q.d0 = apart ? q.r : 2 * q.r;
+    q.d1 = apart ? q.r + half : 2 * q.r + 1;
+    return q;
+  };
+  auto element = [&](int h, int d) -> float {            // (an odd head's last pair has one element)
+    if (d >= a.dim) return 0.0f;
+    const int e = h * a.dim + d;
+    return b != nullptr ? p[e] + b[e] : p[e];
+  };
+  auto weight = [&](int h, int d) -> float { return d < a.dim ? w[h * a.dim + d] : 0.0f; };
+  auto finish = [&](const Pair& q, float u, float v, float wu, float wv, float c, float s, float inv) {
+    u = (u * inv) * wu;
+    v = (v * inv) * wv;
+    if (q.r < half) {
+      const float u0 = u;
       u = u0 * c - v * s;
       v = v * c + u0 * s;
     }
-    put(h, d0, u);
-    put(h, d1, v);
-  }
-}
-
-__device__ __forceinline__ float whole_norm_inv(const float* p, const float* b, int n, float eps, float* red) {
+    put(q.h, q.d0, u);
+    if (q.d1 < a.hd) put(q.h, q.d1, v);
+  };
+  const bool small = pairs <= 256 * PV;
   float acc = 0.0f;
-  for (int i = threadIdx.x; i < n; i += 256) {
-    const float v = b != nullptr ? p[i] + b[i] : p[i];
-    acc = fmaf(v, v, acc);
+  if (small) {
+    float u[PV], v[PV], wu[PV], wv[PV], c[PV], s[PV];
+#pragma unroll
+    for (int j = 0; j < PV; ++j) {
+      u[j] = v[j] = wu[j] = wv[j] = c[j] = s[j] = 0.0f;
+      if (256 * j < pairs) {                             // (scalar)
+        const Pair q = place(min(tid + 256 * j, pairs - 1));
+        u[j] = element(q.h, q.d0);
+        v[j] = element(q.h, q.d1);
+        wu[j] = weight(q.h, q.d0);
+        wv[j] = weight(q.h, q.d1);
+        if (half > 0) {
+          c[j] = ct[min(q.r, half - 1)];
+          s[j] = st[min(q.r, half - 1)];
+        }
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < PV; ++j) {
+      if (tid + 256 * j >= pairs) u[j] = v[j] = 0.0f;
+      acc = fmaf(u[j], u[j], acc);
+      acc = fmaf(v[j], v[j], acc);
+    }
+    const float inv = 1.0f / sqrtf(workgroup_sum_256(acc, red) / (float)(heads * a.dim) + a.eps);
+#pragma unroll
+    for (int j = 0; j < PV; ++j)
+      if (tid + 256 * j < pairs) finish(place(tid + 256 * j), u[j], v[j], wu[j], wv[j], c[j], s[j], inv);
+  } else {
+    for (int i = tid; i < pairs; i += 256) {
+      const Pair q = place(i);
+      const float u = element(q.h, q.d0), v = element(q.h, q.d1);
+      acc = fmaf(u, u, acc);
+      acc = fmaf(v, v, acc);
+    }
+    const float inv = 1.0f / sqrtf(workgroup_sum_256(acc, red) / (float)(heads * a.dim) + a.eps);
+    for (int i = tid; i < pairs; i += 256) {
+      const Pair q = place(i);
+      const float c = q.r < half ? ct[q.r] : 0.0f, s = q.r < half ? st[q.r] : 0.0f;
+      finish(q, element(q.h, q.d0), element(q.h, q.d1), weight(q.h, q.d0), weight(q.h, q.d1), c, s, inv);
+    }
   }
-  return 1.0f / sqrtf(workgroup_sum_256(acc, red) / (float)n + eps);
+  // the padding behind the heads' elements
+  const int from = 2 * per, pad = a.hd - from;
+  for (int i = tid; i < heads * pad; i += 256) put(i / pad, from + i % pad, 0.0f);
 }
 
 // A workgroup for each of a row's three parts (queries, keys, values): each is one chain of loads, a sum and stores.
-template <typename T>
+template <typename T, int PV>
 __global__ __launch_bounds__(256) void whole_norm_kv_kernel(WholeNormArgs a) {
   __shared__ float red[4];
   const int row = blockIdx.x, part = blockIdx.y, tid = threadIdx.x;
@@ -475,20 +521,15 @@ __global__ __launch_bounds__(256) void whole_norm_kv_kernel(WholeNormArgs a) {
   const int qn = a.heads * a.dim, kn = a.kv_heads * a.dim;
   const float* q = a.src + (size_t)row * a.lds;
   if (part == 0) {
-    const float inv_q = whole_norm_inv(q, a.bias, qn, a.eps, red);
     T* qo = reinterpret_cast<T*>(a.q_out) + (size_t)row * a.heads * a.hd;
-    whole_norm_heads(a, q, a.bias, a.q_w, a.heads, inv_q, pos, [&](int h, int d, float v) { gm_store(qo + h * a.hd + d, v); });
+    whole_norm_heads<PV>(a, q, a.bias, a.q_w, a.heads, pos, red, [&](int h, int d, float v) { gm_store(qo + h * a.hd + d, v); });
     return;
   }
-  if (!a.write_cache) return;
   const int page = a.block_table[(size_t)a.row_seq[row] * a.table_stride + pos / a.page_size];
   const int slot = pos % a.page_size;
   if (part == 1) {
-    const float* k = q + qn;
-    const float* kb = a.bias != nullptr ? a.bias + qn : nullptr;
-    const float inv_k = whole_norm_inv(k, kb, kn, a.eps, red);
     T* kc = reinterpret_cast<T*>(a.k_cache);
-    whole_norm_heads(a, k, kb, a.k_w, a.kv_heads, inv_k, pos, [&](int h, int d, float v) {
+    whole_norm_heads<PV>(a, q + qn, a.bias != nullptr ? a.bias + qn : nullptr, a.k_w, a.kv_heads, pos, red, [&](int h, int d, float v) {
       gm_store(kc + (((size_t)page * a.kv_heads + h) * a.page_size + slot) * a.hd + d, v);
     });
     return;
@@ -526,8 +567,13 @@ extern "C" int bw_whole_norm_kv(const float* src, int lds, const int32_t* positi
   if (v_keep != nullptr && v_keep == v_first) return -2;
   WholeNormArgs a{src, positions, row_seq, block_table, q_w, k_w, v_first, lambda, v_keep, q_out, k_cache, v_cache, bias, cos_table,
                   sin_table, lds, ldf, ldk, heads, kv_heads, dim, vdim, hd, page_size, table_stride, write_cache, rot, halves, eps};
-  if (is_bf16) hipLaunchKernelGGL(whole_norm_kv_kernel<bf16_t>, dim3(rows, 3), dim3(256), 0, (hipStream_t)stream, a);
-  else hipLaunchKernelGGL(whole_norm_kv_kernel<float>, dim3(rows, 3), dim3(256), 0, (hipStream_t)stream, a);
+  const dim3 grid(rows, write_cache ? 3 : 1);            // (a layer that reads another's cache has queries only)
+  const bool wide = (long long)heads * ((dim + 1) / 2) > 1024;
+  hipStream_t s = (hipStream_t)stream;
+  if (is_bf16 && wide) hipLaunchKernelGGL((whole_norm_kv_kernel<bf16_t, 8>), grid, dim3(256), 0, s, a);
+  else if (is_bf16) hipLaunchKernelGGL((whole_norm_kv_kernel<bf16_t, 4>), grid, dim3(256), 0, s, a);
+  else if (wide) hipLaunchKernelGGL((whole_norm_kv_kernel<float, 8>), grid, dim3(256), 0, s, a);
+  else hipLaunchKernelGGL((whole_norm_kv_kernel<float, 4>), grid, dim3(256), 0, s, a);
   return BW_LAUNCH_CHECK();
 }
 
@@ -666,7 +712,9 @@ extern "C" int bw_rglru_scan(float* y, int ldy, const float* y_bias, const float
 // place, wts (optional): y is then not the row itself but a table of rows of which this row is a weighted sum,
 // y_row[e] = sum_j wts[row][j] * y[place[row][j]][e], j ascending, one chain an element (what a feed-forward of routed
 // experts leaves: its choices' outputs by sorted place); the sum is formed here instead of by a launch of its own.
-template <typename WT>
+// Rows of up to 256 MAXV elements keep their values in registers, and everything the row needs is asked for before anything is
+// used; longer rows are read twice.
+template <typename WT, int MAXV>
 __global__ __launch_bounds__(256) void norm_add_kernel(const float* __restrict__ y, int ldy, const WT* __restrict__ w, float* __restrict__ x,
                                                        int ldx, bf16_t* __restrict__ rounded, int ldr, int dim, float eps,
                                                        const int32_t* __restrict__ place, const float* __restrict__ wts, int top,
@@ -680,15 +728,20 @@ __global__ __launch_bounds__(256) void norm_add_kernel(const float* __restrict__
     for (int j = 0; j < top; ++j) acc = fmaf(wts[(size_t)row * top + j], y[(size_t)place[(size_t)row * top + j] * ldy + e], acc);
     return acc;
   };
-  constexpr int MAXV = 8;                       // rows of up to 256 * MAXV elements keep their values in registers
-  float v[MAXV];
+  float* xr = x + (size_t)row * ldx;
+  float v[MAXV], xo[MAXV], wp[MAXV];
   float acc = 0.0f;
   if (dim <= 256 * MAXV) {
 #pragma unroll
     for (int j = 0; j < MAXV; ++j) {
-      const int e = tid + 256 * j;
-      v[j] = e < dim ? value(e) : 0.0f;
+      const int e = min(tid + 256 * j, dim - 1);
+      const bool in = 256 * j < dim;                     // (scalar)
+      v[j] = in ? value(e) : 0.0f;
+      xo[j] = in ? xr[e] : 0.0f;
+      wp[j] = in ? gm_load(w + e) : 0.0f;
     }
+#pragma unroll
+    for (int j = 0; j < MAXV; ++j) v[j] = tid + 256 * j < dim ? v[j] : 0.0f;
 #pragma unroll
     for (int j = 0; j < MAXV; ++j) acc = fmaf(v[j], v[j], acc);
   } else {
@@ -702,14 +755,13 @@ __global__ __launch_bounds__(256) void norm_add_kernel(const float* __restrict__
   __syncthreads();
   const float total = ((part[0] + part[1]) + part[2]) + part[3];
   const float inv = 1.0f / sqrtf(total / (float)dim + eps);
-  float* xr = x + (size_t)row * ldx;
   if (dim <= 256 * MAXV) {
 #pragma unroll
     for (int j = 0; j < MAXV; ++j) {
       const int e = tid + 256 * j;
       if (e < dim) {
-        const float normed = (v[j] * inv) * gm_load(w + e);
-        const float nx = scale == 1.0f ? xr[e] + normed : fmaf(scale, normed, xr[e]);
+        const float normed = (v[j] * inv) * wp[j];
+        const float nx = scale == 1.0f ? xo[j] + normed : fmaf(scale, normed, xo[j]);
         xr[e] = nx;
         if (rounded != nullptr) rounded[(size_t)row * ldr + e] = f32_to_bf16(nx);
       }
@@ -727,11 +779,14 @@ __global__ __launch_bounds__(256) void norm_add_kernel(const float* __restrict__
 extern "C" int bw_norm_add(const float* y, int ldy, const void* w, int w_is_bf16, float* x, int ldx, void* rounded, int ldr,
                            int rows, int dim, float eps, const int32_t* place, const float* wts, int top, float scale, void* stream) {
   if (rows <= 0) return 0;
-  const dim3 grid(rows);
-  if (w_is_bf16)
-    hipLaunchKernelGGL(norm_add_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, y, ldy, (const bf16_t*)w, x, ldx, (bf16_t*)rounded, ldr, dim, eps, place, wts, top, scale);
-  else
-    hipLaunchKernelGGL(norm_add_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, y, ldy, (const float*)w, x, ldx, (bf16_t*)rounded, ldr, dim, eps, place, wts, top, scale);
+  hipStream_t s = (hipStream_t)stream;
+  auto launch = [&](auto kernel, auto wt) {
+    hipLaunchKernelGGL(kernel, dim3(rows), dim3(256), 0, s, y, ldy, wt, x, ldx, (bf16_t*)rounded, ldr, dim, eps, place, wts, top, scale);
+  };
+  if (w_is_bf16 && dim <= 2048) launch(norm_add_kernel<bf16_t, 8>, (const bf16_t*)w);
+  else if (w_is_bf16) launch(norm_add_kernel<bf16_t, 16>, (const bf16_t*)w);
+  else if (dim <= 2048) launch(norm_add_kernel<float, 8>, (const float*)w);
+  else launch(norm_add_kernel<float, 16>, (const float*)w);
   return BW_LAUNCH_CHECK();
 }
 
@@ -909,13 +964,12 @@ __global__ __launch_bounds__(256) void scaled_sum_kernel(ScaledSumArgs a, float*
 }
 
 // x[r] += scale * (z / sqrt(mean(z^2) + eps) * w) with z that sum: the norm behind the mixer in the same launch, rounded as in
-// norm_add.  A workgroup a row; rows of up to 2,048 elements stay in registers, longer ones are formed twice (the same
+// norm_add.  A workgroup a row; rows of up to 256 MAXV elements stay in registers, longer ones are formed twice (the same
 // operations): the bits of scaled_sum_kernel followed by norm_add_kernel.
-template <int N>
+template <int N, int MAXV>
 __global__ __launch_bounds__(256) void scaled_sum_norm_add_kernel(ScaledSumArgs a, const float* __restrict__ w, float eps, float scale,
                                                                   float* __restrict__ x, int ldx, bf16_t* __restrict__ rounded, int ldr) {
   __shared__ float part[4];
-  constexpr int MAXV = 8;
   const int row = blockIdx.x, tid = threadIdx.x;
   auto value = [&](int e) -> float {
     float z = a.s[0] * a.y[0][(size_t)row * a.ldy[0] + e];
@@ -999,10 +1053,12 @@ extern "C" int bw_scaled_sum_norm_add(const float* const* y, const int* ldy, con
   if (scaled_sum_args(a, y, ldy, s, n, dim) != 0 || w == nullptr || ldx < dim || (rounded != nullptr && ldr < dim)) return -2;
   hipStream_t st = (hipStream_t)stream;
   bf16_t* r = (bf16_t*)rounded;
-  if (n == 1) hipLaunchKernelGGL(scaled_sum_norm_add_kernel<1>, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr);
-  else if (n == 2) hipLaunchKernelGGL(scaled_sum_norm_add_kernel<2>, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr);
-  else if (n == 3) hipLaunchKernelGGL(scaled_sum_norm_add_kernel<3>, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr);
-  else hipLaunchKernelGGL(scaled_sum_norm_add_kernel<4>, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr);
+  auto launch = [&](auto kernel) { hipLaunchKernelGGL(kernel, dim3(rows), dim3(256), 0, st, a, w, eps, scale, x, ldx, r, ldr); };
+  const bool wide = dim > 2048;
+  if (n == 1) wide ? launch(scaled_sum_norm_add_kernel<1, 16>) : launch(scaled_sum_norm_add_kernel<1, 8>);
+  else if (n == 2) wide ? launch(scaled_sum_norm_add_kernel<2, 16>) : launch(scaled_sum_norm_add_kernel<2, 8>);
+  else if (n == 3) wide ? launch(scaled_sum_norm_add_kernel<3, 16>) : launch(scaled_sum_norm_add_kernel<3, 8>);
+  else wide ? launch(scaled_sum_norm_add_kernel<4, 16>) : launch(scaled_sum_norm_add_kernel<4, 8>);
   return BW_LAUNCH_CHECK();
 }
 

@@ -40,7 +40,7 @@
 //
 // Epilogues: store 32-bit, store bfloat16, add into a 32-bit residual (each output owned
 // by one lane: no atomics), SwiGLU of two products (gate rows n, up rows N+n of a
-// stacked weight) stored as bfloat16: h = g * (1/(1+exp(-g))) * u in 32-bit, or rotary encoding of the
+// stacked weight) stored as bfloat16: h = g * (1/(1+exp(-g))) * u in 32-bit, the exact GELU stored as bfloat16, or rotary encoding of the
 // stacked q|k|v product and the write of k and v to their page slots (heads of 64; up to 64 rows: head sizes
 // in multiples of 64).
 #include <mutex>
@@ -132,6 +132,7 @@ __device__ __forceinline__ void epilogue_store(void* __restrict__ out, size_t o,
                                                float alpha = 1.0f) {
   if constexpr (EPI == EPI_F32) st_f32<DEV>((float*)out + o, v);
   else if constexpr (EPI == EPI_BF16) st_bf16<DEV>((bf16_t*)out + o, f32_to_bf16(v));
+  else if constexpr (EPI == EPI_GELU_BF16) st_bf16<DEV>((bf16_t*)out + o, f32_to_bf16(gelu_erf(v)));
   else if constexpr (EPI == EPI_ADD_F32) st_f32<DEV>((float*)out + o, ld_f32<DEV>((const float*)out + o) + v);
   else if constexpr (EPI == EPI_SWIGLU_BF16) st_bf16<DEV>((bf16_t*)out + o, f32_to_bf16(silu_times(v, u)));
   else if constexpr (EPI == EPI_CLAMPED_GLU_BF16) st_bf16<DEV>((bf16_t*)out + o, f32_to_bf16(clamped_swish_times<true>(v, u, limit, alpha)));
@@ -274,14 +275,15 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
       // (and so does a 32-bit store of up to 16 rows, whose segments those kernels give waves of their own, or with scratch
       // of up to 64 and four segments: 4,096 columns of K = 21,504 at 8 rows took 65 us as 64 workgroups with all of K
       // each, 29 as strips; at 64 rows of K = 8,192 21 us and 17.5, of K = 21,504, where the join weighs more, 33 and 39)
-      const bool whole_k = S == 1 || (EPI != EPI_ADD_F32 && !(EPI == EPI_F32 && (M <= 16 ? S <= 40 : split_ok && S <= 4)));
+      const bool whole_k = S == 1 || (EPI != EPI_ADD_F32 && !(EPI == EPI_F32 && (M <= 16 ? S <= 40 : split_ok && S <= 4)) &&
+                                     !(EPI == EPI_GELU_BF16 && M <= 16 && S <= 40));
       if (whole_k && K % 64 == 0 && wgs >= 64 && fits) {
         if (M <= 16) return launch_mid<EPI, 1, false>(x, w, out, M, N, K, ldx, ldo, wgs, s);
         if (M <= 32) return launch_mid<EPI, 2, false>(x, w, out, M, N, K, ldx, ldo, wgs, s);
         // 33 to 64 rows and so few columns that twice the workgroups still fit the chip at once: two blocks of 32 rows,
         // 32 columns a workgroup, which then pulls half the rows of x and half the weights (4096 columns of K = 2048
         // at 64 rows: 9.5 us against 14.1; 2048 columns, further down: 8.4 against 10.7)
-        if constexpr (EPI == EPI_ADD_F32 || EPI == EPI_F32 || EPI == EPI_BF16) {
+        if constexpr (EPI == EPI_ADD_F32 || EPI == EPI_F32 || EPI == EPI_BF16 || EPI == EPI_GELU_BF16) {
           if (2 * ((N + 31) / 32) <= 256)
             return launch_mid<EPI, 2, false, true>(x, w, out, M, N, K, ldx, ldo, (N + 31) / 32, s, MidNormArgs{}, QkvRopeArgs{}, 1,
                                                    MidSplitArgs{}, 2);
@@ -429,7 +431,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
         return BW_LAUNCH_CHECK();
       }
     }
-    if constexpr (EPI == EPI_F32 || EPI == EPI_BF16) {
+    if constexpr (EPI == EPI_F32 || EPI == EPI_BF16 || EPI == EPI_GELU_BF16) {
       // few enough workgroups of the 64-row kernel to be on the chip at once: all blocks of 64 rows in one launch (a
       // product of 6144 columns at 128 rows 13 us against 20 on 128 x 128 tiles; the SwiGLU product gains nothing)
       const int wgs = (N + 63) / 64, zb = (M + 63) / 64;
@@ -443,7 +445,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
       // (fewer of these tiles than compute units while the 128-row tiles below would fill the chip in one round: a step
       // of those takes half as long, so they win: gate|up of 512 rows 62 us here, half the chip idle)
       bool half_tiles_win = false;
-      if constexpr (EPI == EPI_F32 || EPI == EPI_BF16 || epi_is_glu(EPI)) {
+      if constexpr (EPI == EPI_F32 || EPI == EPI_BF16 || EPI == EPI_GELU_BF16 || epi_is_glu(EPI)) {
         const int t256 = ((M + 127) / 128) * bn;
         half_tiles_win = (t256 + 255) / 256 < 2 * ((bm * bn + 255) / 256);
       }
@@ -459,7 +461,7 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
         return BW_LAUNCH_CHECK();
       }
     }
-    if constexpr (EPI == EPI_F32 || EPI == EPI_BF16 || epi_is_glu(EPI) || EPI == EPI_QKV_ROPE) {
+    if constexpr (EPI == EPI_F32 || EPI == EPI_BF16 || EPI == EPI_GELU_BF16 || epi_is_glu(EPI) || EPI == EPI_QKV_ROPE) {
       // 128 x 256 tiles where they go round the compute units (the 256 x 256 kernel above took what it takes: one
       // segment of K and enough of its tiles); the q|k|v product of 600 to 1,200 rows among them (four heads of 64 a
       // tile, a head a wave as in the 128 x 128 tiles: 1,024 rows 45.8 us there)
@@ -557,6 +559,7 @@ extern "C" int bw_gemm_bf16(const void* x, const void* w, void* out, int M, int 
     case EPI_F32: return launch_gemm_bf16<EPI_F32>(xp, wp, out, M, N, K, ldx, ldo, s);
     case EPI_BF16: return launch_gemm_bf16<EPI_BF16>(xp, wp, out, M, N, K, ldx, ldo, s);
     case EPI_ADD_F32: return launch_gemm_bf16<EPI_ADD_F32>(xp, wp, out, M, N, K, ldx, ldo, s);
+    case EPI_GELU_BF16: return launch_gemm_bf16<EPI_GELU_BF16>(xp, wp, out, M, N, K, ldx, ldo, s);
     case EPI_SWIGLU_BF16: return launch_gemm_bf16<EPI_SWIGLU_BF16>(xp, wp, out, M, N, K, ldx, ldo, s);
   }
   return -2;

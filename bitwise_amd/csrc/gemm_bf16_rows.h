@@ -194,7 +194,7 @@ __device__ __forceinline__ void mid_body(const bf16_t* __restrict__ x, const bf1
         rp.positions += first;
         rp.row_seq += first;
         out = (void*)((bf16_t*)out + (size_t)first * rp.heads * rp.head_dim);
-      } else if constexpr (EPI == EPI_BF16 || EPI == EPI_SWIGLU_BF16) {
+      } else if constexpr (EPI == EPI_BF16 || EPI == EPI_GELU_BF16 || EPI == EPI_SWIGLU_BF16) {
         out = (void*)((bf16_t*)out + (size_t)first * ldo);
       } else {
         out = (void*)((float*)out + (size_t)first * ldo);

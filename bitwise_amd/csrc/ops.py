@@ -15,6 +15,7 @@ import torch
 from . import build as _build
 
 EPI_F32, EPI_BF16, EPI_ADD_F32, EPI_SWIGLU_BF16 = 0, 1, 2, 3
+EPI_GELU_BF16 = 6
 ATT_PART = 64          # keys per partition of the bfloat16 attention fold
 
 
@@ -457,7 +458,7 @@ def gemm_add_scratch(rows: int, N: int, K: int) -> Tuple[int, int]:
 def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, rows: int, epilogue: int,
               scratch: Optional[Tuple[torch.Tensor, torch.Tensor]] = None) -> None:
     """out[:rows] = epilogue(x[:rows] @ w.T) on the matrix cores; see gemm_bf16.hip for the
-    arithmetic.  EPI_SWIGLU_BF16 takes the stacked weight [2N, K] (gate rows, then up rows).
+    arithmetic.  EPI_GELU_BF16 stores the exact GELU of the 32-bit sums, rounded once.  EPI_SWIGLU_BF16 takes the stacked weight [2N, K] (gate rows, then up rows).
     ``scratch`` (EPI_ADD_F32 and EPI_F32): the tensors ``gemm_add_scratch`` asks for (float32, int32
     zeros); the bits do not depend on it.  ``x`` may be a column slice of a wider matrix that starts at a multiple of 8
     elements, and with a 32-bit store ``out`` may be a column slice too."""
@@ -470,7 +471,7 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, rows: int, ep
         if N % 2:
             raise ValueError("gemm_bf16: SwiGLU needs a stacked weight with an even number of rows")
         N //= 2
-    want = torch.bfloat16 if epilogue in (EPI_BF16, EPI_SWIGLU_BF16) else torch.float32
+    want = torch.bfloat16 if epilogue in (EPI_BF16, EPI_SWIGLU_BF16, EPI_GELU_BF16) else torch.float32
     if epilogue == EPI_F32:
         _need_strided(out, want, "out")
     else:

@@ -352,7 +352,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   constexpr bool GATES = MODE == RECUR_SCALAR_GATES;
   constexpr bool BONUS = MODE == RECUR_BONUS_DECAY, FIXED = MODE == RECUR_FIXED_DECAY, STEP = MODE == RECUR_STEP_DECAY;
   constexpr bool DELTA = MODE == RECUR_DELTA;
-  constexpr bool CHANNELS = !GATES && !STEP && !DELTA;   // a decay per channel comes through LDS
+  constexpr bool CHANNELS = !GATES && !STEP && !DELTA && !FIXED;   // a decay per channel comes through LDS
   constexpr int NN = (DPAD + 63) / 64;
   constexpr bool READ_OUT = PHASE != 1;
   constexpr int SPLIT = PHASE == 0 ? recur_split(DPAD) : recur_chunk_split(DPAD);
@@ -441,7 +441,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   const int hk = h / a.heads_per_key;
 
   // a chunk's operands on their way from memory (every load clamped into its row; what lies outside is zeroed on the way to LDS)
-  float rq[NQ], rk[NQ], rz[CHANNELS && !FIXED ? NQ : 1], rv[NV], rg[2];
+  float rq[NQ], rk[NQ], rz[CHANNELS ? NQ : 1], rv[NV], rg[2];
   auto fetch = [&](int t0) {
     if (t0 >= count) return;                             // (scalar)
     const int tc = min(RC, count - t0);
@@ -454,7 +454,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         const float* pr = a.proj + row * a.ldp;
         rq[u] = pr[a.q_off + hk * dim + d];
         rk[u] = pr[a.k_off + hk * dim + d];
-        if constexpr (CHANNELS && !FIXED) rz[u] = a.gate[row * a.ldg + a.gate_off + h * dim + d] + a.bias[h * dim + d];
+        if constexpr (CHANNELS) rz[u] = a.gate[row * a.ldg + a.gate_off + h * dim + d] + a.bias[h * dim + d];
       }
     }
 #pragma unroll
@@ -488,8 +488,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         }
         qs[buf][t][d] = in ? rq[u] * a.qscale : 0.0f;
         ks[buf][t][d] = in ? rk[u] * a.kscale : 0.0f;
-        if constexpr (FIXED) as[buf][t][d] = in ? fixed_decay : 0.0f;
-        else if constexpr (BONUS) as[buf][t][d] = in ? bw_expf(-bw_expf(rz[u])) : 0.0f;
+        if constexpr (BONUS) as[buf][t][d] = in ? bw_expf(-bw_expf(rz[u])) : 0.0f;
         else if constexpr (CHANNELS) as[buf][t][d] = in ? bw_expf(log_sigmoid(rz[u]) * a.param) : 0.0f;
       }
     }
@@ -586,14 +585,14 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
             if constexpr (READ_OUT) o[n] = fmaf(fmaf(ureg[d], kv, Sreg[d]), qr[n][d], o[n]);
             Sreg[d] = fmaf(ar[n][d], Sreg[d], kv);
           } else {
-            Sreg[d] = fmaf(ar[n][d], Sreg[d], kv);
+            Sreg[d] = fmaf(FIXED ? fixed_decay : ar[CHANNELS ? n : 0][CHANNELS ? d : 0], Sreg[d], kv);
             if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
           }
         }
         if constexpr (PHASE == 1) {
 #pragma unroll
           for (int i = 0; i < NN; ++i)
-            if (lane + 64 * i < DPAD) nreg[i] *= as[buf][t + n][lane + 64 * i];
+            if (lane + 64 * i < DPAD) nreg[i] *= FIXED ? fixed_decay : as[CHANNELS ? buf : 0][CHANNELS ? t + n : 0][CHANNELS ? lane + 64 * i : 0];
         }
       } else {
         const float ig = g1[n], fg = g2[n];
@@ -805,8 +804,7 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
 // or sigmoid.  A workgroup per (row, part): thread t owns elements t, t + 256, ... (one chain over its squares), the waves'
 // sums are joined by wave_sum and added in wave order.  Parts of up to 256 GP_MAXV elements keep their values in registers;
 // the same chain either way.
-#define GP_MAXV 8
-template <typename OT, bool BEHIND>
+template <typename OT, bool BEHIND, int GP_MAXV>
 __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __restrict__ o, int ldi, const float* __restrict__ z, int ldz,
                                                               const float* __restrict__ weight, OT* __restrict__ out, int ldo,
                                                               const int32_t* __restrict__ positions, int size, float eps, int gate) {
@@ -906,7 +904,7 @@ __global__ __launch_bounds__(256) void activate_kernel(const float* __restrict__
     if (act == PLAIN_XIELU) {
       h = z > 0.0f ? fmaf(p0 * z, z, 0.5f * z) : fmaf(0.5f + p1, expm1f(z) - z, 0.5f * z);
     } else if (act == PLAIN_GELU_ERF) {
-      h = (0.5f * z) * (1.0f + erff(z * 0.7071067811865476f));
+      h = gelu_erf(z);
     } else {
       const float m = fmaxf(z, 0.0f);
       h = m * m;
@@ -1051,14 +1049,14 @@ extern "C" int bw_gated_part_norm(const float* o, int ldi, const float* z, int l
   if (gate != GATE_SIGMOID && gate != GATE_SILU) return -2;
   const dim3 grid(rows, parts), block(256);
   hipStream_t s = (hipStream_t)stream;
-  if (out_is_bf16 && behind)
-    hipLaunchKernelGGL((gated_part_norm_kernel<bf16_t, true>), grid, block, 0, s, o, ldi, z, ldz, weight, (bf16_t*)out, ldo, positions, size, eps, gate);
-  else if (out_is_bf16)
-    hipLaunchKernelGGL((gated_part_norm_kernel<bf16_t, false>), grid, block, 0, s, o, ldi, z, ldz, weight, (bf16_t*)out, ldo, positions, size, eps, gate);
-  else if (behind)
-    hipLaunchKernelGGL((gated_part_norm_kernel<float, true>), grid, block, 0, s, o, ldi, z, ldz, weight, (float*)out, ldo, positions, size, eps, gate);
-  else
-    hipLaunchKernelGGL((gated_part_norm_kernel<float, false>), grid, block, 0, s, o, ldi, z, ldz, weight, (float*)out, ldo, positions, size, eps, gate);
+  auto launch = [&](auto kernel, auto op) {
+    hipLaunchKernelGGL(kernel, grid, block, 0, s, o, ldi, z, ldz, weight, op, ldo, positions, size, eps, gate);
+  };
+  const bool wide = size > 2048;
+  if (out_is_bf16 && behind) wide ? launch(gated_part_norm_kernel<bf16_t, true, 16>, (bf16_t*)out) : launch(gated_part_norm_kernel<bf16_t, true, 8>, (bf16_t*)out);
+  else if (out_is_bf16) wide ? launch(gated_part_norm_kernel<bf16_t, false, 16>, (bf16_t*)out) : launch(gated_part_norm_kernel<bf16_t, false, 8>, (bf16_t*)out);
+  else if (behind) wide ? launch(gated_part_norm_kernel<float, true, 16>, (float*)out) : launch(gated_part_norm_kernel<float, true, 8>, (float*)out);
+  else wide ? launch(gated_part_norm_kernel<float, false, 16>, (float*)out) : launch(gated_part_norm_kernel<float, false, 8>, (float*)out);
   return BW_LAUNCH_CHECK();
 }
 

@@ -150,7 +150,8 @@ class MLP(FeedForward):
     linear unit with two learned numbers: z > 0: softplus(p) z^2 + z/2; z <= 0: (1/2 + softplus(q)) (e^z - 1 - z) + z/2;
     or "gelu", z/2 (1 + erf(z / sqrt 2)).
     params: width, inter, act, names (up, down and, for xielu, the tensor [p, q]).  The product leaves 32-bit sums, the
-    activation is one 32-bit kernel behind it, which rounds once for the down projection."""
+    activation is one 32-bit kernel behind it, which rounds once for the down projection; on the matrix cores gelu is the
+    product's epilogue (the same function of the same sums)."""
 
     graph_safe = True
     launches_through_ops = True
@@ -197,11 +198,18 @@ class MLP(FeedForward):
         self.up.store(ctx.ws, h, z, ctx.rows)
         return z
 
+    def _inner(self, ctx, h) -> torch.Tensor:
+        if self.act == ops.PLAIN_GELU_ERF and self.up.mfma and h.dtype == torch.bfloat16:
+            act = ctx.ws.buffer("mlp_h", self.inter, torch.bfloat16)
+            ops.gemm_bf16(h, self.up.weight, act, ctx.rows, ops.EPI_GELU_BF16)
+            return act
+        return self._activated(ctx, self._up(ctx, h))
+
     def forward(self, ctx, h, residual) -> None:
-        self.down.add_into(ctx.ws, self._activated(ctx, self._up(ctx, h)), residual, ctx.rows)
+        self.down.add_into(ctx.ws, self._inner(ctx, h), residual, ctx.rows)
 
     def forward_out(self, ctx, h, out) -> None:
-        self.down.store(ctx.ws, self._activated(ctx, self._up(ctx, h)), out, ctx.rows)
+        self.down.store(ctx.ws, self._inner(ctx, h), out, ctx.rows)
 
     def forward_with_norm(self, ctx, x, norm, residual) -> bool:
         z = ctx.ws.buffer("mlp_up", self.inter, torch.float32)
