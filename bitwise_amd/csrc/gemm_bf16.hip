@@ -277,7 +277,11 @@ static int launch_gemm_bf16(const bf16_t* x, const bf16_t* w, void* out, int M, 
       // each, 29 as strips; at 64 rows of K = 8,192 21 us and 17.5, of K = 21,504, where the join weighs more, 33 and 39)
       const bool whole_k = S == 1 || (EPI != EPI_ADD_F32 && !(EPI == EPI_F32 && (M <= 16 ? S <= 40 : split_ok && S <= 4)) &&
                                      !(EPI == EPI_GELU_BF16 && M <= 16 && S <= 40));
-      if (whole_k && K % 64 == 0 && wgs >= 64 && fits) {
+      // (up to 16 rows stored as they are: a wave per strip is faster where the workgroups of 64 columns leave half the compute
+      // units idle or go into a second round: 5,120 columns of K = 2,048 at 8 rows 12.2 us and 7.8, 17,472 columns 23.4
+      // and 19.3)
+      const bool strips_win = (EPI == EPI_F32 || EPI == EPI_GELU_BF16) && M <= 16 && S <= 40 && (wgs < 112 || wgs > 256);
+      if (whole_k && K % 64 == 0 && wgs >= 64 && fits && !strips_win) {
         if (M <= 16) return launch_mid<EPI, 1, false>(x, w, out, M, N, K, ldx, ldo, wgs, s);
         if (M <= 32) return launch_mid<EPI, 2, false>(x, w, out, M, N, K, ldx, ldo, wgs, s);
         // 33 to 64 rows and so few columns that twice the workgroups still fit the chip at once: two blocks of 32 rows,
