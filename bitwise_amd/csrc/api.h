@@ -118,10 +118,11 @@ int bw_norm_shift(const float* x, int ldx, const float* w, const float* mix, flo
 // mode 4: a step size per head, delta = softplus(logit at gate_off + head + bias[head]); decay exp(-bias2[head] delta), the
 // token enters as k (delta v)^T, skip[head] v (optional) joins the read-out.
 // q is multiplied by qscale, k by kscale; heads_per_key neighbouring heads share one q and one k.
-// (silu 1, fixed decay only: q, k and v pass SiLU on their way in)
+// (silu 1, fixed decay only: q, k and v pass SiLU on their way in; few 1: the requests bring a few rows each, which picks the
+// kernel that favours many waves over long walks, the same bits)
 int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_off, int k_off, int v_off, const float* gate, int ldg,
                          int gate_off, int gate2_off, const float* bias, const float* bias2, float param, float qscale,
-                         float kscale, const float* skip, int heads_per_key, int silu, float* state, long long state_ld, float* out,
+                         float kscale, const float* skip, int heads_per_key, int silu, int few, float* state, long long state_ld, float* out,
                          int ldo, const int32_t* seq_rows,
                          const int32_t* slots, const int32_t* positions, int nseq, int heads, int dim, int vdim,
                          const int32_t* chunks, int nchunks, const int32_t* spans, int nspans, float* scan_local,
@@ -186,7 +187,7 @@ int bw_causal_conv(const float* x, int ldx, const float* in_bias, const void* w,
                    const int32_t* positions, int nseq, int max_seq_rows, float* out, int ldo, int silu, void* stream);
 // The convolution with SiLU of causal_conv over [q heads | k heads | v] (key_heads heads of dim channels each, then v_channels),
 // q and k heads made unit vectors, x / sqrt(sum x^2 + eps), q times qscale; and per head of the memory, gates_out[r] =
-// [beta (heads) | g (heads)], beta = sigmoid(gate[b_off + h]), g = exp(-rate[h] softplus(gate[a_off + h] + dt_bias[h]))
+// [beta (heads) | g (heads) | k.q (key_heads)], beta = sigmoid(gate[b_off + h]), g = exp(-rate[h] softplus(gate[a_off + h] + dt_bias[h]))
 int bw_conv_heads(const float* x, int ldx, const float* w, int taps, int key_heads, int dim, int v_channels, float qscale, float eps,
                   float* state, long long state_ld, const float* gate, int ldg, int a_off, int b_off, const float* dt_bias,
                   const float* rate, int heads, float* gates_out, int ldgo, const int32_t* seq_rows, const int32_t* slots,

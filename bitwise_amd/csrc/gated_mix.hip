@@ -134,10 +134,10 @@ extern "C" int bw_causal_conv(const float* x, int ldx, const float* in_bias, con
 // ------------------------------------------------------------------------------ what a delta memory reads
 
 // One launch for everything between the projections and a delta memory's recurrence: a causal convolution with SiLU per
-// channel over [q heads | k heads | v], every q and k head made a unit vector (x / sqrt(sum x^2 + eps), q then times qscale),
-// and a head's step size beta = sigmoid(zb) and decay g = exp(-rate softplus(za + dt_bias)).  A wave a head of q or k (its
-// channels lane, lane + 64, ...), a wave per 64 NC channels of v, a wave for the gates; CONV_HEADS_CHUNK tokens each.  The
-// convolution's sums are those of causal_conv.
+// channel over [q heads | k heads | v], every q and k head made a unit vector (x / sqrt(sum x^2 + eps), q then times qscale), the
+// two vectors' product k.q, and a head's step size beta = sigmoid(zb) and decay g = exp(-rate softplus(za + dt_bias)).  A
+// wave a key head (its q and its k, channels lane, lane + 64, ...), a wave per 64 NC channels of v, a wave for the gates;
+// CONV_HEADS_CHUNK tokens each.  The convolution's sums are those of causal_conv.
 #define CONV_HEADS_CHUNK 16
 
 struct ConvHeadsArgs {
@@ -151,15 +151,72 @@ struct ConvHeadsArgs {
   const float* gate;       // [rows, ldg]: za of head h at a_off + h, zb at b_off + h
   const float* dt_bias;    // [heads]
   const float* rate;       // [heads]
-  float* gates_out;        // [rows, ldgo]: beta of head h at column h, g at heads + h
+  float* gates_out;        // [rows, ldgo]: beta of head h at column h, g at heads + h, k.q of key head j at 2 heads + j
   long long state_ld;
-  int ldx, ldo, channels, ldg, a_off, b_off, ldgo, heads, unit_heads, scaled_heads, dim, items;
+  int ldx, ldo, channels, ldg, a_off, b_off, ldgo, heads, key_heads, dim, items;
   float qscale, eps;
+};
+
+// A lane's NC channels of one stretch (a head, or part of the values): their taps and the inputs before the current token.
+template <int TAPS, int NC>
+struct ConvStretch {
+  static constexpr int P = TAPS > 1 ? TAPS - 1 : 1;
+  float w[NC][TAPS], win[NC][P], old[NC][P];
+  int ch[NC];
+
+  __device__ __forceinline__ void start(const ConvHeadsArgs& a, const float* x, const float* st, int c0, int count, int t0, int lane) {
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      ch[i] = c0 + min(lane + 64 * i, count - 1);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) w[i][j] = a.w[(size_t)ch[i] * TAPS + j];
+      // only the request's first chunk reaches back before the portion, and only its waves touch the slot
+#pragma unroll
+      for (int j = 0; j < P; ++j) old[i][j] = (TAPS > 1 && t0 == 0) ? st[(size_t)j * a.channels + ch[i]] : 0.0f;
+#pragma unroll
+      for (int j = 0; j < P; ++j) {
+        win[i][j] = t0 == 0 ? old[i][j] : x[(size_t)max(t0 - (TAPS - 1) + j, 0) * a.ldx + ch[i]];
+      }
+    }
+  }
+  __device__ __forceinline__ float token(int i, float cur) {
+    float acc = 0.0f;
+    if constexpr (TAPS > 1) {
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) acc = fmaf(w[i][j], win[i][j], acc);
+    }
+    acc = fmaf(w[i][TAPS - 1], cur, acc);
+    acc *= gm_sigmoid(acc);
+    if constexpr (TAPS > 1) {
+#pragma unroll
+      for (int j = 0; j + 1 < TAPS - 1; ++j) win[i][j] = win[i][j + 1];
+      win[i][TAPS - 2] = cur;
+    }
+    return acc;
+  }
+  __device__ __forceinline__ void leave(const ConvHeadsArgs& a, const float* x, float* st, int count, int n, int lane) {
+    if constexpr (TAPS > 1) {
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        if (lane + 64 * i >= count) continue;
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j) {
+          const int idx = n - (TAPS - 1) + j;
+          float v = 0.0f;
+          if (idx >= 0) v = x[(size_t)idx * a.ldx + ch[i]];
+          else {
+#pragma unroll
+            for (int q = 0; q < P; ++q) v = (q == TAPS - 1 + idx) ? old[i][q] : v;
+          }
+          st[(size_t)j * a.channels + ch[i]] = v;
+        }
+      }
+    }
+  }
 };
 
 template <int TAPS, int NC>
 __global__ __launch_bounds__(256) void conv_heads_kernel(ConvHeadsArgs a) {
-  constexpr int P = TAPS > 1 ? TAPS - 1 : 1;
   const int item = blockIdx.x * 4 + wave_index(), lane = threadIdx.x & 63;
   const int seq = blockIdx.y, t0 = blockIdx.z * CONV_HEADS_CHUNK;
   const int first = a.seq_rows[2 * seq], n = a.seq_rows[2 * seq + 1], slot = a.slots[seq];
@@ -176,84 +233,79 @@ __global__ __launch_bounds__(256) void conv_heads_kernel(ConvHeadsArgs a) {
     }
     return;
   }
-  const bool unit = item < a.unit_heads;
-  const int c0 = unit ? item * a.dim : a.unit_heads * a.dim + (item - a.unit_heads) * 64 * NC;
-  const int count = unit ? a.dim : min(64 * NC, a.channels - c0);
-  const float post = item < a.scaled_heads ? a.qscale : 1.0f;
-  float w[NC][TAPS], win[NC][P], old[NC][P];
-  int ch[NC];
-#pragma unroll
-  for (int i = 0; i < NC; ++i) {
-    ch[i] = c0 + min(lane + 64 * i, count - 1);
-#pragma unroll
-    for (int j = 0; j < TAPS; ++j) w[i][j] = a.w[(size_t)ch[i] * TAPS + j];
-  }
   float* st = a.state + (size_t)slot * a.state_ld;
   const float* x = a.x + (size_t)first * a.ldx;
-  // only the request's first chunk reaches back before the portion, and only its waves touch the slot
-#pragma unroll
-  for (int i = 0; i < NC; ++i) {
-#pragma unroll
-    for (int j = 0; j < P; ++j) old[i][j] = (TAPS > 1 && t0 == 0) ? st[(size_t)j * a.channels + ch[i]] : 0.0f;
-#pragma unroll
-    for (int j = 0; j < P; ++j) {
-      const int idx = t0 - (TAPS - 1) + j;
-      win[i][j] = idx >= 0 ? x[(size_t)idx * a.ldx + ch[i]] : old[i][(TAPS - 1 + idx) < 0 ? 0 : (TAPS - 1 + idx)];
-    }
-  }
   float* o = a.out + (size_t)first * a.ldo;
   constexpr int UN = 4;
+  ConvStretch<TAPS, NC> A;
+  if (item < a.key_heads) {
+    ConvStretch<TAPS, NC> B;
+    A.start(a, x, st, item * a.dim, a.dim, t0, lane);
+    B.start(a, x, st, (a.key_heads + item) * a.dim, a.dim, t0, lane);
+    for (int tb = t0; tb < t1; tb += UN) {
+      float ca[UN][NC], cb[UN][NC];
+#pragma unroll
+      for (int u = 0; u < UN; ++u)
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+          const float* xr = x + (size_t)min(tb + u, t1 - 1) * a.ldx;
+          ca[u][i] = xr[A.ch[i]];
+          cb[u][i] = xr[B.ch[i]];
+        }
+#pragma unroll
+      for (int u = 0; u < UN; ++u) {
+        if (tb + u >= t1) continue;                      // (scalar)
+        float q[NC], k[NC], qq = 0.0f, kk = 0.0f, kq = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+          q[i] = A.token(i, ca[u][i]);
+          k[i] = B.token(i, cb[u][i]);
+          if (lane + 64 * i < a.dim) {
+            qq = fmaf(q[i], q[i], qq);
+            kk = fmaf(k[i], k[i], kk);
+            kq = fmaf(k[i], q[i], kq);
+          }
+        }
+        qq = wave_sum(qq);                               // (three sums that wait for nothing but themselves)
+        kk = wave_sum(kk);
+        kq = wave_sum(kq);
+        const float iq = 1.0f / sqrtf(qq + a.eps) * a.qscale, ik = 1.0f / sqrtf(kk + a.eps);
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+          if (lane + 64 * i < a.dim) {
+            o[(size_t)(tb + u) * a.ldo + A.ch[i]] = q[i] * iq;
+            o[(size_t)(tb + u) * a.ldo + B.ch[i]] = k[i] * ik;
+          }
+        }
+        if (lane == 0) a.gates_out[(size_t)(first + tb + u) * a.ldgo + 2 * a.heads + item] = kq * iq * ik;
+      }
+    }
+    if (t0 == 0) {
+      A.leave(a, x, st, a.dim, n, lane);
+      B.leave(a, x, st, a.dim, n, lane);
+    }
+    return;
+  }
+  const int c0 = 2 * a.key_heads * a.dim + (item - a.key_heads) * 64 * NC;
+  const int count = min(64 * NC, a.channels - c0);
+  A.start(a, x, st, c0, count, t0, lane);
   for (int tb = t0; tb < t1; tb += UN) {
     float cur[UN][NC];
 #pragma unroll
     for (int u = 0; u < UN; ++u)
 #pragma unroll
-      for (int i = 0; i < NC; ++i) cur[u][i] = x[(size_t)min(tb + u, t1 - 1) * a.ldx + ch[i]];
+      for (int i = 0; i < NC; ++i) cur[u][i] = x[(size_t)min(tb + u, t1 - 1) * a.ldx + A.ch[i]];
 #pragma unroll
     for (int u = 0; u < UN; ++u) {
-      if (tb + u >= t1) continue;                        // (scalar)
-      float y[NC], ss = 0.0f;
+      if (tb + u >= t1) continue;
 #pragma unroll
       for (int i = 0; i < NC; ++i) {
-        float acc = 0.0f;
-        if constexpr (TAPS > 1) {
-#pragma unroll
-          for (int j = 0; j < TAPS - 1; ++j) acc = fmaf(w[i][j], win[i][j], acc);
-        }
-        acc = fmaf(w[i][TAPS - 1], cur[u][i], acc);
-        acc *= gm_sigmoid(acc);
-        y[i] = acc;
-        if (lane + 64 * i < count) ss = fmaf(acc, acc, ss);
-        if constexpr (TAPS > 1) {
-#pragma unroll
-          for (int j = 0; j + 1 < TAPS - 1; ++j) win[i][j] = win[i][j + 1];
-          win[i][TAPS - 2] = cur[u][i];
-        }
-      }
-      float inv = 1.0f;
-      if (unit) inv = 1.0f / sqrtf(wave_sum(ss) + a.eps);
-#pragma unroll
-      for (int i = 0; i < NC; ++i)
-        if (lane + 64 * i < count) o[(size_t)(tb + u) * a.ldo + ch[i]] = unit ? (y[i] * inv) * post : y[i];
-    }
-  }
-  if (TAPS > 1 && t0 == 0) {
-#pragma unroll
-    for (int i = 0; i < NC; ++i) {
-      if (lane + 64 * i >= count) continue;
-#pragma unroll
-      for (int j = 0; j < TAPS - 1; ++j) {
-        const int idx = n - (TAPS - 1) + j;
-        float v = 0.0f;
-        if (idx >= 0) v = x[(size_t)idx * a.ldx + ch[i]];
-        else {
-#pragma unroll
-          for (int q = 0; q < P; ++q) v = (q == TAPS - 1 + idx) ? old[i][q] : v;
-        }
-        st[(size_t)j * a.channels + ch[i]] = v;
+        const float y = A.token(i, cur[u][i]);
+        if (lane + 64 * i < count) o[(size_t)(tb + u) * a.ldo + A.ch[i]] = y;
       }
     }
   }
+  if (t0 == 0) A.leave(a, x, st, count, n, lane);
 }
 
 template <int NC>
@@ -274,13 +326,13 @@ extern "C" int bw_conv_heads(const float* x, int ldx, const float* w, int taps, 
                              void* stream) {
   if (nseq <= 0 || max_seq_rows <= 0) return 0;
   if (taps < 1 || taps > CONV_MAX_TAPS || (taps > 1 && state == nullptr) || key_heads < 1 || dim < 1 || dim > 256 || v_channels < 1 ||
-      heads < 1 || ldgo < 2 * heads)
+      heads < 1 || ldgo < 2 * heads + key_heads)
     return -2;
   const int channels = 2 * key_heads * dim + v_channels, nc = (dim + 63) / 64;
   if (ldx < channels || ldo < channels || (taps > 1 && state_ld < (long long)(taps - 1) * channels)) return -2;
-  const int items = 2 * key_heads + (v_channels + 64 * nc - 1) / (64 * nc) + 1;
+  const int items = key_heads + (v_channels + 64 * nc - 1) / (64 * nc) + 1;
   ConvHeadsArgs a{x, w, state, out, seq_rows, slots, positions, gate, dt_bias, rate, gates_out, state_ld, ldx, ldo, channels, ldg,
-                  a_off, b_off, ldgo, heads, 2 * key_heads, key_heads, dim, items, qscale, eps};
+                  a_off, b_off, ldgo, heads, key_heads, dim, items, qscale, eps};
   const dim3 grid((items + 3) / 4, nseq, (max_seq_rows + CONV_HEADS_CHUNK - 1) / CONV_HEADS_CHUNK);
   if (grid.y > 65535 || grid.z > 65535) return -2;
   hipStream_t s = (hipStream_t)stream;

@@ -95,7 +95,7 @@ _SIGS = {
     "bw_norm_mean": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_void_p],
     "bw_norm_mean_add": [c_void_p, c_void_p, c_void_p, c_int, c_float, c_void_p, c_float, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
     "bw_linear_recurrence": [c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p,
-                             c_float, c_float, c_float, c_void_p, c_int, c_int, c_void_p, c_longlong, c_void_p, c_int, c_void_p, c_void_p,
+                             c_float, c_float, c_float, c_void_p, c_int, c_int, c_int, c_void_p, c_longlong, c_void_p, c_int, c_void_p, c_void_p,
                              c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_longlong, c_void_p],
     "bw_head_norm_gate": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_int,
                           c_int, c_int, c_float, c_void_p],
@@ -855,7 +855,8 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
                       gate2_off: int, bias: Optional[torch.Tensor], bias2: Optional[torch.Tensor], param: float, qscale: float,
                       state: torch.Tensor, out: torch.Tensor, seq_rows: torch.Tensor, slots: torch.Tensor,
                       positions: torch.Tensor, nseq: int, heads: int, dim: int, vdim: int, scan=None, kscale: float = 1.0,
-                      heads_per_key: int = 1, skip: Optional[torch.Tensor] = None, silu: bool = False) -> None:
+                      heads_per_key: int = 1, skip: Optional[torch.Tensor] = None, silu: bool = False,
+                      few_rows: bool = False) -> None:
     """The recurrence S <- decay * S + k v^T, o = S^T (q * qscale) per head over every request's rows in order, from and
     to ``state`` [slots, elements].  RECUR_DECAY_PER_CHANNEL: decay = exp(logsigmoid(gate + bias) * param) per key
     channel (``gate`` [rows, >= gate_off + heads*dim]).  RECUR_SCALAR_GATES: capped input and forget gates per head
@@ -867,8 +868,10 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
     decay = exp(-bias2[h] delta) (``bias2`` [heads]: the rates), the token enters as k (delta v)^T, and ``skip`` [heads]
     (optional) times v joins the read-out.
     RECUR_DELTA: a step size b and a decay a per head and token, as they are (``gate`` columns gate_off + h and gate2_off + h;
-    ``bias`` None): S <- a S, S <- S + k (b (v - S^T k))^T, then the read-out; always in one pass.
-    ``silu`` (fixed decay): q, k and v are the SiLU of what ``proj`` holds.
+    behind the decays, from gate2_off + heads on, the products k.q of the key heads, as they enter; ``bias`` None):
+    S <- a S, S <- S + k (b (v - S^T k))^T, then the read-out; always in one pass.
+    ``silu`` (fixed decay): q, k and v are the SiLU of what ``proj`` holds.  ``few_rows``: every request brings a few rows (the same
+    bits; a kernel that favours many waves over long walks).
     k is multiplied by ``kscale``; ``heads_per_key`` neighbouring heads share one q and one k.  A head's state lies as
     [value column][key channel].  ``state`` may be a column slice of a wider tensor.
 
@@ -905,7 +908,7 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
             raise ValueError("linear_recurrence: step sizes, their bias or the rates do not fit the heads")
         need = heads * dim * vdim
     elif mode == RECUR_DELTA:
-        if max(gate_off, gate2_off) + heads > gate.shape[1] or scan is not None:
+        if gate_off + heads > gate.shape[1] or gate2_off + heads + heads // max(heads_per_key, 1) > gate.shape[1] or scan is not None:
             raise ValueError("linear_recurrence: step sizes and decays do not fit the heads, or passes over chunks were asked of a delta memory")
         need = heads * dim * vdim
     elif mode == RECUR_FIXED_DECAY:
@@ -948,7 +951,7 @@ def linear_recurrence(mode: int, proj: torch.Tensor, q_off: int, k_off: int, v_o
                                        0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0),
                                        gate_off, gate2_off, 0 if bias is None else bias.data_ptr(),
                                        0 if bias2 is None else bias2.data_ptr(), float(param), float(qscale), float(kscale),
-                                       0 if skip is None else skip.data_ptr(), int(heads_per_key), int(silu), state.data_ptr(),
+                                       0 if skip is None else skip.data_ptr(), int(heads_per_key), int(silu), int(few_rows), state.data_ptr(),
                                        state.stride(0), out.data_ptr(), out.stride(0), seq_rows.data_ptr(), slots.data_ptr(),
                                        positions.data_ptr(), nseq, heads, dim, vdim,
                                        0 if chunks is None else chunks.data_ptr(), nchunks,
@@ -1356,8 +1359,9 @@ def conv_heads(x: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tens
     """What a delta memory reads, in one launch.  ``x`` [rows, q | k | v] float32 (a column slice will do): ``key_heads`` heads of
     ``dim`` channels of queries, as many of keys, then the values' channels.  Every channel passes the causal convolution of
     ``causal_conv`` (weight [channels, taps] float32, ``state`` likewise) and SiLU; a head of q or k is then divided by
-    sqrt(sum x^2 + eps), q also multiplied by ``qscale``; to ``out``, x's layout.  ``gates`` [rows, 2*heads] receives
-    sigmoid(gate[:, b_off + h]) and, behind the heads, exp(-rate[h] * softplus(gate[:, a_off + h] + dt_bias[h]))."""
+    sqrt(sum x^2 + eps), q also multiplied by ``qscale``; to ``out``, x's layout.  ``gates`` [rows, 2*heads + key_heads]
+    receives sigmoid(gate[:, b_off + h]), behind the heads exp(-rate[h] * softplus(gate[:, a_off + h] + dt_bias[h])), and behind
+    those every key head's k.q."""
     for t, what in ((x, "x"), (gate, "gate"), (out, "out"), (gates, "gates")):
         _need_strided(t, torch.float32, what)
     for t, what in ((weight, "weight"), (dt_bias, "dt_bias"), (rate, "rate")):
@@ -1370,7 +1374,7 @@ def conv_heads(x: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tens
         raise ValueError(f"conv_heads: {taps} taps of heads of {dim}; the kernel takes 1 to {CONV_MAX_TAPS} and heads of up to {RECUR_MAX_DIM}")
     if key_heads < 1 or channels <= 2 * key_heads * dim or x.shape[1] < channels or out.shape[1] < channels:
         raise ValueError("conv_heads: x, out or the weight do not fit the heads")
-    if rate.numel() != heads or gates.shape[1] < 2 * heads or max(a_off, b_off) + heads > gate.shape[1] or min(a_off, b_off) < 0:
+    if rate.numel() != heads or gates.shape[1] < 2 * heads + key_heads or max(a_off, b_off) + heads > gate.shape[1] or min(a_off, b_off) < 0:
         raise ValueError("conv_heads: gates, rates or biases do not fit the heads")
     if seq_rows.numel() < 2 * nseq or slots.numel() < nseq:
         raise ValueError("conv_heads: fewer request records than requests")

@@ -271,6 +271,24 @@ __device__ __forceinline__ float join_parts(float v) {
   return v;
 }
 
+// The sums of N values at once, each over the SPLIT lanes of its column: with N = 4 the lanes end with value (bit 5) + 2 (bit 4) of
+// their number, with N = 2 with value (bit 5).  The additions, and so the bits, of join_parts for each.
+template <int SPLIT, int N>
+__device__ __forceinline__ float join_parts_of(const float* v) {
+  static_assert((N == 4 && SPLIT >= 4) || (N == 2 && SPLIT >= 2), "");
+  float y = lane_pair_sum<32>(v[0], v[1]);
+  if constexpr (N == 4) {
+    y = lane_pair_sum<16>(y, lane_pair_sum<32>(v[2], v[3]));
+  } else if constexpr (SPLIT >= 4) {
+    float lower, upper;
+    lane_halves<16>(y, lower, upper);
+    y = lower + upper;
+  }
+  if constexpr (SPLIT >= 8) y += lane_xor<8>(y);
+  if constexpr (SPLIT >= 16) y += lane_xor<4>(y);
+  return y;
+}
+
 struct RecurArgs {
   const float* proj;       // [rows, ldp]: the rows' stacked projections
   int ldp, q_off, k_off, v_off;
@@ -303,7 +321,7 @@ struct RecurArgs {
 // A wave holds the state of 64 / SPLIT value columns of one head in registers: SPLIT lanes a column, each with DH consecutive
 // key channels, so that a head has many short waves; the parts' read-outs are added by lane exchanges in one order whatever
 // runs the head (a single token, a portion, a chunk): the split depends on the head's size alone.  The tokens' q, k, decays
-// and v come through LDS in chunks of RC tokens, shared by the workgroup's waves (neighbouring column blocks of one head);
+// and v come through LDS in chunks of a few tokens, shared by the workgroup's waves (neighbouring column blocks of one head);
 // the next chunk is on its way from memory while one is worked on.  In memory a column's channels lie side by side,
 // [column][channel], so a lane's part is a run of whole vectors.
 //
@@ -320,6 +338,8 @@ struct RecurArgs {
 //   S[d][j] <- e^(-bias2[head] delta) S[d][j] + k[d] (delta v[j]),  o[j] = (S^T q)[j] + skip[head] v[j].
 // RECUR_DELTA:  a step size beta (at gate_off + head) and a decay a (at gate2_off + head) per head and token, as they are;
 //   u[j] = beta (v[j] - a (S^T k)[j]),  S[d][j] <- a S[d][j] + k[d] u[j],  o[j] = (S^T q)[j]: what k reads is replaced towards v.
+//   The read-out is formed from the memory before the write, o = a (S^T q) + (k.q) u, so that only S^T k stands between a token
+//   and the next; k.q comes with the gates (at gate2_off + heads + key group).
 //   (The step of a chunk as a whole is a full matrix and not a decay, so there are no passes over chunks.)
 // (a head's q and k are those of key group head / heads_per_key.)
 // (q is multiplied by qscale and k by kscale on their way into LDS.)
@@ -328,8 +348,9 @@ struct RecurArgs {
 // own: PHASE 1 runs every chunk from a zero state (no read-out) and leaves the chunk's own contribution and its decay;
 // recurrence_scan_kernel walks a request's chunks in order and leaves the state each one starts from; PHASE 3 runs every
 // chunk from there with the read-out, and the request's last chunk leaves the state in the slot.  PHASE 0 walks
-// the whole portion.  The passes differ from PHASE 0 by the rounding of the scan's sums only.
-#define RC 16
+// the whole portion; PHASE 4 does so for steps of a few tokens a request (decoding), where what counts is how many waves are
+// on the chip with their states' loads under way: no groups of tokens, no second buffer, few registers, the same arithmetic.  The passes differ from PHASE 0 by the rounding of the scan's sums only.
+#define RECUR_CHUNK 16   // tokens staged together
 #define RW 4             // waves of a workgroup
 // floats of a chunk's record for one head: S, a vector, two scalars, in whole vectors of four
 __host__ __device__ __forceinline__ size_t recur_record(int dim, int vdim) { return ((size_t)dim * vdim + dim + 2 + 3) & ~(size_t)3; }
@@ -347,6 +368,13 @@ __host__ __device__ constexpr int recur_blocks(int dim, int vdim, bool chunks = 
   return (vdim + recur_columns(dim, chunks) - 1) / recur_columns(dim, chunks);
 }
 
+// What a lane needs of N tokens.
+template <int TOKENS, int DH, bool CHANNELS>
+struct RecurOps {
+  static constexpr int N = TOKENS;
+  float k[N][DH], q[N][DH], a[CHANNELS ? N : 1][CHANNELS ? DH : 1], v[N], g1[N], g2[N], kq[N];
+};
+
 template <int MODE, int DPAD, int PHASE>
 __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a) {
   constexpr bool GATES = MODE == RECUR_SCALAR_GATES;
@@ -355,16 +383,18 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   constexpr bool CHANNELS = !GATES && !STEP && !DELTA && !FIXED;   // a decay per channel comes through LDS
   constexpr int NN = (DPAD + 63) / 64;
   constexpr bool READ_OUT = PHASE != 1;
-  constexpr int SPLIT = PHASE == 0 ? recur_split(DPAD) : recur_chunk_split(DPAD);
+  constexpr bool WALK = PHASE == 0 || PHASE == 4;
+  constexpr int SPLIT = WALK ? recur_split(DPAD) : recur_chunk_split(DPAD);
   constexpr int DH = DPAD / SPLIT, COLS = 64 / SPLIT, WCOLS = RW * COLS;
-  constexpr int TU = PHASE != 0 ? 1 : (SPLIT >= 4 ? 4 : 2);      // tokens worked on together
+  constexpr int TU = PHASE != 0 ? 1 : (SPLIT >= 4 && DH <= 8 ? 4 : 2);      // tokens worked on together (two groups of them fit the registers)
   constexpr int BUFS = PHASE != 0 ? 1 : 2;               // (the passes over chunks hide the loads behind other waves)
+  constexpr int RC = PHASE == 4 && DPAD >= 64 ? 4 : RECUR_CHUNK;
   constexpr int NQ = RC * DPAD / (64 * RW), NV = (RC * WCOLS + 64 * RW - 1) / (64 * RW);
   static_assert(NQ * 64 * RW == RC * DPAD && RC % TU == 0, "a chunk is whole loads and whole groups of tokens");
   __shared__ __attribute__((aligned(16))) float qs[BUFS][RC][DPAD];
   __shared__ __attribute__((aligned(16))) float ks[BUFS][RC][DPAD];
   __shared__ __attribute__((aligned(16))) float as[CHANNELS ? BUFS : 1][CHANNELS ? RC : 1][CHANNELS ? DPAD : 4];
-  __shared__ float gi[BUFS][RC], gf[BUFS][RC];
+  __shared__ float gi[BUFS][RC], gf[BUFS][RC], gd[DELTA ? BUFS : 1][DELTA ? RC : 1];
   __shared__ float vs[BUFS][RC][WCOLS];
   const int lane = threadIdx.x & 63, wv = wave_index();
   const int h = blockIdx.y;
@@ -372,7 +402,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   const size_t rec = recur_record(dim, vdim);
   int first, count, slot;
   bool leaves_state = true;
-  if constexpr (PHASE == 0) {
+  if constexpr (WALK) {
     const int s = blockIdx.z;
     first = a.seq_rows[2 * s];
     count = a.seq_rows[2 * s + 1];
@@ -394,7 +424,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   // (every workgroup of a head carries the normaliser and the maximum, so each keeps a copy of its own in the slot: one that
   // starts late must not find what another has already written)
   const size_t copy = (size_t)a.heads * dim + a.heads;
-  const size_t own = GATES && PHASE == 0 ? blockIdx.x * copy : 0;
+  const size_t own = GATES && WALK ? blockIdx.x * copy : 0;
   float* nv = st + (size_t)a.heads * dim * vdim + own + (size_t)h * dim;
   float* mv = st + (size_t)a.heads * dim * vdim + own + (size_t)a.heads * dim + h;
   // where this wave's state comes from: the slot, nothing, or the chunk's start record
@@ -440,21 +470,47 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   const float skip = STEP && a.skip != nullptr ? a.skip[h] : 0.0f;
   const int hk = h / a.heads_per_key;
 
-  // a chunk's operands on their way from memory (every load clamped into its row; what lies outside is zeroed on the way to LDS)
-  float rq[NQ], rk[NQ], rz[CHANNELS ? NQ : 1], rv[NV], rg[2];
+  // a chunk's operands on their way from memory (every load clamped into its row; what lies outside is zeroed on the way to LDS);
+  // q, k and decay logits as 16-byte vectors where the rows allow it: vector u of a thread is elements 4u .. 4u + 3 of its rq
+  constexpr bool WIDE = NQ % 4 == 0;
+  const bool vectors = WIDE && (dim & 3) == 0 && ((a.q_off | a.k_off | a.ldp) & 3) == 0 && (reinterpret_cast<uintptr_t>(a.proj) & 15) == 0 &&
+                       (!CHANNELS || (((a.ldg | a.gate_off) & 3) == 0 && ((reinterpret_cast<uintptr_t>(a.gate) | reinterpret_cast<uintptr_t>(a.bias)) & 15) == 0));   // (scalar)
+  float rq[NQ], rk[NQ], rz[CHANNELS ? NQ : 1], rv[NV], rg[3];
   auto fetch = [&](int t0) {
     if (t0 >= count) return;                             // (scalar)
     const int tc = min(RC, count - t0);
+    if (vectors) {
 #pragma unroll
-    for (int u = 0; u < NQ; ++u) {
-      if (64 * RW * u < tc * DPAD) {                     // (scalar)
-        const int e = 64 * RW * u + (int)threadIdx.x;
-        const size_t row = (size_t)(first + t0 + min(e / DPAD, tc - 1));
-        const int d = min(e % DPAD, dim - 1);
-        const float* pr = a.proj + row * a.ldp;
-        rq[u] = pr[a.q_off + hk * dim + d];
-        rk[u] = pr[a.k_off + hk * dim + d];
-        if constexpr (CHANNELS) rz[u] = a.gate[row * a.ldg + a.gate_off + h * dim + d] + a.bias[h * dim + d];
+      for (int u = 0; u < NQ / 4; ++u) {
+        if (256 * RW * u < tc * DPAD) {                  // (scalar)
+          const int e = 64 * RW * u + (int)threadIdx.x;
+          const size_t row = (size_t)(first + t0 + min(e / (DPAD / 4), tc - 1));
+          const int d = min(4 * (e % (DPAD / 4)), dim - 4);
+          const float* pr = a.proj + row * a.ldp + hk * dim + d;
+          const f32x4 q4 = *reinterpret_cast<const f32x4*>(pr + a.q_off), k4 = *reinterpret_cast<const f32x4*>(pr + a.k_off);
+          f32x4 z4 = {0.f, 0.f, 0.f, 0.f};
+          if constexpr (CHANNELS)
+            z4 = *reinterpret_cast<const f32x4*>(a.gate + row * a.ldg + a.gate_off + h * dim + d) + *reinterpret_cast<const f32x4*>(a.bias + h * dim + d);
+#pragma unroll
+          for (int x = 0; x < 4; ++x) {
+            rq[4 * u + x] = q4[x];
+            rk[4 * u + x] = k4[x];
+            if constexpr (CHANNELS) rz[4 * u + x] = z4[x];
+          }
+        }
+      }
+    } else {
+#pragma unroll
+      for (int u = 0; u < NQ; ++u) {
+        if (64 * RW * u < tc * DPAD) {                   // (scalar)
+          const int e = 64 * RW * u + (int)threadIdx.x;
+          const size_t row = (size_t)(first + t0 + min(e / DPAD, tc - 1));
+          const int d = min(e % DPAD, dim - 1);
+          const float* pr = a.proj + row * a.ldp;
+          rq[u] = pr[a.q_off + hk * dim + d];
+          rk[u] = pr[a.k_off + hk * dim + d];
+          if constexpr (CHANNELS) rz[u] = a.gate[row * a.ldg + a.gate_off + h * dim + d] + a.bias[h * dim + d];
+        }
       }
     }
 #pragma unroll
@@ -469,35 +525,59 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
       const float* gr = a.gate + (size_t)(first + t0 + min((int)threadIdx.x, tc - 1)) * a.ldg;
       rg[0] = gr[a.gate_off + h];
       rg[1] = GATES || DELTA ? gr[a.gate2_off + h] : 0.0f;
+      rg[2] = DELTA ? gr[a.gate2_off + a.heads + hk] : 0.0f;
     }
   };
+  auto decay_of = [&](float z) { return BONUS ? bw_expf(-bw_expf(z)) : bw_expf(log_sigmoid(z) * a.param); };
   auto stash = [&](int t0, int buf) {
     if (t0 >= count) return;
     const int tc = min(RC, count - t0);
+    if constexpr (FIXED) {
+      if (a.silu) {                                      // (scalar)
 #pragma unroll
-    for (int u = 0; u < NQ; ++u) {
-      if (64 * RW * u < tc * DPAD) {
-        const int e = 64 * RW * u + (int)threadIdx.x;
-        const int t = e / DPAD, d = e % DPAD;
-        const bool in = d < dim;
-        if constexpr (FIXED) {
-          if (a.silu) {                                  // (scalar)
-            rq[u] = silu(rq[u]);
-            rk[u] = silu(rk[u]);
-          }
+        for (int u = 0; u < NQ; ++u) {
+          rq[u] = silu(rq[u]);
+          rk[u] = silu(rk[u]);
         }
-        qs[buf][t][d] = in ? rq[u] * a.qscale : 0.0f;
-        ks[buf][t][d] = in ? rk[u] * a.kscale : 0.0f;
-        if constexpr (BONUS) as[buf][t][d] = in ? bw_expf(-bw_expf(rz[u])) : 0.0f;
-        else if constexpr (CHANNELS) as[buf][t][d] = in ? bw_expf(log_sigmoid(rz[u]) * a.param) : 0.0f;
+#pragma unroll
+        for (int u = 0; u < NV; ++u) rv[u] = silu(rv[u]);
+      }
+    }
+    if (vectors) {
+#pragma unroll
+      for (int u = 0; u < NQ / 4; ++u) {
+        if (256 * RW * u < tc * DPAD) {
+          const int e = 64 * RW * u + (int)threadIdx.x;
+          const int t = e / (DPAD / 4), d = 4 * (e % (DPAD / 4));
+          const bool in = d < dim;
+          f32x4 q4, k4, a4;
+#pragma unroll
+          for (int x = 0; x < 4; ++x) {
+            q4[x] = in ? rq[4 * u + x] * a.qscale : 0.0f;
+            k4[x] = in ? rk[4 * u + x] * a.kscale : 0.0f;
+            if constexpr (CHANNELS) a4[x] = in ? decay_of(rz[4 * u + x]) : 0.0f;
+          }
+          *reinterpret_cast<f32x4*>(&qs[buf][t][d]) = q4;
+          *reinterpret_cast<f32x4*>(&ks[buf][t][d]) = k4;
+          if constexpr (CHANNELS) *reinterpret_cast<f32x4*>(&as[buf][t][d]) = a4;
+        }
+      }
+    } else {
+#pragma unroll
+      for (int u = 0; u < NQ; ++u) {
+        if (64 * RW * u < tc * DPAD) {
+          const int e = 64 * RW * u + (int)threadIdx.x;
+          const int t = e / DPAD, d = e % DPAD;
+          const bool in = d < dim;
+          qs[buf][t][d] = in ? rq[u] * a.qscale : 0.0f;
+          ks[buf][t][d] = in ? rk[u] * a.kscale : 0.0f;
+          if constexpr (CHANNELS) as[buf][t][d] = in ? decay_of(rz[u]) : 0.0f;
+        }
       }
     }
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       const int e = 64 * RW * u + (int)threadIdx.x;
-      if constexpr (FIXED) {
-        if (a.silu) rv[u] = silu(rv[u]);
-      }
       if (64 * RW * u < tc * WCOLS && e < RC * WCOLS) vs[buf][e / WCOLS][e % WCOLS] = j_wg + e % WCOLS < vdim ? rv[u] : 0.0f;
     }
     if constexpr (GATES) {
@@ -511,6 +591,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
       if ((int)threadIdx.x < tc) {
         gi[buf][threadIdx.x] = rg[0];
         gf[buf][threadIdx.x] = rg[1];
+        gd[buf][threadIdx.x] = rg[2];
       }
     }
     if constexpr (STEP) {
@@ -522,10 +603,9 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
     }
   };
 
-  // N tokens from t on: their operands out of LDS together, then one after the other
-  auto tokens = [&](auto count_tag, int t0, int buf, int t) {
-    constexpr int N = decltype(count_tag)::value;
-    float kr[N][DH], qr[N][DH], ar[CHANNELS ? N : 1][CHANNELS ? DH : 1], vr[N], g1[N], g2[N], o[N];
+  // N tokens' operands out of LDS, from token t of the chunk on
+  auto load_tokens = [&](auto& O, int buf, int t) {
+    constexpr int N = std::remove_reference_t<decltype(O)>::N;
 #pragma unroll
     for (int n = 0; n < N; ++n) {
 #pragma unroll
@@ -534,30 +614,37 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         const f32x4 qv = *reinterpret_cast<const f32x4*>(&qs[buf][t + n][dbase + d]);
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          kr[n][d + e] = kv[e];
-          qr[n][d + e] = qv[e];
+          O.k[n][d + e] = kv[e];
+          O.q[n][d + e] = qv[e];
         }
         if constexpr (CHANNELS) {
           const f32x4 av = *reinterpret_cast<const f32x4*>(&as[buf][t + n][dbase + d]);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) ar[n][d + e] = av[e];
+          for (int e = 0; e < 4; ++e) O.a[n][d + e] = av[e];
         }
       }
-      vr[n] = vs[buf][t + n][j_in];
+      O.v[n] = vs[buf][t + n][j_in];
       if constexpr (GATES || STEP || DELTA) {
-        g1[n] = gi[buf][t + n];
-        g2[n] = gf[buf][t + n];
+        O.g1[n] = gi[buf][t + n];
+        O.g2[n] = gf[buf][t + n];
       }
+      if constexpr (DELTA) O.kq[n] = gd[buf][t + n];
     }
+  };
+
+  // those tokens one after the other
+  auto run_tokens = [&](auto& O, int t0, int buf, int t) {
+    constexpr int N = std::remove_reference_t<decltype(O)>::N;
+    float o[N], w[DELTA ? N : 1];
 #pragma unroll
     for (int n = 0; n < N; ++n) {
       o[n] = 0.0f;
       if constexpr (STEP) {
-        const float fa = g2[n], bv = g1[n] * vr[n];
+        const float fa = O.g2[n], bv = O.g1[n] * O.v[n];
 #pragma unroll
         for (int d = 0; d < DH; ++d) {
-          Sreg[d] = fmaf(fa, Sreg[d], kr[n][d] * bv);
-          if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
+          Sreg[d] = fmaf(fa, Sreg[d], O.k[n][d] * bv);
+          if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], O.q[n][d], o[n]);
         }
         if constexpr (PHASE == 1) {
 #pragma unroll
@@ -565,28 +652,32 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         }
       } else if constexpr (DELTA) {
         // (two chains over a lane's channels, then the column's lanes: the one sum the next token waits for)
-        float r0 = 0.0f, r1 = 0.0f;
+        float r0 = 0.0f, r1 = 0.0f, o1 = 0.0f;
 #pragma unroll
         for (int d = 0; d < DH; d += 2) {
-          r0 = fmaf(Sreg[d], kr[n][d], r0);
-          r1 = fmaf(Sreg[d + 1], kr[n][d + 1], r1);
+          r0 = fmaf(Sreg[d], O.k[n][d], r0);
+          r1 = fmaf(Sreg[d + 1], O.k[n][d + 1], r1);
         }
-        const float fa = g2[n], u = g1[n] * fmaf(-fa, join_parts<SPLIT>(r0 + r1), vr[n]);
+        const float fa = O.g2[n], u = O.g1[n] * fmaf(-fa, join_parts<SPLIT>(r0 + r1), O.v[n]);
 #pragma unroll
-        for (int d = 0; d < DH; ++d) {
-          Sreg[d] = fmaf(fa, Sreg[d], kr[n][d] * u);
-          o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
+        for (int d = 0; d < DH; d += 2) {
+          o[n] = fmaf(Sreg[d], O.q[n][d], o[n]);
+          o1 = fmaf(Sreg[d + 1], O.q[n][d + 1], o1);
         }
+        o[n] += o1;
+        w[n] = O.kq[n] * u;
+#pragma unroll
+        for (int d = 0; d < DH; ++d) Sreg[d] = fmaf(fa, Sreg[d], O.k[n][d] * u);
       } else if constexpr (!GATES) {
 #pragma unroll
         for (int d = 0; d < DH; ++d) {
-          const float kv = kr[n][d] * vr[n];
+          const float kv = O.k[n][d] * O.v[n];
           if constexpr (BONUS) {
-            if constexpr (READ_OUT) o[n] = fmaf(fmaf(ureg[d], kv, Sreg[d]), qr[n][d], o[n]);
-            Sreg[d] = fmaf(ar[n][d], Sreg[d], kv);
+            if constexpr (READ_OUT) o[n] = fmaf(fmaf(ureg[d], kv, Sreg[d]), O.q[n][d], o[n]);
+            Sreg[d] = fmaf(O.a[n][d], Sreg[d], kv);
           } else {
-            Sreg[d] = fmaf(FIXED ? fixed_decay : ar[CHANNELS ? n : 0][CHANNELS ? d : 0], Sreg[d], kv);
-            if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
+            Sreg[d] = fmaf(FIXED ? fixed_decay : O.a[CHANNELS ? n : 0][CHANNELS ? d : 0], Sreg[d], kv);
+            if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], O.q[n][d], o[n]);
           }
         }
         if constexpr (PHASE == 1) {
@@ -595,17 +686,17 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
             if (lane + 64 * i < DPAD) nreg[i] *= FIXED ? fixed_decay : as[CHANNELS ? buf : 0][CHANNELS ? t + n : 0][CHANNELS ? lane + 64 * i : 0];
         }
       } else {
-        const float ig = g1[n], fg = g2[n];
+        const float ig = O.g1[n], fg = O.g2[n];
         const float mn = fmaxf(fg + m, ig);
         const float fa = bw_expf(fg + m - mn);
         const float ib = bw_expf(ig - mn);
         m = mn;
         fsum += fg;
-        const float bv = ib * vr[n];
+        const float bv = ib * O.v[n];
 #pragma unroll
         for (int d = 0; d < DH; ++d) {
-          Sreg[d] = fmaf(fa, Sreg[d], kr[n][d] * bv);
-          if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], qr[n][d], o[n]);
+          Sreg[d] = fmaf(fa, Sreg[d], O.k[n][d] * bv);
+          if constexpr (READ_OUT) o[n] = fmaf(Sreg[d], O.q[n][d], o[n]);
         }
         float sum = 0.0f;
 #pragma unroll
@@ -624,18 +715,37 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
       }
     }
     if constexpr (READ_OUT) {
-      // (part n of a column stores token t + n)
-      float mine = 0.0f;
+      float* orow = a.out + (size_t)(first + t0 + t) * a.ldo + h * vdim + j;
+      if constexpr (!GATES && N == TU && (N == 4 || N == 2) && SPLIT >= N) {
+        // the columns' sums of all N tokens at once; a lane ends with the token its number names, the first of a column's
+        // lanes with that token stores it
+        const int mine = N == 4 ? (lane >> 5) + 2 * ((lane >> 4) & 1) : lane >> 5;
+        const bool stores = N == 4 ? (lane & 15) < COLS : (lane & 31) < COLS;
+        float v = join_parts_of<SPLIT, N>(o);
+        auto pick = [&](float x0, float x1, float x2, float x3) {      // (by value: an array by address would go to memory)
+          const float lo = (mine & 1) ? x1 : x0, hi = (mine & 1) ? x3 : x2;
+          return (mine & 2) ? hi : lo;
+        };
+        if constexpr (STEP) v = fmaf(skip, pick(O.v[0], O.v[1], O.v[N - 2], O.v[N - 1]), v);
+        if constexpr (DELTA) v = fmaf(pick(O.g2[0], O.g2[1], O.g2[N - 2], O.g2[N - 1]), v, pick(w[0], w[1], w[N - 2], w[N - 1]));
+        if (live && stores) orow[(size_t)mine * a.ldo] = v;
+      } else {
+        // (part n of a column stores token t + n)
+        float mine = 0.0f;
 #pragma unroll
-      for (int n = 0; n < N; ++n) {
-        float v = o[n];
-        if constexpr (!GATES) v = join_parts<SPLIT>(v);
-        if constexpr (STEP) v = fmaf(skip, vr[n], v);
-        mine = part == n ? v : mine;
+        for (int n = 0; n < N; ++n) {
+          float v = o[n];
+          if constexpr (!GATES) v = join_parts<SPLIT>(v);
+          if constexpr (STEP) v = fmaf(skip, O.v[n], v);
+          if constexpr (DELTA) v = fmaf(O.g2[n], v, w[n]);
+          mine = part == n ? v : mine;
+        }
+        if (live && part < N) orow[(size_t)part * a.ldo] = mine;
       }
-      if (live && part < N) a.out[(size_t)(first + t0 + t + part) * a.ldo + h * vdim + j] = mine;
     }
   };
+  using Group = RecurOps<TU, DH, CHANNELS>;
+  using Single = RecurOps<1, DH, CHANNELS>;
 
   if constexpr (BUFS == 2) {
     fetch(0);
@@ -654,8 +764,31 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
       __syncthreads();
     }
     int t = 0;
-    for (; t + TU <= tc; t += TU) tokens(std::integral_constant<int, TU>{}, t0, buf, t);
-    for (; t < tc; ++t) tokens(std::integral_constant<int, 1>{}, t0, buf, t);
+    if (BUFS == 2 && tc == RC) {
+      // a whole chunk: a group's operands are on their way while the group before it is worked on
+      Group even, odd;
+      load_tokens(even, buf, 0);
+#pragma unroll
+      for (int g = 0; g < RC / TU; g += 2) {
+        load_tokens(odd, buf, (g + 1) * TU);
+        __builtin_amdgcn_sched_barrier(0);
+        run_tokens(even, t0, buf, g * TU);
+        if (g + 2 < RC / TU) load_tokens(even, buf, (g + 2) * TU);
+        __builtin_amdgcn_sched_barrier(0);
+        run_tokens(odd, t0, buf, (g + 1) * TU);
+      }
+      t = RC;
+    }
+    for (; t + TU <= tc; t += TU) {
+      Group group;
+      load_tokens(group, buf, t);
+      run_tokens(group, t0, buf, t);
+    }
+    for (; t < tc; ++t) {
+      Single single;
+      load_tokens(single, buf, t);
+      run_tokens(single, t0, buf, t);
+    }
     if constexpr (BUFS == 2) {
       stash(t0 + RC, buf ^ 1);
       __syncthreads();
@@ -684,7 +817,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         if (dbase + d < dim) S_out[(size_t)j * dim + dbase + d] = Sreg[d];
     }
   }
-  if (wv == 0 && (PHASE == 0 ? GATES : blockIdx.x == 0 && (GATES || PHASE == 1))) {
+  if (wv == 0 && (WALK ? GATES : blockIdx.x == 0 && (GATES || PHASE == 1))) {
     // (the last of the passes leaves every workgroup's copy)
     const int copies = PHASE == 3 ? recur_blocks(dim, vdim) : 1;
     for (int k = 0; k < copies; ++k) {
@@ -741,7 +874,7 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurArgs a, const
 
 template <int MODE, int PHASE>
 int launch_recurrence(const RecurArgs& a, int units, hipStream_t s) {
-  const dim3 grid(recur_blocks(a.dim, a.vdim, PHASE != 0), a.heads, units), block(64 * RW);
+  const dim3 grid(recur_blocks(a.dim, a.vdim, PHASE == 1 || PHASE == 3), a.heads, units), block(64 * RW);
   if (a.dim <= 16) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 16, PHASE>), grid, block, 0, s, a);
   else if (a.dim <= 32) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 32, PHASE>), grid, block, 0, s, a);
   else if (a.dim <= 64) hipLaunchKernelGGL((linear_recurrence_kernel<MODE, 64, PHASE>), grid, block, 0, s, a);
@@ -752,9 +885,9 @@ int launch_recurrence(const RecurArgs& a, int units, hipStream_t s) {
 }
 
 template <int MODE>
-int launch_recurrence_passes(const RecurArgs& a, int nseq, int nchunks, const int32_t* spans, int nspans, hipStream_t s) {
+int launch_recurrence_passes(const RecurArgs& a, int nseq, bool few, int nchunks, const int32_t* spans, int nspans, hipStream_t s) {
   int rc = 0;
-  if (nseq > 0) rc = launch_recurrence<MODE, 0>(a, nseq, s);
+  if (nseq > 0) rc = few ? launch_recurrence<MODE, 4>(a, nseq, s) : launch_recurrence<MODE, 0>(a, nseq, s);
   if (rc != 0 || nchunks <= 0) return rc;
   if constexpr (MODE == RECUR_DELTA) {
     return -2;
@@ -996,7 +1129,7 @@ extern "C" int bw_norm_shift(const float* x, int ldx, const float* w, const floa
 
 extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_off, int k_off, int v_off, const float* gate,
                                     int ldg, int gate_off, int gate2_off, const float* bias, const float* bias2, float param,
-                                    float qscale, float kscale, const float* skip, int heads_per_key, int silu, float* state, long long state_ld, float* out, int ldo,
+                                    float qscale, float kscale, const float* skip, int heads_per_key, int silu, int few, float* state, long long state_ld, float* out, int ldo,
                                     const int32_t* seq_rows, const int32_t* slots, const int32_t* positions, int nseq,
                                     int heads, int dim, int vdim, const int32_t* chunks, int nchunks, const int32_t* spans,
                                     int nspans, float* scan_local, float* scan_start, long long scan_floats, void* stream) {
@@ -1014,12 +1147,12 @@ extern "C" int bw_linear_recurrence(int mode, const float* proj, int ldp, int q_
   RecurArgs a{proj, ldp, q_off, k_off, v_off, gate, ldg, gate_off, gate2_off, bias, bias2, skip, heads_per_key, param, qscale, kscale, silu, state, state_ld,
               out, ldo, seq_rows, slots, positions, heads, dim, vdim, chunks, scan_local, scan_start};
   hipStream_t s = (hipStream_t)stream;
-  if (mode == RECUR_SCALAR_GATES) return launch_recurrence_passes<RECUR_SCALAR_GATES>(a, nseq, nchunks, spans, nspans, s);
-  if (mode == RECUR_DECAY_PER_CHANNEL) return launch_recurrence_passes<RECUR_DECAY_PER_CHANNEL>(a, nseq, nchunks, spans, nspans, s);
-  if (mode == RECUR_BONUS_DECAY) return launch_recurrence_passes<RECUR_BONUS_DECAY>(a, nseq, nchunks, spans, nspans, s);
-  if (mode == RECUR_FIXED_DECAY) return launch_recurrence_passes<RECUR_FIXED_DECAY>(a, nseq, nchunks, spans, nspans, s);
-  if (mode == RECUR_STEP_DECAY) return launch_recurrence_passes<RECUR_STEP_DECAY>(a, nseq, nchunks, spans, nspans, s);
-  if (mode == RECUR_DELTA) return launch_recurrence_passes<RECUR_DELTA>(a, nseq, nchunks, spans, nspans, s);
+  if (mode == RECUR_SCALAR_GATES) return launch_recurrence_passes<RECUR_SCALAR_GATES>(a, nseq, few != 0, nchunks, spans, nspans, s);
+  if (mode == RECUR_DECAY_PER_CHANNEL) return launch_recurrence_passes<RECUR_DECAY_PER_CHANNEL>(a, nseq, few != 0, nchunks, spans, nspans, s);
+  if (mode == RECUR_BONUS_DECAY) return launch_recurrence_passes<RECUR_BONUS_DECAY>(a, nseq, few != 0, nchunks, spans, nspans, s);
+  if (mode == RECUR_FIXED_DECAY) return launch_recurrence_passes<RECUR_FIXED_DECAY>(a, nseq, few != 0, nchunks, spans, nspans, s);
+  if (mode == RECUR_STEP_DECAY) return launch_recurrence_passes<RECUR_STEP_DECAY>(a, nseq, few != 0, nchunks, spans, nspans, s);
+  if (mode == RECUR_DELTA) return launch_recurrence_passes<RECUR_DELTA>(a, nseq, few != 0, nchunks, spans, nspans, s);
   return -2;
 }
 

@@ -81,7 +81,7 @@ class GatedDelta(_MatrixMemoryMixer):
     def _run(self, ctx, call, y, target, add: bool) -> None:
         ws = ctx.ws
         u = ws.buffer("delta_u", self.channels, torch.float32)
-        gates = ws.buffer("delta_gates", 2 * self.heads, torch.float32)
+        gates = ws.buffer("delta_gates", 2 * self.heads + self.kv_heads, torch.float32)
         ops.conv_heads(y, self.conv_w, call.state[:, self.memory:] if self.taps > 1 else None, y, self.offsets["a"], self.offsets["b"],
                        self.dt_bias, self.rate, self.kv_heads, self.dim, ctx.seq_rows, ctx.slots, ctx.positions, ctx.nseq,
                        max_seq_rows(ctx), u, gates, float(self.dim) ** -0.5, self.unit_eps)

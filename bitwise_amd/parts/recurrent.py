@@ -35,6 +35,7 @@ from .gated_attention import max_seq_rows
 from .linear import Linear
 
 
+FEW_SEQ_ROWS = 4         # steps whose requests bring up to so many rows each run the recurrence's kernel for decoding
 SCAN_CHUNK = 32          # rows of a chunk of a long portion
 SCAN_MIN_ROWS = 96       # portions from this many rows on run in three passes over chunks (shorter ones are walked whole),
                          # where the engine allows logits to depend on the cut in their last bits (Workspace.exact_cuts False)
@@ -152,7 +153,8 @@ class _MatrixMemoryMixer(Mixer):
             scan = (chunks, nchunks, spans, nspans, local, start)
         ops.linear_recurrence(self.mode, y, at["r"] if "q" not in at else at["q"], at["k"], at["v"], gate, gate_off, gate2_off,
                               bias, bias2, param, self.qscale, call.state if state is None else state, raw, seq_rows, ctx.slots, ctx.positions, nseq,
-                              self.heads, self.dim, self.vdim, scan=scan, kscale=kscale, heads_per_key=heads_per_key, skip=skip, silu=silu)
+                              self.heads, self.dim, self.vdim, scan=scan, kscale=kscale, heads_per_key=heads_per_key, skip=skip, silu=silu,
+                              few_rows=max_seq_rows(ctx) <= FEW_SEQ_ROWS)
 
     def _finish(self, ctx, y, raw, target, add: bool = True, g_off: Optional[int] = None) -> None:
         act = ctx.ws.buffer("recur_gated", self.heads * self.vdim, self.rt.act_dtype)
@@ -430,7 +432,6 @@ class Lightning(_MatrixMemoryMixer):
     tensors: q, k [heads*dim, width]; v, g [heads*vdim, width]; norm [heads*vdim]; o [width, heads*vdim]."""
 
     mode = ops.RECUR_FIXED_DECAY
-    STAGED_SILU_ROWS = 4      # steps whose requests bring up to so many rows each apply SiLU where the recurrence loads its operands
 
     def __init__(self, params, runtime):
         super().__init__(params, runtime)
@@ -458,7 +459,7 @@ class Lightning(_MatrixMemoryMixer):
         ws, rows, inner = ctx.ws, ctx.rows, self.heads * self.vdim
         y = projected if projected is not None else self._project(ctx, h)
         # (every block of a head's columns stages its q and k again, so a portion's are made once, in place; the same function)
-        staged = max_seq_rows(ctx) <= self.STAGED_SILU_ROWS
+        staged = max_seq_rows(ctx) <= FEW_SEQ_ROWS
         if not staged:
             ops.silu_rows(y[:, :self.offsets["g"]], rows)
         raw = ws.buffer("recur_out", inner, torch.float32)

@@ -20,9 +20,9 @@ pytestmark = pytest.mark.gpu
 # float32: 32-bit sums against float64 ones, a few 1e-6 of a row.  bfloat16: activations rounded where the products and the
 # cache take them, carried through the layers; a row whose sublayer nearly cancels is blown up by the norm behind it, its
 # roundings with it, so in that mode the 90th percentile carries the tight bound.
-TOL = {"float32": 5e-5, "bfloat16": 0.06}
+TOL = {"float32": 2e-5, "bfloat16": 0.06}
 MOST = {"float32": 1.0, "bfloat16": 0.9}
-TYPICAL = {"float32": 1e-5, "bfloat16": 2.5e-2}
+TYPICAL = {"float32": 3e-6, "bfloat16": 3e-2}
 SIGMA = 0.15
 
 
@@ -454,7 +454,7 @@ def test_what_a_delta_memory_reads_against_plain(gpu, key_heads, heads, dim, vdi
         u = torch.cat([(q * dim ** -0.5).reshape(n, qk), k.reshape(n, qk), u[:, 2 * qk:]], 1)
         beta = torch.sigmoid(s[:, channels + heads:].double())
         decay = torch.exp(-rate.double() * pn.softplus(s[:, channels:channels + heads].double() + bias.double()))
-        want.append((u, torch.cat([beta, decay], 1)))
+        want.append((u, torch.cat([beta, decay, (q * k).sum(-1) * dim ** -0.5], 1)))
 
     def run(steps):
         state = torch.full((2, max(1, (taps - 1) * channels) + 3), float("nan"), device=gpu)
@@ -469,7 +469,7 @@ def test_what_a_delta_memory_reads_against_plain(gpu, key_heads, heads, dim, vdi
                 pos += list(range(at[r], at[r] + m))
                 slots.append(slot_of[r])
             xd = torch.cat(x).to(gpu)[:, 2:]
-            out, gates = torch.zeros(len(pos), channels, device=gpu), torch.zeros(len(pos), 2 * heads, device=gpu)
+            out, gates = torch.zeros(len(pos), channels, device=gpu), torch.zeros(len(pos), 2 * heads + key_heads, device=gpu)
             ops.conv_heads(xd, wc.to(gpu), state[:, 3:] if taps > 1 else None, xd, channels, channels + heads, bias.to(gpu), rate.to(gpu),
                            key_heads, dim, dev(seq_rows), dev(slots), dev(pos), len(step), max(m for _, m in step), out, gates, dim ** -0.5, 1e-6)
             o = 0
@@ -501,7 +501,8 @@ def test_delta_recurrence_against_plain(gpu, heads, key_heads, dim, vdim):
     want = pn.delta_recurrence(q.double().view(T, key_heads, dim), k.double().view(T, key_heads, dim), v.double().view(T, heads, vdim),
                                decay.double(), beta.double())
     dev = _dev(gpu)
-    u, gates = torch.cat([q, k, v], 1).to(gpu), torch.cat([beta, decay], 1).to(gpu)
+    kq = (k.double() * q.double()).view(T, key_heads, dim).sum(-1).float()
+    u, gates = torch.cat([q, k, v], 1).to(gpu), torch.cat([beta, decay, kq], 1).to(gpu)
     positions = dev(list(range(T)))
 
     def run(cuts):
@@ -511,7 +512,8 @@ def test_delta_recurrence_against_plain(gpu, heads, key_heads, dim, vdim):
             rows = slice(at, at + n)
             o = torch.zeros(n, hv, device=gpu)
             ops.linear_recurrence(ops.RECUR_DELTA, u[rows], 0, qk, 2 * qk, gates[rows], 0, heads, None, None, 0.0, 1.0, state, o, dev([0, n]),
-                                  dev([1]), positions[rows].contiguous(), 1, heads, dim, vdim, heads_per_key=heads // key_heads)
+                                  dev([1]), positions[rows].contiguous(), 1, heads, dim, vdim, heads_per_key=heads // key_heads,
+                                  few_rows=n <= 2)
             out[rows] = o
             at += n
         return out
@@ -558,7 +560,7 @@ def test_fading_recurrence_with_silu_against_plain(gpu, heads, dim, vdim):
                         torch.zeros(len(chunks) * rec, device=gpu), torch.zeros(len(chunks) * rec, device=gpu))
                 seq_rows, nseq = dev([0, 0]), 0
             ops.linear_recurrence(ops.RECUR_FIXED_DECAY, yd[rows], 0, hd, 2 * hd, None, 0, 0, dd, None, 0.0, 1.0, state, o, seq_rows, dev([0]),
-                                  positions[rows].contiguous(), nseq, heads, dim, vdim, scan=scan, silu=staged)
+                                  positions[rows].contiguous(), nseq, heads, dim, vdim, scan=scan, silu=staged, few_rows=n <= 2)
             out[rows] = o
             at += n
         return out
