@@ -113,16 +113,6 @@ __device__ __forceinline__ void lane_halves(float v, float& lower, float& upper)
   upper = __uint_as_float(r[1]);
 }
 
-// Two values at once: the lanes whose bit OFF is clear get the sum of a over the pair (l, l ^ OFF), the others the sum of b.
-template <int OFF>
-__device__ __forceinline__ float lane_pair_sum(float a, float b) {
-  static_assert(OFF == 32 || OFF == 16, "halves of the wave or of its halves");
-  typedef __attribute__((ext_vector_type(2))) unsigned u2;
-  const unsigned ua = __float_as_uint(a), ub = __float_as_uint(b);
-  const u2 r = OFF == 32 ? __builtin_amdgcn_permlane32_swap(ua, ub, false, false) : __builtin_amdgcn_permlane16_swap(ua, ub, false, false);
-  return __uint_as_float(r[0]) + __uint_as_float(r[1]);
-}
-
 template <int OFF>
 __device__ __forceinline__ float lane_xor(float v) {
   const int u = (int)__float_as_uint(v);

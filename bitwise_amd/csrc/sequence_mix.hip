@@ -254,39 +254,17 @@ __global__ __launch_bounds__(256) void norm_shift_row_kernel(const float* __rest
 
 enum { RECUR_DECAY_PER_CHANNEL = 0, RECUR_SCALAR_GATES = 1, RECUR_BONUS_DECAY = 2, RECUR_FIXED_DECAY = 3, RECUR_STEP_DECAY = 4, RECUR_DELTA = 5 };
 
-// The sum over the SPLIT lanes that hold the parts of one column, l, l + 64/SPLIT, ... (every one of them gets it).
+// The sum over the SPLIT neighbouring lanes that hold the parts of one column (every one of them gets it): an addition a
+// stage whose second operand comes through a data-parallel move within a row of 16 lanes.  Behind the first two stages the
+// lanes of a quad hold the same value, so the mirror images of 8 and of 16 lanes fetch the other half's.
 template <int SPLIT>
 __device__ __forceinline__ float join_parts(float v) {
-  if constexpr (SPLIT >= 2) {
-    float lower, upper;
-    lane_halves<32>(v, lower, upper);
-    v = lower + upper;
-    if constexpr (SPLIT >= 4) {
-      lane_halves<16>(v, lower, upper);
-      v = lower + upper;
-    }
-    if constexpr (SPLIT >= 8) v += lane_xor<8>(v);
-    if constexpr (SPLIT >= 16) v += lane_xor<4>(v);
-  }
+  static_assert(SPLIT <= 16, "a column's parts lie within a row of 16 lanes");
+  if constexpr (SPLIT >= 2) v += lane_xor<1>(v);
+  if constexpr (SPLIT >= 4) v += lane_xor<2>(v);
+  if constexpr (SPLIT >= 8) v += __uint_as_float((unsigned)__builtin_amdgcn_mov_dpp((int)__float_as_uint(v), 0x141, 0xf, 0xf, true));      // row_half_mirror
+  if constexpr (SPLIT >= 16) v += __uint_as_float((unsigned)__builtin_amdgcn_mov_dpp((int)__float_as_uint(v), 0x140, 0xf, 0xf, true));     // row_mirror
   return v;
-}
-
-// The sums of N values at once, each over the SPLIT lanes of its column: with N = 4 the lanes end with value (bit 5) + 2 (bit 4) of
-// their number, with N = 2 with value (bit 5).  The additions, and so the bits, of join_parts for each.
-template <int SPLIT, int N>
-__device__ __forceinline__ float join_parts_of(const float* v) {
-  static_assert((N == 4 && SPLIT >= 4) || (N == 2 && SPLIT >= 2), "");
-  float y = lane_pair_sum<32>(v[0], v[1]);
-  if constexpr (N == 4) {
-    y = lane_pair_sum<16>(y, lane_pair_sum<32>(v[2], v[3]));
-  } else if constexpr (SPLIT >= 4) {
-    float lower, upper;
-    lane_halves<16>(y, lower, upper);
-    y = lower + upper;
-  }
-  if constexpr (SPLIT >= 8) y += lane_xor<8>(y);
-  if constexpr (SPLIT >= 16) y += lane_xor<4>(y);
-  return y;
 }
 
 struct RecurArgs {
@@ -318,7 +296,7 @@ struct RecurArgs {
   float* start;            // per chunk: the state it starts from (S; scalar gates: n, m)
 };
 
-// A wave holds the state of 64 / SPLIT value columns of one head in registers: SPLIT lanes a column, each with DH consecutive
+// A wave holds the state of 64 / SPLIT value columns of one head in registers: SPLIT lanes a column, each with DH
 // key channels, so that a head has many short waves; the parts' read-outs are added by lane exchanges in one order whatever
 // runs the head (a single token, a portion, a chunk): the split depends on the head's size alone.  The tokens' q, k, decays
 // and v come through LDS in chunks of a few tokens, shared by the workgroup's waves (neighbouring column blocks of one head);
@@ -336,7 +314,7 @@ struct RecurArgs {
 // RECUR_FIXED_DECAY:  as per channel with one constant decay a head, alpha[d] = bias[head]; no logits are read.
 // RECUR_STEP_DECAY:  a step size per head and token, delta = softplus(z + bias[head]) with z at gate_off + head;
 //   S[d][j] <- e^(-bias2[head] delta) S[d][j] + k[d] (delta v[j]),  o[j] = (S^T q)[j] + skip[head] v[j].
-// RECUR_DELTA:  a step size beta (at gate_off + head) and a decay a (at gate2_off + head) per head and token, as they are;
+// RECUR_DELTA:  a step size beta (at gate_off + head) and a decay a (at gate2_off + head) per head and token;
 //   u[j] = beta (v[j] - a (S^T k)[j]),  S[d][j] <- a S[d][j] + k[d] u[j],  o[j] = (S^T q)[j]: what k reads is replaced towards v.
 //   The read-out is formed from the memory before the write, o = a (S^T q) + (k.q) u, so that only S^T k stands between a token
 //   and the next; k.q comes with the gates (at gate2_off + heads + key group).
@@ -416,7 +394,9 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   }
   if (count <= 0 || slot < 0) return;
   if (a.positions[first] < 0) return;
-  const int col = lane % COLS, part = lane / COLS, dbase = part * DH;
+  const int col = lane / SPLIT, part = lane % SPLIT;
+  // a lane's channels: runs of four, the column's lanes side by side (what they read together lies side by side, too)
+  auto channel = [&](int d) { return (d >> 2) * 4 * SPLIT + 4 * part + (d & 3); };
   const int j_wg = blockIdx.x * WCOLS, j_in = wv * COLS + col, j = j_wg + j_in;
   const bool live = j < vdim;
   float* st = a.state + (size_t)slot * a.state_ld;
@@ -443,13 +423,13 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
     const f32x4* src = reinterpret_cast<const f32x4*>(S_in + (size_t)min(j, vdim - 1) * dim);
 #pragma unroll
     for (int d = 0; d < DH; d += 4) {
-      const f32x4 v = src[min(dbase + d, dim - 4) >> 2];
+      const f32x4 v = src[min(channel(d), dim - 4) >> 2];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) Sreg[d + e] = live && dbase + d < dim ? v[e] : 0.0f;
+      for (int e = 0; e < 4; ++e) Sreg[d + e] = live && channel(d) < dim ? v[e] : 0.0f;
     }
   } else {
 #pragma unroll
-    for (int d = 0; d < DH; ++d) Sreg[d] = (PHASE != 1 && live && dbase + d < dim) ? S_in[(size_t)j * dim + dbase + d] : 0.0f;
+    for (int d = 0; d < DH; ++d) Sreg[d] = (PHASE != 1 && live && channel(d) < dim) ? S_in[(size_t)j * dim + channel(d)] : 0.0f;
   }
   float nreg[NN];          // scalar gates: the normaliser; otherwise in PHASE 1: the product of the chunk's decays
   float m = 0.0f, fsum = 0.0f;
@@ -464,7 +444,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   float ureg[BONUS ? DH : 1];
   if constexpr (BONUS) {
 #pragma unroll
-    for (int d = 0; d < DH; ++d) ureg[d] = dbase + d < dim ? a.bias2[h * dim + dbase + d] : 0.0f;
+    for (int d = 0; d < DH; ++d) ureg[d] = channel(d) < dim ? a.bias2[h * dim + channel(d)] : 0.0f;
   }
   const float fixed_decay = FIXED ? a.bias[h] : 0.0f;
   const float skip = STEP && a.skip != nullptr ? a.skip[h] : 0.0f;
@@ -610,15 +590,15 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
     for (int n = 0; n < N; ++n) {
 #pragma unroll
       for (int d = 0; d < DH; d += 4) {
-        const f32x4 kv = *reinterpret_cast<const f32x4*>(&ks[buf][t + n][dbase + d]);
-        const f32x4 qv = *reinterpret_cast<const f32x4*>(&qs[buf][t + n][dbase + d]);
+        const f32x4 kv = *reinterpret_cast<const f32x4*>(&ks[buf][t + n][channel(d)]);
+        const f32x4 qv = *reinterpret_cast<const f32x4*>(&qs[buf][t + n][channel(d)]);
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           O.k[n][d + e] = kv[e];
           O.q[n][d + e] = qv[e];
         }
         if constexpr (CHANNELS) {
-          const f32x4 av = *reinterpret_cast<const f32x4*>(&as[buf][t + n][dbase + d]);
+          const f32x4 av = *reinterpret_cast<const f32x4*>(&as[buf][t + n][channel(d)]);
 #pragma unroll
           for (int e = 0; e < 4; ++e) O.a[n][d + e] = av[e];
         }
@@ -651,14 +631,16 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
           for (int i = 0; i < NN; ++i) nreg[i] *= fa;
         }
       } else if constexpr (DELTA) {
-        // (two chains over a lane's channels, then the column's lanes: the one sum the next token waits for)
+        // (what the next token waits for: two chains over a lane's channels, the column's lanes, and then one fused
+        // multiply-add for u and one for each channel)
+        const float fa = O.g2[n], step_v = O.g1[n] * O.v[n], step_a = -(O.g1[n] * fa);
         float r0 = 0.0f, r1 = 0.0f, o1 = 0.0f;
 #pragma unroll
         for (int d = 0; d < DH; d += 2) {
           r0 = fmaf(Sreg[d], O.k[n][d], r0);
           r1 = fmaf(Sreg[d + 1], O.k[n][d + 1], r1);
         }
-        const float fa = O.g2[n], u = O.g1[n] * fmaf(-fa, join_parts<SPLIT>(r0 + r1), O.v[n]);
+        const float u = fmaf(step_a, join_parts<SPLIT>(r0 + r1), step_v);
 #pragma unroll
         for (int d = 0; d < DH; d += 2) {
           o[n] = fmaf(Sreg[d], O.q[n][d], o[n]);
@@ -667,7 +649,7 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
         o[n] += o1;
         w[n] = O.kq[n] * u;
 #pragma unroll
-        for (int d = 0; d < DH; ++d) Sreg[d] = fmaf(fa, Sreg[d], O.k[n][d] * u);
+        for (int d = 0; d < DH; ++d) Sreg[d] = fmaf(O.k[n][d], u, fa * Sreg[d]);
       } else if constexpr (!GATES) {
 #pragma unroll
         for (int d = 0; d < DH; ++d) {
@@ -716,32 +698,17 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
     }
     if constexpr (READ_OUT) {
       float* orow = a.out + (size_t)(first + t0 + t) * a.ldo + h * vdim + j;
-      if constexpr (!GATES && N == TU && (N == 4 || N == 2) && SPLIT >= N) {
-        // the columns' sums of all N tokens at once; a lane ends with the token its number names, the first of a column's
-        // lanes with that token stores it
-        const int mine = N == 4 ? (lane >> 5) + 2 * ((lane >> 4) & 1) : lane >> 5;
-        const bool stores = N == 4 ? (lane & 15) < COLS : (lane & 31) < COLS;
-        float v = join_parts_of<SPLIT, N>(o);
-        auto pick = [&](float x0, float x1, float x2, float x3) {      // (by value: an array by address would go to memory)
-          const float lo = (mine & 1) ? x1 : x0, hi = (mine & 1) ? x3 : x2;
-          return (mine & 2) ? hi : lo;
-        };
-        if constexpr (STEP) v = fmaf(skip, pick(O.v[0], O.v[1], O.v[N - 2], O.v[N - 1]), v);
-        if constexpr (DELTA) v = fmaf(pick(O.g2[0], O.g2[1], O.g2[N - 2], O.g2[N - 1]), v, pick(w[0], w[1], w[N - 2], w[N - 1]));
-        if (live && stores) orow[(size_t)mine * a.ldo] = v;
-      } else {
-        // (part n of a column stores token t + n)
-        float mine = 0.0f;
+      // (part n of a column stores token t + n)
+      float mine = 0.0f;
 #pragma unroll
-        for (int n = 0; n < N; ++n) {
-          float v = o[n];
-          if constexpr (!GATES) v = join_parts<SPLIT>(v);
-          if constexpr (STEP) v = fmaf(skip, O.v[n], v);
-          if constexpr (DELTA) v = fmaf(O.g2[n], v, w[n]);
-          mine = part == n ? v : mine;
-        }
-        if (live && part < N) orow[(size_t)part * a.ldo] = mine;
+      for (int n = 0; n < N; ++n) {
+        float v = o[n];
+        if constexpr (!GATES) v = join_parts<SPLIT>(v);
+        if constexpr (STEP) v = fmaf(skip, O.v[n], v);
+        if constexpr (DELTA) v = fmaf(O.g2[n], v, w[n]);
+        mine = part == n ? v : mine;
       }
+      if (live && part < N) orow[(size_t)part * a.ldo] = mine;
     }
   };
   using Group = RecurOps<TU, DH, CHANNELS>;
@@ -810,11 +777,11 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
       f32x4* dst = reinterpret_cast<f32x4*>(S_out + (size_t)j * dim);
 #pragma unroll
       for (int d = 0; d < DH; d += 4)
-        if (dbase + d < dim) dst[(dbase + d) >> 2] = (f32x4){Sreg[d], Sreg[d + 1], Sreg[d + 2], Sreg[d + 3]};
+        if (channel(d) < dim) dst[channel(d) >> 2] = (f32x4){Sreg[d], Sreg[d + 1], Sreg[d + 2], Sreg[d + 3]};
     } else {
 #pragma unroll
       for (int d = 0; d < DH; ++d)
-        if (dbase + d < dim) S_out[(size_t)j * dim + dbase + d] = Sreg[d];
+        if (channel(d) < dim) S_out[(size_t)j * dim + channel(d)] = Sreg[d];
     }
   }
   if (wv == 0 && (WALK ? GATES : blockIdx.x == 0 && (GATES || PHASE == 1))) {
