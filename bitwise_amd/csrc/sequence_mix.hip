@@ -328,7 +328,6 @@ struct RecurArgs {
 // chunk from there with the read-out, and the request's last chunk leaves the state in the slot.  PHASE 0 walks
 // the whole portion; PHASE 4 does so for steps of a few tokens a request (decoding), where what counts is how many waves are
 // on the chip with their states' loads under way: no groups of tokens, no second buffer, few registers, the same arithmetic.  The passes differ from PHASE 0 by the rounding of the scan's sums only.
-#define RECUR_CHUNK 16   // tokens staged together
 #define RW 4             // waves of a workgroup
 // floats of a chunk's record for one head: S, a vector, two scalars, in whole vectors of four
 __host__ __device__ __forceinline__ size_t recur_record(int dim, int vdim) { return ((size_t)dim * vdim + dim + 2 + 3) & ~(size_t)3; }
@@ -364,9 +363,9 @@ __global__ __launch_bounds__(64 * RW) void linear_recurrence_kernel(RecurArgs a)
   constexpr bool WALK = PHASE == 0 || PHASE == 4;
   constexpr int SPLIT = WALK ? recur_split(DPAD) : recur_chunk_split(DPAD);
   constexpr int DH = DPAD / SPLIT, COLS = 64 / SPLIT, WCOLS = RW * COLS;
-  constexpr int TU = PHASE != 0 ? 1 : (SPLIT >= 4 && DH <= 8 ? 4 : 2);      // tokens worked on together (two groups of them fit the registers)
+  constexpr int TU = PHASE != 0 ? 1 : (SPLIT >= 4 && DPAD <= 64 ? 4 : 2);      // tokens of a group (two groups' operands fit the registers, with room for a second wave)
   constexpr int BUFS = PHASE != 0 ? 1 : 2;               // (the passes over chunks hide the loads behind other waves)
-  constexpr int RC = PHASE == 4 && DPAD >= 64 ? 4 : RECUR_CHUNK;
+  constexpr int RC = PHASE == 4 && DPAD >= 64 ? 4 : (PHASE == 0 && DPAD <= 128 ? 32 : 16);     // tokens staged together
   constexpr int NQ = RC * DPAD / (64 * RW), NV = (RC * WCOLS + 64 * RW - 1) / (64 * RW);
   static_assert(NQ * 64 * RW == RC * DPAD && RC % TU == 0, "a chunk is whole loads and whole groups of tokens");
   __shared__ __attribute__((aligned(16))) float qs[BUFS][RC][DPAD];
