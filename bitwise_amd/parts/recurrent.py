@@ -39,7 +39,6 @@ FEW_SEQ_ROWS = 4         # steps whose requests bring up to so many rows each ru
 SCAN_CHUNK = 32          # rows of a chunk of a long portion
 SCAN_MIN_ROWS = 96       # portions from this many rows on run in three passes over chunks (shorter ones are walked whole),
                          # where the engine allows logits to depend on the cut in their last bits (Workspace.exact_cuts False)
-SCAN_MAX_STATE = 1 << 20  # memories of a layer with so many elements and more fill the chip when a portion is walked whole: no passes
 
 
 def _scan_plan(ctx):
@@ -80,7 +79,8 @@ class _MatrixMemoryMixer(Mixer):
     mode = -1
     gate_kind = ops.GATE_SIGMOID
     per_head_norm_weight = True
-    passes = True                             # long portions may run in passes over chunks
+    passes = True             # long portions may run in passes over chunks
+    walk_from = 1 << 19       # memories of a layer with so many elements and more fill the chip when a portion is walked whole: no passes
 
     def __init__(self, params, runtime):
         super().__init__(params, runtime)
@@ -142,7 +142,7 @@ class _MatrixMemoryMixer(Mixer):
         """``at``: where q (or r), k and v lie in a row of ``y``, if not at the stacked projection's own
         offsets.  ``state``: the memories' part of the slots, if they do not fill them."""
         at = self.offsets if at is None else at
-        plan = _scan_plan(ctx) if self.passes and self.heads * self.dim * self.vdim < SCAN_MAX_STATE else None
+        plan = _scan_plan(ctx) if self.passes and self.heads * self.dim * self.vdim < self.walk_from else None
         seq_rows, nseq, scan = ctx.seq_rows, ctx.nseq, None
         if plan is not None:
             seq_rows, nseq, chunks, nchunks, spans, nspans = plan
@@ -220,6 +220,7 @@ class MatrixLSTM(_MatrixMemoryMixer):
     i.b, f.b [heads]; norm [heads*vdim]; o [width, heads*vdim]."""
 
     mode = ops.RECUR_SCALAR_GATES
+    walk_from = 1 << 20       # (the walk carries the normaliser along: the passes win for longer)
     gate_kind = ops.GATE_SIGMOID
     per_head_norm_weight = True
 
