@@ -38,6 +38,9 @@ int bw_gemm_bf16(const void* x, const void* w, void* out, int M, int N, int K, i
 int bw_gemm_clamped_glu_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo, float limit,
                              float alpha, void* stream);
 int bw_gemm_add_scratch(int M, int N, int K, long long* scratch_floats, int* counters);
+// out = bf16(gelu_tanh(x W^T) * table[token of the row]): up to 16 rows, K in steps of 64, fewer than 4,096 columns (-7: another shape)
+int bw_gemm_side_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo, const int32_t* tokens,
+                      const int32_t* feedback, const void* table, int ldt, int vocab, void* stream);
 int bw_gemm_store_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo, float* scratch,
                        long long scratch_floats, int32_t* counters, int num_counters, void* stream);   // (bw_gemm_bf16's 32-bit store)
 int bw_gemm_add_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo, float* scratch,

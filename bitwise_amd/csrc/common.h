@@ -97,6 +97,12 @@ __device__ __forceinline__ float clamped_swish_times(float g, float u, float lim
 // The exact GELU, z/2 (1 + erf(z / sqrt 2)), as the activation kernel and the products' epilogue both compute it.
 __device__ __forceinline__ float gelu_erf(float z) { return (0.5f * z) * (1.0f + erff(z * 0.7071067811865476f)); }
 
+// GELU in its tanh form, 32-bit.
+__device__ __forceinline__ float gelu_tanh(float z) {
+  const float inner = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+  return 0.5f * z * (1.0f + tanhf(inner));
+}
+
 // Lane exchanges from register to register (no trip through LDS).  The halves and quarters of the wave by gfx950's
 // lane swaps: of (v, v) swapped, the first result holds in every lane the value of its partner or its own in the
 // lower half (32: lanes 0-31; 16: the even rows of 16 lanes), the second the one in the upper half; an operation

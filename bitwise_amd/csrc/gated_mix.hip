@@ -678,11 +678,6 @@ struct RglruArgs {
   int ldy, ldu, ldg, ldo, channels, bs;
 };
 
-__device__ __forceinline__ float gm_gelu_tanh(float z) {
-  const float inner = 0.7978845608028654f * (z + 0.044715f * z * z * z);
-  return 0.5f * z * (1.0f + tanhf(inner));
-}
-
 // What a token adds to its channel's state and the factor the state keeps: independent of the state itself.
 __device__ __forceinline__ void rglru_terms(float zr, float zi, float u, float br, float bi, float c, float& a, float& b) {
   const float r = gm_sigmoid(zr + br), i = gm_sigmoid(zi + bi);
@@ -704,7 +699,7 @@ __global__ __launch_bounds__(256) void rglru_terms_kernel(RglruArgs p, int rows)
   rglru_terms(zr[0], zr[p.bs], p.u[(size_t)row * p.ldu + c], p.ra_bias[c], p.ri_bias[c], p.decay[c], a, b);
   zr[0] = a;
   zr[p.bs] = b;
-  *yy = gm_gelu_tanh(p.y_bias != nullptr ? *yy + p.y_bias[c] : *yy);
+  *yy = gelu_tanh(p.y_bias != nullptr ? *yy + p.y_bias[c] : *yy);
 }
 
 template <typename TO>
@@ -1128,7 +1123,7 @@ __global__ __launch_bounds__(256) void side_gate_kernel(const float* __restrict_
     int tok = tokens[row];
     if (tok == BW_TOKEN_FROM_FEEDBACK && feedback != nullptr) tok = feedback[row];
     float v = 0.0f;
-    if (tok >= 0 && tok < vocab) v = gm_gelu_tanh(z[(size_t)row * ldz + e]) * gm_load(table + (size_t)tok * ldt + e);
+    if (tok >= 0 && tok < vocab) v = gelu_tanh(z[(size_t)row * ldz + e]) * gm_load(table + (size_t)tok * ldt + e);
     gm_store(out + (size_t)row * ldo + e, v);
   }
 }

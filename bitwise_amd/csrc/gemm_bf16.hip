@@ -138,6 +138,30 @@ __device__ __forceinline__ void epilogue_store(void* __restrict__ out, size_t o,
   else if constexpr (EPI == EPI_CLAMPED_GLU_BF16) st_bf16<DEV>((bf16_t*)out + o, f32_to_bf16(clamped_swish_times<true>(v, u, limit, alpha)));
 }
 
+// EPI_SIDE_BF16 (up to 16 rows): an output is the GELU (tanh form) of its sum times the element of its row's token in a table, rounded
+// to bfloat16: the statements of side_gate_kernel on the sums while they are still in registers.
+struct SideGateArgs {
+  const int32_t* tokens = nullptr;
+  const int32_t* feedback = nullptr;
+  const bf16_t* table = nullptr;       // [vocab] rows of ldt elements, column n of the product at element n
+  int ldt = 0, vocab = 0;
+};
+template <int EPI>
+__device__ __forceinline__ int side_token(const SideGateArgs& sg, int m) {
+  if constexpr (EPI == EPI_SIDE_BF16) {
+    int tok = sg.tokens[m];
+    if (tok == BW_TOKEN_FROM_FEEDBACK && sg.feedback != nullptr) tok = sg.feedback[m];
+    return tok;
+  } else {
+    return 0;
+  }
+}
+__device__ __forceinline__ void side_store(const SideGateArgs& sg, int tok, int n, bf16_t* out, float z) {
+  float v = 0.0f;
+  if (tok >= 0 && tok < sg.vocab) v = gelu_tanh(z) * bf16_to_f32(sg.table[(size_t)tok * sg.ldt + n]);
+  *out = f32_to_bf16(v);
+}
+
 // (host) The phases asked for while a chain is open wait in a list and leave as one launch (further down).
 struct MidCall;
 struct RowsCall;
@@ -539,6 +563,21 @@ extern "C" int bw_gemm_add_bf16(const void* x, const void* w, void* out, int M, 
   if ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) return -3;
   return launch_gemm_bf16<EPI_ADD_F32>((const bf16_t*)x, (const bf16_t*)w, out, M, N, K, ldx, ldo, (hipStream_t)stream,
                                        QkvRopeArgs{}, MidSplitArgs{scratch, counters}, (size_t)scratch_floats, num_counters);
+}
+
+// out[m][n] = bf16(gelu_tanh(x W^T [m][n]) * table[token of m][n]) for up to 16 rows and fewer than 4,096 columns, K in steps of 64:
+// the bits of bw_gemm_bf16's 32-bit store followed by bw_side_gate.  -7: not this shape.
+extern "C" int bw_gemm_side_bf16(const void* x, const void* w, void* out, int M, int N, int K, int ldx, int ldo, const int32_t* tokens,
+                                 const int32_t* feedback, const void* table, int ldt, int vocab, void* stream) {
+  if (M <= 0 || N <= 0) return 0;
+  if (K <= 0 || ldx < K || (ldx % 8) || ldo < N || ldt < N || vocab <= 0 || tokens == nullptr || table == nullptr) return -2;
+  if ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) return -3;
+  const int S = (K + GEMM_SEG - 1) / GEMM_SEG;
+  if (M > 16 || K % 64 || S > 40 || (N + 15) / 16 >= 256 || (size_t)M * ldx * 2 >= ((size_t)1 << 31)) return -7;
+  const SideGateArgs sg{tokens, feedback, (const bf16_t*)table, ldt, vocab};
+  hipStream_t s = (hipStream_t)stream;
+  if (K <= 64 * BURST_STEPS) return launch_burst<EPI_SIDE_BF16>((const bf16_t*)x, (const bf16_t*)w, out, M, N, K, ldx, ldo, s, sg);
+  return launch_stream<EPI_SIDE_BF16, 8>((const bf16_t*)x, (const bf16_t*)w, out, M, N, K, ldx, ldo, S, s, sg);
 }
 
 // out = x W^T (32-bit store) with that scratch: the bits of bw_gemm_bf16's store.

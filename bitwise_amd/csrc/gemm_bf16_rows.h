@@ -680,7 +680,7 @@ __device__ __forceinline__ void stream_issue(unsigned char* ring, __amdgpu_buffe
 // flight); x, old values and outputs travel at device scope.
 template <int EPI, int CW, int XR, bool CH, int DEPTH = 24>
 __device__ __forceinline__ void stream_body(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, void* __restrict__ out, int M, int N,
-                                            int K, int ldx, int ldo, int S, const ChainCtx& cc) {
+                                            int K, int ldx, int ldo, int S, const ChainCtx& cc, const SideGateArgs& sg = SideGateArgs{}) {
   using SH = StreamShape<CW, XR, DEPTH>;
   extern __shared__ __attribute__((aligned(16))) unsigned char stream_lds[];   // [waves][ring], then [S][4][64] floats when S > 1
   const int wave = wave_index(), lane = threadIdx.x & 63, nwaves = cc.waves;
@@ -713,7 +713,16 @@ __device__ __forceinline__ void stream_body(const bf16_t* __restrict__ x, const 
   // A residual add: the wave that stores asks for its outputs' old values before anything else (loads older than
   // the ring's, so every wait below covers them); asked for at the end they were one more trip to memory.
   float old_out[4] = {0.f, 0.f, 0.f, 0.f};
+  int tokens[4] = {-1, -1, -1, -1};
   auto ask_old = [&]() {
+    if constexpr (EPI == EPI_SIDE_BF16) {                // (the rows' tokens likewise)
+      if (wave == 0 && n_ok) {
+#pragma unroll
+        for (int q = 0; q < 4; ++q)
+          if (4 * g + q < M) tokens[q] = side_token<EPI>(sg, 4 * g + q);
+      }
+      asm volatile("" ::: "memory");
+    }
     if constexpr (EPI == EPI_ADD_F32) {
       if (wave == 0 && n_ok) {
 #pragma unroll
@@ -794,6 +803,8 @@ __device__ __forceinline__ void stream_body(const bf16_t* __restrict__ x, const 
     if constexpr (EPI == EPI_ADD_F32) {
       // (several segments: the residual is in already; one: old + sum, the addition of the store that reads)
       st_f32<CH>((float*)out + (size_t)m * ldo + n0 + c, S > 1 ? acc[q] : old_out[q] + acc[q]);
+    } else if constexpr (EPI == EPI_SIDE_BF16) {
+      side_store(sg, tokens[q], n0 + c, (bf16_t*)out + (size_t)m * ldo + n0 + c, acc[q]);
     } else {
       epilogue_store<EPI, CH>(out, (size_t)m * ldo + n0 + c, acc[q], acc[q]);
     }
@@ -803,13 +814,14 @@ __device__ __forceinline__ void stream_body(const bf16_t* __restrict__ x, const 
 template <int EPI, int CW, int XR = 16, int DEPTH = 24>
 __global__ __launch_bounds__(DEPTH == 24 ? 256 : 512) void gemm_bf16_stream_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                                                                                    void* __restrict__ out, int M, int N, int K, int ldx,
-                                                                                   int ldo, int S) {
-  stream_body<EPI, CW, XR, false, DEPTH>(x, w, out, M, N, K, ldx, ldo, S, launch_ctx());
+                                                                                   int ldo, int S, SideGateArgs sg) {
+  stream_body<EPI, CW, XR, false, DEPTH>(x, w, out, M, N, K, ldx, ldo, S, launch_ctx(), sg);
 }
 
 // Five to eight segments of K and no more than 8 rows: a wave a segment, all at once, with shallower rings.
 template <int EPI, int CW>
-static int launch_stream_many(const bf16_t* x, const bf16_t* w, void* out, int M, int N, int K, int ldx, int ldo, int S, hipStream_t s) {
+static int launch_stream_many(const bf16_t* x, const bf16_t* w, void* out, int M, int N, int K, int ldx, int ldo, int S, hipStream_t s,
+                         const SideGateArgs& sg = SideGateArgs{}) {
   constexpr int DEPTH = STREAM_DEPTH_MANY(CW);
   using SH = StreamShape<CW, 8, DEPTH>;
   const size_t lds_bytes = (size_t)S * SH::RING + (size_t)S * 4 * 64 * sizeof(float);
@@ -819,15 +831,16 @@ static int launch_stream_many(const bf16_t* x, const bf16_t* w, void* out, int M
     (void)hipFuncSetAttribute((const void*)gemm_bf16_stream_kernel<EPI, CW, 8, DEPTH>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     allowed = true;
   }
-  BW_LAUNCH((gemm_bf16_stream_kernel<EPI, CW, 8, DEPTH>), dim3((N + CW - 1) / CW), dim3(64 * S), lds_bytes, s, x, w, out, M, N, K, ldx, ldo, S);
+  BW_LAUNCH((gemm_bf16_stream_kernel<EPI, CW, 8, DEPTH>), dim3((N + CW - 1) / CW), dim3(64 * S), lds_bytes, s, x, w, out, M, N, K, ldx, ldo, S, sg);
   return BW_LAUNCH_CHECK();
 }
 
 template <int EPI, int CW, int XR>
-static int launch_stream_rows(const bf16_t* x, const bf16_t* w, void* out, int M, int N, int K, int ldx, int ldo, int S, hipStream_t s) {
+static int launch_stream_rows(const bf16_t* x, const bf16_t* w, void* out, int M, int N, int K, int ldx, int ldo, int S, hipStream_t s,
+                         const SideGateArgs& sg = SideGateArgs{}) {
   using SH = StreamShape<CW, XR>;
   if constexpr (XR == 8) {
-    const int rc = launch_stream_many<EPI, CW>(x, w, out, M, N, K, ldx, ldo, S, s);
+    const int rc = launch_stream_many<EPI, CW>(x, w, out, M, N, K, ldx, ldo, S, s, sg);
     if (rc != -7) return rc;
   }
   const int waves = S < 4 ? S : 4;
@@ -843,15 +856,16 @@ static int launch_stream_rows(const bf16_t* x, const bf16_t* w, void* out, int M
     if constexpr (kind >= 0) return chain_record_rows(kind, RowsCall{x, w, out, M, N, K, ldx, ldo, S}, (N + CW - 1) / CW, waves, (int)lds_bytes, s);
   }
   BW_LAUNCH((gemm_bf16_stream_kernel<EPI, CW, XR>), dim3((N + CW - 1) / CW), dim3(64 * waves), lds_bytes, s, x, w, out, M, N,
-                     K, ldx, ldo, S);
+                     K, ldx, ldo, S, sg);
   return BW_LAUNCH_CHECK();
 }
 
 template <int EPI, int CW>
-static int launch_stream(const bf16_t* x, const bf16_t* w, void* out, int M, int N, int K, int ldx, int ldo, int S, hipStream_t s) {
+static int launch_stream(const bf16_t* x, const bf16_t* w, void* out, int M, int N, int K, int ldx, int ldo, int S, hipStream_t s,
+                         const SideGateArgs& sg = SideGateArgs{}) {
   // (how many rows a stage holds changes no bit: the chain of a row is the same statements on the same values)
-  if (M <= 8) return launch_stream_rows<EPI, CW, 8>(x, w, out, M, N, K, ldx, ldo, S, s);
-  return launch_stream_rows<EPI, CW, 16>(x, w, out, M, N, K, ldx, ldo, S, s);
+  if (M <= 8) return launch_stream_rows<EPI, CW, 8>(x, w, out, M, N, K, ldx, ldo, S, s, sg);
+  return launch_stream_rows<EPI, CW, 16>(x, w, out, M, N, K, ldx, ldo, S, s, sg);
 }
 
 // ------------------------------------------------------------------------------ up to 16 rows, few columns, one segment
@@ -871,7 +885,7 @@ static int launch_stream(const bf16_t* x, const bf16_t* w, void* out, int M, int
 // then the old values and x at device scope; a wave's q-th step is there when all but its last 2 * (7 - q) loads are.
 template <int EPI, bool CH>
 __device__ __forceinline__ void burst_body(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, void* __restrict__ out, int M, int N,
-                                           int K, int ldx, int ldo, const ChainCtx& cc) {
+                                           int K, int ldx, int ldo, const ChainCtx& cc, const SideGateArgs& sg = SideGateArgs{}) {
   extern __shared__ __attribute__((aligned(16))) unsigned char burst_lds[];   // [BURST_STEPS][BURST_STAGE]
   typedef __attribute__((address_space(3))) void* lds_ptr;
   const int wave = wave_index(), lane = threadIdx.x & 63;
@@ -893,7 +907,16 @@ __device__ __forceinline__ void burst_body(const bf16_t* __restrict__ x, const b
   // A residual add: the wave that stores asks for its outputs' old values before anything else (older than its loads
   // of the steps, so every wait below covers them); asked for at the end they were one more trip to memory.
   float old_out[4] = {0.f, 0.f, 0.f, 0.f};
+  int tokens[4] = {-1, -1, -1, -1};
   auto ask_old = [&]() {
+    if constexpr (EPI == EPI_SIDE_BF16) {                // (the rows' tokens likewise)
+      if (wave == 0 && n_ok) {
+#pragma unroll
+        for (int q = 0; q < 4; ++q)
+          if (4 * g + q < M) tokens[q] = side_token<EPI>(sg, 4 * g + q);
+      }
+      asm volatile("" ::: "memory");
+    }
     if constexpr (EPI == EPI_ADD_F32) {
       if (wave == 0 && n_ok) {
 #pragma unroll
@@ -984,18 +1007,20 @@ __device__ __forceinline__ void burst_body(const bf16_t* __restrict__ x, const b
     const int m = 4 * g + q;
     if (m >= M) continue;
     if constexpr (EPI == EPI_ADD_F32) st_f32<CH>((float*)out + (size_t)m * ldo + n0 + c, old_out[q] + acc[q]);
+    else if constexpr (EPI == EPI_SIDE_BF16) side_store(sg, tokens[q], n0 + c, (bf16_t*)out + (size_t)m * ldo + n0 + c, acc[q]);
     else epilogue_store<EPI, CH>(out, (size_t)m * ldo + n0 + c, acc[q], acc[q]);
   }
 }
 
 template <int EPI>
 __global__ __launch_bounds__(256) void gemm_bf16_burst_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
-                                                              void* __restrict__ out, int M, int N, int K, int ldx, int ldo) {
-  burst_body<EPI, false>(x, w, out, M, N, K, ldx, ldo, launch_ctx());
+                                                              void* __restrict__ out, int M, int N, int K, int ldx, int ldo, SideGateArgs sg) {
+  burst_body<EPI, false>(x, w, out, M, N, K, ldx, ldo, launch_ctx(), sg);
 }
 
 template <int EPI>
-static int launch_burst(const bf16_t* x, const bf16_t* w, void* out, int M, int N, int K, int ldx, int ldo, hipStream_t s) {
+static int launch_burst(const bf16_t* x, const bf16_t* w, void* out, int M, int N, int K, int ldx, int ldo, hipStream_t s,
+                        const SideGateArgs& sg = SideGateArgs{}) {
   static bool allowed = false;                       // more than 64 KB of dynamic LDS has to be asked for once
   if (!allowed) {
     (void)hipFuncSetAttribute((const void*)gemm_bf16_burst_kernel<EPI>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
@@ -1005,6 +1030,6 @@ static int launch_burst(const bf16_t* x, const bf16_t* w, void* out, int M, int 
     if constexpr (EPI == EPI_ADD_F32) return chain_record_rows(CK_BURST_ADD, RowsCall{x, w, out, M, N, K, ldx, ldo, 1}, (N + 7) / 8, 4, BURST_STEPS * BURST_STAGE, s);
   }
   BW_LAUNCH((gemm_bf16_burst_kernel<EPI>), dim3((N + 7) / 8), dim3(256), BURST_STEPS * BURST_STAGE, s, x, w, out, M, N, K,
-                     ldx, ldo);
+                     ldx, ldo, sg);
   return BW_LAUNCH_CHECK();
 }

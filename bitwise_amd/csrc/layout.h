@@ -14,7 +14,7 @@
 #define BW_HD inline
 #endif
 
-enum { EPI_F32 = 0, EPI_BF16 = 1, EPI_ADD_F32 = 2, EPI_SWIGLU_BF16 = 3, EPI_QKV_ROPE = 4, EPI_CLAMPED_GLU_BF16 = 5, EPI_GELU_BF16 = 6 };
+enum { EPI_F32 = 0, EPI_BF16 = 1, EPI_ADD_F32 = 2, EPI_SWIGLU_BF16 = 3, EPI_QKV_ROPE = 4, EPI_CLAMPED_GLU_BF16 = 5, EPI_GELU_BF16 = 6, EPI_SIDE_BF16 = 7 };
 
 // Epilogues that take the stacked weight [gate rows; up rows] and store act(gate) * up.
 BW_HD constexpr bool epi_is_glu(int epi) { return epi == EPI_SWIGLU_BF16 || epi == EPI_CLAMPED_GLU_BF16; }

@@ -52,6 +52,8 @@ _SIGS = {
     "bw_gemm_add_scratch": [c_int, c_int, c_int, c_void_p, c_void_p],
     "bw_gemm_add_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_longlong, c_void_p,
                          c_int, c_void_p],
+    "bw_gemm_side_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
+                          c_void_p],
     "bw_gemm_store_bf16": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_longlong, c_void_p,
                            c_int, c_void_p],
     "bw_gemm_add_bf16_static": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
@@ -1609,6 +1611,36 @@ def scaled_sum_norm_add(ys: Sequence[torch.Tensor], scales: Sequence[float], wei
     _check(_fn("bw_scaled_sum_norm_add")(yp, ld, sc, n, weight.data_ptr(), float(eps), float(scale), x.data_ptr(), x.stride(0),
                                          0 if rounded is None else rounded.data_ptr(), 0 if rounded is None else rounded.stride(0),
                                          rows, dim, _stream()), "scaled_sum_norm_add")
+
+
+def side_gemm_ok(rows: int, weight: torch.Tensor, table: torch.Tensor) -> bool:
+    """Whether ``gemm_side_bf16`` takes this step: few rows, columns and an inner size its kernels take, a bfloat16 table."""
+    n, k = weight.shape
+    return rows <= 16 and k % 64 == 0 and k <= 40 * 2048 and n <= 4080 and table.dtype == torch.bfloat16
+
+
+def gemm_side_bf16(x: torch.Tensor, w: torch.Tensor, tokens: torch.Tensor, feedback: Optional[torch.Tensor], table: torch.Tensor,
+                   out: torch.Tensor, rows: int) -> None:
+    """out[r, d] = gelu_tanh((x @ w.T)[r, d]) * table[token of r, d], one launch for up to 16 rows: the bits of ``gemm_bf16`` with a
+    32-bit store followed by ``side_gate`` into a bfloat16 ``out``."""
+    _need_strided(x, torch.bfloat16, "x")
+    _need(w, torch.bfloat16, "weight")
+    _need(tokens, torch.int32, "tokens")
+    _need(out, torch.bfloat16, "out")
+    if table.dtype != torch.bfloat16 or not table.is_cuda or table.dim() != 2 or table.stride(1) != 1:
+        raise ValueError("gemm_side_bf16: the table must be a bfloat16 GPU matrix with contiguous rows")
+    n, k = w.shape
+    if x.shape[1] != k or out.shape[1] != n or table.shape[1] != n or min(x.shape[0], out.shape[0], tokens.numel()) < rows:
+        raise ValueError("gemm_side_bf16: x, w, table and out do not fit")
+    if not side_gemm_ok(rows, w, table):
+        raise ValueError("gemm_side_bf16: up to 16 rows of an inner size in steps of 64")
+    if feedback is not None:
+        _need(feedback, torch.int32, "feedback")
+        if feedback.numel() < rows:
+            raise ValueError("gemm_side_bf16: feedback is shorter than the rows")
+    _check(_fn("bw_gemm_side_bf16")(x.data_ptr(), w.data_ptr(), out.data_ptr(), rows, n, k, x.stride(0), out.stride(0), tokens.data_ptr(),
+                                    0 if feedback is None else feedback.data_ptr(), table.data_ptr(), table.stride(0), table.shape[0],
+                                    _stream()), "gemm_side_bf16")
 
 
 def side_gate(z: torch.Tensor, tokens: torch.Tensor, feedback: Optional[torch.Tensor], table: torch.Tensor, out: torch.Tensor,

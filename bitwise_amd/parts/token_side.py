@@ -52,10 +52,14 @@ class TokenSide(SideInput):
         table = ctx.forward_notes.get("token_side_table")
         if table is None or table.shape[1] < self.offset + self.dim:
             raise ValueError("token_side: the embedding holds no side table with this layer's columns")
-        z = ws.buffer("side_gate", self.dim, torch.float32)
-        self.gate.store(ws, h, z, rows)
+        e, feedback = table[:, self.offset:self.offset + self.dim], getattr(ctx, "token_feedback", None)
         g = ws.buffer("side_gated", self.dim, self.rt.act_dtype)
-        ops.side_gate(z, ctx.tokens, getattr(ctx, "token_feedback", None), table[:, self.offset:self.offset + self.dim], g, rows)
+        if self.gate.mfma and h.dtype == torch.bfloat16 and ops.side_gemm_ok(rows, self.gate.weight, e):
+            ops.gemm_side_bf16(h, self.gate.weight, ctx.tokens, feedback, e, g, rows)      # (decode steps: one launch, the same bits)
+        else:
+            z = ws.buffer("side_gate", self.dim, torch.float32)
+            self.gate.store(ws, h, z, rows)
+            ops.side_gate(z, ctx.tokens, feedback, e, g, rows)
         y = ws.buffer("side_out", self.width, torch.float32)
         self.proj.store(ws, g, y, rows)
         ops.norm_add(y, self.norm_weight, x, rows, self.eps, rounded)

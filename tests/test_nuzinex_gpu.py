@@ -696,6 +696,33 @@ def test_stores_and_gelu_of_products_do_not_depend_on_the_rows(gpu, N, K):
     assert ((act[:1].cpu().double() - gelu[:1]).abs() <= 2 ** -7 * gelu[:1].abs() + 1e-5).all()
 
 
+@pytest.mark.parametrize("N,K", [(16, 64), (256, 2048), (40, 4096), (256, 8192), (1000, 1024), (7, 12288)])
+def test_side_gate_in_the_product_of_few_rows(gpu, N, K):
+    """The gate of the side input as the product's epilogue: the bits of the product followed by the gate's launch, with given
+    tokens, tokens the step before sampled, and padding."""
+    from bitwise_amd.csrc import ops
+    torch.manual_seed(N + K)
+    w, x = (torch.randn(N, K, device=gpu) * K ** -0.5).to(torch.bfloat16), torch.randn(16, K, device=gpu).to(torch.bfloat16)
+    table = torch.randn(37, N + 24, device=gpu).to(torch.bfloat16)[:, 8:8 + N]
+    tokens = torch.randint(0, 37, (16,)).tolist()
+    feedback = torch.randint(0, 37, (16,), dtype=torch.int32, device=gpu)
+    for rows in (1, 5, 8, 16):
+        given = list(tokens)
+        given[rows - 1] = -2
+        if rows > 3:
+            given[2] = -1
+        given = _dev(gpu)(given)
+        z, want, got = torch.zeros(16, N, device=gpu), *(torch.full((16, N), 3.0, dtype=torch.bfloat16, device=gpu) for _ in range(2))
+        ops.gemm_bf16(x, w, z, rows, ops.EPI_F32)
+        ops.side_gate(z, given, feedback, table, want, rows)
+        ops.gemm_side_bf16(x, w, given, feedback, table, got, rows)
+        assert torch.equal(got, want), rows
+    assert (got[2] == 0).all() and not (got[0] == 0).all()
+    with pytest.raises(ValueError):
+        ops.gemm_side_bf16(torch.zeros(17, K, dtype=torch.bfloat16, device=gpu), w, torch.zeros(17, dtype=torch.int32, device=gpu), None, table,
+                           torch.zeros(17, N, dtype=torch.bfloat16, device=gpu), 17)
+
+
 def test_exact_gelu_against_plain(gpu):
     from bitwise_amd.csrc import ops
     x = torch.cat([torch.randn(7, 300, generator=torch.Generator().manual_seed(1)) * 4, torch.tensor([0.0, -1e-6, 1e-6, -80.0, 80.0]).repeat(7, 1)], 1)
