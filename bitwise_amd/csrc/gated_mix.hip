@@ -518,25 +518,44 @@ __device__ __forceinline__ void whole_norm_heads(const WholeNormArgs& a, const f
   const bool small = pairs <= 256 * PV;
   float acc = 0.0f;
   if (small) {
-    float u[PV], v[PV], wu[PV], wv[PV], c[PV], s[PV];
+    // (loads only, every index clamped into the row: all of them are asked for before the first is waited for)
+    float u[PV], v[PV], bu[PV], bv[PV], wu[PV], wv[PV], c[PV], s[PV];
 #pragma unroll
     for (int j = 0; j < PV; ++j) {
-      u[j] = v[j] = wu[j] = wv[j] = c[j] = s[j] = 0.0f;
-      if (256 * j < pairs) {                             // (scalar)
+      const Pair q = place(min(tid + 256 * j, pairs - 1));
+      const int e0 = q.h * a.dim + q.d0, e1 = q.h * a.dim + min(q.d1, a.dim - 1);
+      u[j] = p[e0];
+      v[j] = p[e1];
+      wu[j] = w[e0];
+      wv[j] = w[e1];
+    }
+    if (b != nullptr) {                                  // (scalar)
+#pragma unroll
+      for (int j = 0; j < PV; ++j) {
         const Pair q = place(min(tid + 256 * j, pairs - 1));
-        u[j] = element(q.h, q.d0);
-        v[j] = element(q.h, q.d1);
-        wu[j] = weight(q.h, q.d0);
-        wv[j] = weight(q.h, q.d1);
-        if (half > 0) {
-          c[j] = ct[min(q.r, half - 1)];
-          s[j] = st[min(q.r, half - 1)];
-        }
+        bu[j] = b[q.h * a.dim + q.d0];
+        bv[j] = b[q.h * a.dim + min(q.d1, a.dim - 1)];
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < PV; ++j) c[j] = s[j] = 0.0f;
+    if (half > 0) {                                      // (scalar)
+#pragma unroll
+      for (int j = 0; j < PV; ++j) {
+        const int r = min(place(min(tid + 256 * j, pairs - 1)).r, half - 1);
+        c[j] = ct[r];
+        s[j] = st[r];
       }
     }
 #pragma unroll
     for (int j = 0; j < PV; ++j) {
-      if (tid + 256 * j >= pairs) u[j] = v[j] = 0.0f;
+      if (b != nullptr) {
+        u[j] += bu[j];
+        v[j] += bv[j];
+      }
+      const bool in = tid + 256 * j < pairs;
+      if (!in) u[j] = 0.0f;
+      if (!in || place(min(tid + 256 * j, pairs - 1)).d1 >= a.dim) v[j] = 0.0f;      // (an odd head's last pair has one element)
       acc = fmaf(u[j], u[j], acc);
       acc = fmaf(v[j], v[j], acc);
     }
@@ -1029,16 +1048,21 @@ __global__ __launch_bounds__(256) void scaled_sum_norm_add_kernel(ScaledSumArgs 
   float z[MAXV], xo[MAXV], wp[MAXV];
   float acc = 0.0f;
   if (small) {
+    // (loads only, no branch between them: everything is asked for before the first value is waited for)
+    float yv[N][MAXV];
 #pragma unroll
     for (int j = 0; j < MAXV; ++j) {
       const int e = min(tid + 256 * j, a.dim - 1);
-      const bool in = 256 * j < a.dim;                   // (scalar)
-      z[j] = in ? value(e) : 0.0f;
-      xo[j] = in ? xr[e] : 0.0f;
-      wp[j] = in ? w[e] : 0.0f;
+#pragma unroll
+      for (int b = 0; b < N; ++b) yv[b][j] = a.y[b][(size_t)row * a.ldy[b] + e];
+      xo[j] = xr[e];
+      wp[j] = w[e];
     }
 #pragma unroll
     for (int j = 0; j < MAXV; ++j) {
+      z[j] = a.s[0] * yv[0][j];
+#pragma unroll
+      for (int b = 1; b < N; ++b) z[j] = fmaf(a.s[b], yv[b][j], z[j]);
       if (tid + 256 * j >= a.dim) z[j] = 0.0f;
       acc = fmaf(z[j], z[j], acc);
     }

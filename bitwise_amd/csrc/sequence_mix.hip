@@ -924,15 +924,16 @@ __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __res
     return BEHIND ? y * act(zv) : y;
   };
   const bool small = size <= 256 * GP_MAXV;
-  float v[GP_MAXV], zv[GP_MAXV];
+  float v[GP_MAXV], zv[GP_MAXV], wv[GP_MAXV];
   float acc = 0.0f;
   if (small) {
     float ov[GP_MAXV];
 #pragma unroll
     for (int j = 0; j < GP_MAXV; ++j) {
       const int e = min(tid + 256 * j, size - 1);
-      ov[j] = 256 * j < size ? orow[e] : 0.0f;
-      zv[j] = 256 * j < size ? zrow[e] : 0.0f;
+      ov[j] = orow[e];
+      zv[j] = zrow[e];
+      wv[j] = wr[e];
     }
 #pragma unroll
     for (int j = 0; j < GP_MAXV; ++j) {
@@ -953,7 +954,7 @@ __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __res
 #pragma unroll
     for (int j = 0; j < GP_MAXV; ++j) {
       const int e = tid + 256 * j;
-      if (e < size) store_act(dst + e, after(v[j], inv, wr[e], zv[j]));
+      if (e < size) store_act(dst + e, after(v[j], inv, wv[j], zv[j]));
     }
   } else {
     for (int e = tid; e < size; e += 256) store_act(dst + e, after(before(orow[e], zrow[e]), inv, wr[e], zrow[e]));
